@@ -117,6 +117,18 @@ int tg_model_load_weights_mem(tg_model *m, const void *image, size_t n);
 size_t tg_weight_file_bytes(const tg_config *cfg);
 void tg_model_destroy(tg_model *m);
 
+/* Any model the library knows by its folder: config.json ("architecture" selects the design, the other keys give its layers
+ * and sizes) and model.safetensors.  No counterpart in the reference, whose models are built in.
+ * Designs: "Madevik" (layers of gated linear attention and of latent attention, element-wise tanh norms, mixtures of experts).
+ * dtype: TG_DTYPE_BF16 (weights and matrix operands bfloat16; residual stream, norms, scores, routers and recurrent state
+ * fp32) or TG_DTYPE_F32 (everything fp32).  The model comes with its weights; an unknown design or mixer is
+ * TG_ERR_UNSUPPORTED_SHAPE, a missing tensor or a wrong shape TG_ERR_BAD_ARG. */
+enum { TG_DTYPE_BF16 = 0, TG_DTYPE_F32 = 1 };
+int tg_model_open(const char *dir, int dtype, tg_model **out);
+/* sizes of a model (of one opened from a folder: hidden_size, n_layers, n_vocab; the other fields are 0) */
+int tg_model_config(const tg_model *m, tg_config *out);
+const char *tg_model_architecture(const tg_model *m); /* "Gemma3", or config.json's name */
+
 /* What gemma::generate builds before the first forward (transformer.hpp:193-202): both RoPE
  * tables, the GeLU table, the DecodeState (KV caches + counters) and the logits buffer.
  * Like the reference's forward_* the tables are parameters: pass host arrays to use the caller's
@@ -125,6 +137,9 @@ void tg_model_destroy(tg_model *m);
 int tg_session_create(tg_model *m, const float *rope_cos, const float *rope_sin, const float *rope_sw_cos,
                       const float *rope_sw_sin, const float *gelu_table, float gelu_min, float gelu_max, int gelu_size,
                       tg_session **out);
+/* A session of any model with the library's own tables.  max_tokens: positions a session of a model opened from a folder can
+ * hold (its caches are allocated for them); Gemma sessions always hold n_pos. */
+int tg_session_open(tg_model *m, int max_tokens, tg_session **out);
 int tg_session_reset(tg_session *s); /* empty KV caches, position 0 */
 void tg_session_destroy(tg_session *s);
 int tg_session_position(const tg_session *s);
@@ -137,6 +152,13 @@ int tg_session_release_workspace(tg_session *s);
 int tg_forward_prefill(tg_session *s, const int32_t *ids, int n, float *logits, int32_t *argmax);
 /* gemma::forward_decode (transformer.hpp:75) + argmax */
 int tg_forward_decode(tg_session *s, int32_t id, float *logits, int32_t *argmax);
+/* The next n tokens of the session's sequence, at whatever position it is: a prompt may come in portions of any size.
+ * want[n_want]: ascending places among them whose logits go to logits (host, [n_want][n_vocab]); argmax (may be NULL): the pick
+ * behind the last one.  The result does not depend on how a sequence is cut into portions, beyond rounding.  Models opened
+ * from a folder run a portion of more than one token through their prefill kernels; a Gemma model does so for a whole
+ * prompt of which only the end is wanted, and takes anything else token by token.  Afterwards the token log
+ * (tg_session_read_ids) starts with this pick, as behind a prefill, unless the portion went token by token. */
+int tg_forward_tokens(tg_session *s, const int32_t *ids, int n, const int32_t *want, int n_want, float *logits, int32_t *argmax);
 /* greedy branch of gemma::generate (transformer.hpp:204-250) without tokenizer/EOS stop:
  * out_ids gets n_decode+1 ids (the first from the prefill logits); seconds are wall clock around
  * forward_prefill+argmax and around the decode loop (the tok/s definitions of gemma.cpp:53-58). */

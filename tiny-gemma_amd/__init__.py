@@ -14,7 +14,8 @@ import numpy as np
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libtinygemma_hip.so")
 CSRC = os.path.join(HERE, "csrc")
-SOURCES = ["tg_api.hip", "tg_gemv.hip", "tg_attn.hip", "tg_attn_prefill.hip", "tg_rows.hip", "tg_gemm_mfma.hip", "tg_sample.hip", "tg_repack.hip", "tg_probe.hip", "tg_decode_fused.hip"]
+SOURCES = ["tg_api.hip", "tg_gemv.hip", "tg_attn.hip", "tg_attn_prefill.hip", "tg_rows.hip", "tg_gemm_mfma.hip", "tg_sample.hip", "tg_repack.hip", "tg_probe.hip", "tg_decode_fused.hip",
+           "tg_linear.hip", "tg_gla.hip", "tg_latent.hip", "tg_moe.hip", "tg_net.hip"]
 HIPCC_FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",
                "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-function",
                # leading scalar kernel arguments are preloaded into SGPRs by the dispatcher (no s_load round trip)
@@ -23,6 +24,9 @@ HIPCC_FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",
 c_f32p = C.POINTER(C.c_float)
 c_i8p = C.POINTER(C.c_int8)
 c_i32p = C.POINTER(C.c_int32)
+
+
+DTYPES = {"bfloat16": 0, "float32": 1}
 
 
 class TgError(RuntimeError):
@@ -45,7 +49,7 @@ def build_library(verbose=False, changed_only=False):
     objdir = os.path.join(HERE, "build")
     os.makedirs(objdir, exist_ok=True)
     flags = [f for f in HIPCC_FLAGS if f != "-shared"]
-    headers = [os.path.join(CSRC, h) for h in ("tg_internal.h", "tg_gemv_parts.h", "tg_attn_decode.h")] + [os.path.join(HERE, "..", "include", "tinygemma_hip.h")]
+    headers = [os.path.join(CSRC, h) for h in sorted(os.listdir(CSRC)) if h.endswith(".h")] + [os.path.join(HERE, "..", "include", "tinygemma_hip.h")]
 
     def compile_one(src):
         path, obj = os.path.join(CSRC, src), os.path.join(objdir, src + ".o")
@@ -106,6 +110,12 @@ def lib():
     L.tg_model_destroy.argtypes = [C.c_void_p]
     L.tg_session_create.argtypes = [C.c_void_p, c_f32p, c_f32p, c_f32p, c_f32p, c_f32p, C.c_float, C.c_float, C.c_int,
                                     C.POINTER(C.c_void_p)]
+    L.tg_model_open.argtypes = [C.c_char_p, C.c_int, C.POINTER(C.c_void_p)]
+    L.tg_model_config.argtypes = [C.c_void_p, C.POINTER(Config)]
+    L.tg_model_architecture.argtypes = [C.c_void_p]
+    L.tg_model_architecture.restype = C.c_char_p
+    L.tg_session_open.argtypes = [C.c_void_p, C.c_int, C.POINTER(C.c_void_p)]
+    L.tg_forward_tokens.argtypes = [C.c_void_p, c_i32p, C.c_int, c_i32p, C.c_int, c_f32p, c_i32p]
     L.tg_session_reset.argtypes = [C.c_void_p]
     L.tg_session_release_workspace.argtypes = [C.c_void_p]
     L.tg_session_destroy.argtypes = [C.c_void_p]
@@ -282,6 +292,20 @@ class Transformer:
         self.h = C.c_void_p()
         check(lib().tg_model_create(C.byref(cfg), C.byref(self.h)))
 
+    @classmethod
+    def from_dir(cls, path, dtype="bfloat16"):
+        """A model from its folder (config.json + model.safetensors), in one of DTYPES."""
+        self = cls.__new__(cls)
+        self.h = C.c_void_p()
+        check(lib().tg_model_open(os.fsencode(path), DTYPES[dtype], C.byref(self.h)))
+        self.cfg = Config()
+        check(lib().tg_model_config(self.h, C.byref(self.cfg)))
+        return self
+
+    @property
+    def architecture(self):
+        return lib().tg_model_architecture(self.h).decode()
+
     def read_weights(self, path):
         check(lib().tg_model_load_weights(self.h, path.encode()))
 
@@ -294,6 +318,13 @@ class Transformer:
 
     def session(self, rope=None, rope_sw=None, gelu_table=None, gmin=-4.0, gmax=4.0, gsize=1024):
         return Session(self, rope, rope_sw, gelu_table, gmin, gmax, gsize)
+
+    def open_session(self, max_tokens):
+        """A session of any model with the library's own tables and room for max_tokens positions."""
+        s = Session.__new__(Session)
+        s.model, s.cfg, s.h = self, self.cfg, C.c_void_p()
+        check(lib().tg_session_open(self.h, int(max_tokens), C.byref(s.h)))
+        return s
 
     def free(self):
         if self.h:
@@ -340,6 +371,17 @@ class Session:
         logits = np.empty(self.cfg.n_vocab, np.float32) if want_logits else None
         arg = C.c_int32(-1)
         check(lib().tg_forward_decode(self.h, int(tok), _f(logits), C.byref(arg)))
+        return arg.value, logits
+
+    def forward(self, ids, want=None):
+        """The next tokens of the sequence, a portion of any size: (argmax behind the last, logits [len(want), vocab]).
+        want: ascending places among them (default: the last)."""
+        ids = np.ascontiguousarray(ids, np.int32)
+        want = np.ascontiguousarray([ids.size - 1] if want is None else want, np.int32)
+        logits = np.empty((want.size, self.cfg.n_vocab), np.float32)
+        arg = C.c_int32(-1)
+        check(lib().tg_forward_tokens(self.h, ids.ctypes.data_as(c_i32p), ids.size, want.ctypes.data_as(c_i32p), want.size, _f(logits),
+                                      C.byref(arg)))
         return arg.value, logits
 
     def greedy(self, prompt, n_decode):

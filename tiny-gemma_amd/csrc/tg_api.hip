@@ -14,6 +14,7 @@
 #include <map>
 
 #include "tg_internal.h"
+#include "tg_net.h"
 
 // ---------------------------------------------------------------------------------------------
 // library state and errors
@@ -229,6 +230,7 @@ struct tg_model {
 	float *rmsw = nullptr;
 	PackedMat lm;
 	std::vector<LayerDev> L;
+	TgNet *net = nullptr;   // a layer-list model opened from a folder; the fields above except cfg, loaded and the counts are then unused
 };
 
 namespace {
@@ -291,6 +293,8 @@ struct AttnPlanDev {
 
 struct tg_session {
 	tg_model *m = nullptr;
+	TgNetSeq *seq = nullptr;  // caches and states of a layer-list model (kc, vc and the other Gemma buffers below are then unused)
+	int capacity = 0;         // positions the session holds
 	float *cos_g = nullptr, *sin_g = nullptr, *cos_l = nullptr, *sin_l = nullptr;  // [n_pos][head_dim/2]
 	float *lut = nullptr;
 	float gmin = 0, geps = 0;
@@ -655,12 +659,44 @@ int tg_model_create(const tg_config *cfg, tg_model **out) {
 	return TG_OK;
 }
 
+static void model_free_weights(tg_model *m);
+
+int tg_model_open(const char *dir, int dtype, tg_model **out) {
+	if (int rc = ensure_init()) return rc;
+	if (!dir || !out) return tg_fail(TG_ERR_BAD_ARG, "null argument");
+	TgNet *net = nullptr;
+	if (int rc = tg_net_open(dir, dtype, g_n_cu, g_stream, &net)) return rc;
+	tg_model *m = new tg_model();
+	memset(&m->cfg, 0, sizeof(m->cfg));
+	const TgNetCfg &c = tg_net_cfg(net);
+	m->cfg.hidden_size = c.width;
+	m->cfg.n_layers = (int)c.layers.size();
+	m->cfg.n_vocab = c.vocab;
+	m->net = net;
+	m->loaded = true;
+	*out = m;
+	return TG_OK;
+}
+
+int tg_model_config(const tg_model *m, tg_config *out) {
+	if (!m || !out) return tg_fail(TG_ERR_BAD_ARG, "null argument");
+	*out = m->cfg;
+	return TG_OK;
+}
+
+const char *tg_model_architecture(const tg_model *m) {
+	if (!m) return "";
+	return m->net ? tg_net_cfg(m->net).arch.c_str() : "Gemma3";
+}
+
 static void model_free_weights(tg_model *m) {
 	(void)hipStreamSynchronize(g_stream);
 	if (m->wte) (void)hipFree(m->wte);
 	if (m->wte_scales) (void)hipFree(m->wte_scales);
 	if (m->rmsw) (void)hipFree(m->rmsw);
 	m->wte = nullptr; m->wte_scales = nullptr; m->rmsw = nullptr;
+	tg_net_free(m->net);
+	m->net = nullptr;
 	free_packed(&m->lm);
 	for (auto &L : m->L) {
 		free_packed(&L.qkv); free_packed(&L.o); free_packed(&L.ug); free_packed(&L.d);
@@ -688,8 +724,7 @@ void tg_model_destroy(tg_model *m) {
 // The file goes to the device as it is (the reference layout, transformer.hpp:122-160), in chunks through two
 // pinned staging buffers so that producing a chunk (file read or memcpy) overlaps the DMA of the previous one.
 // fill(dst, off, len) must produce bytes [off, off + len) of the file at dst.
-template <typename Fill>
-static int stage_image(uint8_t *d_raw, size_t n, Fill fill) {
+int tg_stage_image(uint8_t *d_raw, size_t n, const TgFill &fill) {
 	constexpr size_t CHUNK = (size_t)32 << 20;
 	void *pin[2] = {nullptr, nullptr};
 	hipEvent_t ev[2] = {nullptr, nullptr};
@@ -791,12 +826,13 @@ static int build_from_image(tg_model *m, const uint8_t *d_raw) {
 template <typename Fill>
 static int load_weights_impl(tg_model *m, Fill fill) {
 	// a session holds device pointers into the weights (and captured graphs bake them in): no reload under a live session
+	if (m->net) return tg_fail(TG_ERR_STATE, "a model opened from a folder has its weights");
 	if (m->n_sessions > 0) return tg_fail(TG_ERR_STATE, "the model has live sessions: destroy them before loading weights again");
 	model_free_weights(m);
 	const size_t n = tg_weight_file_bytes(&m->cfg);
 	uint8_t *d_raw = nullptr;
 	if (hipMalloc((void **)&d_raw, n) != hipSuccess) return tg_fail(TG_ERR_HIP, "hipMalloc of the file image failed");
-	int rc = stage_image(d_raw, n, fill);
+	int rc = tg_stage_image(d_raw, n, fill);
 	if (rc == TG_OK) rc = build_from_image(m, d_raw);
 	(void)hipStreamSynchronize(g_stream);
 	(void)hipFree(d_raw);
@@ -886,6 +922,7 @@ void tg_session_destroy(tg_session *s) {
 		if (p) (void)hipFree(p);
 	s->pf_plan.release();
 	s->pf_plan_local.release();
+	tg_net_seq_free(s->seq);
 	for (float *p : s->kc)
 		if (p) (void)hipFree(p);
 	for (float *p : s->vc)
@@ -903,6 +940,7 @@ int tg_session_create(tg_model *m, const float *rope_cos, const float *rope_sin,
                       tg_session **out) {
 	if (!m || !out) return tg_fail(TG_ERR_BAD_ARG, "null argument");
 	if (!m->loaded) return tg_fail(TG_ERR_STATE, "model has no weights");
+	if (m->net) return tg_fail(TG_ERR_BAD_ARG, "a model opened from a folder has no tables: tg_session_open");
 	if (gelu_size < 1 || !(gelu_max > gelu_min)) return tg_fail(TG_ERR_BAD_ARG, "bad GeLU table range");
 	const tg_config &c = m->cfg;
 	tg_session *s = new tg_session();
@@ -943,6 +981,7 @@ int tg_session_create(tg_model *m, const float *rope_cos, const float *rope_sin,
 		if (hipMalloc((void **)&s->kc[(size_t)l], bytes) != hipSuccess || hipMalloc((void **)&s->vc[(size_t)l], bytes) != hipSuccess)
 			return fail(tg_fail(TG_ERR_HIP, "KV cache allocation failed"));
 	}
+	s->capacity = c.n_pos;
 	s->tok_log_cap = c.n_pos + 1;
 #define TG_ALLOC(ptr, bytes)                                                                         \
 	if (hipMalloc((void **)&(ptr), (bytes)) != hipSuccess) return fail(tg_fail(TG_ERR_HIP, "session allocation failed: " #ptr))
@@ -976,6 +1015,7 @@ int tg_session_create(tg_model *m, const float *rope_cos, const float *rope_sin,
 int tg_session_reset(tg_session *s) {
 	if (!s) return tg_fail(TG_ERR_BAD_ARG, "null session");
 	const tg_config &c = s->m->cfg;
+	if (s->seq && !s->m->loaded) return tg_fail(TG_ERR_STATE, "the session's model has been destroyed");
 	TG_HIP(hipStreamSynchronize(g_stream));
 	for (size_t l = 0; l < s->kc.size(); l++) {
 		const size_t bytes = sizeof(float) * (size_t)s->max_pos[l] * c.head_dim;
@@ -983,7 +1023,10 @@ int tg_session_reset(tg_session *s) {
 		TG_HIP(hipMemset(s->vc[l], 0, bytes));
 	}
 	TG_HIP(hipMemset(s->ctr, 0, sizeof(int) * 8));
-	TG_HIP(hipMemset(s->xr, 0, sizeof(float) * (size_t)(2 * c.n_layers + 1) * c.hidden_size));
+	if (s->seq) {
+		if (int rc = tg_net_seq_reset(s->seq)) return rc;
+	} else
+		TG_HIP(hipMemset(s->xr, 0, sizeof(float) * (size_t)(2 * c.n_layers + 1) * c.hidden_size));
 	TG_HIP(hipDeviceSynchronize());
 	s->pos = s->bp_local = s->bp_global = s->steps = 0;
 	s->pick_pending = false;
@@ -993,6 +1036,41 @@ int tg_session_reset(tg_session *s) {
 }
 
 int tg_session_position(const tg_session *s) { return s ? s->pos : -1; }
+
+// A session of any model, with the library's own tables.
+int tg_session_open(tg_model *m, int max_tokens, tg_session **out) {
+	if (!m || !out) return tg_fail(TG_ERR_BAD_ARG, "null argument");
+	if (!m->loaded) return tg_fail(TG_ERR_STATE, "model has no weights");
+	if (!m->net) {
+		if (max_tokens > m->cfg.n_pos) return tg_fail(TG_ERR_BAD_ARG, "more positions than the model has");
+		return tg_session_create(m, nullptr, nullptr, nullptr, nullptr, nullptr, -4.0f, 4.0f, 1024, out);  // transformer.hpp:197
+	}
+	if (max_tokens < 1) return tg_fail(TG_ERR_BAD_ARG, "a session needs room for at least one token");
+	tg_session *s = new tg_session();
+	s->m = m;
+	s->capacity = max_tokens;
+	s->tok_log_cap = max_tokens + 1;
+	auto fail = [&](int code) {
+		tg_session_destroy(s);
+		return code;
+	};
+	if (int rc = tg_net_seq_create(m->net, max_tokens, &s->seq)) return fail(rc);
+	const size_t nb = (size_t)tg_net_head_blocks(m->net);
+	if (hipMalloc((void **)&s->logits, sizeof(float) * (size_t)tg_net_vocab_padded(m->net)) != hipSuccess ||
+	    hipMalloc((void **)&s->blk_val, sizeof(float) * nb) != hipSuccess || hipMalloc((void **)&s->blk_idx, sizeof(int) * nb) != hipSuccess ||
+	    hipMalloc((void **)&s->ctr, sizeof(int) * 8) != hipSuccess ||
+	    hipMalloc((void **)&s->tok_log, sizeof(int) * (size_t)s->tok_log_cap) != hipSuccess)
+		return fail(tg_fail(TG_ERR_HIP, "session allocation failed"));
+	if (int rc = tg_session_reset(s)) return fail(rc);
+	m->n_sessions += 1;
+	s->counted = true;
+	*out = s;
+	return TG_OK;
+}
+
+static TgHead head_of(tg_session *s) { return TgHead{s->logits, s->blk_val, s->blk_idx, s->ctr}; }
+// pairs of (maximum, index) that the head's launch leaves for the argmax
+static int head_blocks(const tg_session *s) { return s->m->net ? tg_net_head_blocks(s->m->net) : s->m->lm.ntiles; }
 
 // ---------------------------------------------------------------------------------------------
 // forward_decode: 5 launches per layer + 1 for the head
@@ -1342,8 +1420,19 @@ static void launch_lmhead(tg_session *s, const float *pend, const float *w_post,
 // The finishing launch of a pending greedy pick (see tg_session::pick_pending).
 static void flush_pick(tg_session *s) {
 	if (!s->pick_pending) return;
-	tg_launch_argmax_finish(s->blk_val, s->blk_idx, s->m->lm.ntiles, s->ctr, s->tok_log, 1, g_stream);
+	tg_launch_argmax_finish(s->blk_val, s->blk_idx, head_blocks(s), s->ctr, s->tok_log, 1, g_stream);
 	s->pick_pending = false;
+}
+
+// The end of a decode step: draw the token or take the argmax; may_stay: a greedy pick may stay pending.
+static void finish_pick(tg_session *s, bool may_stay) {
+	if (s->sampling)
+		tg_launch_minp(s->logits, s->m->cfg.n_vocab, s->s_minp, s->s_temp, s->randf, -1, s->rand_base, s->probs, s->seg, s->bsum, s->bmax,
+		               s->ctr, s->tok_log, 0, nullptr, g_stream);
+	else if (may_stay)
+		s->pick_pending = true;
+	else
+		tg_launch_argmax_finish(s->blk_val, s->blk_idx, head_blocks(s), s->ctr, s->tok_log, 1, g_stream);
 }
 
 // One decode step.  chain: the greedy pick may stay pending for the next step's first launch to finish (the caller
@@ -1353,8 +1442,19 @@ static int enqueue_decode_step(tg_session *s, StepProfile *prof, bool full_grid,
 	tg_model *m = s->m;
 	const tg_config &c = m->cfg;
 	const int L = c.n_layers, h = c.hidden_size;
-	if (s->pos >= c.n_pos) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
+	if (s->pos >= s->capacity) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
 	if (s->steps >= s->tok_log_cap) return tg_fail(TG_ERR_STATE, "token log is full");
+	if (m->net) {
+		if (prof || only) return tg_fail(TG_ERR_BAD_ARG, "per-launch profiling is for the Gemma models");
+		if (int rc = tg_net_step(s->seq, head_of(s), s->pos, !full_grid, s->pos)) return rc;
+		finish_pick(s, false);
+		TG_HIP(hipGetLastError());
+		s->pos += 1;
+		s->bp_local += 1;
+		s->bp_global += 1;
+		s->steps += 1;
+		return TG_OK;
+	}
 #define TG_DO(k, l, stmt)                                                        \
 	if (!only || (only->kclass == (k) && only->layer == (l)))                        \
 		for (int r_ = 0; r_ < (only ? only->repeat : 1); r_++) {                     \
@@ -1397,15 +1497,7 @@ static int enqueue_decode_step(tg_session *s, StepProfile *prof, bool full_grid,
 	TG_MARK(TG_KC_LMHEAD);
 	TG_DO(TG_KC_LMHEAD, 0, launch_lmhead(s, last_pend, m->L[(size_t)L - 1].mpost, s->xr + (size_t)(2 * L - 1) * h, s->xr + (size_t)(2 * L) * h));
 	TG_MARK(TG_KC_ARGMAX);
-	if (!only) {
-		if (s->sampling)
-			tg_launch_minp(s->logits, c.n_vocab, s->s_minp, s->s_temp, s->randf, -1, s->rand_base, s->probs, s->seg, s->bsum, s->bmax,
-			               s->ctr, s->tok_log, 0, nullptr, g_stream);
-		else if (chain && !prof && !full_grid)
-			s->pick_pending = true;
-		else
-			tg_launch_argmax_finish(s->blk_val, s->blk_idx, m->lm.ntiles, s->ctr, s->tok_log, 1, g_stream);
-	}
+	if (!only) finish_pick(s, chain && !prof && !full_grid);
 	TG_MARK(-1);
 #undef TG_MARK
 #undef TG_DO
@@ -1607,7 +1699,7 @@ static int decode_graph_mode_of(const tg_config &c) {
 	const double bytes = c.n_layers * (h * (qo + 2 * kv) + qo * h + 3 * h * f) + h * c.n_vocab;
 	return bytes / (5.0 * c.n_layers + 1.0) < 5e6 ? 2 : 0;
 }
-static int decode_graph_mode(const tg_session *s) { return decode_graph_mode_of(s->m->cfg); }
+static int decode_graph_mode(const tg_session *s) { return s->m->net ? 0 : decode_graph_mode_of(s->m->cfg); }
 
 int tg_plan_decode_launch_mode(const tg_config *cfg) {
 	if (!cfg || cfg->n_layers < 1) return -1;
@@ -1642,7 +1734,7 @@ int tg_decode_enqueue(tg_session *s, int n_steps) {
 			} else {
 				// a capture or a node update the runtime refuses leaves nothing enqueued: the session's counters go back
 				// and this and all later steps of the session are plain launches
-				if (s->pos >= c.n_pos) rc = tg_fail(TG_ERR_STATE, "context is full (n_pos)");
+				if (s->pos >= s->capacity) rc = tg_fail(TG_ERR_STATE, "context is full (n_pos)");
 				else if (s->steps >= s->tok_log_cap) rc = tg_fail(TG_ERR_STATE, "token log is full");
 				else {
 					// several steps per graph launch where the batch, the context and the token log have room for them and
@@ -1650,7 +1742,7 @@ int tg_decode_enqueue(tg_session *s, int n_steps) {
 					// (the first step of a batch goes out alone: the device would otherwise wait until the host has updated the
 					// nodes of four steps, 0.4 ms, before it sees the first launch)
 					int ns = 1;
-					if (i > 0 && n_steps - i >= TG_GRAPH_STEPS && s->pos + TG_GRAPH_STEPS <= c.n_pos && s->steps + TG_GRAPH_STEPS <= s->tok_log_cap) {
+					if (i > 0 && n_steps - i >= TG_GRAPH_STEPS && s->pos + TG_GRAPH_STEPS <= s->capacity && s->steps + TG_GRAPH_STEPS <= s->tok_log_cap) {
 						ns = TG_GRAPH_STEPS;
 						for (int k = 1; k < TG_GRAPH_STEPS; k++)
 							if (patched_graph_topology(s, k) != patched_graph_topology(s, 0)) ns = 1;
@@ -1699,7 +1791,7 @@ int tg_decode_enqueue(tg_session *s, int n_steps) {
 			s->graphs[key] = exec;
 			TG_HIP(hipGraphLaunch(exec, g_stream));
 		} else {
-			if (s->pos >= c.n_pos) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
+			if (s->pos >= s->capacity) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
 			if (s->steps >= s->tok_log_cap) return tg_fail(TG_ERR_STATE, "token log is full");
 			TG_HIP(hipGraphLaunch(it->second, g_stream));
 			s->pos += 1;
@@ -1782,6 +1874,11 @@ int tg_set_gemm_split(int enable) {
 }
 
 int tg_session_release_workspace(tg_session *s) {
+	if (s && s->seq) {
+		TG_HIP(hipStreamSynchronize(g_stream));
+		tg_net_seq_release_workspace(s->seq);
+		return TG_OK;
+	}
 	if (!s) return tg_fail(TG_ERR_BAD_ARG, "null session");
 	TG_HIP(hipStreamSynchronize(g_stream));
 	if (s->pf_ws) (void)hipFree(s->pf_ws);
@@ -2154,6 +2251,48 @@ int set_counters_after_prefill(tg_session *s, int n) {
 }
 }  // namespace
 
+// A portion of several tokens of a layer-list model, behind whatever the session holds.  The token log starts anew with
+// the portion's pick, as behind a prefill.
+static int net_extend(tg_session *s, const int32_t *ids, int n, const int32_t *want, int n_want, float *want_logits, float *logits, int32_t *argmax) {
+	if (int rc = tg_net_rows(s->seq, ids, n, s->pos, want, n_want, want_logits, head_of(s), g_keep_taps)) return rc;
+	s->pos += n;
+	s->bp_local = s->bp_global = s->pos;
+	s->steps = 1;
+	const int ctr[4] = {s->pos, s->pos, s->pos, 0};
+	TG_HIP(hipMemcpyAsync(s->ctr, ctr, sizeof(ctr), hipMemcpyHostToDevice, g_stream));
+	tg_launch_argmax_finish(s->blk_val, s->blk_idx, head_blocks(s), s->ctr, s->tok_log, 0, g_stream);
+	TG_HIP(hipGetLastError());
+	if (logits) TG_HIP(hipMemcpyAsync(logits, s->logits, sizeof(float) * (size_t)s->m->cfg.n_vocab, hipMemcpyDeviceToHost, g_stream));
+	int32_t tok = -1;
+	TG_HIP(hipMemcpyAsync(&tok, s->ctr + 4, sizeof(int), hipMemcpyDeviceToHost, g_stream));
+	TG_HIP(hipStreamSynchronize(g_stream));
+	if (argmax) *argmax = tok;
+	return TG_OK;
+}
+
+int tg_forward_tokens(tg_session *s, const int32_t *ids, int n, const int32_t *want, int n_want, float *logits, int32_t *argmax) {
+	if (!s || !ids || n_want < 0 || (n_want > 0 && (!want || !logits))) return tg_fail(TG_ERR_BAD_ARG, "bad argument");
+	if (int rc = session_usable(s)) return rc;
+	const tg_config &c = s->m->cfg;
+	if (n < 1) return tg_fail(TG_ERR_BAD_ARG, "empty portion");
+	for (int i = 0; i < n; i++)
+		if (ids[i] < 0 || ids[i] >= c.n_vocab) return tg_fail(TG_ERR_BAD_ARG, "token id outside the vocabulary");
+	for (int i = 0; i < n_want; i++)
+		if (want[i] < 0 || want[i] >= n || (i > 0 && want[i] <= want[i - 1])) return tg_fail(TG_ERR_BAD_ARG, "wanted places must ascend within the portion");
+	if (s->pos + n > s->capacity) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
+	flush_pick(s);
+	if (s->m->net && n > 1) return net_extend(s, ids, n, want, n_want, logits, nullptr, argmax);
+	// a whole prompt of which only the end is wanted is a prefill; anything else of a Gemma model goes token by token
+	if (!s->m->net && s->pos == 0 && n > 1 && (n_want == 0 || (n_want == 1 && want[0] == n - 1)))
+		return tg_forward_prefill(s, ids, n, n_want ? logits : nullptr, argmax);
+	for (int i = 0, w = 0; i < n; i++) {
+		const bool is = w < n_want && want[w] == i;
+		if (int rc = tg_forward_decode(s, ids[i], is ? logits + (size_t)w * c.n_vocab : nullptr, argmax)) return rc;
+		w += is ? 1 : 0;
+	}
+	return TG_OK;
+}
+
 int tg_forward_prefill(tg_session *s, const int32_t *ids, int n, float *logits, int32_t *argmax) {
 	if (!s || !ids) return tg_fail(TG_ERR_BAD_ARG, "null argument");
 	if (int rc = session_usable(s)) return rc;
@@ -2161,7 +2300,8 @@ int tg_forward_prefill(tg_session *s, const int32_t *ids, int n, float *logits, 
 	const tg_config &c = m->cfg;
 	if (n < 1) return tg_fail(TG_ERR_BAD_ARG, "empty prompt");
 	if (s->pos != 0) return tg_fail(TG_ERR_STATE, "prefill needs an empty session (decode.hpp:78-79)");
-	if (n > c.n_pos) return tg_fail(TG_ERR_STATE, "prompt longer than n_pos");
+	if (n > s->capacity) return tg_fail(TG_ERR_STATE, "prompt longer than n_pos");
+	if (m->net) return net_extend(s, ids, n, nullptr, 0, nullptr, logits, argmax);
 	const int L = c.n_layers, h = c.hidden_size;
 	const size_t S = (size_t)n;
 	PrefillCtx p;
@@ -2208,6 +2348,7 @@ int tg_forward_prefill(tg_session *s, const int32_t *ids, int n, float *logits, 
 // block level (parity checks of one modules::attention / mlp / lm_head call at a time)
 // ---------------------------------------------------------------------------------------------
 static int block_args_ok(tg_session *s, int layer, const float *x, int rows) {
+	if (s && s->seq) return tg_fail(TG_ERR_BAD_ARG, "block-level calls are for the Gemma models");
 	if (int rc = session_usable(s)) return rc;
 	const tg_config &c = s->m->cfg;
 	if (!x || rows < 1 || layer < 0 || layer >= c.n_layers) return tg_fail(TG_ERR_BAD_ARG, "bad argument");
@@ -2348,9 +2489,8 @@ namespace {
 // scratch of the sampler + room for n draws, uploaded from the host
 int sampler_prepare(tg_session *s, const float *randf, int n) {
 	const tg_config &c = s->m->cfg;
-	if (c.n_vocab % 1024 != 0) return tg_fail(TG_ERR_UNSUPPORTED_SHAPE, "sampler needs a vocabulary that is a multiple of 1024");
 	if (!s->probs) {
-		TG_HIP(hipMalloc((void **)&s->probs, sizeof(float) * (size_t)c.n_vocab));
+		TG_HIP(hipMalloc((void **)&s->probs, sizeof(float) * tg_minp_padded(c.n_vocab)));
 		TG_HIP(hipMalloc((void **)&s->seg, sizeof(float) * tg_minp_segments(c.n_vocab)));
 		TG_HIP(hipMalloc((void **)&s->bsum, sizeof(float) * tg_minp_blocks(c.n_vocab)));
 		TG_HIP(hipMalloc((void **)&s->bmax, sizeof(float) * tg_minp_blocks(c.n_vocab)));
@@ -2450,6 +2590,7 @@ int tg_session_tap(tg_session *s, int b, float *out, int rows) {
 	if (b < 0 || b > 2 * c.n_layers) return tg_fail(TG_ERR_BAD_ARG, "no such block");
 	TG_HIP(hipStreamSynchronize(g_stream));
 	if (int rc = fused_check(s)) return rc;
+	if (s->seq) return s->m->loaded ? tg_net_tap(s->seq, b, out, rows) : tg_fail(TG_ERR_STATE, "the session's model has been destroyed");
 	const size_t h = (size_t)c.hidden_size;
 	if (s->taps) {
 		if (rows != s->tap_rows)
@@ -2466,6 +2607,7 @@ int tg_session_kv(tg_session *s, int layer, float *keys, float *values, int *pos
 	if (!s) return tg_fail(TG_ERR_BAD_ARG, "null session");
 	const tg_config &c = s->m->cfg;
 	if (layer < 0 || layer >= c.n_layers) return tg_fail(TG_ERR_BAD_ARG, "no such layer");
+	if (s->seq) return tg_fail(TG_ERR_BAD_ARG, "the session's model has no key/value cache");
 	TG_HIP(hipStreamSynchronize(g_stream));
 	if (int rc = fused_check(s)) return rc;
 	const size_t bytes = sizeof(float) * (size_t)s->max_pos[(size_t)layer] * c.head_dim;

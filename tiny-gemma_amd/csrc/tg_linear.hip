@@ -1,0 +1,502 @@
+// Products with bfloat16 or float32 weights: packing, one-row products (decode) and tiled products (prefill).
+// Layout and number formats: tg_linear.h.
+
+#include "tg_linear.h"
+
+namespace {
+
+// ---- packing (load time) -----------------------------------------------------------------------------------------------
+__device__ __forceinline__ float pack_read(const TgPack &p, int i, int j) {
+	const int gi = i / p.gp, ri = i - gi * p.gp, gj = j / p.kgp, rj = j - gj * p.kgp;
+	const int r = gi * p.g + ri, c = gj * p.kg + rj;
+	if (ri >= p.g || rj >= p.kg || r >= p.rsrc || c >= p.ksrc) return 0.0f;
+	const size_t at = p.transpose ? (size_t)c * p.src_ld + r : (size_t)r * p.src_ld + c;
+	return p.src_f32 ? ((const float *)p.src)[at] : (float)((const __bf16 *)p.src)[at];
+}
+
+template <class TR>
+__global__ __launch_bounds__(256) void pack_kernel(typename TR::T *dst, int k, TgPack p) {
+	const long long total = (long long)p.rows * p.cols;
+	for (long long e = (long long)blockIdx.x * 256 + threadIdx.x; e < total; e += (long long)gridDim.x * 256) {
+		const int i = (int)(e / p.cols), j = (int)(e - (long long)i * p.cols);
+		const int row = (i / 16) * 16 * p.frag_step + p.frag_off * 16 + i % 16;
+		const size_t frag = (size_t)(row / 16) * (k / TR::KF) + j / TR::KF;
+		const int lane = row % 16 + 16 * ((j % TR::KF) / TR::KV);
+		dst[frag * 64 * TR::KV + lane * TR::KV + j % TR::KV] = (typename TR::T)pack_read(p, i, j);
+	}
+}
+
+__global__ __launch_bounds__(256) void unpack_f32_kernel(float *dst, int ld, TgPack p) {
+	const long long total = (long long)p.rows * p.cols;
+	for (long long e = (long long)blockIdx.x * 256 + threadIdx.x; e < total; e += (long long)gridDim.x * 256) {
+		const int i = (int)(e / p.cols), j = (int)(e - (long long)i * p.cols);
+		dst[(size_t)i * ld + j] = pack_read(p, i, j);
+	}
+}
+
+// ---- one-row products ----------------------------------------------------------------------------------------------------
+constexpr int NT = 256;
+
+// Experts by rank: expert e is chosen when fewer than `top` experts have a larger choice score (or the same one and a
+// lower index).  s_sel / s_val (LDS, top entries): the chosen experts in rank order and their scores.
+__device__ __forceinline__ void choose_experts(const float *logits, const float *correction, int E, int top, float *s_choice, int *s_sel,
+                                               float *s_val) {
+	for (int e = threadIdx.x; e < E; e += NT) s_choice[e] = tg_sigmoid(logits[e]) + correction[e];
+	__syncthreads();
+	for (int e = threadIdx.x; e < E; e += NT) {
+		const float c = s_choice[e];
+		int rank = 0;
+		for (int o = 0; o < E; o++) {
+			const float co = s_choice[o];
+			rank += (co > c || (co == c && o < e)) ? 1 : 0;
+		}
+		if (rank < top) {
+			s_sel[rank] = e;
+			s_val[rank] = tg_sigmoid(logits[e]);
+		}
+	}
+	__syncthreads();
+}
+
+// NTL: tiles per wave (2: a gate|up pair); KW: waves that share a tile's K (4), or 1: every wave has tiles of its own;
+// U: fragments in flight per lane and tile
+template <class TR, int PRO, int EPI, int NTL, int KW, int U>
+__global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
+	typedef typename TR::T T;
+	typedef typename TR::Frag Frag;
+	extern __shared__ __align__(16) unsigned char smem[];
+	T *xs = reinterpret_cast<T *>(smem);
+	__shared__ float s_red[4][NTL * 16];
+	__shared__ float s_misc[64];
+	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int part = blockIdx.y, z = blockIdx.z;
+	const int per = (p.kfrags + p.ksplit - 1) / p.ksplit;
+	const int kb = part * per, ke = min(p.kfrags, kb + per), nk = max(ke - kb, 0);
+	const int k0 = kb * TR::KF, kn = nk * TR::KF;
+
+	int zw = z;
+	if constexpr (PRO == TG_VP_EXPERT) {
+		// LDS: choice scores [experts] | selected [top] | their scores [top] behind the vector
+		float *s_choice = reinterpret_cast<float *>(smem + sizeof(T) * (size_t)(per + KW * U) * TR::KF);
+		int *s_sel = reinterpret_cast<int *>(s_choice + p.experts);
+		float *s_val = reinterpret_cast<float *>(s_sel + p.top);
+		choose_experts(p.logits, p.correction, p.experts, p.top, s_choice, s_sel, s_val);
+		zw = s_sel[z];
+		if (blockIdx.x == 0 && part == 0 && z == 0) {
+			for (int k = tid; k < p.top; k += NT) {
+				float sum = 0.0f;
+				for (int o = 0; o < p.top; o++) sum += s_val[o];
+				p.sel[k] = s_sel[k];
+				p.wgt[k] = s_val[k] / (sum + 1e-20f) * p.rscale;
+			}
+		}
+	}
+	if constexpr (EPI == TG_VE_WEIGHTED) zw = p.sel[z];
+
+	const int group = KW == 4 ? (int)blockIdx.x : (int)blockIdx.x * 4 + w;  // tile group of this wave
+	const bool live = group * NTL < p.ntiles;
+	const int tile0 = live ? group * NTL : 0;
+	const Frag *W = reinterpret_cast<const Frag *>(p.W) + ((size_t)zw * p.zfrags + (size_t)tile0 * p.kfrags) * 64 + lane;
+	const int step = KW, kf0 = kb + (KW == 4 ? w : 0);
+	Frag wr[NTL][U];
+	auto load = [&](int kf) {
+#pragma unroll
+		for (int u = 0; u < U; u++) {
+			const int kk = kf + u * step, kc = min(kk, p.kfrags - 1);
+#pragma unroll
+			for (int t = 0; t < NTL; t++) wr[t][u] = W[((size_t)t * p.kfrags + kc) * 64];
+		}
+	};
+
+	// the vector's prologue: elements [k0, k0 + kn), then zeros that the surplus steps of the last round multiply
+	if constexpr (PRO == TG_VP_PLAIN || PRO == TG_VP_EXPERT) {
+		load(kf0);
+		const float *x = p.x + (PRO == TG_VP_PLAIN ? (size_t)z * p.x_zstride : 0);
+		for (int j = tid; j < kn; j += NT) xs[j] = (T)x[k0 + j];
+	} else if constexpr (PRO == TG_VP_DYT) {
+		load(kf0);
+		int row = 0;
+		if (p.embed) {
+			row = p.ctr[4];
+			row = row < 0 ? 0 : (row >= p.vocab ? p.vocab - 1 : row);
+		}
+		for (int j = tid; j < kn; j += NT) {
+			const int c = k0 + j, cc = c < p.width ? c : 0;
+			float x = p.embed ? (float)((const __bf16 *)p.embed)[(size_t)row * p.embed_ld + cc] : p.x[cc];
+			float add = 0.0f;
+			for (int q = 0; q < p.nparts; q++) add += p.pend[(size_t)q * p.pend_stride + cc];
+			if (p.nparts) x = x + p.mult * add;
+			const float h = tanhf(p.alpha * x) * p.nw[cc] + p.nb[cc];
+			const bool in = c < p.width;
+			xs[j] = (T)(in ? h : 0.0f);
+			if (blockIdx.x == 0 && z == 0) {
+				if (p.x_out) p.x_out[c] = in ? x : 0.0f;
+				if (p.h_out) p.h_out[c] = in ? h : 0.0f;
+			}
+		}
+	} else if constexpr (PRO == TG_VP_HEADNORM) {
+		load(kf0);
+		// head by head, a wave each: sum of squares, then the head's elements that lie in this part of K
+		const int h_lo = k0 / p.vdimp, h_hi = min((k0 + kn - 1) / p.vdimp, p.heads16 - 1);
+		for (int j = tid; j < kn; j += NT)
+			if ((k0 + j) / p.vdimp >= p.heads16) xs[j] = (T)0.0f;
+		for (int a = h_lo + w; a <= h_hi; a += 4) {
+			const float *o = p.x + (size_t)a * p.vdimp, *g = p.gate + (size_t)a * p.vdimp;
+			float ss = 0.0f;
+			for (int v = lane; v < p.vdim; v += 64) ss = fmaf(o[v], o[v], ss);
+			ss = tg_wave_sum(ss);
+			const float inv = 1.0f / sqrtf(ss / (float)p.vdim + p.eps);
+			for (int v = lane; v < p.vdimp; v += 64) {
+				const int j = a * p.vdimp + v - k0;
+				const bool in = v < p.vdim;
+				const int vc = in ? v : 0;
+				const float r = o[vc] * inv * p.nw[vc] * tg_silu(g[vc]);
+				if (j >= 0 && j < kn) xs[j] = (T)(in ? r : 0.0f);
+			}
+		}
+	} else {  // MERGE
+		load(kf0);
+		float m = -INFINITY;
+		for (int b = 0; b < p.nmerge; b++) m = fmaxf(m, p.part_ml[((size_t)b * p.heads16 + z) * 2]);
+		float l = 0.0f;
+		for (int b = 0; b < p.nmerge; b++) {
+			const float *ml = p.part_ml + ((size_t)b * p.heads16 + z) * 2;
+			const float f = expf(ml[0] - m);
+			l += f * ml[1];
+			if (tid == 0) s_misc[b] = f;
+		}
+		__syncthreads();
+		const float inv = 1.0f / l;
+		for (int j = tid; j < kn; j += NT) {
+			float a = 0.0f;
+			for (int b = 0; b < p.nmerge; b++) a = fmaf(s_misc[b], p.part_acc[((size_t)b * p.heads16 + z) * p.x_zstride + k0 + j], a);
+			xs[j] = (T)(a * inv);
+		}
+	}
+	for (int j = kn + tid; j < kn + KW * U * TR::KF; j += NT) xs[j] = (T)0.0f;
+	__syncthreads();
+
+	f32x4_t acc[NTL];
+#pragma unroll
+	for (int t = 0; t < NTL; t++) acc[t] = f32x4_t{0, 0, 0, 0};
+	const T *xl = xs + (lane >> 4) * TR::KV;
+	for (int kf = kf0; kf < ke; kf += step * U) {
+		Frag cur[NTL][U];
+#pragma unroll
+		for (int t = 0; t < NTL; t++)
+#pragma unroll
+			for (int u = 0; u < U; u++) cur[t][u] = wr[t][u];
+		if (kf + step * U < ke) load(kf + step * U);
+#pragma unroll
+		for (int u = 0; u < U; u++) {
+			const Frag xf = *reinterpret_cast<const Frag *>(xl + (size_t)(kf + u * step - kb) * TR::KF);
+#pragma unroll
+			for (int t = 0; t < NTL; t++) acc[t] = TR::mma(xf, cur[t][u], acc[t]);
+		}
+	}
+	// all 16 rows of the first operand are the vector: element 0 of lane l is output l % 16 of the tile
+	if constexpr (KW == 4) {
+		if (lane < 16) {
+#pragma unroll
+			for (int t = 0; t < NTL; t++) s_red[w][t * 16 + lane] = acc[t][0];
+		}
+		__syncthreads();
+		if (tid < 16) {
+			float v[NTL];
+#pragma unroll
+			for (int t = 0; t < NTL; t++) v[t] = (s_red[0][t * 16 + tid] + s_red[1][t * 16 + tid]) + (s_red[2][t * 16 + tid] + s_red[3][t * 16 + tid]);
+			float *y = p.y + (size_t)part * p.part_stride + (size_t)z * p.y_zstride;
+			if constexpr (EPI == TG_VE_SWIGLU) {
+				y[group * 16 + tid] = tg_silu(v[0]) * v[NTL - 1];
+			} else {
+				float r = v[0];
+				if constexpr (EPI == TG_VE_GATE) r *= tg_sigmoid(p.gate[z]);
+				if constexpr (EPI == TG_VE_WEIGHTED) r *= p.wgt[z];
+				y[group * 16 + tid] = r;
+				if constexpr (EPI == TG_VE_LOGITS) {
+					float bv = group * 16 + tid < p.nout ? r : -INFINITY;
+					int bi = group * 16 + tid;
+#pragma unroll
+					for (int o = 8; o > 0; o >>= 1) {
+						const float ov = __shfl_xor(bv, o, 16);
+						const int oi = __shfl_xor(bi, o, 16);
+						if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+					}
+					if (tid == 0) { p.blk_val[blockIdx.x] = bv; p.blk_idx[blockIdx.x] = bi; }
+				}
+			}
+		}
+	} else {
+		if (lane < 16) {
+			const float r = acc[0][0];
+			const int o = group * 16 + lane;
+			if (live) p.y[(size_t)z * p.y_zstride + o] = r;
+			if constexpr (EPI == TG_VE_LOGITS) s_red[w][lane] = live && o < p.nout ? r : -INFINITY;
+		}
+		if constexpr (EPI == TG_VE_LOGITS) {
+			__syncthreads();
+			if (tid < 64) {
+				float bv = s_red[tid >> 4][tid & 15];
+				int bi = (int)blockIdx.x * 64 + tid;
+#pragma unroll
+				for (int o = 32; o > 0; o >>= 1) {
+					const float ov = __shfl_xor(bv, o, 64);
+					const int oi = __shfl_xor(bi, o, 64);
+					if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+				}
+				if (tid == 0) { p.blk_val[blockIdx.x] = bv; p.blk_idx[blockIdx.x] = bi; }
+			}
+		}
+	}
+}
+
+bool vec_wide(const TgVec &v, int epi) { return (epi == TG_VE_STORE || epi == TG_VE_LOGITS) && v.ksplit == 1 && v.nz == 1 && v.ntiles >= 2048; }
+
+template <class TR, int PRO, int EPI>
+void launch_vec_t(const TgVec &v, hipStream_t s) {
+	constexpr int NTL = EPI == TG_VE_SWIGLU ? 2 : 1;
+	const int per = (v.kfrags + v.ksplit - 1) / v.ksplit;
+	const unsigned bx = (unsigned)tg_vec_blocks(v, EPI);
+	auto lds = [&](int pad) {
+		size_t b = sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF;
+		if (PRO == TG_VP_EXPERT) b += sizeof(float) * (size_t)(v.experts + 2 * v.top);
+		return b;
+	};
+	if constexpr (EPI == TG_VE_STORE || EPI == TG_VE_LOGITS) {
+		if (vec_wide(v, EPI)) {
+			hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, 1, 1, 8>), dim3(bx, 1, 1), dim3(NT), lds(8), s, v);
+			return;
+		}
+	}
+	hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 4>), dim3(bx, (unsigned)v.ksplit, (unsigned)v.nz), dim3(NT), lds(16), s, v);
+}
+
+template <class TR>
+void launch_vec_dt(const TgVec &v, int pro, int epi, hipStream_t s) {
+	if (pro == TG_VP_PLAIN && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_PLAIN, TG_VE_STORE>(v, s);
+	else if (pro == TG_VP_DYT && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_DYT, TG_VE_STORE>(v, s);
+	else if (pro == TG_VP_DYT && epi == TG_VE_LOGITS) launch_vec_t<TR, TG_VP_DYT, TG_VE_LOGITS>(v, s);
+	else if (pro == TG_VP_HEADNORM) launch_vec_t<TR, TG_VP_HEADNORM, TG_VE_STORE>(v, s);
+	else if (pro == TG_VP_MERGE) launch_vec_t<TR, TG_VP_MERGE, TG_VE_GATE>(v, s);
+	else if (pro == TG_VP_EXPERT) launch_vec_t<TR, TG_VP_EXPERT, TG_VE_SWIGLU>(v, s);
+	else if (pro == TG_VP_PLAIN && epi == TG_VE_GATE) launch_vec_t<TR, TG_VP_PLAIN, TG_VE_GATE>(v, s);
+	else launch_vec_t<TR, TG_VP_PLAIN, TG_VE_WEIGHTED>(v, s);
+}
+
+// ---- tiled products --------------------------------------------------------------------------------------------------------
+// A workgroup computes BM x BN with WM x WN waves of (16 MI) x (16 NI) each.  K advances by two fragments (128 bytes of a
+// row) per stage: both operands go global -> registers -> LDS in fragment order, the next stage's loads in flight during
+// the matrix instructions of this one, one LDS-only barrier per stage.
+template <class TR, int EPI, int WM, int WN, int MI, int NI, bool GROUPED>
+__global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
+	typedef typename TR::T T;
+	typedef typename TR::Frag Frag;
+	constexpr int BM = WM * MI * 16, BN = WN * NI * 16;
+	constexpr int AF = BM / 16, BF = BN / 16, NF = 2 * (AF + BF), PW = NF / 4;  // fragments per stage, per wave
+	static_assert(NF % 4 == 0 && WM * WN == 4, "four waves share a stage's fragments");
+	__shared__ __align__(16) Frag lds[2][NF * 64];
+	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int ntn = (g.N + BN - 1) / BN;
+
+	// Workgroups go to the 8 XCDs in turn: give each XCD a contiguous run of the tile order, so that the workgroups it
+	// runs side by side share weight tiles and activation rows in its L2.  (A list of groups launches as many workgroups
+	// as it could have tiles: the run lengths come from the tiles it has.)
+	const int mrows = EPI == TG_GE_TRANS ? g.rows_out : g.M;
+	const int ntm = GROUPED ? *g.ntiles : (mrows + BM - 1) / BM;
+	int b;
+	{
+		const int total = ntm * ntn, q = total >> 3, r = total & 7, x = (int)blockIdx.x & 7, i = (int)blockIdx.x >> 3;
+		if (i >= q + (x < r ? 1 : 0)) return;
+		b = x * q + min(x, r) + i;
+	}
+	int m0, m1, tn;
+	const Frag *W = reinterpret_cast<const Frag *>(g.W);
+	if constexpr (GROUPED) {
+		const int t = b / ntn;
+		tn = b - t * ntn;
+		const int4 tile = g.tiles[t];
+		m0 = tile.y;
+		m1 = tile.z;
+		W += (size_t)tile.x * g.group_frags * 64;
+	} else {
+		tn = b / ntm;
+		m0 = (b - tn * ntm) * BM;
+		m1 = g.M;
+	}
+	const int kfr = g.K / TR::KF, nst = kfr / 2, nfr = g.N / 16;
+
+	// this wave's fragments of a stage: f = w * PW + i; the first 2 AF are A (row tile f / 2, k half f % 2), then B
+	const unsigned char *src[PW];
+	int adv[PW];
+#pragma unroll
+	for (int i = 0; i < PW; i++) {
+		const int f = w * PW + i;
+		if (f < 2 * AF) {
+			int r = min(m0 + (f >> 1) * 16 + (lane & 15), m1 - 1);
+			if (g.row_src) r = g.row_src[r];
+			src[i] = reinterpret_cast<const unsigned char *>(g.A) + ((size_t)r * g.lda + (f & 1) * TR::KF) * sizeof(T) + (lane >> 4) * 16;
+			adv[i] = 128;
+		} else {
+			const int fb = f - 2 * AF, nf = min(tn * BF + (fb >> 1), nfr - 1);
+			src[i] = reinterpret_cast<const unsigned char *>(W + ((size_t)nf * kfr + (fb & 1)) * 64 + lane);
+			adv[i] = 2048;
+		}
+	}
+	Frag st[PW];
+	auto fetch = [&](int s) {
+#pragma unroll
+		for (int i = 0; i < PW; i++) st[i] = *reinterpret_cast<const Frag *>(src[i] + (size_t)s * adv[i]);
+	};
+	auto put = [&](int buf) {
+#pragma unroll
+		for (int i = 0; i < PW; i++) lds[buf][(w * PW + i) * 64 + lane] = st[i];
+	};
+	const int wm = w / WN, wn = w - wm * WN;
+	f32x4_t acc[MI][NI];
+#pragma unroll
+	for (int i = 0; i < MI; i++)
+#pragma unroll
+		for (int j = 0; j < NI; j++) acc[i][j] = f32x4_t{0, 0, 0, 0};
+
+	fetch(0);
+	put(0);
+	tg_lds_barrier();
+	for (int s = 0; s < nst; s++) {
+		const int buf = s & 1;
+		fetch(s + 1 < nst ? s + 1 : s);
+#pragma unroll
+		for (int kh = 0; kh < 2; kh++) {
+			Frag a[MI], bb[NI];
+#pragma unroll
+			for (int i = 0; i < MI; i++) a[i] = lds[buf][((wm * MI + i) * 2 + kh) * 64 + lane];
+#pragma unroll
+			for (int j = 0; j < NI; j++) bb[j] = lds[buf][(2 * AF + (wn * NI + j) * 2 + kh) * 64 + lane];
+#pragma unroll
+			for (int i = 0; i < MI; i++)
+#pragma unroll
+				for (int j = 0; j < NI; j++) acc[i][j] = EPI == TG_GE_TRANS ? TR::mma(a[i], bb[j], acc[i][j]) : TR::mma(bb[j], a[i], acc[i][j]);
+		}
+		put(buf ^ 1);
+		tg_lds_barrier();
+	}
+
+	const int lr = lane & 15, lg = lane >> 4;
+	if constexpr (EPI == TG_GE_TRANS) {
+		// lane: column n = lr, rows m = 4 lg + i, four consecutive keys of a 32-key (bf16) or 16-key (fp32) operand block
+#pragma unroll
+		for (int i = 0; i < MI; i++)
+#pragma unroll
+			for (int j = 0; j < NI; j++) {
+				const int n = tn * BN + (wn * NI + j) * 16 + lr, m = m0 + (wm * MI + i) * 16 + 4 * lg;
+				if (n >= g.N || m >= g.rows_out) continue;
+				int at = m;
+				if constexpr (TR::DT == TG_DT_BF16) at = (m & ~31) + lg * 8 + ((m >> 4) & 1) * 4;
+				tg_store4((T *)g.C + (size_t)n * g.ldc + at, acc[i][j]);
+			}
+	} else {
+		// lane: row m = lr, columns n = 4 lg + i
+#pragma unroll
+		for (int i = 0; i < MI; i++) {
+			const int m = m0 + (wm * MI + i) * 16 + lr;
+			if (m >= m1) continue;
+			if constexpr (EPI == TG_GE_SWIGLU) {
+#pragma unroll
+				for (int j = 0; j < NI; j += 2) {
+					const int n = tn * BN + (wn * NI + j) * 16;  // of the interleaved rows
+					if (n >= g.N) continue;
+					f32x4_t r;
+#pragma unroll
+					for (int e = 0; e < 4; e++) r[e] = tg_silu(acc[i][j][e]) * acc[i][j + 1][e];
+					tg_store4((T *)g.C + (size_t)m * g.ldc + n / 2 + 4 * lg, r);
+				}
+			} else {
+#pragma unroll
+				for (int j = 0; j < NI; j++) {
+					const int n = tn * BN + (wn * NI + j) * 16 + 4 * lg;
+					if (n >= g.N) continue;
+					if constexpr (EPI == TG_GE_STORE) {
+						if (n < g.n_split) tg_store4((T *)g.C + (size_t)m * g.ldc + n, acc[i][j]);
+						else tg_store4(g.C2 + (size_t)m * g.ldc2 + n - g.n_split, acc[i][j]);
+					} else if constexpr (EPI == TG_GE_F32) {
+						tg_store4(g.C2 + (size_t)m * g.ldc2 + n, acc[i][j]);
+					} else {
+						float *c = g.C2 + (size_t)m * g.ldc2 + n;
+						f32x4_t x = tg_load4(c);
+#pragma unroll
+						for (int e = 0; e < 4; e++) x[e] = x[e] + g.mult * acc[i][j][e];
+						tg_store4(c, x);
+					}
+				}
+			}
+		}
+	}
+}
+
+template <class TR, int EPI>
+void launch_linear_t(const TgGemm &g, hipStream_t s) {
+	if (g.tiles) {
+		if constexpr (EPI == TG_GE_STORE || EPI == TG_GE_SWIGLU) {
+			const unsigned grid = (unsigned)g.max_tiles * (unsigned)((g.N + 127) / 128);
+			if (g.tile_rows == 128)
+				hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 4, 4, true>), dim3(grid), dim3(256), 0, s, g);
+			else
+				hipLaunchKernelGGL((linear_kernel<TR, EPI, 1, 4, 2, 2, true>), dim3(grid), dim3(256), 0, s, g);
+		}
+		return;
+	}
+	const int ntn = (g.N + 127) / 128, rows = EPI == TG_GE_TRANS ? g.rows_out : g.M;
+	// 128-row tiles from the point where they fill the device's compute units once
+	if ((rows + 127) / 128 * ntn >= 256 && rows > 64)
+		hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 4, 4, false>), dim3((unsigned)((rows + 127) / 128 * ntn)), dim3(256), 0, s, g);
+	else
+		hipLaunchKernelGGL((linear_kernel<TR, EPI, 1, 4, 2, 2, false>), dim3((unsigned)((rows + 31) / 32 * ntn)), dim3(256), 0, s, g);
+}
+
+template <class TR>
+void launch_linear_dt(const TgGemm &g, int epi, hipStream_t s) {
+	switch (epi) {
+		case TG_GE_STORE: launch_linear_t<TR, TG_GE_STORE>(g, s); break;
+		case TG_GE_F32: launch_linear_t<TR, TG_GE_F32>(g, s); break;
+		case TG_GE_RESID: launch_linear_t<TR, TG_GE_RESID>(g, s); break;
+		case TG_GE_SWIGLU: launch_linear_t<TR, TG_GE_SWIGLU>(g, s); break;
+		default: launch_linear_t<TR, TG_GE_TRANS>(g, s); break;
+	}
+}
+
+unsigned pack_grid(const TgPack &p) {
+	const long long n = ((long long)p.rows * p.cols + 255) / 256;
+	return (unsigned)(n < 16384 ? (n > 0 ? n : 1) : 16384);
+}
+
+}  // namespace
+
+void tg_launch_pack(const TgMat &dst, int dt, const TgPack &p, hipStream_t s) {
+	if (dt == TG_DT_BF16) hipLaunchKernelGGL((pack_kernel<TgB16>), dim3(pack_grid(p)), dim3(256), 0, s, (__bf16 *)dst.w, dst.k, p);
+	else hipLaunchKernelGGL((pack_kernel<TgF32>), dim3(pack_grid(p)), dim3(256), 0, s, (float *)dst.w, dst.k, p);
+}
+
+void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s) {
+	hipLaunchKernelGGL(unpack_f32_kernel, dim3(pack_grid(p)), dim3(256), 0, s, dst, ld, p);
+}
+
+int tg_vec_blocks(const TgVec &v, int epi) {
+	if (vec_wide(v, epi)) return (v.ntiles + 3) / 4;
+	return epi == TG_VE_SWIGLU ? (v.ntiles + 1) / 2 : v.ntiles;
+}
+
+// Parts of K for a product whose consumer adds them: enough workgroups for the device, at least 8 fragments per part.
+int tg_vec_ksplit(int ntiles, int nz, int kfrags, int n_cu) {
+	int p = 1;
+	while (p < 8 && ntiles * nz * p < n_cu && kfrags / (2 * p) >= 8) p *= 2;
+	return p;
+}
+
+void tg_launch_vec(const TgVec &v, int dt, int pro, int epi, hipStream_t s) {
+	if (dt == TG_DT_BF16) launch_vec_dt<TgB16>(v, pro, epi, s);
+	else launch_vec_dt<TgF32>(v, pro, epi, s);
+}
+
+void tg_launch_linear(const TgGemm &g, int dt, int epi, hipStream_t s) {
+	if (dt == TG_DT_BF16) launch_linear_dt<TgB16>(g, epi, s);
+	else launch_linear_dt<TgF32>(g, epi, s);
+}

@@ -1,0 +1,146 @@
+// Routing of a prefill's tokens to experts, and the row step between the blocks: tg_moe.h.
+
+#include "tg_moe.h"
+
+namespace {
+
+// a wave per token; the workgroup counts its tokens' choices per expert
+__global__ __launch_bounds__(256) void moe_route_kernel(TgMoeRoute r) {
+	extern __shared__ __align__(16) float sm[];
+	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, E = r.experts;
+	int *s_cnt = (int *)sm;
+	float *s_choice = sm + E + w * E, *s_val = sm + 5 * E + w * r.top;
+	int *s_sel = (int *)(sm + 5 * E + 4 * r.top) + w * r.top;
+	for (int e = tid; e < E; e += 256) s_cnt[e] = 0;
+	__syncthreads();
+	for (int i = w; i < TG_MOE_BLOCK; i += 4) {
+		const int t = blockIdx.x * TG_MOE_BLOCK + i;
+		if (t < r.n) {
+			const float *lg = r.logits + (size_t)t * r.ld;
+			for (int e = lane; e < E; e += 64) s_choice[e] = tg_sigmoid(lg[e]) + r.correction[e];
+			__builtin_amdgcn_wave_barrier();
+			asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+			for (int e = lane; e < E; e += 64) {
+				const float c = s_choice[e];
+				int rank = 0;
+				for (int o = 0; o < E; o++) {
+					const float co = s_choice[o];
+					rank += (co > c || (co == c && o < e)) ? 1 : 0;
+				}
+				if (rank < r.top) {
+					s_sel[rank] = e;
+					s_val[rank] = tg_sigmoid(lg[e]);
+				}
+			}
+			__builtin_amdgcn_wave_barrier();
+			asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+			for (int k = lane; k < r.top; k += 64) {
+				float sum = 0.0f;
+				for (int o = 0; o < r.top; o++) sum += s_val[o];
+				const size_t at = (size_t)t * r.top + k;
+				r.sel[at] = s_sel[k];
+				r.wgt[at] = s_val[k] / (sum + 1e-20f) * r.scale;
+				r.slot[at] = atomicAdd(&s_cnt[s_sel[k]], 1);
+			}
+		}
+	}
+	__syncthreads();
+	for (int e = tid; e < E; e += 256) r.count[(size_t)blockIdx.x * E + e] = s_cnt[e];
+}
+
+// one workgroup, a thread per expert: first slot of every (block, expert), and the tile list
+__global__ __launch_bounds__(TG_MOE_MAX_EXPERTS) void moe_offsets_kernel(TgMoeRoute r, int blocks) {
+	__shared__ int s_n[TG_MOE_MAX_EXPERTS], s_t[TG_MOE_MAX_EXPERTS];
+	const int e = threadIdx.x, E = r.experts;
+	int cnt = 0;
+	if (e < E)
+		for (int b = 0; b < blocks; b++) cnt += r.count[(size_t)b * E + e];
+	const int nt = (cnt + r.tile_rows - 1) / r.tile_rows;
+	s_n[e] = cnt;
+	s_t[e] = nt;
+	__syncthreads();
+	for (int o = 1; o < TG_MOE_MAX_EXPERTS; o <<= 1) {  // inclusive sums
+		const int a = e >= o ? s_n[e - o] : 0, b = e >= o ? s_t[e - o] : 0;
+		__syncthreads();
+		s_n[e] += a;
+		s_t[e] += b;
+		__syncthreads();
+	}
+	const int first = s_n[e] - cnt, t0 = s_t[e] - nt;
+	if (e < E) {
+		int run = first;
+		for (int b = 0; b < blocks; b++) {
+			const int c = r.count[(size_t)b * E + e];
+			r.count[(size_t)b * E + e] = run;
+			run += c;
+		}
+		for (int i = 0; i < nt; i++) r.tiles[t0 + i] = int4{e, first + i * r.tile_rows, min(first + (i + 1) * r.tile_rows, first + cnt), 0};
+	}
+	if (e == E - 1) *r.ntiles = s_t[e];
+}
+
+__global__ __launch_bounds__(256) void moe_scatter_kernel(TgMoeRoute r) {
+	const int i = blockIdx.x * 256 + threadIdx.x;
+	if (i >= r.n * r.top) return;
+	const int t = i / r.top;
+	const int slot = r.count[(size_t)(t / TG_MOE_BLOCK) * r.experts + r.sel[i]] + r.slot[i];
+	r.slot[i] = slot;
+	r.row_src[slot] = t;
+}
+
+// a wave per row, four columns per lane and pass
+template <class TR>
+__global__ __launch_bounds__(256) void rows_dyt_kernel(TgRowsDyt r) {
+	typedef typename TR::T T;
+	const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+	if (t >= r.n) return;
+	float *xr = r.x + (size_t)(r.gather ? r.gather[t] : t) * r.ldx;
+	int id = 0;
+	if (r.embed) {
+		id = r.ids[t];
+		id = id < 0 ? 0 : (id >= r.vocab ? r.vocab - 1 : id);
+	}
+	for (int c = 4 * lane; c < r.ldx; c += 256) {
+		f32x4_t x = r.embed ? tg_load4((const __bf16 *)r.embed + (size_t)id * r.ldx + c) : tg_load4(xr + c);
+		if (r.y) {
+			f32x4_t add = {0, 0, 0, 0};
+			for (int k = 0; k < r.top; k++) {
+				const float g = r.wgt[(size_t)t * r.top + k];
+				const f32x4_t y = tg_load4((const T *)r.y + (size_t)r.slot[(size_t)t * r.top + k] * r.ldx + c);
+#pragma unroll
+				for (int e = 0; e < 4; e++) add[e] = fmaf(g, y[e], add[e]);
+			}
+#pragma unroll
+			for (int e = 0; e < 4; e++) x[e] = x[e] + r.mult * add[e];
+		}
+		if (r.embed || r.y) tg_store4(xr + c, x);
+		if (r.out) {
+			const f32x4_t nw = tg_load4(r.nw + c), nb = tg_load4(r.nb + c);
+			f32x4_t h;
+#pragma unroll
+			for (int e = 0; e < 4; e++) h[e] = tanhf(r.alpha * x[e]) * nw[e] + nb[e];
+			tg_store4((T *)r.out + (size_t)t * r.ldx + c, h);
+		}
+	}
+}
+
+}  // namespace
+
+int tg_moe_max_tiles(int n, int experts, int top, int tile_rows) {
+	const int rows = n * top;
+	return rows / tile_rows + (experts < rows ? experts : rows);
+}
+
+void tg_launch_moe_route(const TgMoeRoute &r, hipStream_t s) {
+	const int blocks = (r.n + TG_MOE_BLOCK - 1) / TG_MOE_BLOCK;
+	const size_t lds = sizeof(float) * (5 * (size_t)r.experts + 8 * (size_t)r.top);
+	hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)blocks), dim3(256), lds, s, r);
+	hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(TG_MOE_MAX_EXPERTS), 0, s, r, blocks);
+	hipLaunchKernelGGL(moe_scatter_kernel, dim3((unsigned)((r.n * r.top + 255) / 256)), dim3(256), 0, s, r);
+}
+
+void tg_launch_rows_dyt(const TgRowsDyt &r, int dt, hipStream_t s) {
+	const dim3 grid((unsigned)((r.n + 3) / 4));
+	if (dt == TG_DT_BF16) hipLaunchKernelGGL((rows_dyt_kernel<TgB16>), grid, dim3(256), 0, s, r);
+	else hipLaunchKernelGGL((rows_dyt_kernel<TgF32>), grid, dim3(256), 0, s, r);
+}

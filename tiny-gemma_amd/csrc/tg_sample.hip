@@ -32,11 +32,20 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ float wave_max(float v) { return tg_wave_max(v); }
 __device__ __forceinline__ float wave_sum(float v) { return tg_wave_sum(v); }
 
+// four consecutive logits; entries past the vocabulary (its last workgroup may be partial) count as -inf
+__device__ __forceinline__ f32x4 load_logits(const float *logits, int i, int n) {
+	if (i + 4 <= n) return *reinterpret_cast<const f32x4 *>(logits + i);
+	f32x4 l;
+#pragma unroll
+	for (int e = 0; e < 4; e++) l[e] = i + e < n ? logits[i + e] : -INFINITY;
+	return l;
+}
+
 // bmax[b] = max over the workgroup's 1024 elements of logits[i] / temp
-__global__ __launch_bounds__(SNT) void minp_max_kernel(const float *logits, float temp, float *bmax) {
+__global__ __launch_bounds__(SNT) void minp_max_kernel(const float *logits, int n, float temp, float *bmax) {
 	__shared__ float sm[SNT / 64];
 	const int tid = threadIdx.x;
-	const f32x4 l = *reinterpret_cast<const f32x4 *>(logits + (size_t)blockIdx.x * SCHUNK + 4 * tid);
+	const f32x4 l = load_logits(logits, (int)blockIdx.x * SCHUNK + 4 * tid, n);
 	float m = fmaxf(fmaxf(l[0] / temp, l[1] / temp), fmaxf(l[2] / temp, l[3] / temp));
 	m = wave_max(m);
 	if ((tid & 63) == 0) sm[tid >> 6] = m;
@@ -46,11 +55,11 @@ __global__ __launch_bounds__(SNT) void minp_max_kernel(const float *logits, floa
 
 // probs[i] = exp(logits[i] / temp - rowmax); seg[s] = sum of segment s; bsum[b] = sum of the workgroup's
 // probabilities that are >= cut.  maxp is exp(0) = 1 (the maximum element itself), so cut = minp.
-__global__ __launch_bounds__(SNT) void minp_prob_kernel(const float *logits, float temp, float minp, const float *bmax, int nblocks,
+__global__ __launch_bounds__(SNT) void minp_prob_kernel(const float *logits, int n, float temp, float minp, const float *bmax, int nblocks,
                                                         float *probs, float *seg, float *bsum) {
 	__shared__ float sm[SNT / 64], ss[SNT / 64];
 	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-	const f32x4 l = *reinterpret_cast<const f32x4 *>(logits + (size_t)blockIdx.x * SCHUNK + 4 * tid);
+	const f32x4 l = load_logits(logits, (int)blockIdx.x * SCHUNK + 4 * tid, n);
 	float m = -INFINITY;
 	for (int i = tid; i < nblocks; i += SNT) m = fmaxf(m, bmax[i]);
 	m = wave_max(m);
@@ -84,7 +93,7 @@ __global__ __launch_bounds__(SNT) void minp_prob_kernel(const float *logits, flo
 // randf: the draw of this token is randf[rand_idx], or randf[ctr[3] - rand_base] when rand_idx < 0.
 __global__ __launch_bounds__(FNT) void minp_finish_kernel(const float *probs, const float *seg, const float *bsum, int nblocks, int nseg,
                                                           const float *randf, int rand_idx, int rand_base, int *ctr, int *tok_log,
-                                                          int mode, int *out_tok) {
+                                                          int mode, int *out_tok, int n) {
 	__shared__ float s_w[FNT / 64];
 	__shared__ float s_scan[FNT / 64];
 	__shared__ int s_seg;
@@ -162,7 +171,7 @@ __global__ __launch_bounds__(FNT) void minp_finish_kernel(const float *probs, co
 #pragma unroll
 		for (int o = 32; o > 0; o >>= 1) first = min(first, __shfl_xor(first, o, 64));
 		if (first == NONE) first = SEG - 1;  // rounding: the segment's end reached r, its re-scan did not
-		token = cs * SEG + first;
+		token = min(cs * SEG + first, n - 1);
 	}
 	if (tid == 0) {
 		if (out_tok) *out_tok = token;
@@ -183,15 +192,16 @@ __global__ __launch_bounds__(FNT) void minp_finish_kernel(const float *probs, co
 
 }  // namespace
 
-size_t tg_minp_blocks(int n) { return (size_t)n / SCHUNK; }
-size_t tg_minp_segments(int n) { return (size_t)n / SEG; }
+size_t tg_minp_blocks(int n) { return ((size_t)n + SCHUNK - 1) / SCHUNK; }
+size_t tg_minp_padded(int n) { return tg_minp_blocks(n) * SCHUNK; }
+size_t tg_minp_segments(int n) { return tg_minp_padded(n) / SEG; }
 
-// logits[n] (n a multiple of 1024) -> token; probs[n], seg[n/256], bsum[n/1024], bmax[n/1024] are scratch
+// logits[n] -> token; probs[tg_minp_padded(n)], seg[tg_minp_segments(n)], bsum and bmax[tg_minp_blocks(n)] are scratch
 void tg_launch_minp(const float *logits, int n, float minp, float temp, const float *randf, int rand_idx, int rand_base, float *probs,
                     float *seg, float *bsum, float *bmax, int *ctr, int *tok_log, int mode, int *out_tok, hipStream_t s) {
-	const int nb = n / SCHUNK, nseg = n / SEG;
-	hipLaunchKernelGGL(minp_max_kernel, dim3((unsigned)nb), dim3(SNT), 0, s, logits, temp, bmax);
-	hipLaunchKernelGGL(minp_prob_kernel, dim3((unsigned)nb), dim3(SNT), 0, s, logits, temp, minp, bmax, nb, probs, seg, bsum);
+	const int nb = (int)tg_minp_blocks(n), nseg = (int)tg_minp_segments(n);
+	hipLaunchKernelGGL(minp_max_kernel, dim3((unsigned)nb), dim3(SNT), 0, s, logits, n, temp, bmax);
+	hipLaunchKernelGGL(minp_prob_kernel, dim3((unsigned)nb), dim3(SNT), 0, s, logits, n, temp, minp, bmax, nb, probs, seg, bsum);
 	hipLaunchKernelGGL(minp_finish_kernel, dim3(1), dim3(FNT), 0, s, probs, seg, bsum, nb, nseg, randf, rand_idx, rand_base, ctr, tok_log,
-	                   mode, out_tok);
+	                   mode, out_tok, n);
 }
