@@ -15,6 +15,7 @@
 //   gemma::generate_greedy, gemma::generate_ids   transformer.hpp:167-258 on token ids (argmax / min-p branch)
 //   gemma::generate                               transformer.hpp:167-258 on text, streaming (with tokenizer.hpp)
 //   sentencepiece::Tokenizer                      tokenizer.hpp:14-239 (in host/tokenizer.hpp)
+//   model::Model, model::Session                  models opened from a folder (no counterpart in the reference)
 //
 // Errors: the reference throws std::runtime_error for an unknown dimension ("Unsupported ROW/COL
 // dimension: N") and an unopenable weight file ("Could not open file."), and assert()s on shape
@@ -248,9 +249,10 @@ inline std::tuple<int, std::vector<int>, float, float> generate_ids(const std::v
 // come back once per burst, so text appears burst by burst; 1 = token by token); with terminate_on_end the text
 // stops before the first <end_of_turn> and the count is that of the steps before it, as in the reference.
 // Where the reference's tokenizer throws on a byte token (see tokenizer.hpp) the byte itself is printed.
-inline std::tuple<int, std::string, float, float> generate(std::string prompt, int n_decode, sentencepiece::Tokenizer *tokenizer,
-                                                           Transformer *t, const float minp, const float temp,
-                                                           const bool terminate_on_end, int burst = 16) {
+// `open` makes the session once the prompt's length is known.
+template <typename Open>
+inline std::tuple<int, std::string, float, float> generate_on(Open open, std::string prompt, int n_decode, sentencepiece::Tokenizer *tokenizer,
+                                                              const float minp, const float temp, const bool terminate_on_end, int burst) {
 	using clk = std::chrono::high_resolution_clock;
 	auto t_prefill_s = clk::now();
 	std::random_device rd;
@@ -274,17 +276,14 @@ inline std::tuple<int, std::string, float, float> generate(std::string prompt, i
 		}
 	};
 
-	decode::RoPE rope(&t->cfg, false), rope_sw(&t->cfg, true);
-	lut::GeLUTable table{-4.0, 4.0, 1024};  // transformer.hpp:197
-	decode::DecodeState d(1, &t->cfg);
-	bind_session(t, &d, &rope, &rope_sw, &table);
+	tg_session *session = open((int)prompt_len);
 
 	std::vector<float> randf((size_t)std::max(n_decode, 0) + 1, 0.0f);
 	if (sampling)
 		for (float &r : randf) r = unif(gen);
 	std::vector<int> out((size_t)std::max(n_decode, 0) + 1);
 	// prefill and the first token (from the prefill logits)
-	check(tg_generate(d.session, ids.data(), (int)prompt_len, 0, minp, temp, randf.data(), out.data(), nullptr, nullptr));
+	check(tg_generate(session, ids.data(), (int)prompt_len, 0, minp, temp, randf.data(), out.data(), nullptr, nullptr));
 	int prev_token = ids[ids.size() - 1];
 	std::cout << piece_of(out[0], prev_token) << std::flush;
 	prev_token = out[0];
@@ -296,10 +295,10 @@ inline std::tuple<int, std::string, float, float> generate(std::string prompt, i
 	if (burst < 1) burst = 1;
 	while (done < n_decode && !stop) {
 		const int n = std::min(burst, n_decode - done);
-		if (sampling) check(tg_decode_enqueue_sampled(d.session, n, minp, temp, randf.data() + 1 + done));
-		else check(tg_decode_enqueue(d.session, n));
+		if (sampling) check(tg_decode_enqueue_sampled(session, n, minp, temp, randf.data() + 1 + done));
+		else check(tg_decode_enqueue(session, n));
 		int got = 0;
-		check(tg_session_read_ids(d.session, out.data(), done + 1 + n, &got));
+		check(tg_session_read_ids(session, out.data(), done + 1 + n, &got));
 		if (got != done + 1 + n) throw std::runtime_error("token log incomplete");
 		for (int i = 0; i < n; i++) {
 			const int tok = out[(size_t)done + 1];
@@ -319,7 +318,72 @@ inline std::tuple<int, std::string, float, float> generate(std::string prompt, i
 	const double s_decode = std::chrono::duration<double>(t_decode_e - t_decode_s).count();
 	return {done, decoded, (float)s_prefill, (float)s_decode};
 }
+
+inline std::tuple<int, std::string, float, float> generate(std::string prompt, int n_decode, sentencepiece::Tokenizer *tokenizer,
+                                                           Transformer *t, const float minp, const float temp,
+                                                           const bool terminate_on_end, int burst = 16) {
+	decode::RoPE rope(&t->cfg, false), rope_sw(&t->cfg, true);
+	lut::GeLUTable table{-4.0, 4.0, 1024};  // transformer.hpp:197
+	decode::DecodeState d(1, &t->cfg);
+	return generate_on(
+	    [&](int) {
+		    bind_session(t, &d, &rope, &rope_sw, &table);
+		    return d.session;
+	    },
+	    std::move(prompt), n_decode, tokenizer, minp, temp, terminate_on_end, burst);
+}
 }  // namespace gemma
+
+// Models opened from a folder (config.json + model.safetensors); the design is config.json's "architecture".
+namespace model {
+struct Model {
+	tg_model *h = nullptr;
+	tg_config cfg{};
+	Model(const std::string &dir, const std::string &dtype) {
+		if (dtype != "bfloat16" && dtype != "float32") throw std::runtime_error("dtype: bfloat16 or float32");
+		check(tg_model_open(dir.c_str(), dtype == "float32" ? TG_DTYPE_F32 : TG_DTYPE_BF16, &h));
+		check(tg_model_config(h, &cfg));
+	}
+	Model(const Model &) = delete;
+	Model &operator=(const Model &) = delete;
+	~Model() { tg_model_destroy(h); }
+	std::string architecture() const { return tg_model_architecture(h); }
+};
+
+struct Session {
+	tg_session *h = nullptr;
+	Session() = default;
+	Session(const Model &m, int max_tokens) { check(tg_session_open(m.h, max_tokens, &h)); }
+	Session(const Session &) = delete;
+	Session &operator=(const Session &) = delete;
+	~Session() { tg_session_destroy(h); }
+};
+
+// {n_generated, ids (n_generated + 1), s_prefill, s_decode}: gemma::generate_ids for these models
+inline std::tuple<int, std::vector<int>, float, float> generate_ids(const std::vector<int> &prompt, int n_decode, const Model &m, const float minp,
+                                                                    const float temp, std::mt19937 &gen) {
+	std::uniform_real_distribution<float> unif(0.0, 1.0);
+	std::vector<float> randf((size_t)n_decode + 1);
+	for (float &r : randf) r = unif(gen);
+	Session s(m, (int)prompt.size() + n_decode + 1);
+	std::vector<int> ids((size_t)n_decode + 1);
+	double sp = 0, sd = 0;
+	check(tg_generate(s.h, prompt.data(), (int)prompt.size(), n_decode, minp, temp, randf.data(), ids.data(), &sp, &sd));
+	return {n_decode, ids, (float)sp, (float)sd};
+}
+
+// gemma::generate (text in, text out) for these models
+inline std::tuple<int, std::string, float, float> generate(std::string prompt, int n_decode, sentencepiece::Tokenizer *tokenizer, const Model &m,
+                                                           const float minp, const float temp, const bool terminate_on_end, int burst = 16) {
+	std::unique_ptr<Session> s;
+	return gemma::generate_on(
+	    [&](int prompt_len) {
+		    s = std::make_unique<Session>(m, prompt_len + std::max(n_decode, 0) + 1);
+		    return s->h;
+	    },
+	    std::move(prompt), n_decode, tokenizer, minp, temp, terminate_on_end, burst);
+}
+}  // namespace model
 
 namespace ops {
 // strict '>' scan from index 0: the lowest index wins ties

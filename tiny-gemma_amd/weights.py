@@ -9,7 +9,13 @@ py/gemma.py:27-77 writes and csrc/include/transformer.hpp:99-165 reads:
     lm_head int8[hidden][vocab] + f32[vocab]        (tied: the transpose of the fp32 wte, re-quantized)
 
 Matrices are [in][out] row-major with one fp32 scale per output column.
+
+random_model_dir writes a random-init model folder (config.json + model.safetensors, bfloat16) of a layer-list model.
 """
+import json
+import os
+import struct
+
 import numpy as np
 
 
@@ -88,3 +94,81 @@ def random_weight_image(cfg, seed, std=0.02, norm_std=0.1):
     put(lm_s)
     assert pos == out.size
     return out
+
+
+# ---- model folders (layer-list models) ---------------------------------------------------------------------------
+def madevik_tensors(cfg, decay_rank):
+    """[(name, shape, kind)] of a Madevik model in file order; kind: "w" matrix, "one" norm weight, "zero" bias,
+    "alpha" scalar of the element-wise tanh norm, "decay" bias of the decay projection."""
+    D, V = cfg["width"], cfg["vocab"]
+    out = [("embed", (V, D), "w")]
+
+    def norm(name):
+        out.extend([(name, (D,), "one"), (name + ".b", (D,), "zero"), (name + ".alpha", (), "alpha")])
+
+    for i, l in enumerate(cfg["layers"]):
+        if l.get("weights_of") is not None:
+            continue
+        m, p = l["mixer"], f"l{i}.mix."
+        H, d, v = m["heads"], m["dim"], m["vdim"]
+        norm(f"l{i}.norm1")
+        if l["type"] == "gla":
+            out += [(p + "q", (H * d, D), "w"), (p + "k", (H * d, D), "w"), (p + "v", (H * v, D), "w"), (p + "g", (H * v, D), "w"),
+                    (p + "o", (D, H * v), "w"), (p + "norm", (v,), "one"), (p + "a1", (decay_rank, D), "w"), (p + "a2", (H * d, decay_rank), "w"),
+                    (p + "a2.b", (H * d,), "decay")]
+        else:
+            r = m["kv_rank"]
+            out += [(p + "q", (H * d, D), "w"), (p + "dkv", (r, D), "w"), (p + "dkv.norm", (r,), "one"), (p + "uk", (H * d, r), "w"),
+                    (p + "uv", (H * v, r), "w"), (p + "g", (H, D), "w"), (p + "o", (D, H * v), "w")]
+        if l.get("mlp") is not None:
+            norm(f"l{i}.norm2")
+            E, ff, q = l["mlp"]["router"]["experts"], l["mlp"]["expert"]["ff"], f"l{i}.mlp."
+            for e in range(E):
+                out += [(f"{q}e{e}.gate", (ff, D), "w"), (f"{q}e{e}.up", (ff, D), "w"), (f"{q}e{e}.down", (D, ff), "w")]
+            out += [(q + "router", (E, D), "w"), (q + "correction", (E,), "zero")]
+    norm("final.norm")
+    out.append(("head", (V, D), "w"))
+    return out
+
+
+def random_model_dir(path, cfg, seed, decay_rank=16, block=1 << 22):
+    """Writes config.json and model.safetensors of a random-init model (matrices N(0, 1 / inputs)) into `path`.  Matrices are
+    cut at random places out of one block of normal numbers per scale: large models are written at the speed of the disk."""
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    rng = np.random.default_rng(seed)
+    base = rng.standard_normal(block, dtype=np.float32)
+
+    def bf16(a):
+        u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+        return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+    blocks = {}
+    head, off = {}, 0
+    tensors = madevik_tensors(cfg, decay_rank)
+    for name, shape, _ in tensors:
+        n = 2 * int(np.prod(shape, dtype=np.int64))
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [off, off + n]}
+        off += n
+    text = json.dumps(head).encode()
+    text += b" " * (-len(text) % 8)
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(text)) + text)
+        for _, shape, kind in tensors:
+            n = int(np.prod(shape, dtype=np.int64))
+            if kind == "w":
+                std = float(shape[-1]) ** -0.5
+                if std not in blocks:
+                    blocks[std] = bf16(base * np.float32(std))
+                b = blocks[std]
+                while n > 0:
+                    k = min(n, block // 2)
+                    at = int(rng.integers(0, block - k + 1))
+                    f.write(b[at:at + k].tobytes())
+                    n -= k
+            else:
+                a = {"one": 1.0, "zero": 0.0, "alpha": 0.7, "decay": 3.0}[kind] * np.ones(n, np.float32)
+                if kind in ("one", "zero"):
+                    a += rng.standard_normal(n, dtype=np.float32) * np.float32(0.1)
+                f.write(bf16(a).tobytes())
