@@ -147,8 +147,112 @@ def _cpu_baseline_run(orc, image_path, cfg_name, prompt, n_decode):
     }
 
 
+# ---- layer-list models (--design): shapes that resemble a real model's layers, random weights -------------------------------
+def _design_layers(n, unique, every, gla, latent, moe):
+    """n layers, the last of every `every` latent attention, the others gated linear attention; layers behind the first
+    `unique` share the weights of the layer a multiple of `unique` before them."""
+    out = []
+    for i in range(n):
+        l = dict(latent if i % every == every - 1 else gla, mlp=moe)
+        if i >= unique:
+            l["weights_of"] = i % unique
+        out.append(l)
+    return out
+
+
+def design_config(size):
+    """(config, Gemma shape of equal width or None).  The layers' parameters that a token uses are as many as those of the
+    Gemma shape of equal width (640: 4.9 M per layer, 1152: 27 M); sharing weights bounds the file, not the bytes a step
+    streams: the distinct layers exceed the 256 MB memory-side cache."""
+    def cfg(width, vocab, layers):
+        return {"architecture": "Madevik", "width": width, "vocab": vocab, "residual_mult": 0.5, "norm": {"eps": 1e-5}, "layers": layers}
+
+    def gla(heads, dim, vdim):
+        return {"type": "gla", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "tau": 16.0}}
+
+    def lat(heads, dim, vdim, rank):
+        return {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "kv_rank": rank, "scale": dim ** -0.5}}
+
+    def moe(experts, top, ff):
+        return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "scale": 2.5}}
+
+    if size == "640":
+        return cfg(640, 262144, _design_layers(18, 18, 3, gla(4, 64, 128), lat(4, 64, 64, 128), moe(8, 2, 768))), "270m"
+    if size == "1152":
+        return cfg(1152, 262144, _design_layers(26, 8, 4, gla(4, 128, 256), lat(8, 128, 128, 256), moe(16, 4, 1728))), "1B"
+    return cfg(2048, 131072, _design_layers(24, 4, 4, gla(16, 128, 128), lat(16, 128, 128, 512), moe(64, 6, 1024))), None
+
+
+def design_bench(args):
+    """Prefill and decode throughput of the design, and of the Gemma shape of equal width in the same process."""
+    import importlib
+    import shutil
+    import tempfile
+    tg = ge.load_package()
+    tgw = importlib.import_module("tiny_gemma_amd.weights")
+    dev = tg.init(0)
+    rng = np.random.default_rng(args.seed)
+
+    def rates(sess, n_vocab, prompts, steps):
+        out = {}
+        for n in prompts:
+            ids = rng.integers(0, n_vocab, n).astype(np.int32)
+            best = None
+            for _ in range(3):          # the first run allocates the workspace
+                sess.reset()
+                tg.synchronize()
+                t0 = time.perf_counter()
+                sess.prefill(ids, want_logits=False)
+                best = min(best or 1e9, time.perf_counter() - t0)
+            sess.decode_enqueue(16)
+            tg.synchronize()
+            time.sleep(2e-3)
+            t0 = time.perf_counter()
+            sess.decode_enqueue(steps)
+            te = time.perf_counter() - t0
+            tg.synchronize()
+            td = time.perf_counter() - t0
+            out[str(n)] = {"prefill_ms": 1e3 * best, "prefill_tok_s": n / best, "decode_tok_s": steps / td, "decode_ms_per_step": 1e3 * td / steps,
+                           "host_enqueue_ms_per_step": 1e3 * te / steps}
+        return out
+
+    result = {}
+    sizes = [args.size] if args.size else ["640", "1152", "2048"]
+    prompts = [int(x) for x in args.prompts.split(",")]
+    for size in sizes:
+        cfg, gemma = design_config(size)
+        d = tempfile.mkdtemp(prefix="tg_bench_")
+        try:
+            tgw.random_model_dir(d, cfg, args.seed)
+            t0 = time.perf_counter()
+            model = tg.Transformer.from_dir(d, args.dtype)
+            t_load = time.perf_counter() - t0
+        finally:
+            shutil.rmtree(d)
+        sess = model.open_session(max(prompts) + args.design_steps + 32)
+        r = {"layers": len(cfg["layers"]), "dtype": args.dtype, "load_s": t_load, args.design: rates(sess, cfg["vocab"], prompts, args.design_steps)}
+        del sess, model
+        if gemma and not args.headline_only:
+            gcfg = tg.named_config(gemma)
+            gm = tg.Transformer(gcfg)
+            gm.read_weights_mem(tgw.random_weight_image(gcfg, args.seed))
+            gs = gm.session()
+            r[f"gemma3_{gemma}_int8"] = rates(gs, gcfg.n_vocab, prompts, args.design_steps)
+            del gs, gm
+        result[size] = r
+        print(f"{size}: {json.dumps(r)}", file=sys.stderr, flush=True)
+    print(json.dumps({"metric": "design_tokens_per_s", "design": args.design, "unit": "tok/s", "data": "synthetic", "n_gpus": 1, "sizes": result,
+                      "device": dev}))
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--design", choices=["madevik"], default=None,
+                    help="instead of the default workload: prefill and decode rates of this design at --size, beside the Gemma shape of equal width")
+    ap.add_argument("--size", choices=["640", "1152", "2048"], default=None, help="with --design: width (default: all)")
+    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="with --design")
+    ap.add_argument("--prompts", default="178,1024,4096", help="with --design: prompt lengths")
+    ap.add_argument("--design-steps", type=int, default=256, help="with --design: decode steps behind each prompt")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=1024)
     ap.add_argument("--warmup", type=int, default=16)
@@ -170,6 +274,9 @@ def main():
                     help="for rocprofv3 --pmc, no timing.  decode (default): prefill, a few decode steps and 4 launches of a "
                          "256 MiB copy kernel; gemm: 4 launches of the prefill GEMM at 4096 x 1152 x 6912 and nothing else")
     args = ap.parse_args()
+    if args.design:
+        design_bench(args)
+        return
     if args.gpus != 1:
         print("bench.py: this path is single-GPU (batch-1 decode has no data parallelism to spread); run with --gpus 1",
               file=sys.stderr)

@@ -31,7 +31,16 @@ __global__ __launch_bounds__(256) void gla_step_kernel(const float *y, TgGla g, 
 	for (int d = tid; d < g.dimp; d += 256) {
 		const size_t c = (size_t)h * g.dimp + d;
 		float z = 0.0f;
-		for (int j = 0; j < g.rank; j++) z = fmaf(g.a2[(size_t)j * hd + c], y[a_off + j], z);
+		for (int j0 = 0; j0 < g.rank; j0 += 16) {
+			float wa[16], ya[16];
+#pragma unroll
+			for (int j = 0; j < 16; j++) {
+				wa[j] = g.a2[(size_t)min(j0 + j, g.rank - 1) * hd + c];
+				ya[j] = y[a_off + min(j0 + j, g.rank - 1)];
+			}
+#pragma unroll
+			for (int j = 0; j < 16; j++) z = j0 + j < g.rank ? fmaf(wa[j], ya[j], z) : z;
+		}
 		s_a[d] = expf(tg_log_sigmoid(z + g.a2b[c]) * g.inv_tau);
 		s_q[d] = y[c] * g.qscale;
 		s_k[d] = y[k_off + c];
@@ -72,29 +81,51 @@ __global__ __launch_bounds__(256) void gla_step_kernel(const float *y, TgGla g, 
 	}
 }
 
-// ---- running sums of log alpha inside every chunk --------------------------------------------------------------------------
+// ---- running sums of log alpha inside every chunk: 64 channels per workgroup, a wave per 16 tokens ----------------------------
 __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld_low, TgGla g, int n, float *b) {
-	const int hd = g.heads * g.dimp, c = blockIdx.y * 256 + threadIdx.x, t0 = blockIdx.x * C;
-	if (c >= hd) return;
-	const bool real = c % g.dimp < g.dim;
-	const float bias = g.a2b[c];
-	float run = 0.0f;
-	for (int i0 = 0; i0 < C; i0 += 8) {
-		float z[8];
+	__shared__ __align__(16) float s_low[C][20];
+	__shared__ float s_sum[4][64];
+	const int hd = g.heads * g.dimp, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, t0 = blockIdx.x * C;
+	const int c = blockIdx.y * 64 + lane, cc = min(c, hd - 1);
+	const bool real = c < hd && cc % g.dimp < g.dim;
+	const float bias = g.a2b[cc];
+	float z[16];
 #pragma unroll
-		for (int i = 0; i < 8; i++) z[i] = 0.0f;
-		for (int j = 0; j < g.rank; j++) {
-			const float wj = g.a2[(size_t)j * hd + c];
+	for (int i = 0; i < 16; i++) z[i] = bias;
+	for (int j0 = 0; j0 < g.rank; j0 += 16) {
+		float wj[16];
 #pragma unroll
-			for (int i = 0; i < 8; i++) z[i] = fmaf(wj, low[(size_t)min(t0 + i0 + i, n - 1) * ld_low + j], z[i]);
-		}
+		for (int j = 0; j < 16; j++) wj[j] = g.a2[(size_t)min(j0 + j, g.rank - 1) * hd + cc];
+		// (the rows of `low` are padded to a multiple of 16)
+		const f32x4_t v = tg_load4(low + (size_t)min(t0 + (tid >> 2), n - 1) * ld_low + j0 + (tid & 3) * 4);
+		__syncthreads();
+		tg_store4(&s_low[tid >> 2][(tid & 3) * 4], v);
+		__syncthreads();
 #pragma unroll
-		for (int i = 0; i < 8; i++) {
-			const int t = t0 + i0 + i;
-			if (real && t < n) run += tg_log_sigmoid(z[i] + bias) * g.inv_tau;  // past the end: the sum stays
-			b[(size_t)t * hd + c] = run;
-		}
+		for (int j = 0; j < 16; j++)
+			if (j0 + j >= g.rank) wj[j] = 0.0f;
+#pragma unroll
+		for (int i = 0; i < 16; i++)
+#pragma unroll
+			for (int j4 = 0; j4 < 4; j4++) {
+				const f32x4_t l = tg_load4(&s_low[16 * w + i][4 * j4]);
+#pragma unroll
+				for (int e = 0; e < 4; e++) z[i] = fmaf(wj[4 * j4 + e], l[e], z[i]);
+			}
 	}
+	float run = 0.0f;
+#pragma unroll
+	for (int i = 0; i < 16; i++) {
+		if (real && t0 + 16 * w + i < n) run += tg_log_sigmoid(z[i]) * g.inv_tau;  // past the end: the sum stays
+		z[i] = run;
+	}
+	s_sum[w][lane] = run;
+	__syncthreads();
+	float before = 0.0f;
+	for (int q = 0; q < w; q++) before += s_sum[q][lane];
+	if (c < hd)
+#pragma unroll
+		for (int i = 0; i < 16; i++) b[(size_t)(t0 + 16 * w + i) * hd + c] = before + z[i];
 }
 
 // ---- A: a workgroup per chunk and head, a wave per block of 16 rows ---------------------------------------------------------
@@ -319,7 +350,7 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
 	const T *x = (const T *)qkv;
 	const unsigned chunks = (unsigned)((n + C - 1) / C), H = (unsigned)g.heads, hd = (unsigned)(g.heads * g.dimp);
 	const unsigned ndb = (unsigned)((g.dimp + 63) / 64), nvb = (unsigned)((g.vdimp + 63) / 64);
-	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (hd + 255) / 256), dim3(256), 0, s, low, ld_low, g, n, t.b);
+	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (hd + 63) / 64), dim3(256), 0, s, low, ld_low, g, n, t.b);
 	hipLaunchKernelGGL((gla_intra_kernel<TR>), dim3(chunks, H), dim3(256), 0, s, x, ld, k_off, g, n, t.b, t.a);
 	hipLaunchKernelGGL((gla_state_kernel<TR>), dim3(chunks, H, ndb * nvb), dim3(256), 0, s, x, ld, k_off, v_off, g, n, t.b, t.u);
 	const size_t per = (size_t)hd * g.vdimp;

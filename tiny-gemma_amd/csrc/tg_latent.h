@@ -9,8 +9,10 @@
 
 #include "tg_linear.h"
 
-#define TG_LATENT_MAX_PARTS 16     // partials that the value product merges in its prologue
+#define TG_LATENT_MAX_PARTS TG_VEC_MERGE_MAX  // partials that the value product merges in its prologue
 #define TG_LATENT_MAX_BLOCKS 256   // key parts per launch
+#define TG_LATENT_TILE 32
+#define TG_LATENT_LDS_MAX (150 * 1024)
 #define TG_LATENT_HEAD_MAX 256     // largest padded head size of the tiled kernel
 
 struct TgLatentStep {
@@ -22,10 +24,11 @@ struct TgLatentStep {
 	void *cache;                   // [capacity][rankp] in the model's format; the new row is written here
 	const int *ctr;                // device counters; ctr[0] = position
 	int host_pos;                  // the position, or -1: read the counter
-	int chunk, nb;                 // keys per part (multiple of 64), parts
+	int chunk, nb;                 // keys per part (multiple of TG_LATENT_TILE), parts
 	float *part_acc, *part_ml;     // [nb][heads16][rankp], [nb][heads16][2]
 };
 void tg_launch_latent_step(const TgLatentStep &a, int dt, hipStream_t s);
+size_t tg_latent_step_lds(int rankp, int dt);  // LDS the step asks for, besides its static 7 KiB
 // folds nb > TG_LATENT_MAX_PARTS partials into one
 void tg_launch_latent_fold(const float *acc, const float *ml, int nb, int heads16, int rankp, float *out_acc, float *out_ml, hipStream_t s);
 

@@ -5,115 +5,192 @@
 namespace {
 
 // ---- one token -------------------------------------------------------------------------------------------------------------
-// A workgroup takes one part of the keys for 16 heads and (blockIdx.z) 512 latent columns of the value sum.  Scores of a tile
-// of 64 keys come from the matrix instructions (wave w: keys 16 w ...), the running softmax is a wave's work for 4 heads, the
-// value sum stays on the vector units in fp32: a lane owns two latent columns of all 16 heads.
+// A workgroup takes one part of the keys for 16 heads (HT of which exist), tile by tile of 32.  A tile's latent rows go to LDS
+// in one round trip (the first tile's loads are requested before anything else is done), row pitch 16 bytes more than the row.
+// Scores come from the matrix instructions, wave w: keys 16 (w % 2) ..., half w / 2 of the latent; the running softmax is a
+// wave's work for 4 heads; the value sum stays on the vector units in fp32: a lane owns two latent columns of all heads, for
+// every G-th key (G = 1, 2 or 4 groups of lanes, added at the end), in passes of 512 columns (blockIdx.z).
+constexpr int ST = 32;         // keys per tile
+constexpr int ST_LOADS = 8;    // 16-byte pieces per lane and round of the tile copy
+
 template <class TR>
+size_t latent_step_lds(int rankp) {  // q' fragments | tile | (reused) sums of the lane groups
+	const size_t row = (size_t)rankp * sizeof(typename TR::T);
+	return 16 * row + ST * (row + 16);
+}
+
+template <class TR, int HT>
 __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
 	extern __shared__ __align__(16) unsigned char smem[];
+	const int row = a.rankp * (int)sizeof(T), pitch = row + 16, ppr = row / 16;  // bytes; 16-byte pieces per row
 	Frag *s_q = reinterpret_cast<Frag *>(smem);  // [rankp / KF][64]
-	__shared__ __align__(16) float s_p[64][20];
+	unsigned char *s_c = smem + 16 * row;
+	__shared__ float s_half[2][ST][16];
+	__shared__ __align__(16) float s_p[ST][20];
 	__shared__ float s_corr[16], s_sq[4];
 	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
 	const int part = blockIdx.x, h0 = blockIdx.y * 16, heads16 = (int)gridDim.y * 16;
 	const int pos = a.host_pos >= 0 ? a.host_pos : a.ctr[0], ctx = pos + 1;
 	const int kb = part * a.chunk, ke = min(ctx, kb + a.chunk);
 	T *cache = (T *)a.cache;
+	typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+	u32x4 piece[ST_LOADS];
+	// pieces [base, base + 256 * ST_LOADS) of a tile; the new token's row is not in memory yet: it is written to LDS below
+	auto request = [&](int k0, int base) {
+#pragma unroll
+		for (int i = 0; i < ST_LOADS; i++) {
+			const int e = min(base + tid + 256 * i, ST * ppr - 1), r = e / ppr, key = max(min(min(k0 + r, ke - 1), pos - 1), 0);
+			piece[i] = *reinterpret_cast<const u32x4 *>((const unsigned char *)cache + (size_t)key * row + (e - r * ppr) * 16);
+		}
+	};
+	auto place = [&](int base) {
+#pragma unroll
+		for (int i = 0; i < ST_LOADS; i++) {
+			const int e = base + tid + 256 * i, r = e / ppr;
+			if (e < ST * ppr) *reinterpret_cast<u32x4 *>(s_c + (size_t)r * pitch + (e - r * ppr) * 16) = piece[i];
+		}
+	};
+	const bool mine = pos >= kb && pos < kb + a.chunk;
+	float raw[2], nrm[2];
+#pragma unroll
+	for (int i = 0; i < 2; i++) {
+		const int j = min(tid + 256 * i, a.rank - 1);
+		raw[i] = a.dkv[j];
+		nrm[i] = a.norm[j];
+	}
+	request(kb, 0);
 
-	// the new token's row, by the workgroup(s) whose part it ends
-	if (pos >= kb && pos < kb + a.chunk) {
+	// q' in operand order: lane = head, 16 bytes of the latent
+	for (int e = tid; e < 4 * a.rankp; e += 256) {
+		const int h = e / (a.rankp / 4), j = (e - h * (a.rankp / 4)) * 4, hh = h0 + h;
+		f32x4_t v = tg_load4(a.q + (size_t)min(hh, a.heads - 1) * a.rankp + j);
+		if (hh >= a.heads) v = f32x4_t{0, 0, 0, 0};
+		tg_store4(reinterpret_cast<T *>(s_q) + ((size_t)(j / TR::KF) * 64 + h + 16 * ((j % TR::KF) / TR::KV)) * TR::KV + j % TR::KV, v);
+	}
+	// the new token's latent, normalised, by the workgroups whose part it ends
+	float inv = 0.0f;
+	if (mine) {
 		float ss = 0.0f;
-		for (int j = tid; j < a.rank; j += 256) ss = fmaf(a.dkv[j], a.dkv[j], ss);
+		for (int j = tid, i = 0; j < a.rank; j += 256, i++) {
+			const float x = i < 2 ? raw[i & 1] : a.dkv[j];
+			ss = fmaf(x, x, ss);
+		}
 		ss = tg_wave_sum(ss);
 		if (lane == 0) s_sq[w] = ss;
 		__syncthreads();
-		const float inv = 1.0f / sqrtf(((s_sq[0] + s_sq[1]) + (s_sq[2] + s_sq[3])) / (float)a.rank + a.eps);
-		for (int j = tid; j < a.rankp; j += 256) {
-			const int jc = j < a.rank ? j : 0;
-			const float c = a.dkv[jc] * inv * a.norm[jc];
-			cache[(size_t)pos * a.rankp + j] = (T)(j < a.rank ? c : 0.0f);
-		}
+		inv = 1.0f / sqrtf(((s_sq[0] + s_sq[1]) + (s_sq[2] + s_sq[3])) / (float)a.rank + a.eps);
 	}
-	// q' in operand order: lane = head, 16 bytes of the latent
-	for (int e = tid; e < 16 * a.rankp; e += 256) {
-		const int h = e / a.rankp, j = e - h * a.rankp, hh = h0 + h;
-		const float v = hh < a.heads ? a.q[(size_t)hh * a.rankp + j] : 0.0f;
-		reinterpret_cast<T *>(s_q)[((size_t)(j / TR::KF) * 64 + h + 16 * ((j % TR::KF) / TR::KV)) * TR::KV + j % TR::KV] = (T)v;
-	}
-	__syncthreads();
 
-	const int col = blockIdx.z * 512 + 2 * tid;
-	const bool cin = col < a.rankp;
+	const int cols = min(a.rankp, 512) / 2, G = cols <= 64 ? 4 : (cols <= 128 ? 2 : 1), per = 256 / G;
+	const int grp = tid / per, cl = tid - grp * per, col = blockIdx.z * 512 + 2 * cl;
+	const bool cin = cl < cols && col < a.rankp;
 	const int colc = cin ? col : 0;
-	float acc[16][2];
+	float acc[HT][2];
 #pragma unroll
-	for (int h = 0; h < 16; h++) acc[h][0] = acc[h][1] = 0.0f;
+	for (int h = 0; h < HT; h++) acc[h][0] = acc[h][1] = 0.0f;
 	float m[4], l[4];
 #pragma unroll
 	for (int i = 0; i < 4; i++) { m[i] = -INFINITY; l[i] = 0.0f; }
-	const int kfr = a.rankp / TR::KF;
-	for (int k0 = kb; k0 < ke; k0 += 64) {
-		{
-			const int key = min(k0 + 16 * w + lr, ke - 1);
-			const T *row = cache + (size_t)key * a.rankp + lg * TR::KV;
-			f32x4_t sc = {0, 0, 0, 0};
-			for (int kf = 0; kf < kfr; kf++) sc = TR::mma(*reinterpret_cast<const Frag *>(row + (size_t)kf * TR::KF), s_q[kf * 64 + lane], sc);
-#pragma unroll
-			for (int e = 0; e < 4; e++) s_p[16 * w + 4 * lg + e][lr] = k0 + 16 * w + 4 * lg + e < ke ? sc[e] * a.scale : -INFINITY;
+	const int kfr = a.rankp / TR::KF, kh = (kfr + 1) / 2, kf_lo = (w >> 1) * kh, kf_hi = min(kfr, kf_lo + kh);
+	for (int k0 = kb; k0 < ke; k0 += ST) {
+		for (int base = 0; base < ST * ppr; base += 256 * ST_LOADS) {
+			if (base) request(k0, base);
+			place(base);
 		}
 		__syncthreads();
-#pragma unroll
-		for (int i = 0; i < 4; i++) {
-			const float s = s_p[lane][4 * w + i];
-			const float mn = fmaxf(m[i], tg_wave_max(s)), f = expf(m[i] - mn), p = expf(s - mn);
-			s_p[lane][4 * w + i] = p;
-			l[i] = l[i] * f + tg_wave_sum(p);
-			m[i] = mn;
-			if (lane == 0) s_corr[4 * w + i] = f;
-		}
-		__syncthreads();
-#pragma unroll
-		for (int h = 0; h < 16; h++) {
-			acc[h][0] *= s_corr[h];
-			acc[h][1] *= s_corr[h];
-		}
-		const int kn = min(64, ke - k0);
-		const T *base = cache + (size_t)k0 * a.rankp + colc;
-		for (int k = 0; k < kn; k += 8) {
-			float c0[8], c1[8];
-#pragma unroll
-			for (int u = 0; u < 8; u++) {
-				const T *p = base + (size_t)min(k + u, kn - 1) * a.rankp;
-				c0[u] = (float)p[0];
-				c1[u] = (float)p[1];
+		if (mine && pos < k0 + ST) {
+			for (int j = tid, i = 0; j < a.rankp; j += 256, i++) {
+				const int jc = j < a.rank ? j : 0;
+				const float x = i < 2 ? raw[i & 1] : a.dkv[jc], g = i < 2 ? nrm[i & 1] : a.norm[jc];
+				const T c = (T)(j < a.rank ? x * inv * g : 0.0f);
+				*reinterpret_cast<T *>(s_c + (size_t)(pos - k0) * pitch + (size_t)j * sizeof(T)) = c;
+				cache[(size_t)pos * a.rankp + j] = c;
 			}
+			__syncthreads();
+		}
+		if (k0 + ST < ke) request(k0 + ST, 0);
+		{
+			const unsigned char *rp = s_c + (size_t)(16 * (w & 1) + lr) * pitch + lg * 16;
+			f32x4_t sc = {0, 0, 0, 0};
+			for (int kf = kf_lo; kf < kf_hi; kf++) sc = TR::mma(*reinterpret_cast<const Frag *>(rp + kf * 64), s_q[kf * 64 + lane], sc);
 #pragma unroll
-			for (int u = 0; u < 8; u++) {  // rows past the part's end have probability 0
-				const int kk = k + u;
+			for (int e = 0; e < 4; e++) s_half[w >> 1][16 * (w & 1) + 4 * lg + e][lr] = sc[e];
+		}
+		__syncthreads();
+		{
+			// lane: key lane % 32, heads 4 w + lane / 32 and 4 w + 2 + lane / 32
+			const int key = lane & 31;
 #pragma unroll
-				for (int h4 = 0; h4 < 4; h4++) {
-					const f32x4_t p = tg_load4(&s_p[kk][4 * h4]);
+			for (int i = 0; i < 2; i++) {
+				const int h = 4 * w + 2 * i + (lane >> 5);
+				const float s = k0 + key < ke ? (s_half[0][key][h] + s_half[1][key][h]) * a.scale : -INFINITY;
+				float mx = fmaxf(s, tg_red_partner<16>(s));
+				mx = tg_row16_max(mx);
+				const float mn = fmaxf(m[i], mx), f = expf(m[i] - mn), p = expf(s - mn);
+				float sum = p + tg_red_partner<16>(p);
+				sum = tg_row16_sum(sum);
+				s_p[key][h] = p;
+				l[i] = l[i] * f + sum;
+				m[i] = mn;
+				if (key == 0) s_corr[h] = f;
+			}
+		}
+		__syncthreads();
+		if (k0 > kb) {
 #pragma unroll
-					for (int e = 0; e < 4; e++) {
-						acc[4 * h4 + e][0] = fmaf(p[e], c0[u], acc[4 * h4 + e][0]);
-						acc[4 * h4 + e][1] = fmaf(p[e], c1[u], acc[4 * h4 + e][1]);
-					}
+			for (int h = 0; h < HT; h++) {
+				acc[h][0] *= s_corr[h];
+				acc[h][1] *= s_corr[h];
+			}
+		}
+		// rows past the part's end repeat its last row, with probability 0
+#pragma unroll 4
+		for (int k = grp; k < ST; k += G) {
+			const T *c = reinterpret_cast<const T *>(s_c + (size_t)k * pitch) + colc;
+			const float c0 = (float)c[0], c1 = (float)c[1];
+#pragma unroll
+			for (int h4 = 0; h4 < HT / 4; h4++) {
+				const f32x4_t p = tg_load4(&s_p[k][4 * h4]);
+#pragma unroll
+				for (int e = 0; e < 4; e++) {
+					acc[4 * h4 + e][0] = fmaf(p[e], c0, acc[4 * h4 + e][0]);
+					acc[4 * h4 + e][1] = fmaf(p[e], c1, acc[4 * h4 + e][1]);
 				}
 			}
 		}
 		__syncthreads();
 	}
-	if (cin) {
+	// the lane groups' sums meet in LDS (the tile's place: HT heads of at most 256 columns)
+	if (G > 1) {
+		float *s_s = reinterpret_cast<float *>(smem);
+		for (int g = 1; g < G; g++) {
+			if (grp == g && cin) {
+#pragma unroll
+				for (int h = 0; h < HT; h++) *reinterpret_cast<float2 *>(s_s + ((size_t)h * cols + cl) * 2) = float2{acc[h][0], acc[h][1]};
+			}
+			__syncthreads();
+			if (grp == 0) {
+#pragma unroll
+				for (int h = 0; h < HT; h++) {
+					const float2 v = *reinterpret_cast<const float2 *>(s_s + ((size_t)h * cols + cl) * 2);
+					acc[h][0] += v.x;
+					acc[h][1] += v.y;
+				}
+			}
+			__syncthreads();
+		}
+	}
+	if (cin && grp == 0) {
 		float *o = a.part_acc + ((size_t)part * heads16 + h0) * a.rankp + col;
 #pragma unroll
-		for (int h = 0; h < 16; h++) *reinterpret_cast<float2 *>(o + (size_t)h * a.rankp) = float2{acc[h][0], acc[h][1]};
+		for (int h = 0; h < HT; h++) *reinterpret_cast<float2 *>(o + (size_t)h * a.rankp) = float2{acc[h][0], acc[h][1]};
 	}
-	if (blockIdx.z == 0 && lane == 0) {
+	if (blockIdx.z == 0 && (lane & 31) == 0) {
 #pragma unroll
-		for (int i = 0; i < 4; i++) {
-			float *ml = a.part_ml + ((size_t)part * heads16 + h0 + 4 * w + i) * 2;
+		for (int i = 0; i < 2; i++) {
+			float *ml = a.part_ml + ((size_t)part * heads16 + h0 + 4 * w + 2 * i + (lane >> 5)) * 2;
 			ml[0] = m[i];
 			ml[1] = l[i];
 		}
@@ -176,16 +253,21 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const float *dkv, int 
 // registers -> LDS, the next tile's loads in flight during this one's arithmetic.  Scores are taken as K Q^T, so a lane holds
 // four consecutive keys of one query and the probabilities are already the second operand of V^T P^T; in the bf16 format they
 // enter it as two bf16 planes (value and remainder).
-template <class TR, int DMAX, int KT, int QT>
-__global__ __launch_bounds__(256) void latent_attn_kernel(TgLatentRows a) {
+// Sizes are compile-time buckets (DM >= dimp, VM >= vdimp): query elements past the head are zero, value rows past it are
+// computed from repeated rows and not stored, so that no branch stands between the LDS reads and matrix instructions.
+template <class TR, int DM, int VM, int KT, int QT>
+__global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
-	constexpr int ND = DMAX / TR::KF, NV = DMAX / 16, NK = KT / 16, NB = KT / TR::KF;
+	constexpr int ND = DM / TR::KF, NV = VM / 16, NK = KT / 16, NB = KT / TR::KF;
 	constexpr int KFRAGS = NK * ND, NF = KFRAGS + NV * NB, PW = NF / 4;
 	static_assert(NF % 4 == 0 && NB >= 1, "");
 	__shared__ __align__(16) Frag lds[NF * 64];
 	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
-	const int h = blockIdx.x, qb = ((int)gridDim.y - 1 - (int)blockIdx.y) * 64 * QT;  // the longest rows first
+	// Query tiles from both ends: the first half of the launch takes the long rows, longest first, the second half the
+	// short ones, shortest first, so that the workgroups that meet on a compute unit have about the same work together.
+	const int nqt = (int)gridDim.y, y = (int)blockIdx.y, half = (nqt + 1) / 2;
+	const int h = blockIdx.x, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
 	const int kd = a.dimp / TR::KF, nv = a.vdimp / 16;
 	const T *Q = (const T *)a.q, *K = (const T *)a.k + (size_t)h * a.dimp, *V = (const T *)a.vt + (size_t)h * a.vdimp * a.ldv;
 	const float sl2 = a.scale * 1.44269504088896340736f;
@@ -197,7 +279,10 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(TgLatentRows a) {
 		qi[s] = qb + w * 16 * QT + s * 16 + lr;
 		const T *row = Q + (size_t)min(qi[s], a.n - 1) * a.ldq + (size_t)h * a.dimp + lg * TR::KV;
 #pragma unroll
-		for (int d = 0; d < ND; d++) qf[s][d] = *reinterpret_cast<const Frag *>(row + (d < kd ? d : 0) * TR::KF);
+		for (int d = 0; d < ND; d++) {
+			qf[s][d] = *reinterpret_cast<const Frag *>(row + (d < kd ? d : 0) * TR::KF);
+			if (d >= kd) qf[s][d] = Frag{};
+		}
 	}
 	f32x4_t o[QT][NV];
 	float m[QT], l[QT];
@@ -242,12 +327,11 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(TgLatentRows a) {
 #pragma unroll
 			for (int s = 0; s < QT; s++) sc[s][kt] = f32x4_t{0, 0, 0, 0};
 #pragma unroll
-			for (int d = 0; d < ND; d++)
-				if (d < kd) {
-					const Frag kf = lds[(kt * ND + d) * 64 + lane];
+			for (int d = 0; d < ND; d++) {
+				const Frag kf = lds[(kt * ND + d) * 64 + lane];
 #pragma unroll
-					for (int s = 0; s < QT; s++) sc[s][kt] = TR::mma(kf, qf[s][d], sc[s][kt]);
-				}
+				for (int s = 0; s < QT; s++) sc[s][kt] = TR::mma(kf, qf[s][d], sc[s][kt]);
+			}
 		}
 #pragma unroll
 		for (int s = 0; s < QT; s++) {
@@ -298,15 +382,14 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(TgLatentRows a) {
 				}
 			}
 #pragma unroll
-			for (int v = 0; v < NV; v++)
-				if (v < nv) {
-					const Frag vf = lds[(KFRAGS + v * NB + b) * 64 + lane];
+			for (int v = 0; v < NV; v++) {
+				const Frag vf = lds[(KFRAGS + v * NB + b) * 64 + lane];
 #pragma unroll
-					for (int s = 0; s < QT; s++) {
-						o[s][v] = TR::mma(vf, ph[s], o[s][v]);
-						if constexpr (TR::DT == TG_DT_BF16) o[s][v] = TR::mma(vf, pl[s], o[s][v]);
-					}
+				for (int s = 0; s < QT; s++) {
+					o[s][v] = TR::mma(vf, ph[s], o[s][v]);
+					if constexpr (TR::DT == TG_DT_BF16) o[s][v] = TR::mma(vf, pl[s], o[s][v]);
 				}
+			}
 		}
 		tg_lds_barrier();
 		put();
@@ -333,30 +416,52 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(TgLatentRows a) {
 	}
 }
 
+template <class TR, int DM, int VM, int KT>
+void launch_bucket(const TgLatentRows &a, hipStream_t s) {
+	// 128-query tiles (half the LDS reads per product) where they fill the device twice
+	if constexpr (TR::DT == TG_DT_BF16 && DM <= 128 && VM <= 128) {
+		if (a.heads * ((a.n + 127) / 128) >= 512) {
+			hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 2>), dim3((unsigned)a.heads, (unsigned)((a.n + 127) / 128)), dim3(256), 0, s, a);
+			return;
+		}
+	}
+	hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 1>), dim3((unsigned)a.heads, (unsigned)((a.n + 63) / 64)), dim3(256), 0, s, a);
+}
+
 template <class TR>
 void launch_attention(const TgLatentRows &a, hipStream_t s) {
-	const int d = a.dimp > a.vdimp ? a.dimp : a.vdimp;
-	const dim3 g1((unsigned)a.heads, (unsigned)((a.n + 63) / 64)), g2((unsigned)a.heads, (unsigned)((a.n + 127) / 128));
-	const bool two = TR::DT == TG_DT_BF16 && a.heads * ((a.n + 127) / 128) >= 512;  // 128-query tiles where they fill the device twice
-	if (d <= 64) {
-		if (two) hipLaunchKernelGGL((latent_attn_kernel<TR, 64, 64, 2>), g2, dim3(256), 0, s, a);
-		else hipLaunchKernelGGL((latent_attn_kernel<TR, 64, 64, 1>), g1, dim3(256), 0, s, a);
-	} else if (d <= 128) {
-		if (two) hipLaunchKernelGGL((latent_attn_kernel<TR, 128, 64, 2>), g2, dim3(256), 0, s, a);
-		else hipLaunchKernelGGL((latent_attn_kernel<TR, 128, 64, 1>), g1, dim3(256), 0, s, a);
-	} else {
-		hipLaunchKernelGGL((latent_attn_kernel<TR, 256, 32, 1>), g1, dim3(256), 0, s, a);
-	}
+	constexpr int W = TR::DT == TG_DT_BF16 ? 64 : 32;  // keys per tile of the wide buckets
+	const int d = a.dimp, v = a.vdimp;
+	if (d <= 64 && v <= 64) launch_bucket<TR, 64, 64, 64>(a, s);
+	else if (d <= 64 && v <= 128) launch_bucket<TR, 64, 128, 64>(a, s);
+	else if (d <= 128 && v <= 64) launch_bucket<TR, 128, 64, 64>(a, s);
+	else if (d <= 128 && v <= 128) launch_bucket<TR, 128, 128, W>(a, s);
+	else if (d <= 192 && v <= 128) launch_bucket<TR, 192, 128, 32>(a, s);
+	else launch_bucket<TR, 256, 256, 32>(a, s);
 }
 
 }  // namespace
 
-void tg_launch_latent_step(const TgLatentStep &a, int dt, hipStream_t s) {
+namespace {
+template <class TR>
+void launch_step(const TgLatentStep &a, hipStream_t s) {
 	const dim3 grid((unsigned)a.nb, (unsigned)((a.heads + 15) / 16), (unsigned)((a.rankp + 511) / 512));
-	const size_t lds = 16 * (size_t)a.rankp * tg_dt_bytes(dt);
-	if (dt == TG_DT_BF16) hipLaunchKernelGGL((latent_step_kernel<TgB16>), grid, dim3(256), lds, s, a);
-	else hipLaunchKernelGGL((latent_step_kernel<TgF32>), grid, dim3(256), lds, s, a);
+	const size_t lds = latent_step_lds<TR>(a.rankp);
+	if (lds > 48 * 1024) {
+		(void)hipFuncSetAttribute((const void *)latent_step_kernel<TR, 8>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+		(void)hipFuncSetAttribute((const void *)latent_step_kernel<TR, 16>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+	}
+	if (a.heads <= 8) hipLaunchKernelGGL((latent_step_kernel<TR, 8>), grid, dim3(256), lds, s, a);
+	else hipLaunchKernelGGL((latent_step_kernel<TR, 16>), grid, dim3(256), lds, s, a);
 }
+}  // namespace
+
+void tg_launch_latent_step(const TgLatentStep &a, int dt, hipStream_t s) {
+	if (dt == TG_DT_BF16) launch_step<TgB16>(a, s);
+	else launch_step<TgF32>(a, s);
+}
+
+size_t tg_latent_step_lds(int rankp, int dt) { return dt == TG_DT_BF16 ? latent_step_lds<TgB16>(rankp) : latent_step_lds<TgF32>(rankp); }
 
 void tg_launch_latent_fold(const float *acc, const float *ml, int nb, int heads16, int rankp, float *out_acc, float *out_ml, hipStream_t s) {
 	hipLaunchKernelGGL(latent_fold_kernel, dim3((unsigned)heads16, (unsigned)(rankp / 64)), dim3(256), 0, s, acc, ml, nb, heads16, rankp, out_acc,

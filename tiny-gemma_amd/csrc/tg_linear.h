@@ -79,6 +79,7 @@ void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s);
 // y = W x for one vector, or for `nz` of them at once (head blocks, experts).  A workgroup owns one tile of 16 outputs (two
 // for the gate|up pair) over its part of K, or, where there are thousands of tiles, four of them.  The vector is prepared by
 // every workgroup in a prologue and held in LDS.
+#define TG_VEC_MERGE_MAX 16  // attention partials a prologue merges
 enum {
 	TG_VP_PLAIN = 0,   // x[z]
 	TG_VP_DYT,         // residual sum, then the element-wise tanh norm
@@ -110,7 +111,6 @@ struct TgVec {
 	float *x_out, *h_out;      // DYT: the new residual and the normalised vector (may be null)
 	const void *embed;         // DYT: x is row ctr[4] of this table instead (null: x)
 	int embed_ld, vocab;
-	int width;                 // DYT: elements of the vector (the rest of K is padding)
 	const int *ctr;
 	const float *gate;         // HEADNORM: gate vector laid out like x; GATE: one value per z
 	int vdim, vdimp;           // HEADNORM: head size and its padded size

@@ -41,14 +41,16 @@ constexpr int NT = 256;
 // lower index).  s_sel / s_val (LDS, top entries): the chosen experts in rank order and their scores.
 __device__ __forceinline__ void choose_experts(const float *logits, const float *correction, int E, int top, float *s_choice, int *s_sel,
                                                float *s_val) {
-	for (int e = threadIdx.x; e < E; e += NT) s_choice[e] = tg_sigmoid(logits[e]) + correction[e];
+	const int E4 = (E + 3) & ~3;  // s_choice has room for a multiple of four
+	for (int e = threadIdx.x; e < E4; e += NT) s_choice[e] = e < E ? tg_sigmoid(logits[e]) + correction[e] : -INFINITY;
 	__syncthreads();
 	for (int e = threadIdx.x; e < E; e += NT) {
 		const float c = s_choice[e];
 		int rank = 0;
-		for (int o = 0; o < E; o++) {
-			const float co = s_choice[o];
-			rank += (co > c || (co == c && o < e)) ? 1 : 0;
+		for (int o = 0; o < E4; o += 4) {
+			const f32x4_t co = tg_load4(s_choice + o);
+#pragma unroll
+			for (int i = 0; i < 4; i++) rank += (co[i] > c || (co[i] == c && o + i < e)) ? 1 : 0;
 		}
 		if (rank < top) {
 			s_sel[rank] = e;
@@ -57,6 +59,10 @@ __device__ __forceinline__ void choose_experts(const float *logits, const float 
 	}
 	__syncthreads();
 }
+
+// A launch is a chain of dependent memory round trips, so every prologue requests all of its inputs before it uses one
+// (clamped indices, no loads under branches), and the first round of the weight stream right behind them: waits are in
+// order, the prologue's arithmetic then runs while the weights are on their way.
 
 // NTL: tiles per wave (2: a gate|up pair); KW: waves that share a tile's K (4), or 1: every wave has tiles of its own;
 // U: fragments in flight per lane and tile
@@ -76,9 +82,9 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 
 	int zw = z;
 	if constexpr (PRO == TG_VP_EXPERT) {
-		// LDS: choice scores [experts] | selected [top] | their scores [top] behind the vector
+		// LDS: choice scores [experts, padded] | selected [top] | their scores [top] behind the vector
 		float *s_choice = reinterpret_cast<float *>(smem + sizeof(T) * (size_t)(per + KW * U) * TR::KF);
-		int *s_sel = reinterpret_cast<int *>(s_choice + p.experts);
+		int *s_sel = reinterpret_cast<int *>(s_choice + ((p.experts + 3) & ~3));
 		float *s_val = reinterpret_cast<float *>(s_sel + p.top);
 		choose_experts(p.logits, p.correction, p.experts, p.top, s_choice, s_sel, s_val);
 		zw = s_sel[z];
@@ -110,67 +116,131 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 
 	// the vector's prologue: elements [k0, k0 + kn), then zeros that the surplus steps of the last round multiply
 	if constexpr (PRO == TG_VP_PLAIN || PRO == TG_VP_EXPERT) {
-		load(kf0);
-		const float *x = p.x + (PRO == TG_VP_PLAIN ? (size_t)z * p.x_zstride : 0);
-		for (int j = tid; j < kn; j += NT) xs[j] = (T)x[k0 + j];
+		const float *x = p.x + (PRO == TG_VP_PLAIN ? (size_t)z * p.x_zstride : 0) + k0;
+		for (int b = 0; b == 0 || b < kn; b += 8 * NT) {
+			f32x4_t v[2];
+#pragma unroll
+			for (int i = 0; i < 2; i++) v[i] = tg_load4(x + min(b + 4 * (tid + i * NT), max(kn - 4, 0)));
+			if (b == 0) load(kf0);
+#pragma unroll
+			for (int i = 0; i < 2; i++)
+				if (b + 4 * (tid + i * NT) < kn) tg_store4(xs + b + 4 * (tid + i * NT), v[i]);
+		}
 	} else if constexpr (PRO == TG_VP_DYT) {
-		load(kf0);
 		int row = 0;
 		if (p.embed) {
 			row = p.ctr[4];
 			row = row < 0 ? 0 : (row >= p.vocab ? p.vocab - 1 : row);
 		}
-		for (int j = tid; j < kn; j += NT) {
-			const int c = k0 + j, cc = c < p.width ? c : 0;
-			float x = p.embed ? (float)((const __bf16 *)p.embed)[(size_t)row * p.embed_ld + cc] : p.x[cc];
-			float add = 0.0f;
-			for (int q = 0; q < p.nparts; q++) add += p.pend[(size_t)q * p.pend_stride + cc];
-			if (p.nparts) x = x + p.mult * add;
-			const float h = tanhf(p.alpha * x) * p.nw[cc] + p.nb[cc];
-			const bool in = c < p.width;
-			xs[j] = (T)(in ? h : 0.0f);
-			if (blockIdx.x == 0 && z == 0) {
-				if (p.x_out) p.x_out[c] = in ? x : 0.0f;
-				if (p.h_out) p.h_out[c] = in ? h : 0.0f;
+		// two elements per lane and pass; the padding behind the vector is zero in x, the parts, the norm and the table
+		constexpr int PER = 3, PQ = 8;
+		for (int b = 0; b == 0 || b < kn; b += 2 * PER * NT) {
+			float2 x[PER], nw[PER], nb[PER], pq[PER][PQ];
+			int c[PER];
+#pragma unroll
+			for (int i = 0; i < PER; i++) {
+				const int j = b + 2 * (tid + i * NT);
+				c[i] = k0 + min(j, max(kn - 2, 0));
+				if (p.embed) {
+					const unsigned u = *reinterpret_cast<const unsigned *>((const __bf16 *)p.embed + (size_t)row * p.embed_ld + c[i]);
+					x[i] = float2{__uint_as_float(u << 16), __uint_as_float(u & 0xffff0000u)};
+				} else {
+					x[i] = *reinterpret_cast<const float2 *>(p.x + c[i]);
+				}
+				nw[i] = *reinterpret_cast<const float2 *>(p.nw + c[i]);
+				nb[i] = *reinterpret_cast<const float2 *>(p.nb + c[i]);
+			}
+			float2 add[PER];
+#pragma unroll
+			for (int i = 0; i < PER; i++) add[i] = float2{0.0f, 0.0f};
+			for (int q0 = 0; q0 < p.nparts; q0 += PQ) {
+#pragma unroll
+				for (int q = 0; q < PQ; q++)
+#pragma unroll
+					for (int i = 0; i < PER; i++)
+						pq[i][q] = *reinterpret_cast<const float2 *>(p.pend + (size_t)min(q0 + q, p.nparts - 1) * p.pend_stride + c[i]);
+				if (b == 0 && q0 == 0) load(kf0);
+#pragma unroll
+				for (int q = 0; q < PQ; q++)
+					if (q0 + q < p.nparts)
+#pragma unroll
+						for (int i = 0; i < PER; i++) {
+							add[i].x += pq[i][q].x;
+							add[i].y += pq[i][q].y;
+						}
+			}
+			if (b == 0 && p.nparts == 0) load(kf0);
+#pragma unroll
+			for (int i = 0; i < PER; i++) {
+				const int j = b + 2 * (tid + i * NT);
+				if (p.nparts) {
+					x[i].x = x[i].x + p.mult * add[i].x;
+					x[i].y = x[i].y + p.mult * add[i].y;
+				}
+				const float2 h = {tanhf(p.alpha * x[i].x) * nw[i].x + nb[i].x, tanhf(p.alpha * x[i].y) * nw[i].y + nb[i].y};
+				if (j < kn) {
+					xs[j] = (T)h.x;
+					xs[j + 1] = (T)h.y;
+					if (blockIdx.x == 0 && z == 0) {
+						if (p.x_out) *reinterpret_cast<float2 *>(p.x_out + c[i]) = x[i];
+						if (p.h_out) *reinterpret_cast<float2 *>(p.h_out + c[i]) = h;
+					}
+				}
 			}
 		}
 	} else if constexpr (PRO == TG_VP_HEADNORM) {
-		load(kf0);
-		// head by head, a wave each: sum of squares, then the head's elements that lie in this part of K
-		const int h_lo = k0 / p.vdimp, h_hi = min((k0 + kn - 1) / p.vdimp, p.heads16 - 1);
-		for (int j = tid; j < kn; j += NT)
-			if ((k0 + j) / p.vdimp >= p.heads16) xs[j] = (T)0.0f;
+		// head by head, a wave each, four elements per lane and pass: sum of squares, then the head's elements that lie in
+		// this part of K
+		const int h_lo = k0 / p.vdimp, h_hi = min((k0 + kn - 1) / p.vdimp, p.heads16 - 1), vl = p.vdimp - 4;
+		bool first = true;
 		for (int a = h_lo + w; a <= h_hi; a += 4) {
 			const float *o = p.x + (size_t)a * p.vdimp, *g = p.gate + (size_t)a * p.vdimp;
+			const f32x4_t o0 = tg_load4(o + min(4 * lane, vl)), g0 = tg_load4(g + min(4 * lane, vl)), w0 = tg_load4(p.nw + min(4 * lane, vl));
+			if (first) load(kf0);
+			first = false;
 			float ss = 0.0f;
-			for (int v = lane; v < p.vdim; v += 64) ss = fmaf(o[v], o[v], ss);
+			for (int v = 4 * lane; v < p.vdimp; v += 256) {  // the padding is zero
+				const f32x4_t ov = v < 256 ? o0 : tg_load4(o + v);
+#pragma unroll
+				for (int e = 0; e < 4; e++) ss = fmaf(ov[e], ov[e], ss);
+			}
 			ss = tg_wave_sum(ss);
 			const float inv = 1.0f / sqrtf(ss / (float)p.vdim + p.eps);
-			for (int v = lane; v < p.vdimp; v += 64) {
+			for (int v = 4 * lane; v < p.vdimp; v += 256) {
+				const f32x4_t ov = v < 256 ? o0 : tg_load4(o + v), gv = v < 256 ? g0 : tg_load4(g + v), wv = v < 256 ? w0 : tg_load4(p.nw + v);
 				const int j = a * p.vdimp + v - k0;
-				const bool in = v < p.vdim;
-				const int vc = in ? v : 0;
-				const float r = o[vc] * inv * p.nw[vc] * tg_silu(g[vc]);
-				if (j >= 0 && j < kn) xs[j] = (T)(in ? r : 0.0f);
+				f32x4_t r;
+#pragma unroll
+				for (int e = 0; e < 4; e++) r[e] = ov[e] * inv * wv[e] * tg_silu(gv[e]);
+				if (j >= 0 && j < kn) tg_store4(xs + j, r);
 			}
 		}
-	} else {  // MERGE
+		if (first) load(kf0);
+		for (int j = tid; j < kn; j += NT)
+			if ((k0 + j) / p.vdimp >= p.heads16) xs[j] = (T)0.0f;
+	} else {  // MERGE: at most 16 partials
+		const int bl = min(lane & 15, p.nmerge - 1);
+		const float2 ml = *reinterpret_cast<const float2 *>(p.part_ml + ((size_t)bl * p.heads16 + z) * 2);
+		float a[TG_VEC_MERGE_MAX];
+		const float *pa = p.part_acc + (size_t)z * p.x_zstride + k0;
+#pragma unroll
+		for (int b = 0; b < TG_VEC_MERGE_MAX; b++)
+			a[b] = pa[(size_t)min(b, p.nmerge - 1) * p.heads16 * p.x_zstride + min(tid, max(kn - 1, 0))];
 		load(kf0);
-		float m = -INFINITY;
-		for (int b = 0; b < p.nmerge; b++) m = fmaxf(m, p.part_ml[((size_t)b * p.heads16 + z) * 2]);
-		float l = 0.0f;
-		for (int b = 0; b < p.nmerge; b++) {
-			const float *ml = p.part_ml + ((size_t)b * p.heads16 + z) * 2;
-			const float f = expf(ml[0] - m);
-			l += f * ml[1];
-			if (tid == 0) s_misc[b] = f;
-		}
+		const bool in = (lane & 15) < p.nmerge;
+		const float m = tg_row16_max(in ? ml.x : -INFINITY);
+		const float f = in ? expf(ml.x - m) : 0.0f;
+		const float inv = 1.0f / tg_row16_sum(f * ml.y);
+		if (tid < 16) s_misc[tid] = f * inv;
 		__syncthreads();
-		const float inv = 1.0f / l;
 		for (int j = tid; j < kn; j += NT) {
-			float a = 0.0f;
-			for (int b = 0; b < p.nmerge; b++) a = fmaf(s_misc[b], p.part_acc[((size_t)b * p.heads16 + z) * p.x_zstride + k0 + j], a);
-			xs[j] = (T)(a * inv);
+			float r = 0.0f;
+#pragma unroll
+			for (int b = 0; b < TG_VEC_MERGE_MAX; b++) {
+				if (j != tid) a[b] = pa[(size_t)min(b, p.nmerge - 1) * p.heads16 * p.x_zstride + j];
+				r = fmaf(s_misc[b], a[b], r);
+			}
+			xs[j] = (T)r;
 		}
 	}
 	for (int j = kn + tid; j < kn + KW * U * TR::KF; j += NT) xs[j] = (T)0.0f;
@@ -259,7 +329,7 @@ void launch_vec_t(const TgVec &v, hipStream_t s) {
 	const unsigned bx = (unsigned)tg_vec_blocks(v, EPI);
 	auto lds = [&](int pad) {
 		size_t b = sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF;
-		if (PRO == TG_VP_EXPERT) b += sizeof(float) * (size_t)(v.experts + 2 * v.top);
+		if (PRO == TG_VP_EXPERT) b += sizeof(float) * (size_t)(((v.experts + 3) & ~3) + 2 * v.top);
 		return b;
 	};
 	if constexpr (EPI == TG_VE_STORE || EPI == TG_VE_LOGITS) {
@@ -268,7 +338,13 @@ void launch_vec_t(const TgVec &v, hipStream_t s) {
 			return;
 		}
 	}
-	hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 4>), dim3(bx, (unsigned)v.ksplit, (unsigned)v.nz), dim3(NT), lds(16), s, v);
+	// fragments in flight: all of a wave's where they fit, else in as few equal rounds as possible
+	const dim3 grid(bx, (unsigned)v.ksplit, (unsigned)v.nz);
+	const int n = (per + 3) / 4;
+	if (n <= 2) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 2>), grid, dim3(NT), lds(8), s, v);
+	else if (n <= 4) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 4>), grid, dim3(NT), lds(16), s, v);
+	else if (n <= 6 || (n > 9 && n <= 12)) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 6>), grid, dim3(NT), lds(24), s, v);
+	else hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 9>), grid, dim3(NT), lds(36), s, v);
 }
 
 template <class TR>
@@ -285,17 +361,17 @@ void launch_vec_dt(const TgVec &v, int pro, int epi, hipStream_t s) {
 
 // ---- tiled products --------------------------------------------------------------------------------------------------------
 // A workgroup computes BM x BN with WM x WN waves of (16 MI) x (16 NI) each.  K advances by two fragments (128 bytes of a
-// row) per stage: both operands go global -> registers -> LDS in fragment order, the next stage's loads in flight during
-// the matrix instructions of this one, one LDS-only barrier per stage.
+// row) per stage: both operands go global -> registers -> LDS in fragment order (two LDS buffers, two sets of registers: the
+// loads of the next two stages are in flight during the matrix instructions of this one), one LDS-only barrier per stage.
 template <class TR, int EPI, int WM, int WN, int MI, int NI, bool GROUPED>
-__global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
+__global__ __launch_bounds__(256, 2) void linear_kernel(TgGemm g) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
 	constexpr int BM = WM * MI * 16, BN = WN * NI * 16;
 	constexpr int AF = BM / 16, BF = BN / 16, NF = 2 * (AF + BF), PW = NF / 4;  // fragments per stage, per wave
 	static_assert(NF % 4 == 0 && WM * WN == 4, "four waves share a stage's fragments");
 	__shared__ __align__(16) Frag lds[2][NF * 64];
-	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
 	const int ntn = (g.N + BN - 1) / BN;
 
 	// Workgroups go to the 8 XCDs in turn: give each XCD a contiguous run of the tile order, so that the workgroups it
@@ -326,7 +402,9 @@ __global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
 	const int kfr = g.K / TR::KF, nst = kfr / 2, nfr = g.N / 16;
 
 	// this wave's fragments of a stage: f = w * PW + i; the first 2 AF are A (row tile f / 2, k half f % 2), then B
-	const unsigned char *src[PW];
+	// (addresses: a base that the wave shares, 32-bit offsets per lane; operands are below 4 GiB)
+	const unsigned char *base[PW];
+	unsigned off[PW];
 	int adv[PW];
 #pragma unroll
 	for (int i = 0; i < PW; i++) {
@@ -334,22 +412,25 @@ __global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
 		if (f < 2 * AF) {
 			int r = min(m0 + (f >> 1) * 16 + (lane & 15), m1 - 1);
 			if (g.row_src) r = g.row_src[r];
-			src[i] = reinterpret_cast<const unsigned char *>(g.A) + ((size_t)r * g.lda + (f & 1) * TR::KF) * sizeof(T) + (lane >> 4) * 16;
+			base[i] = reinterpret_cast<const unsigned char *>(g.A) + (f & 1) * 64;
+			off[i] = (unsigned)r * (unsigned)(g.lda * (int)sizeof(T)) + (unsigned)(lane >> 4) * 16u;
 			adv[i] = 128;
 		} else {
 			const int fb = f - 2 * AF, nf = min(tn * BF + (fb >> 1), nfr - 1);
-			src[i] = reinterpret_cast<const unsigned char *>(W + ((size_t)nf * kfr + (fb & 1)) * 64 + lane);
+			base[i] = reinterpret_cast<const unsigned char *>(W + ((size_t)nf * kfr + (fb & 1)) * 64);
+			off[i] = (unsigned)lane * 16u;
 			adv[i] = 2048;
 		}
 	}
-	Frag st[PW];
-	auto fetch = [&](int s) {
+	Frag st[2][PW];
+	auto fetch = [&](int set, int s) {
+		s = min(s, nst - 1);
 #pragma unroll
-		for (int i = 0; i < PW; i++) st[i] = *reinterpret_cast<const Frag *>(src[i] + (size_t)s * adv[i]);
+		for (int i = 0; i < PW; i++) st[set][i] = *reinterpret_cast<const Frag *>(base[i] + (size_t)s * adv[i] + off[i]);
 	};
-	auto put = [&](int buf) {
+	auto put = [&](int set) {
 #pragma unroll
-		for (int i = 0; i < PW; i++) lds[buf][(w * PW + i) * 64 + lane] = st[i];
+		for (int i = 0; i < PW; i++) lds[set][(w * PW + i) * 64 + lane] = st[set][i];
 	};
 	const int wm = w / WN, wn = w - wm * WN;
 	f32x4_t acc[MI][NI];
@@ -358,26 +439,32 @@ __global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
 #pragma unroll
 		for (int j = 0; j < NI; j++) acc[i][j] = f32x4_t{0, 0, 0, 0};
 
-	fetch(0);
+	fetch(0, 0);
+	fetch(1, 1);
 	put(0);
+	fetch(0, 2);
 	tg_lds_barrier();
-	for (int s = 0; s < nst; s++) {
-		const int buf = s & 1;
-		fetch(s + 1 < nst ? s + 1 : s);
+	// buffer and register set of a stage: its parity
+	auto stage = [&](int s, int par) {
 #pragma unroll
 		for (int kh = 0; kh < 2; kh++) {
 			Frag a[MI], bb[NI];
 #pragma unroll
-			for (int i = 0; i < MI; i++) a[i] = lds[buf][((wm * MI + i) * 2 + kh) * 64 + lane];
+			for (int i = 0; i < MI; i++) a[i] = lds[par][((wm * MI + i) * 2 + kh) * 64 + lane];
 #pragma unroll
-			for (int j = 0; j < NI; j++) bb[j] = lds[buf][(2 * AF + (wn * NI + j) * 2 + kh) * 64 + lane];
+			for (int j = 0; j < NI; j++) bb[j] = lds[par][(2 * AF + (wn * NI + j) * 2 + kh) * 64 + lane];
 #pragma unroll
 			for (int i = 0; i < MI; i++)
 #pragma unroll
 				for (int j = 0; j < NI; j++) acc[i][j] = EPI == TG_GE_TRANS ? TR::mma(a[i], bb[j], acc[i][j]) : TR::mma(bb[j], a[i], acc[i][j]);
 		}
-		put(buf ^ 1);
+		put(par ^ 1);
+		fetch(par ^ 1, s + 3);
 		tg_lds_barrier();
+	};
+	for (int s = 0; s < nst; s += 2) {
+		stage(s, 0);
+		if (s + 1 < nst) stage(s + 1, 1);
 	}
 
 	const int lr = lane & 15, lg = lane >> 4;
@@ -432,8 +519,55 @@ __global__ __launch_bounds__(256) void linear_kernel(TgGemm g) {
 	}
 }
 
+// Few columns (a router): 16 rows x 64 columns per workgroup, the waves share K, operands straight from memory in fragment
+// order, partial sums meet in LDS.
+template <class TR>
+__global__ __launch_bounds__(256) void linear_thin_kernel(TgGemm g) {
+	typedef typename TR::T T;
+	typedef typename TR::Frag Frag;
+	constexpr int NI = 4, U = 4;
+	__shared__ f32x4_t s_acc[4][NI][64];
+	const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
+	const int m0 = blockIdx.x * 16, n0 = blockIdx.y * NI, kfr = g.K / TR::KF, nfr = g.N / 16;
+	const T *A = (const T *)g.A + (size_t)min(m0 + lr, g.M - 1) * g.lda + lg * TR::KV;
+	const Frag *W = reinterpret_cast<const Frag *>(g.W) + lane;
+	f32x4_t acc[NI];
+#pragma unroll
+	for (int j = 0; j < NI; j++) acc[j] = f32x4_t{0, 0, 0, 0};
+	for (int kf = w; kf < kfr; kf += 4 * U) {
+		Frag a[U], b[U][NI];
+#pragma unroll
+		for (int u = 0; u < U; u++) {
+			const int kc = min(kf + 4 * u, kfr - 1);
+			a[u] = *reinterpret_cast<const Frag *>(A + (size_t)kc * TR::KF);
+#pragma unroll
+			for (int j = 0; j < NI; j++) b[u][j] = W[((size_t)min(n0 + j, nfr - 1) * kfr + kc) * 64];
+		}
+#pragma unroll
+		for (int u = 0; u < U; u++) {
+			if (kf + 4 * u >= kfr) a[u] = Frag{};
+#pragma unroll
+			for (int j = 0; j < NI; j++) acc[j] = TR::mma(b[u][j], a[u], acc[j]);
+		}
+	}
+#pragma unroll
+	for (int j = 0; j < NI; j++) s_acc[w][j][lane] = acc[j];
+	__syncthreads();
+	// wave w: column fragment w
+	f32x4_t r;
+#pragma unroll
+	for (int e = 0; e < 4; e++) r[e] = (s_acc[0][w][lane][e] + s_acc[1][w][lane][e]) + (s_acc[2][w][lane][e] + s_acc[3][w][lane][e]);
+	if (m0 + lr < g.M && n0 + w < nfr) tg_store4(g.C2 + (size_t)(m0 + lr) * g.ldc2 + (n0 + w) * 16 + 4 * lg, r);
+}
+
 template <class TR, int EPI>
 void launch_linear_t(const TgGemm &g, hipStream_t s) {
+	if constexpr (EPI == TG_GE_F32) {
+		if (g.N <= 256) {
+			hipLaunchKernelGGL((linear_thin_kernel<TR>), dim3((unsigned)((g.M + 15) / 16), (unsigned)((g.N + 63) / 64)), dim3(256), 0, s, g);
+			return;
+		}
+	}
 	if (g.tiles) {
 		if constexpr (EPI == TG_GE_STORE || EPI == TG_GE_SWIGLU) {
 			const unsigned grid = (unsigned)g.max_tiles * (unsigned)((g.N + 127) / 128);

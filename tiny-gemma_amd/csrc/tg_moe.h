@@ -5,7 +5,7 @@
 #include "tg_linear.h"
 
 #define TG_MOE_MAX_EXPERTS 1024
-#define TG_MOE_BLOCK 64  // tokens per routing workgroup
+#define TG_MOE_BLOCK 16  // tokens per routing workgroup
 
 // Routing of n tokens: logits [n][ld] fp32.  Expert e's rows are the slots [offset(e), offset(e + 1)); tiles of tile_rows slots
 // of one expert each, as the grouped products take them.

@@ -48,35 +48,55 @@ __global__ __launch_bounds__(256) void moe_route_kernel(TgMoeRoute r) {
 	for (int e = tid; e < E; e += 256) r.count[(size_t)blockIdx.x * E + e] = s_cnt[e];
 }
 
-// one workgroup, a thread per expert: first slot of every (block, expert), and the tile list
-__global__ __launch_bounds__(TG_MOE_MAX_EXPERTS) void moe_offsets_kernel(TgMoeRoute r, int blocks) {
-	__shared__ int s_n[TG_MOE_MAX_EXPERTS], s_t[TG_MOE_MAX_EXPERTS];
-	const int e = threadIdx.x, E = r.experts;
-	int cnt = 0;
-	if (e < E)
-		for (int b = 0; b < blocks; b++) cnt += r.count[(size_t)b * E + e];
-	const int nt = (cnt + r.tile_rows - 1) / r.tile_rows;
-	s_n[e] = cnt;
-	s_t[e] = nt;
+// One workgroup: first slot of every (block, expert), and the tile list.  A thread per expert and segment of the blocks
+// (ep = experts rounded up to a power of two, TG_MOE_MAX_EXPERTS / ep segments).
+__global__ __launch_bounds__(TG_MOE_MAX_EXPERTS) void moe_offsets_kernel(TgMoeRoute r, int blocks, int ep) {
+	__shared__ int s_seg[TG_MOE_MAX_EXPERTS], s_n[TG_MOE_MAX_EXPERTS], s_t[TG_MOE_MAX_EXPERTS];
+	const int E = r.experts, tid = threadIdx.x, e = tid & (ep - 1), seg = tid / ep, segs = TG_MOE_MAX_EXPERTS / ep;
+	const int per = (blocks + segs - 1) / segs, b0 = min(seg * per, blocks), b1 = min(b0 + per, blocks);
+	const int ec = min(e, E - 1);
+	int own = 0;
+	for (int b = b0; b < b1; b += 8) {
+		int c[8];
+#pragma unroll
+		for (int i = 0; i < 8; i++) c[i] = r.count[(size_t)min(b + i, b1 - 1) * E + ec];
+#pragma unroll
+		for (int i = 0; i < 8; i++) own += (b + i < b1 && e < E) ? c[i] : 0;
+	}
+	s_seg[tid] = own;
 	__syncthreads();
-	for (int o = 1; o < TG_MOE_MAX_EXPERTS; o <<= 1) {  // inclusive sums
-		const int a = e >= o ? s_n[e - o] : 0, b = e >= o ? s_t[e - o] : 0;
+	for (int o = 1; o < segs; o <<= 1) {  // inclusive sums over the segments of an expert
+		const int v = seg >= o ? s_seg[tid - o * ep] : 0;
 		__syncthreads();
-		s_n[e] += a;
-		s_t[e] += b;
+		s_seg[tid] += v;
+		__syncthreads();
+	}
+	const int cnt = s_seg[(segs - 1) * ep + e], nt = (cnt + r.tile_rows - 1) / r.tile_rows, before = s_seg[tid] - own;
+	if (tid < ep) {
+		s_n[e] = cnt;
+		s_t[e] = nt;
+	}
+	__syncthreads();
+	for (int o = 1; o < ep; o <<= 1) {  // inclusive sums over the experts
+		const int a = tid < ep && e >= o ? s_n[e - o] : 0, b = tid < ep && e >= o ? s_t[e - o] : 0;
+		__syncthreads();
+		if (tid < ep) {
+			s_n[e] += a;
+			s_t[e] += b;
+		}
 		__syncthreads();
 	}
 	const int first = s_n[e] - cnt, t0 = s_t[e] - nt;
 	if (e < E) {
-		int run = first;
-		for (int b = 0; b < blocks; b++) {
+		int run = first + before;
+		for (int b = b0; b < b1; b++) {
 			const int c = r.count[(size_t)b * E + e];
 			r.count[(size_t)b * E + e] = run;
 			run += c;
 		}
-		for (int i = 0; i < nt; i++) r.tiles[t0 + i] = int4{e, first + i * r.tile_rows, min(first + (i + 1) * r.tile_rows, first + cnt), 0};
+		for (int i = seg; i < nt; i += segs) r.tiles[t0 + i] = int4{e, first + i * r.tile_rows, min(first + (i + 1) * r.tile_rows, first + cnt), 0};
 	}
-	if (e == E - 1) *r.ntiles = s_t[e];
+	if (tid == E - 1) *r.ntiles = s_t[e];
 }
 
 __global__ __launch_bounds__(256) void moe_scatter_kernel(TgMoeRoute r) {
@@ -135,7 +155,9 @@ void tg_launch_moe_route(const TgMoeRoute &r, hipStream_t s) {
 	const int blocks = (r.n + TG_MOE_BLOCK - 1) / TG_MOE_BLOCK;
 	const size_t lds = sizeof(float) * (5 * (size_t)r.experts + 8 * (size_t)r.top);
 	hipLaunchKernelGGL(moe_route_kernel, dim3((unsigned)blocks), dim3(256), lds, s, r);
-	hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(TG_MOE_MAX_EXPERTS), 0, s, r, blocks);
+	int ep = 1;
+	while (ep < r.experts) ep *= 2;
+	hipLaunchKernelGGL(moe_offsets_kernel, dim3(1), dim3(TG_MOE_MAX_EXPERTS), 0, s, r, blocks, ep);
 	hipLaunchKernelGGL(moe_scatter_kernel, dim3((unsigned)((r.n * r.top + 255) / 256)), dim3(256), 0, s, r);
 }
 

@@ -502,14 +502,13 @@ void norm_prologue(const TgNet *n, TgVec *v, const Norm &nm) {
 	v->nw = nm.w;
 	v->nb = nm.b;
 	v->alpha = nm.alpha;
-	v->width = n->cfg.width;
 	v->mult = n->cfg.residual_mult;
 }
 
 // Latent attention of one token: keys per workgroup and the number of parts for a context of ctx keys.
 void latent_parts(int ctx, int *chunk, int *nb) {
 	const int c = (ctx + TG_LATENT_MAX_BLOCKS - 1) / TG_LATENT_MAX_BLOCKS;
-	*chunk = tg_up(c, 64);
+	*chunk = tg_up(c, TG_LATENT_TILE);
 	*nb = (ctx + *chunk - 1) / *chunk;
 }
 
@@ -537,6 +536,9 @@ int tg_net_open(const char *dir, int dt, int n_cu, hipStream_t s, TgNet **out) {
 	int rc = tg_fail(TG_ERR_UNSUPPORTED_SHAPE, "unknown architecture '" + a->str + "'");
 	for (const Arch &k : ARCHS)
 		if (a->str == k.name) rc = k.parse(j, &n->cfg);
+	for (const TgNetLayerCfg &l : n->cfg.layers)
+		if (!rc && l.mix.kind == TG_MIX_LATENT && tg_latent_step_lds(tg_up(l.mix.rank, 64), dt) > TG_LATENT_LDS_MAX)
+			rc = tg_fail(TG_ERR_UNSUPPORTED_SHAPE, "kv_rank " + std::to_string(l.mix.rank) + " does not fit the LDS in this number format");
 	if (!rc) rc = load_weights(n, std::string(dir) + "/model.safetensors");
 	if (rc) {
 		tg_net_free(n);
@@ -610,6 +612,8 @@ int tg_net_seq_create(TgNet *n, int capacity, TgNetSeq **out) {
 		void *p = nullptr;
 		if (hipMalloc(&p, bytes) != hipSuccess) return fail("layer state");
 		q->state.push_back(p);
+		// (a tile of the latent cache is read whole, its rows behind the sequence with weight 0: they must hold numbers)
+		if (hipMemset(p, 0, bytes) != hipSuccess) return fail("layer state");
 		q->state_bytes.push_back(bytes);
 		if (c.mlp) {
 			lg = std::max(lg, (size_t)w.router.n);
