@@ -6,6 +6,7 @@
 #include "tg_linear.h"
 
 #define TG_GLA_CHUNK 64
+#define TG_GLA_VDIM_MAX 512  // largest padded value size of the chunked form
 
 struct TgGla {
 	int heads, dim, dimp, vdim, vdimp, rank;
@@ -20,10 +21,9 @@ void tg_launch_gla_step(const TgGla &g, const float *y, int k_off, int v_off, in
 // n tokens: qkv [n][ld] in the model's format (q at column 0, offsets in elements), low [n][ld_low] fp32 (the decay's low-rank input).
 // Scratch: see tg_gla_scratch.  out [n][ld_out]: the normalised, gated heads.
 struct TgGlaScratch {
-	float *b;       // [chunks * 64][heads * dimp] running sums of log alpha inside a chunk
+	float *b;       // [chunks * 64][heads * dimp] running sums of log2 alpha inside a chunk
 	float *a;       // [chunks][heads][64][64]
 	float *u;       // [chunks][heads][dimp][vdimp]
-	float *o;       // [n][heads * vdimp]
 };
 size_t tg_gla_scratch(const TgGla &g, int n, TgGlaScratch *t, unsigned char *base);  // bytes; fills *t when base is not null
 void tg_launch_gla_rows(const TgGla &g, int dt, const void *qkv, int ld, int k_off, int v_off, int g_off, const float *low, int ld_low, int n,

@@ -3,8 +3,8 @@
 // Chunked form.  With b_t the sum of log alpha over the chunk's tokens up to and including t, a chunk of 64 tokens that
 // starts from state S contributes
 //     o_i = (q_i e^{b_i})^T S + sum_{j <= i} A_ij v_j,   A_ij = sum_d q_id k_jd e^{b_id - b_jd},
-//     S'  = diag(e^{b_end}) S + sum_j (k_j e^{b_end - b_j}) v_j^T,
-// all exponents <= 0, whatever the decay: A's blocks of 16 x 16 below the diagonal take the exponent apart at the row
+//     S'  = diag(e^{b_end}) S + sum_j (k_j e^{b_end - b_j}) v_j^T
+// (b is kept in units of log 2, so every exponential is one v_exp_f32), all exponents <= 0, whatever the decay: A's blocks of 16 x 16 below the diagonal take the exponent apart at the row
 // block's first token (both halves <= 0) and run on the fp32 matrix instructions, the diagonal blocks are summed pair by
 // pair.  Four launches: b; A and the chunks' own state contributions U, all chunks at once; the states in front of every
 // chunk, one pass over U; the outputs, all chunks at once.  Everything is fp32 (q, k, v are read in the model's format).
@@ -14,6 +14,7 @@
 namespace {
 
 constexpr int C = TG_GLA_CHUNK;
+__device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // ---- one token -----------------------------------------------------------------------------------------------------------
 // A workgroup owns 32 value columns of a head: lane = 4 columns, 32 groups of key channels.
@@ -41,7 +42,7 @@ __global__ __launch_bounds__(256) void gla_step_kernel(const float *y, TgGla g, 
 #pragma unroll
 			for (int j = 0; j < 16; j++) z = j0 + j < g.rank ? fmaf(wa[j], ya[j], z) : z;
 		}
-		s_a[d] = expf(tg_log_sigmoid(z + g.a2b[c]) * g.inv_tau);
+		s_a[d] = pow2(tg_log2_sigmoid(z + g.a2b[c]) * g.inv_tau);
 		s_q[d] = y[c] * g.qscale;
 		s_k[d] = y[k_off + c];
 	}
@@ -116,7 +117,7 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld
 	float run = 0.0f;
 #pragma unroll
 	for (int i = 0; i < 16; i++) {
-		if (real && t0 + 16 * w + i < n) run += tg_log_sigmoid(z[i]) * g.inv_tau;  // past the end: the sum stays
+		if (real && t0 + 16 * w + i < n) run += tg_log2_sigmoid(z[i]) * g.inv_tau;  // past the end: the sum stays
 		z[i] = run;
 	}
 	s_sum[w][lane] = run;
@@ -160,11 +161,11 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 			for (int st = 0; st < SL / 4; st++) {
 				const int d = 4 * st + lg;
 				const float ref = s_b[16 * w - 1][d];
-				const float qv = s_q[qi][d] * expf(s_b[qi][d] - ref);
+				const float qv = s_q[qi][d] * pow2(s_b[qi][d] - ref);
 #pragma unroll
 				for (int j = 0; j < 3; j++)
 					if (j < w) {
-						const float kv = s_k[16 * j + lr][d] * expf(ref - s_b[16 * j + lr][d]);
+						const float kv = s_k[16 * j + lr][d] * pow2(ref - s_b[16 * j + lr][d]);
 						off[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv, kv, off[j], 0, 0, 0);
 					}
 			}
@@ -177,7 +178,7 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 				const f32x4_t k = tg_load4(&s_k[kj][d]), bj = tg_load4(&s_b[kj][d]);
 				if (kj <= qi) {
 #pragma unroll
-					for (int e = 0; e < 4; e++) dia[j] = fmaf(q[e] * k[e], expf(bi[e] - bj[e]), dia[j]);
+					for (int e = 0; e < 4; e++) dia[j] = fmaf(q[e] * k[e], pow2(bi[e] - bj[e]), dia[j]);
 				}
 			}
 		}
@@ -194,153 +195,189 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 	}
 }
 
-// ---- U = sum_j (k_j e^{b_end - b_j}) v_j^T: 64 key channels x 64 value columns per workgroup ----------------------------------
-constexpr int BP = 68;
-template <class TR>
-__global__ __launch_bounds__(256) void gla_state_kernel(const typename TR::T *qkv, int ld, int k_off, int v_off, TgGla g, int n, const float *b,
+// ---- U = sum_j (k_j e^{b_end - b_j}) v_j^T: 128 key channels x VB value columns per workgroup, 8 waves of 64 x VB / 4 -----------
+template <class TR, int VB>
+__global__ __launch_bounds__(512) void gla_state_kernel(const typename TR::T *qkv, int ld, int k_off, int v_off, TgGla g, int n, const float *b,
                                                         float *U) {
-	__shared__ __align__(16) float s_k[C][BP], s_v[C][BP];
-	const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-	const int nvb = (g.vdimp + 63) / 64, d0 = (int)(blockIdx.z / nvb) * 64, v0 = (int)(blockIdx.z % nvb) * 64;
+	constexpr int KP = 128 + 16, VP = VB + 16, NI = VB / 64;  // pitches: four rows side by side meet all banks
+	__shared__ __align__(16) float s_k[C][KP], s_v[C][VP];
+	const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, wd = (w & 1) * 64, wv = (w >> 1) * (VB / 4);
+	const int nvb = (g.vdimp + VB - 1) / VB, d0 = (int)(blockIdx.z / nvb) * 128, v0 = (int)(blockIdx.z % nvb) * VB;
 	const int lr = lane & 15, lg = lane >> 4, hd = g.heads * g.dimp, t0 = ch * C;
-	for (int e = tid; e < C * 16; e += 256) {
-		const int r = e >> 4, c4 = (e & 15) * 4, t = t0 + r, tc = min(t, n - 1);
-		const bool kin = t < n && d0 + c4 < g.dimp, vin = t < n && v0 + c4 < g.vdimp;
-		const size_t kc = (size_t)h * g.dimp + (kin ? d0 + c4 : 0), vc = (size_t)h * g.vdimp + (vin ? v0 + c4 : 0);
-		const f32x4_t k = tg_load4(qkv + (size_t)tc * ld + k_off + kc), v = tg_load4(qkv + (size_t)tc * ld + v_off + vc);
-		const f32x4_t be = tg_load4(b + (size_t)(t0 + C - 1) * hd + kc), bj = tg_load4(b + (size_t)t * hd + kc);
-		f32x4_t ks, vs;
 #pragma unroll
-		for (int i = 0; i < 4; i++) {
-			ks[i] = kin ? k[i] * expf(be[i] - bj[i]) : 0.0f;
-			vs[i] = vin ? v[i] : 0.0f;
-		}
+	for (int i = 0; i < C * 32 / 512; i++) {
+		const int e = tid + 512 * i, r = e >> 5, c4 = (e & 31) * 4, t = t0 + r, tc = min(t, n - 1);
+		const bool in = t < n && d0 + c4 < g.dimp;
+		const size_t kc = (size_t)h * g.dimp + (in ? d0 + c4 : 0);
+		const f32x4_t k = tg_load4(qkv + (size_t)tc * ld + k_off + kc);
+		const f32x4_t be = tg_load4(b + (size_t)(t0 + C - 1) * hd + kc), bj = tg_load4(b + (size_t)t * hd + kc);
+		f32x4_t ks;
+#pragma unroll
+		for (int q = 0; q < 4; q++) ks[q] = in ? k[q] * pow2(be[q] - bj[q]) : 0.0f;
 		tg_store4(&s_k[r][c4], ks);
-		tg_store4(&s_v[r][c4], vs);
+	}
+#pragma unroll
+	for (int i = 0; i < C * VB / 4 / 512; i++) {
+		const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4, t = t0 + r, tc = min(t, n - 1);
+		const bool in = t < n && v0 + c4 < g.vdimp;
+		f32x4_t v = tg_load4(qkv + (size_t)tc * ld + v_off + (size_t)h * g.vdimp + (in ? v0 + c4 : 0));
+		if (!in) v = f32x4_t{0, 0, 0, 0};
+		tg_store4(&s_v[r][c4], v);
 	}
 	__syncthreads();
-	f32x4_t acc[4];
+	f32x4_t acc[4][NI];
 #pragma unroll
-	for (int j = 0; j < 4; j++) acc[j] = f32x4_t{0, 0, 0, 0};
+	for (int i = 0; i < 4; i++)
+#pragma unroll
+		for (int j = 0; j < NI; j++) acc[i][j] = f32x4_t{0, 0, 0, 0};
 #pragma unroll 4
 	for (int t = 0; t < C; t += 4) {
-		const float a = s_k[t + lg][16 * w + lr];
+		float a[4], v[NI];
 #pragma unroll
-		for (int j = 0; j < 4; j++) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, s_v[t + lg][16 * j + lr], acc[j], 0, 0, 0);
+		for (int i = 0; i < 4; i++) a[i] = s_k[t + lg][wd + 16 * i + lr];
+#pragma unroll
+		for (int j = 0; j < NI; j++) v[j] = s_v[t + lg][wv + 16 * j + lr];
+		// value columns are the first operand: a lane holds four of them for one key channel
+#pragma unroll
+		for (int i = 0; i < 4; i++)
+#pragma unroll
+			for (int j = 0; j < NI; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[j], a[i], acc[i][j], 0, 0, 0);
 	}
 	float *out = U + ((size_t)ch * g.heads + h) * g.dimp * g.vdimp;
 #pragma unroll
-	for (int j = 0; j < 4; j++)
+	for (int i = 0; i < 4; i++)
 #pragma unroll
-		for (int e = 0; e < 4; e++) {
-			const int d = d0 + 16 * w + 4 * lg + e, v = v0 + 16 * j + lr;
-			if (d < g.dimp && v < g.vdimp) out[(size_t)d * g.vdimp + v] = acc[j][e];
+		for (int j = 0; j < NI; j++) {
+			const int d = d0 + wd + 16 * i + lr, v = v0 + wv + 16 * j + 4 * lg;
+			if (d < g.dimp && v < g.vdimp) tg_store4(out + (size_t)d * g.vdimp + v, acc[i][j]);
 		}
 }
 
 // ---- U becomes the state in front of its chunk; the state behind the last chunk goes to the sequence ---------------------------
 __global__ __launch_bounds__(256) void gla_scan_kernel(float *U, const float *b, TgGla g, int chunks) {
-	const size_t per = (size_t)g.heads * g.dimp * g.vdimp, e = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+	constexpr int AHEAD = 8;  // chunks whose loads are in flight
+	const size_t per = (size_t)g.heads * g.dimp * g.vdimp, e = (size_t)blockIdx.x * 256 + threadIdx.x;
 	if (e >= per) return;
 	const int hd = g.heads * g.dimp, c = (int)(e / g.vdimp);
-	f32x4_t s = tg_load4(g.state + e), nxt = tg_load4(U + e);
-	float bn = b[(size_t)(C - 1) * hd + c];
-	for (int ch = 0; ch < chunks; ch++) {
-		const f32x4_t u = nxt;
-		const float dec = expf(bn);
-		if (ch + 1 < chunks) {
-			nxt = tg_load4(U + (size_t)(ch + 1) * per + e);
-			bn = b[(size_t)((ch + 1) * C + C - 1) * hd + c];
-		}
-		tg_store4(U + (size_t)ch * per + e, s);
+	float s = g.state[e], u[AHEAD], bn[AHEAD];
+	auto load = [&](int i, int ch) {
+		ch = min(ch, chunks - 1);
+		u[i] = U[(size_t)ch * per + e];
+		bn[i] = b[(size_t)(ch * C + C - 1) * hd + c];
+	};
 #pragma unroll
-		for (int i = 0; i < 4; i++) s[i] = fmaf(dec, s[i], u[i]);
+	for (int i = 0; i < AHEAD; i++) load(i, i);
+	for (int ch = 0; ch < chunks; ch += AHEAD) {
+#pragma unroll
+		for (int i = 0; i < AHEAD; i++) {
+			if (ch + i < chunks) {
+				U[(size_t)(ch + i) * per + e] = s;
+				s = fmaf(pow2(bn[i]), s, u[i]);
+			}
+			load(i, ch + i + AHEAD);  // (past the end: the last chunk again, unused)
+		}
 	}
-	tg_store4(g.state + e, s);
+	g.state[e] = s;
 }
 
-// ---- o = (q e^b)^T S + A v: 64 tokens x 64 value columns per workgroup -----------------------------------------------------------
-template <class TR>
-__global__ __launch_bounds__(256) void gla_out_kernel(const typename TR::T *qkv, int ld, int v_off, TgGla g, int n, const float *b, const float *A,
-                                                      const float *U, float *o) {
-	__shared__ __align__(16) float s_a[C][BP], s_b[C][BP];
-	const int ch = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * 64, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+// ---- o = (q e^b)^T S + A v, the head's root mean square norm and silu(gate): 64 tokens x the whole head per workgroup -------------
+// 8 waves: 16 tokens x half of the value columns each.  Slabs of 32: first the key channels (rows q e^b, columns of S), then
+// the chunk's own tokens (rows A, columns v); a slab's loads are in flight during the one before it.
+template <class TR, int VB>
+__global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv, int ld, int v_off, int g_off, TgGla g, int n, const float *b,
+                                                      const float *A, const float *U, typename TR::T *out, int ld_out) {
+	constexpr int XP = 36, YP = VB + 16, NI = VB / 32, NY = 32 * VB / 4 / 512;
+	__shared__ __align__(16) float s_x[C][XP], s_y[32][YP];
+	__shared__ float s_sq[2][C];
+	const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, wt = (w & 3) * 16, wv = (w >> 2) * (VB / 2);
 	const int lr = lane & 15, lg = lane >> 4, hd = g.heads * g.dimp, t0 = ch * C;
 	const float *S = U + ((size_t)ch * g.heads + h) * g.dimp * g.vdimp;
-	f32x4_t acc[4];
+	const int slabs = g.dimp / 32;  // dimp is a multiple of 32
+	f32x4_t x, bx, y[NY];
+	const int xr = tid >> 3, xc = (tid & 7) * 4;
+	auto fetch = [&](int sl) {
+		if (sl < slabs) {
+			const size_t qc = (size_t)h * g.dimp + sl * 32 + xc;
+			x = tg_load4(qkv + (size_t)min(t0 + xr, n - 1) * ld + qc);
+			bx = tg_load4(b + (size_t)(t0 + xr) * hd + qc);
 #pragma unroll
-	for (int j = 0; j < 4; j++) acc[j] = f32x4_t{0, 0, 0, 0};
-	// slabs of 64: the key channels (rows q e^b, columns of S), last the chunk's own tokens (rows A, columns v)
-	const int slabs = (g.dimp + 63) / 64;
-	for (int sl = 0; sl <= slabs; sl++) {
-		__syncthreads();
-		for (int e = tid; e < C * 16; e += 256) {
-			const int r = e >> 4, c4 = (e & 15) * 4;
-			const bool vin = v0 + c4 < g.vdimp;
-			f32x4_t x, y;
-			if (sl < slabs) {
-				const int t = t0 + r, d = sl * 64 + c4;
-				const bool qin = t < n && d < g.dimp, sin = sl * 64 + r < g.dimp && vin;
-				const size_t qc = (size_t)h * g.dimp + (qin ? d : 0);
-				const f32x4_t q = tg_load4(qkv + (size_t)min(t, n - 1) * ld + qc), bq = tg_load4(b + (size_t)t * hd + qc);
-				const f32x4_t sv = tg_load4(S + (size_t)(sin ? sl * 64 + r : 0) * g.vdimp + (sin ? v0 + c4 : 0));
-#pragma unroll
-				for (int i = 0; i < 4; i++) {
-					x[i] = qin ? q[i] * g.qscale * expf(bq[i]) : 0.0f;
-					y[i] = sin ? sv[i] : 0.0f;
-				}
-			} else {
-				const int t = t0 + r;
-				const bool in = t < n && vin;
-				x = tg_load4(A + (((size_t)ch * g.heads + h) * C + r) * C + c4);
-				const f32x4_t v = tg_load4(qkv + (size_t)min(t, n - 1) * ld + v_off + (size_t)h * g.vdimp + (vin ? v0 + c4 : 0));
-#pragma unroll
-				for (int i = 0; i < 4; i++) y[i] = in ? v[i] : 0.0f;
+			for (int i = 0; i < NY; i++) {
+				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
+				y[i] = tg_load4(S + (size_t)(sl * 32 + r) * g.vdimp + (c4 < g.vdimp ? c4 : 0));
 			}
-			tg_store4(&s_a[r][c4], x);
-			tg_store4(&s_b[r][c4], y);
-		}
-		__syncthreads();
-#pragma unroll 4
-		for (int d = 0; d < 64; d += 4) {
-			const float a = s_a[16 * w + lr][d + lg];
+		} else {
+			const int j0 = (sl - slabs) * 32;
+			x = tg_load4(A + (((size_t)ch * g.heads + h) * C + xr) * C + j0 + xc);
 #pragma unroll
-			for (int j = 0; j < 4; j++) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, s_b[d + lg][16 * j + lr], acc[j], 0, 0, 0);
+			for (int i = 0; i < NY; i++) {
+				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
+				y[i] = tg_load4(qkv + (size_t)min(t0 + j0 + r, n - 1) * ld + v_off + (size_t)h * g.vdimp + (c4 < g.vdimp ? c4 : 0));
+			}
+		}
+	};
+	auto put = [&](int sl) {
+		if (sl < slabs) {
+#pragma unroll
+			for (int e = 0; e < 4; e++) x[e] = x[e] * g.qscale * pow2(bx[e]);
+		}
+		tg_store4(&s_x[xr][xc], x);
+#pragma unroll
+		for (int i = 0; i < NY; i++) {
+			const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
+			tg_store4(&s_y[r][c4], c4 < g.vdimp ? y[i] : f32x4_t{0, 0, 0, 0});  // (rows of v past the end meet zeros of A)
+		}
+	};
+	f32x4_t acc[NI];
+#pragma unroll
+	for (int j = 0; j < NI; j++) acc[j] = f32x4_t{0, 0, 0, 0};
+	fetch(0);
+	for (int sl = 0; sl < slabs + 2; sl++) {
+		put(sl);
+		tg_lds_barrier();
+		if (sl + 1 < slabs + 2) fetch(sl + 1);
+#pragma unroll
+		for (int d = 0; d < 32; d += 4) {
+			const float a = s_x[wt + lr][d + lg];
+#pragma unroll
+			for (int j = 0; j < NI; j++) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(s_y[d + lg][wv + 16 * j + lr], a, acc[j], 0, 0, 0);
+		}
+		tg_lds_barrier();
+	}
+	// a lane holds token wt + lr, value columns wv + 16 j + 4 lg ...
+	float ss = 0.0f;
+#pragma unroll
+	for (int j = 0; j < NI; j++)
+#pragma unroll
+		for (int e = 0; e < 4; e++) ss = fmaf(acc[j][e], acc[j][e], ss);
+	ss += tg_red_partner<32>(ss);
+	ss += tg_red_partner<16>(ss);
+	if (lg == 0) s_sq[w >> 2][wt + lr] = ss;
+	__syncthreads();
+	const int t = t0 + wt + lr;
+	if (t >= n) return;
+	const float inv = 1.0f / sqrtf((s_sq[0][wt + lr] + s_sq[1][wt + lr]) / (float)g.vdim + g.eps);
+	typename TR::T *dst = out + (size_t)t * ld_out + (size_t)h * g.vdimp;
+	const typename TR::T *gate = qkv + (size_t)t * ld + g_off + (size_t)h * g.vdimp;
+#pragma unroll
+	for (int j = 0; j < NI; j++) {
+		const int v = wv + 16 * j + 4 * lg;
+		if (v < g.vdimp) {
+			const f32x4_t gv = tg_load4(gate + v), nw = tg_load4(g.norm + v);
+			f32x4_t r;
+#pragma unroll
+			for (int e = 0; e < 4; e++) r[e] = acc[j][e] * inv * nw[e] * tg_silu(gv[e]);
+			tg_store4(dst + v, r);
 		}
 	}
-#pragma unroll
-	for (int j = 0; j < 4; j++)
-#pragma unroll
-		for (int e = 0; e < 4; e++) {
-			const int t = t0 + 16 * w + 4 * lg + e, v = v0 + 16 * j + lr;
-			if (t < n && v < g.vdimp) o[(size_t)t * g.heads * g.vdimp + (size_t)h * g.vdimp + v] = acc[j][e];
-		}
+	if (h == g.heads - 1)  // the columns behind the heads
+		for (int v = g.heads * g.vdimp + (w >> 2) * 16 + 4 * lg; v < ld_out; v += 32) tg_store4(out + (size_t)t * ld_out + v, f32x4_t{0, 0, 0, 0});
 }
 
-// ---- every head over its root mean square, times the norm's weight and silu(gate); a wave per (token, head) ------------------------
-template <class TR>
-__global__ __launch_bounds__(256) void gla_norm_gate_kernel(const float *o, const typename TR::T *gate, int ld, TgGla g, int n, typename TR::T *out,
-                                                            int ld_out) {
-	const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-	const int per = g.heads + 1;  // the last "head" of a token clears the columns behind the heads
-	if (row >= n * per) return;
-	const int t = row / per, h = row - t * per;
-	typename TR::T *dst = out + (size_t)t * ld_out + (size_t)h * g.vdimp;
-	if (h == g.heads) {
-		for (int v = h * g.vdimp + lane; v < ld_out; v += 64) out[(size_t)t * ld_out + v] = (typename TR::T)0.0f;
-		return;
-	}
-	const float *x = o + ((size_t)t * g.heads + h) * g.vdimp;
-	float ss = 0.0f;
-	for (int v = lane; v < g.vdim; v += 64) ss = fmaf(x[v], x[v], ss);
-	ss = tg_wave_sum(ss);
-	const float inv = 1.0f / sqrtf(ss / (float)g.vdim + g.eps);
-	for (int v = lane; v < g.vdimp; v += 64) {
-		const bool in = v < g.vdim;
-		const int vc = in ? v : 0;
-		const float r = x[vc] * inv * g.norm[vc] * tg_silu((float)gate[(size_t)t * ld + (size_t)h * g.vdimp + vc]);
-		dst[v] = (typename TR::T)(in ? r : 0.0f);
-	}
+template <class TR, int VB>
+void launch_out(const TgGla &g, const typename TR::T *x, int ld, int v_off, int g_off, int n, const TgGlaScratch &t, typename TR::T *out, int ld_out,
+                hipStream_t s) {
+	hipLaunchKernelGGL((gla_out_kernel<TR, VB>), dim3((unsigned)((n + C - 1) / C), (unsigned)g.heads), dim3(512), 0, s, x, ld, v_off, g_off, g, n, t.b,
+	                   t.a, t.u, out, ld_out);
 }
 
 template <class TR>
@@ -348,16 +385,21 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
                  const TgGlaScratch &t, void *out, int ld_out, hipStream_t s) {
 	typedef typename TR::T T;
 	const T *x = (const T *)qkv;
-	const unsigned chunks = (unsigned)((n + C - 1) / C), H = (unsigned)g.heads, hd = (unsigned)(g.heads * g.dimp);
-	const unsigned ndb = (unsigned)((g.dimp + 63) / 64), nvb = (unsigned)((g.vdimp + 63) / 64);
+	T *o = (T *)out;
+	const unsigned chunks = (unsigned)((n + C - 1) / C), H = (unsigned)g.heads, hd = (unsigned)(g.heads * g.dimp), nd = (unsigned)((g.dimp + 127) / 128);
 	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (hd + 63) / 64), dim3(256), 0, s, low, ld_low, g, n, t.b);
 	hipLaunchKernelGGL((gla_intra_kernel<TR>), dim3(chunks, H), dim3(256), 0, s, x, ld, k_off, g, n, t.b, t.a);
-	hipLaunchKernelGGL((gla_state_kernel<TR>), dim3(chunks, H, ndb * nvb), dim3(256), 0, s, x, ld, k_off, v_off, g, n, t.b, t.u);
+	if (g.vdimp <= 64)
+		hipLaunchKernelGGL((gla_state_kernel<TR, 64>), dim3(chunks, H, nd), dim3(512), 0, s, x, ld, k_off, v_off, g, n, t.b, t.u);
+	else
+		hipLaunchKernelGGL((gla_state_kernel<TR, 128>), dim3(chunks, H, nd * (unsigned)((g.vdimp + 127) / 128)), dim3(512), 0, s, x, ld, k_off, v_off, g,
+		                   n, t.b, t.u);
 	const size_t per = (size_t)hd * g.vdimp;
-	hipLaunchKernelGGL(gla_scan_kernel, dim3((unsigned)((per / 4 + 255) / 256)), dim3(256), 0, s, t.u, t.b, g, (int)chunks);
-	hipLaunchKernelGGL((gla_out_kernel<TR>), dim3(chunks, H, nvb), dim3(256), 0, s, x, ld, v_off, g, n, t.b, t.a, t.u, t.o);
-	const long long rows = (long long)n * (g.heads + 1);
-	hipLaunchKernelGGL((gla_norm_gate_kernel<TR>), dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, s, t.o, x + g_off, ld, g, n, (T *)out, ld_out);
+	hipLaunchKernelGGL(gla_scan_kernel, dim3((unsigned)((per + 255) / 256)), dim3(256), 0, s, t.u, t.b, g, (int)chunks);
+	if (g.vdimp <= 64) launch_out<TR, 64>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
+	else if (g.vdimp <= 128) launch_out<TR, 128>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
+	else if (g.vdimp <= 256) launch_out<TR, 256>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
+	else launch_out<TR, TG_GLA_VDIM_MAX>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
 }
 
 }  // namespace
@@ -379,7 +421,6 @@ size_t tg_gla_scratch(const TgGla &g, int n, TgGlaScratch *t, unsigned char *bas
 	take(&t->b, chunks * C * hd);
 	take(&t->a, chunks * g.heads * C * C);
 	take(&t->u, chunks * hd * g.vdimp);
-	take(&t->o, (size_t)n * g.heads * g.vdimp);
 	return off;
 }
 

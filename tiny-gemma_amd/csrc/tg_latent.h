@@ -10,7 +10,7 @@
 #include "tg_linear.h"
 
 #define TG_LATENT_MAX_PARTS TG_VEC_MERGE_MAX  // partials that the value product merges in its prologue
-#define TG_LATENT_MAX_BLOCKS 256   // key parts per launch
+#define TG_LATENT_MAX_BLOCKS 128   // key parts per launch
 #define TG_LATENT_TILE 32
 #define TG_LATENT_LDS_MAX (150 * 1024)
 #define TG_LATENT_HEAD_MAX 256     // largest padded head size of the tiled kernel

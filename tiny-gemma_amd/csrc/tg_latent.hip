@@ -5,21 +5,21 @@
 namespace {
 
 // ---- one token -------------------------------------------------------------------------------------------------------------
-// A workgroup takes one part of the keys for 16 heads (HT of which exist), tile by tile of 32.  A tile's latent rows go to LDS
-// in one round trip (the first tile's loads are requested before anything else is done), row pitch 16 bytes more than the row.
-// Scores come from the matrix instructions, wave w: keys 16 (w % 2) ..., half w / 2 of the latent; the running softmax is a
-// wave's work for 4 heads; the value sum stays on the vector units in fp32: a lane owns two latent columns of all heads, for
-// every G-th key (G = 1, 2 or 4 groups of lanes, added at the end), in passes of 512 columns (blockIdx.z).
+// A workgroup takes one part of the keys for 16 heads, tile by tile of 32.  A tile's latent rows go to LDS in one round trip
+// (the first tile's loads are requested before anything else is done), row pitch 16 bytes more than the row.  Scores: wave w
+// takes keys 16 (w % 2) ... and half w / 2 of the latent; the running softmax is a wave's work for 4 heads; the value sum is
+// a product of the probabilities [16 heads x 32 keys] (in the bf16 format two planes, value and remainder) with the tile,
+// wave w the column tiles w, w + 4, ..., in passes of 512 columns (blockIdx.z).
 constexpr int ST = 32;         // keys per tile
 constexpr int ST_LOADS = 8;    // 16-byte pieces per lane and round of the tile copy
 
 template <class TR>
-size_t latent_step_lds(int rankp) {  // q' fragments | tile | (reused) sums of the lane groups
+size_t latent_step_lds(int rankp) {  // q' fragments | tile
 	const size_t row = (size_t)rankp * sizeof(typename TR::T);
 	return 16 * row + ST * (row + 16);
 }
 
-template <class TR, int HT>
+template <class TR>
 __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
@@ -28,7 +28,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	Frag *s_q = reinterpret_cast<Frag *>(smem);  // [rankp / KF][64]
 	unsigned char *s_c = smem + 16 * row;
 	__shared__ float s_half[2][ST][16];
-	__shared__ __align__(16) float s_p[ST][20];
+	__shared__ __align__(16) float s_p[16][ST + 4];
 	__shared__ float s_corr[16], s_sq[4];
 	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
 	const int part = blockIdx.x, h0 = blockIdx.y * 16, heads16 = (int)gridDim.y * 16;
@@ -63,11 +63,21 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	request(kb, 0);
 
 	// q' in operand order: lane = head, 16 bytes of the latent
-	for (int e = tid; e < 4 * a.rankp; e += 256) {
-		const int h = e / (a.rankp / 4), j = (e - h * (a.rankp / 4)) * 4, hh = h0 + h;
-		f32x4_t v = tg_load4(a.q + (size_t)min(hh, a.heads - 1) * a.rankp + j);
-		if (hh >= a.heads) v = f32x4_t{0, 0, 0, 0};
-		tg_store4(reinterpret_cast<T *>(s_q) + ((size_t)(j / TR::KF) * 64 + h + 16 * ((j % TR::KF) / TR::KV)) * TR::KV + j % TR::KV, v);
+	const int q4 = a.rankp / 4;
+	for (int base = 0; base < 16 * q4; base += 256 * 8) {
+		f32x4_t v[8];
+#pragma unroll
+		for (int i = 0; i < 8; i++) {
+			const int e = min(base + tid + 256 * i, 16 * q4 - 1), h = e / q4;
+			v[i] = tg_load4(a.q + (size_t)min(h0 + h, a.heads - 1) * a.rankp + (e - h * q4) * 4);
+		}
+#pragma unroll
+		for (int i = 0; i < 8; i++) {
+			const int e = base + tid + 256 * i, h = e / q4, j = (e - h * q4) * 4;
+			if (h0 + h >= a.heads) v[i] = f32x4_t{0, 0, 0, 0};
+			if (e < 16 * q4)
+				tg_store4(reinterpret_cast<T *>(s_q) + ((size_t)(j / TR::KF) * 64 + h + 16 * ((j % TR::KF) / TR::KV)) * TR::KV + j % TR::KV, v[i]);
+		}
 	}
 	// the new token's latent, normalised, by the workgroups whose part it ends
 	float inv = 0.0f;
@@ -83,16 +93,14 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		inv = 1.0f / sqrtf(((s_sq[0] + s_sq[1]) + (s_sq[2] + s_sq[3])) / (float)a.rank + a.eps);
 	}
 
-	const int cols = min(a.rankp, 512) / 2, G = cols <= 64 ? 4 : (cols <= 128 ? 2 : 1), per = 256 / G;
-	const int grp = tid / per, cl = tid - grp * per, col = blockIdx.z * 512 + 2 * cl;
-	const bool cin = cl < cols && col < a.rankp;
-	const int colc = cin ? col : 0;
-	float acc[HT][2];
+	constexpr int NC = 8;  // column tiles per wave
+	const int ct0 = blockIdx.z * 32 + w, nct = a.rankp / 16;
+	f32x4_t acc[NC];
 #pragma unroll
-	for (int h = 0; h < HT; h++) acc[h][0] = acc[h][1] = 0.0f;
-	float m[4], l[4];
+	for (int c = 0; c < NC; c++) acc[c] = f32x4_t{0, 0, 0, 0};
+	float m[2], l[2];
 #pragma unroll
-	for (int i = 0; i < 4; i++) { m[i] = -INFINITY; l[i] = 0.0f; }
+	for (int i = 0; i < 2; i++) { m[i] = -INFINITY; l[i] = 0.0f; }
 	const int kfr = a.rankp / TR::KF, kh = (kfr + 1) / 2, kf_lo = (w >> 1) * kh, kf_hi = min(kfr, kf_lo + kh);
 	for (int k0 = kb; k0 < ke; k0 += ST) {
 		for (int base = 0; base < ST * ppr; base += 256 * ST_LOADS) {
@@ -131,7 +139,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 				const float mn = fmaxf(m[i], mx), f = expf(m[i] - mn), p = expf(s - mn);
 				float sum = p + tg_red_partner<16>(p);
 				sum = tg_row16_sum(sum);
-				s_p[key][h] = p;
+				s_p[h][key] = p;
 				l[i] = l[i] * f + sum;
 				m[i] = mn;
 				if (key == 0) s_corr[h] = f;
@@ -140,52 +148,46 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		__syncthreads();
 		if (k0 > kb) {
 #pragma unroll
-			for (int h = 0; h < HT; h++) {
-				acc[h][0] *= s_corr[h];
-				acc[h][1] *= s_corr[h];
+			for (int e = 0; e < 4; e++) {
+				const float f = s_corr[4 * lg + e];
+#pragma unroll
+				for (int c = 0; c < NC; c++) acc[c][e] *= f;
 			}
 		}
 		// rows past the part's end repeat its last row, with probability 0
-#pragma unroll 4
-		for (int k = grp; k < ST; k += G) {
-			const T *c = reinterpret_cast<const T *>(s_c + (size_t)k * pitch) + colc;
-			const float c0 = (float)c[0], c1 = (float)c[1];
 #pragma unroll
-			for (int h4 = 0; h4 < HT / 4; h4++) {
-				const f32x4_t p = tg_load4(&s_p[k][4 * h4]);
+		for (int b = 0; b < ST / TR::KF; b++) {
+			Frag ph, pl;
+			f32x4_t pv[TR::KV / 4];
 #pragma unroll
-				for (int e = 0; e < 4; e++) {
-					acc[4 * h4 + e][0] = fmaf(p[e], c0, acc[4 * h4 + e][0]);
-					acc[4 * h4 + e][1] = fmaf(p[e], c1, acc[4 * h4 + e][1]);
-				}
+			for (int i = 0; i < TR::KV / 4; i++) pv[i] = tg_load4(&s_p[lr][b * TR::KF + lg * TR::KV + 4 * i]);
+#pragma unroll
+			for (int i = 0; i < TR::KV; i++) {
+				const T hi = (T)pv[i / 4][i % 4];
+				ph[i] = hi;
+				pl[i] = (T)(pv[i / 4][i % 4] - (float)hi);
+			}
+#pragma unroll
+			for (int c = 0; c < NC; c++) {
+				const int ct = min(ct0 + 4 * c, nct - 1);
+				const T *col = reinterpret_cast<const T *>(s_c + (size_t)(b * TR::KF + lg * TR::KV) * pitch) + ct * 16 + lr;
+				Frag cf;
+#pragma unroll
+				for (int i = 0; i < TR::KV; i++) cf[i] = *reinterpret_cast<const T *>(reinterpret_cast<const unsigned char *>(col) + i * pitch);
+				acc[c] = TR::mma(ph, cf, acc[c]);
+				if constexpr (TR::DT == TG_DT_BF16) acc[c] = TR::mma(pl, cf, acc[c]);
 			}
 		}
 		__syncthreads();
 	}
-	// the lane groups' sums meet in LDS (the tile's place: HT heads of at most 256 columns)
-	if (G > 1) {
-		float *s_s = reinterpret_cast<float *>(smem);
-		for (int g = 1; g < G; g++) {
-			if (grp == g && cin) {
+	float *o = a.part_acc + ((size_t)part * heads16 + h0) * a.rankp;
 #pragma unroll
-				for (int h = 0; h < HT; h++) *reinterpret_cast<float2 *>(s_s + ((size_t)h * cols + cl) * 2) = float2{acc[h][0], acc[h][1]};
-			}
-			__syncthreads();
-			if (grp == 0) {
+	for (int c = 0; c < NC; c++) {
+		const int ct = ct0 + 4 * c;
+		if (ct < nct) {
 #pragma unroll
-				for (int h = 0; h < HT; h++) {
-					const float2 v = *reinterpret_cast<const float2 *>(s_s + ((size_t)h * cols + cl) * 2);
-					acc[h][0] += v.x;
-					acc[h][1] += v.y;
-				}
-			}
-			__syncthreads();
+			for (int e = 0; e < 4; e++) o[(size_t)(4 * lg + e) * a.rankp + ct * 16 + lr] = acc[c][e];
 		}
-	}
-	if (cin && grp == 0) {
-		float *o = a.part_acc + ((size_t)part * heads16 + h0) * a.rankp + col;
-#pragma unroll
-		for (int h = 0; h < HT; h++) *reinterpret_cast<float2 *>(o + (size_t)h * a.rankp) = float2{acc[h][0], acc[h][1]};
 	}
 	if (blockIdx.z == 0 && (lane & 31) == 0) {
 #pragma unroll
@@ -224,7 +226,13 @@ __global__ __launch_bounds__(256) void latent_fold_kernel(const float *acc, cons
 	}
 	const int j = blockIdx.y * 64 + lane;  // a wave per quarter of the parts
 	float a = 0.0f;
-	for (int b = w; b < nb; b += 4) a = fmaf(s_f[b], acc[((size_t)b * heads16 + h) * rankp + j], a);
+	for (int b = w; b < nb; b += 64) {
+		float v[16];
+#pragma unroll
+		for (int i = 0; i < 16; i++) v[i] = acc[((size_t)min(b + 4 * i, nb - 1) * heads16 + h) * rankp + j];
+#pragma unroll
+		for (int i = 0; i < 16; i++) a = fmaf(b + 4 * i < nb ? s_f[min(b + 4 * i, nb - 1)] : 0.0f, v[i], a);
+	}
 	__shared__ float s_a[4][64];
 	s_a[w][lane] = a;
 	__syncthreads();
@@ -270,7 +278,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	const int h = blockIdx.x, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
 	const int kd = a.dimp / TR::KF, nv = a.vdimp / 16;
 	const T *Q = (const T *)a.q, *K = (const T *)a.k + (size_t)h * a.dimp, *V = (const T *)a.vt + (size_t)h * a.vdimp * a.ldv;
-	const float sl2 = a.scale * 1.44269504088896340736f;
+	const float sl2 = fabsf(a.scale) * 1.44269504088896340736f;  // (the sign goes to the queries: maxima are taken before scaling)
+	const bool neg = a.scale < 0.0f;
 
 	Frag qf[QT][ND];
 	int qi[QT];
@@ -282,6 +291,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 		for (int d = 0; d < ND; d++) {
 			qf[s][d] = *reinterpret_cast<const Frag *>(row + (d < kd ? d : 0) * TR::KF);
 			if (d >= kd) qf[s][d] = Frag{};
+			if (neg) qf[s][d] = -qf[s][d];
 		}
 	}
 	f32x4_t o[QT][NV];
@@ -333,36 +343,44 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 				for (int s = 0; s < QT; s++) sc[s][kt] = TR::mma(kf, qf[s][d], sc[s][kt]);
 			}
 		}
+		// keys past a query only in the tiles that reach the wave's first query
+		const bool masked = k0 + KT - 1 > a.past + qb + w * 16 * QT;
 #pragma unroll
 		for (int s = 0; s < QT; s++) {
-			const int lim = a.past + qi[s];
+			if (masked) {
+				const int lim = a.past + qi[s] - k0 - 4 * lg;
+#pragma unroll
+				for (int kt = 0; kt < NK; kt++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) sc[s][kt][e] = kt * 16 + e <= lim ? sc[s][kt][e] : -INFINITY;
+			}
 			float mt = -INFINITY;
 #pragma unroll
 			for (int kt = 0; kt < NK; kt++)
 #pragma unroll
-				for (int e = 0; e < 4; e++) {
-					const float v = k0 + kt * 16 + 4 * lg + e <= lim ? sc[s][kt][e] * sl2 : -INFINITY;
-					sc[s][kt][e] = v;
-					mt = fmaxf(mt, v);
-				}
+				for (int e = 0; e < 4; e++) mt = fmaxf(mt, sc[s][kt][e]);
 			mt = fmaxf(mt, tg_red_partner<32>(mt));
 			mt = fmaxf(mt, tg_red_partner<16>(mt));
-			const float mn = fmaxf(m[s], mt), f = exp2f(m[s] - mn);  // key 0 is in the first tile: mn is finite
-			m[s] = mn;
+			const float mn = fmaxf(m[s], mt * sl2);  // key 0 is in the first tile: finite
+			if (__ballot(mn > m[s])) {
+				const float f = __builtin_amdgcn_exp2f(m[s] - mn);
+				l[s] *= f;
+#pragma unroll
+				for (int v = 0; v < NV; v++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) o[s][v][e] *= f;
+				m[s] = mn;
+			}
 			float sum = 0.0f;
 #pragma unroll
 			for (int kt = 0; kt < NK; kt++)
 #pragma unroll
 				for (int e = 0; e < 4; e++) {
-					const float p = exp2f(sc[s][kt][e] - mn);
+					const float p = __builtin_amdgcn_exp2f(fmaf(sc[s][kt][e], sl2, -mn));
 					sc[s][kt][e] = p;
 					sum += p;
 				}
-			l[s] = l[s] * f + sum;
-#pragma unroll
-			for (int v = 0; v < NV; v++)
-#pragma unroll
-				for (int e = 0; e < 4; e++) o[s][v][e] *= f;
+			l[s] += sum;
 		}
 #pragma unroll
 		for (int b = 0; b < NB; b++) {
@@ -447,12 +465,8 @@ template <class TR>
 void launch_step(const TgLatentStep &a, hipStream_t s) {
 	const dim3 grid((unsigned)a.nb, (unsigned)((a.heads + 15) / 16), (unsigned)((a.rankp + 511) / 512));
 	const size_t lds = latent_step_lds<TR>(a.rankp);
-	if (lds > 48 * 1024) {
-		(void)hipFuncSetAttribute((const void *)latent_step_kernel<TR, 8>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-		(void)hipFuncSetAttribute((const void *)latent_step_kernel<TR, 16>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-	}
-	if (a.heads <= 8) hipLaunchKernelGGL((latent_step_kernel<TR, 8>), grid, dim3(256), lds, s, a);
-	else hipLaunchKernelGGL((latent_step_kernel<TR, 16>), grid, dim3(256), lds, s, a);
+	if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void *)latent_step_kernel<TR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+	hipLaunchKernelGGL((latent_step_kernel<TR>), grid, dim3(256), lds, s, a);
 }
 }  // namespace
 

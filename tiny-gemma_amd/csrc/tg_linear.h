@@ -43,7 +43,13 @@ struct TgF32 {
 };
 __device__ __forceinline__ float tg_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float tg_silu(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float tg_log_sigmoid(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
+// log2(sigmoid(z)) = min(z, 0) log2 e - log2(1 + e^-|z|); for a small second term its series, which keeps it exact to the last bits
+__device__ __forceinline__ float tg_log2_sigmoid(float z) {
+	const float L2E = 1.44269504088896340736f;
+	const float x = __builtin_amdgcn_exp2f(-fabsf(z) * L2E);
+	const float series = x * fmaf(x, fmaf(x, fmaf(x, fmaf(x, 0.2f, -0.25f), 1.0f / 3.0f), -0.5f), 1.0f) * L2E;
+	return fminf(z, 0.0f) * L2E - (x < 0.0625f ? series : __builtin_amdgcn_logf(1.0f + x));
+}
 // four consecutive values as one store
 __device__ __forceinline__ void tg_store4(float *p, f32x4_t v) { *reinterpret_cast<f32x4_t *>(p) = v; }
 __device__ __forceinline__ void tg_store4(__bf16 *p, f32x4_t v) { *reinterpret_cast<bf16x4_t *>(p) = __builtin_convertvector(v, bf16x4_t); }
@@ -157,7 +163,7 @@ struct TgGemm {
 	const int4 *tiles;     // null: one matrix
 	const int *ntiles;     // device: tiles in the list
 	int max_tiles;
-	int tile_rows;         // rows per tile: 128 or 32
+	int tile_rows;         // rows per tile: 128, 64 or 32
 	const int *row_src;    // row r of the product reads row row_src[r] of A (null: r)
 	long long group_frags; // fragments between the matrices of consecutive groups
 };

@@ -101,7 +101,7 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 
 	const int group = KW == 4 ? (int)blockIdx.x : (int)blockIdx.x * 4 + w;  // tile group of this wave
 	const bool live = group * NTL < p.ntiles;
-	const int tile0 = live ? group * NTL : 0;
+	const int tile0 = live ? group * NTL : 0, tiles_here = min(NTL, p.ntiles - tile0);
 	const Frag *W = reinterpret_cast<const Frag *>(p.W) + ((size_t)zw * p.zfrags + (size_t)tile0 * p.kfrags) * 64 + lane;
 	const int step = KW, kf0 = kb + (KW == 4 ? w : 0);
 	Frag wr[NTL][U];
@@ -110,7 +110,7 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 		for (int u = 0; u < U; u++) {
 			const int kk = kf + u * step, kc = min(kk, p.kfrags - 1);
 #pragma unroll
-			for (int t = 0; t < NTL; t++) wr[t][u] = W[((size_t)t * p.kfrags + kc) * 64];
+			for (int t = 0; t < NTL; t++) wr[t][u] = W[((size_t)(t < tiles_here ? t : 0) * p.kfrags + kc) * 64];
 		}
 	};
 
@@ -133,7 +133,7 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 			row = row < 0 ? 0 : (row >= p.vocab ? p.vocab - 1 : row);
 		}
 		// two elements per lane and pass; the padding behind the vector is zero in x, the parts, the norm and the table
-		constexpr int PER = 3, PQ = 8;
+		constexpr int PER = 4, PQ = 8;
 		for (int b = 0; b == 0 || b < kn; b += 2 * PER * NT) {
 			float2 x[PER], nw[PER], nb[PER], pq[PER][PQ];
 			int c[PER];
@@ -282,7 +282,10 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 				float r = v[0];
 				if constexpr (EPI == TG_VE_GATE) r *= tg_sigmoid(p.gate[z]);
 				if constexpr (EPI == TG_VE_WEIGHTED) r *= p.wgt[z];
-				y[group * 16 + tid] = r;
+				y[group * NTL * 16 + tid] = r;
+				if constexpr (NTL == 2) {
+					if (group * 2 + 1 < p.ntiles) y[group * 32 + 16 + tid] = v[1];
+				}
 				if constexpr (EPI == TG_VE_LOGITS) {
 					float bv = group * 16 + tid < p.nout ? r : -INFINITY;
 					int bi = group * 16 + tid;
@@ -322,10 +325,24 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 
 bool vec_wide(const TgVec &v, int epi) { return (epi == TG_VE_STORE || epi == TG_VE_LOGITS) && v.ksplit == 1 && v.nz == 1 && v.ntiles >= 2048; }
 
+// Two tiles per workgroup where one each would be two workgroups per compute unit and more: the prologue (with its reads of
+// the parts of the residual) is done half as often.
+bool vec_pairs(const TgVec &v, int epi) { return epi == TG_VE_STORE && v.nparts > 0 && v.nz == 1 && v.ksplit == 1 && v.ntiles >= 448; }
+
 template <class TR, int PRO, int EPI>
 void launch_vec_t(const TgVec &v, hipStream_t s) {
 	constexpr int NTL = EPI == TG_VE_SWIGLU ? 2 : 1;
 	const int per = (v.kfrags + v.ksplit - 1) / v.ksplit;
+	if constexpr (PRO == TG_VP_DYT && EPI == TG_VE_STORE) {
+		if (!vec_wide(v, EPI) && vec_pairs(v, EPI)) {
+			const int n = (per + 3) / 4;
+			auto lds = [&](int pad) { return sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF; };
+			const dim3 grid((unsigned)tg_vec_blocks(v, EPI), (unsigned)v.ksplit, (unsigned)v.nz);
+			if (n <= 6) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, 2, 4, 6>), grid, dim3(NT), lds(24), s, v);
+			else hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, 2, 4, 8>), grid, dim3(NT), lds(32), s, v);
+			return;
+		}
+	}
 	const unsigned bx = (unsigned)tg_vec_blocks(v, EPI);
 	auto lds = [&](int pad) {
 		size_t b = sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF;
@@ -344,6 +361,7 @@ void launch_vec_t(const TgVec &v, hipStream_t s) {
 	if (n <= 2) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 2>), grid, dim3(NT), lds(8), s, v);
 	else if (n <= 4) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 4>), grid, dim3(NT), lds(16), s, v);
 	else if (n <= 6 || (n > 9 && n <= 12)) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 6>), grid, dim3(NT), lds(24), s, v);
+	else if (n <= 8 || (n > 12 && n <= 16) || (n > 18 && n <= 24)) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 8>), grid, dim3(NT), lds(32), s, v);
 	else hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, NTL, 4, 9>), grid, dim3(NT), lds(36), s, v);
 }
 
@@ -439,33 +457,67 @@ __global__ __launch_bounds__(256, 2) void linear_kernel(TgGemm g) {
 #pragma unroll
 		for (int j = 0; j < NI; j++) acc[i][j] = f32x4_t{0, 0, 0, 0};
 
+	// Two sets of operand registers as well: the LDS reads of one half of a stage are in flight during the matrix
+	// instructions of the half before it.
+	Frag fa[2][MI], fb[2][NI];
+	auto read = [&](int kh, int par) {
+#pragma unroll
+		for (int i = 0; i < MI; i++) fa[kh][i] = lds[par][((wm * MI + i) * 2 + kh) * 64 + lane];
+#pragma unroll
+		for (int j = 0; j < NI; j++) fb[kh][j] = lds[par][(2 * AF + (wn * NI + j) * 2 + kh) * 64 + lane];
+	};
+	auto multiply = [&](int kh) {
+#pragma unroll
+		for (int i = 0; i < MI; i++)
+#pragma unroll
+			for (int j = 0; j < NI; j++)
+				acc[i][j] = EPI == TG_GE_TRANS ? TR::mma(fa[kh][i], fb[kh][j], acc[i][j]) : TR::mma(fb[kh][j], fa[kh][i], acc[i][j]);
+	};
 	fetch(0, 0);
 	fetch(1, 1);
 	put(0);
 	fetch(0, 2);
 	tg_lds_barrier();
-	// buffer and register set of a stage: its parity
+	read(0, 0);
+	// LDS buffer and register set of a stage: its parity
+	// (the order is pinned: left to itself the scheduler moves every LDS read down to its use)
+	constexpr int MM = MI * NI * (TR::DT == TG_DT_BF16 ? 1 : 4), RD = MI + NI;
+	constexpr int MR = MM / 2 / RD > 0 ? MM / 2 / RD : 1, MP = MM / 2 / PW > 0 ? MM / 2 / PW : 1;
 	auto stage = [&](int s, int par) {
-#pragma unroll
-		for (int kh = 0; kh < 2; kh++) {
-			Frag a[MI], bb[NI];
-#pragma unroll
-			for (int i = 0; i < MI; i++) a[i] = lds[par][((wm * MI + i) * 2 + kh) * 64 + lane];
-#pragma unroll
-			for (int j = 0; j < NI; j++) bb[j] = lds[par][(2 * AF + (wn * NI + j) * 2 + kh) * 64 + lane];
-#pragma unroll
-			for (int i = 0; i < MI; i++)
-#pragma unroll
-				for (int j = 0; j < NI; j++) acc[i][j] = EPI == TG_GE_TRANS ? TR::mma(a[i], bb[j], acc[i][j]) : TR::mma(bb[j], a[i], acc[i][j]);
-		}
+		read(1, par);
+		multiply(0);
 		put(par ^ 1);
 		fetch(par ^ 1, s + 3);
+#pragma unroll
+		for (int i = 0; i < RD; i++) {
+			__builtin_amdgcn_sched_group_barrier(0x100, 1, 0);        // LDS read
+			__builtin_amdgcn_sched_group_barrier(0x008, MR, 0);  // matrix instructions
+		}
+#pragma unroll
+		for (int i = 0; i < PW; i++) {
+			__builtin_amdgcn_sched_group_barrier(0x008, MP, 0);
+			__builtin_amdgcn_sched_group_barrier(0x200, 1, 0);        // LDS write
+			__builtin_amdgcn_sched_group_barrier(0x020, 1, 0);        // global load
+		}
+		__builtin_amdgcn_sched_barrier(0);
 		tg_lds_barrier();
+		__builtin_amdgcn_sched_barrier(0);
+		read(0, par ^ 1);
+		multiply(1);
+#pragma unroll
+		for (int i = 0; i < RD; i++) {
+			__builtin_amdgcn_sched_group_barrier(0x100, 1, 1);
+			__builtin_amdgcn_sched_group_barrier(0x008, MM / RD > 0 ? MM / RD : 1, 1);
+		}
+		__builtin_amdgcn_sched_barrier(0);
 	};
-	for (int s = 0; s < nst; s += 2) {
+	// (pairs without a branch between them: across one, the waits for the older register set would cover the newer one too)
+	int s = 0;
+	for (; s + 1 < nst; s += 2) {
 		stage(s, 0);
-		if (s + 1 < nst) stage(s + 1, 1);
+		stage(s + 1, 1);
 	}
+	if (s < nst) stage(s, 0);
 
 	const int lr = lane & 15, lg = lane >> 4;
 	if constexpr (EPI == TG_GE_TRANS) {
@@ -573,15 +625,20 @@ void launch_linear_t(const TgGemm &g, hipStream_t s) {
 			const unsigned grid = (unsigned)g.max_tiles * (unsigned)((g.N + 127) / 128);
 			if (g.tile_rows == 128)
 				hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 4, 4, true>), dim3(grid), dim3(256), 0, s, g);
+			else if (g.tile_rows == 64)
+				hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 2, 4, true>), dim3(grid), dim3(256), 0, s, g);
 			else
 				hipLaunchKernelGGL((linear_kernel<TR, EPI, 1, 4, 2, 2, true>), dim3(grid), dim3(256), 0, s, g);
 		}
 		return;
 	}
 	const int ntn = (g.N + 127) / 128, rows = EPI == TG_GE_TRANS ? g.rows_out : g.M;
-	// 128-row tiles from the point where they fill the device's compute units once
-	if ((rows + 127) / 128 * ntn >= 256 && rows > 64)
+	// 128-row tiles where they fill the device's 512 places (two workgroups per compute unit), then 64 rows, then 32
+	const int t128 = (rows + 127) / 128 * ntn, t64 = (rows + 63) / 64 * ntn;
+	if (t128 >= 448)
 		hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 4, 4, false>), dim3((unsigned)((rows + 127) / 128 * ntn)), dim3(256), 0, s, g);
+	else if (t64 >= 256)
+		hipLaunchKernelGGL((linear_kernel<TR, EPI, 2, 2, 2, 4, false>), dim3((unsigned)t64), dim3(256), 0, s, g);
 	else
 		hipLaunchKernelGGL((linear_kernel<TR, EPI, 1, 4, 2, 2, false>), dim3((unsigned)((rows + 31) / 32 * ntn)), dim3(256), 0, s, g);
 }
@@ -615,7 +672,7 @@ void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s) {
 
 int tg_vec_blocks(const TgVec &v, int epi) {
 	if (vec_wide(v, epi)) return (v.ntiles + 3) / 4;
-	return epi == TG_VE_SWIGLU ? (v.ntiles + 1) / 2 : v.ntiles;
+	return epi == TG_VE_SWIGLU || vec_pairs(v, epi) ? (v.ntiles + 1) / 2 : v.ntiles;
 }
 
 // Parts of K for a product whose consumer adds them: enough workgroups for the device, at least 8 fragments per part.

@@ -108,11 +108,11 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(TgMoeRoute r) {
 	r.row_src[slot] = t;
 }
 
-// a wave per row, four columns per lane and pass
-template <class TR>
+// four columns per lane and pass; a wave per row, or where there are few rows (WPR = 4) a workgroup per row
+template <class TR, int WPR>
 __global__ __launch_bounds__(256) void rows_dyt_kernel(TgRowsDyt r) {
 	typedef typename TR::T T;
-	const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+	const int t = blockIdx.x * (4 / WPR) + (threadIdx.x >> 6) / WPR, lane = threadIdx.x & (64 * WPR - 1);
 	if (t >= r.n) return;
 	float *xr = r.x + (size_t)(r.gather ? r.gather[t] : t) * r.ldx;
 	int id = 0;
@@ -120,15 +120,23 @@ __global__ __launch_bounds__(256) void rows_dyt_kernel(TgRowsDyt r) {
 		id = r.ids[t];
 		id = id < 0 ? 0 : (id >= r.vocab ? r.vocab - 1 : id);
 	}
-	for (int c = 4 * lane; c < r.ldx; c += 256) {
+	for (int c = 4 * lane; c < r.ldx; c += 256 * WPR) {
 		f32x4_t x = r.embed ? tg_load4((const __bf16 *)r.embed + (size_t)id * r.ldx + c) : tg_load4(xr + c);
 		if (r.y) {
 			f32x4_t add = {0, 0, 0, 0};
-			for (int k = 0; k < r.top; k++) {
-				const float g = r.wgt[(size_t)t * r.top + k];
-				const f32x4_t y = tg_load4((const T *)r.y + (size_t)r.slot[(size_t)t * r.top + k] * r.ldx + c);
+			for (int k0 = 0; k0 < r.top; k0 += 8) {
+				f32x4_t y[8];
+				float g[8];
 #pragma unroll
-				for (int e = 0; e < 4; e++) add[e] = fmaf(g, y[e], add[e]);
+				for (int k = 0; k < 8; k++) {
+					const size_t at = (size_t)t * r.top + min(k0 + k, r.top - 1);
+					g[k] = k0 + k < r.top ? r.wgt[at] : 0.0f;
+					y[k] = tg_load4((const T *)r.y + (size_t)r.slot[at] * r.ldx + c);
+				}
+#pragma unroll
+				for (int k = 0; k < 8; k++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) add[e] = fmaf(g[k], y[k][e], add[e]);
 			}
 #pragma unroll
 			for (int e = 0; e < 4; e++) x[e] = x[e] + r.mult * add[e];
@@ -162,7 +170,13 @@ void tg_launch_moe_route(const TgMoeRoute &r, hipStream_t s) {
 }
 
 void tg_launch_rows_dyt(const TgRowsDyt &r, int dt, hipStream_t s) {
-	const dim3 grid((unsigned)((r.n + 3) / 4));
-	if (dt == TG_DT_BF16) hipLaunchKernelGGL((rows_dyt_kernel<TgB16>), grid, dim3(256), 0, s, r);
-	else hipLaunchKernelGGL((rows_dyt_kernel<TgF32>), grid, dim3(256), 0, s, r);
+	const bool few = r.n < 2048;
+	const dim3 grid((unsigned)(few ? r.n : (r.n + 3) / 4));
+	if (dt == TG_DT_BF16) {
+		if (few) hipLaunchKernelGGL((rows_dyt_kernel<TgB16, 4>), grid, dim3(256), 0, s, r);
+		else hipLaunchKernelGGL((rows_dyt_kernel<TgB16, 1>), grid, dim3(256), 0, s, r);
+	} else {
+		if (few) hipLaunchKernelGGL((rows_dyt_kernel<TgF32, 4>), grid, dim3(256), 0, s, r);
+		else hipLaunchKernelGGL((rows_dyt_kernel<TgF32, 1>), grid, dim3(256), 0, s, r);
+	}
 }

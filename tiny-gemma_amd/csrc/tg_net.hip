@@ -75,6 +75,7 @@ int parse_madevik(const TgJson &j, TgNetCfg *c) {
 		} else if (type->str == "gla") {
 			lc.mix.kind = TG_MIX_GLA;
 			if (int rc = need_float(mix, "tau", where, &lc.mix.tau)) return rc;
+			if (lc.mix.vdimp() > TG_GLA_VDIM_MAX) return tg_fail(TG_ERR_UNSUPPORTED_SHAPE, where + ": value size above " + std::to_string(TG_GLA_VDIM_MAX));
 		} else {
 			return tg_fail(TG_ERR_UNSUPPORTED_SHAPE, where + ": unknown mixer '" + type->str + "'");
 		}
@@ -507,8 +508,13 @@ void norm_prologue(const TgNet *n, TgVec *v, const Norm &nm) {
 
 // Latent attention of one token: keys per workgroup and the number of parts for a context of ctx keys.
 void latent_parts(int ctx, int *chunk, int *nb) {
-	const int c = (ctx + TG_LATENT_MAX_BLOCKS - 1) / TG_LATENT_MAX_BLOCKS;
-	*chunk = tg_up(c, TG_LATENT_TILE);
+	// As many parts of one tile as a prologue merges; longer contexts need a fold, whose bytes (a partial sum is as large as
+	// 32 keys with 16 heads) bound the number of parts from above.
+	*chunk = TG_LATENT_TILE;
+	if (ctx > TG_LATENT_TILE * TG_LATENT_MAX_PARTS) {
+		const int want = (ctx + TG_LATENT_MAX_BLOCKS - 1) / TG_LATENT_MAX_BLOCKS;
+		*chunk = std::max(2 * TG_LATENT_TILE, tg_up(want, TG_LATENT_TILE));
+	}
 	*nb = (ctx + *chunk - 1) / *chunk;
 }
 
@@ -958,6 +964,14 @@ static int net_pass(TgNetSeq *q, const int32_t *ids, int rows, int pos, const in
 		g.ldc = g.n_split = w.n_split;
 		g.C2 = r.low;
 		g.ldc2 = w.in.n - w.n_split;
+		if (w.in.n - w.n_split <= 64 && rows >= 128) {
+			// a few fp32 columns behind the others would start another column of tiles: a product of their own
+			TgGemm low = g;
+			low.W = (const unsigned char *)w.in.w + frags(dt, w.n_split, w.in.k) * 1024;
+			g.N = w.n_split;
+			low.N = w.in.n - w.n_split;
+			tg_launch_linear(low, dt, TG_GE_F32, s);
+		}
 		tg_launch_linear(g, dt, TG_GE_STORE, s);
 		if (m.kind == TG_MIX_GLA) {
 			const TgGla ga = gla_of(n, l, q);
@@ -1015,7 +1029,8 @@ static int net_pass(TgNetSeq *q, const int32_t *ids, int rows, int pos, const in
 		mr.n = rows;
 		mr.experts = e.experts;
 		mr.top = e.top;
-		mr.tile_rows = (long long)rows * e.top >= 64LL * e.experts ? 128 : 32;
+		const long long per_expert = (long long)rows * e.top / e.experts;
+		mr.tile_rows = per_expert >= 128 ? 128 : (per_expert >= 48 ? 64 : 32);
 		mr.scale = e.scale;
 		mr.sel = r.sel;
 		mr.wgt = r.wgt;
