@@ -382,6 +382,32 @@ def test_greedy_generation(tg, folder, name):
     assert (lg.max(-1) - lg[np.arange(7), one]).max() <= 1e-4 * max(lg.std(), 1e-3)
 
 
+def test_captured_steps_equal_stream_launches(tg, folder):
+    """Decode steps replayed from captured graphs (position read on the device, launches sized for a bound of the context):
+    the same picks, logits and residual stream as stream launches, over many replays, with prefills and other work between
+    them and across a change of the bound."""
+    cfg = nm.MODELS["flat"]
+    path, om = folder("flat", cfg, seed=20)
+    model = tg.Transformer.from_dir(path, "bfloat16")
+    prompt = ids_of(cfg, 480, 77)
+    runs = {}
+    for mode in (0, 1):
+        tg.check(tg.lib().tg_set_graphs(mode))
+        s = model.open_session(640)
+        out = []
+        for rep in range(3):
+            s.reset()
+            s.prefill(prompt[:480 - rep], want_logits=False)
+            for n in (1, 7, 50, 3, 20):
+                s.decode_enqueue(n)
+                out.append(s.read_ids(640).tolist())
+            out.append(s.tap(2 * len(cfg["layers"]))[0].tolist())
+            out.append(s.decode(5)[1].tolist())
+        runs[mode] = out
+    assert runs[0] == runs[1]
+    tg.check(tg.lib().tg_set_graphs(-1))
+
+
 def test_sampled_generation(tg, folder):
     """The min-p sampler on a vocabulary that is no multiple of its blocks: every draw lies where the cumulative
     distribution of the oracle's logits crosses the uniform number."""

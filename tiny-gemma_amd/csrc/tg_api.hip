@@ -1699,7 +1699,51 @@ static int decode_graph_mode_of(const tg_config &c) {
 	const double bytes = c.n_layers * (h * (qo + 2 * kv) + qo * h + 3 * h * f) + h * c.n_vocab;
 	return bytes / (5.0 * c.n_layers + 1.0) < 5e6 ? 2 : 0;
 }
-static int decode_graph_mode(const tg_session *s) { return s->m->net ? 0 : decode_graph_mode_of(s->m->cfg); }
+static int decode_graph_mode(const tg_session *s) {
+	if (!s->m->net) return decode_graph_mode_of(s->m->cfg);
+	if (g_use_graphs >= 0) return g_use_graphs;
+	if (profiler_attached()) return 0;
+	double bytes = 0.0;
+	int launches = 1;
+	tg_net_step_cost(s->m->net, &bytes, &launches);
+	return bytes / launches < 5e6 ? 1 : 0;
+}
+
+// Greedy steps of a layer-list model from captured graphs.  A captured step reads its position from device memory; its
+// latent attention launches serve every position below a bound, so there is one graph per bound (and number of steps).
+static int net_context_bound(const tg_session *s) {
+	int b = 512;
+	while (b <= s->pos) b += b < 4096 ? b : 4096;
+	return std::min(b, s->capacity);
+}
+static int enqueue_net_graph_steps(tg_session *s, int bound, int nsteps) {
+	const uint64_t key = (uint64_t)bound | ((uint64_t)nsteps << 32);
+	auto it = s->graphs.find(key);
+	if (it == s->graphs.end()) {
+		TG_HIP(hipStreamBeginCapture(g_stream, hipStreamCaptureModeThreadLocal));
+		int rc = TG_OK;
+		for (int k = 0; k < nsteps && rc == TG_OK; k++) {
+			rc = tg_net_step(s->seq, head_of(s), s->pos + k, false, bound - 1);
+			tg_launch_argmax_finish(s->blk_val, s->blk_idx, head_blocks(s), s->ctr, s->tok_log, 1, g_stream);
+		}
+		hipGraph_t graph = nullptr;
+		const hipError_t e = hipStreamEndCapture(g_stream, &graph);
+		hipGraphExec_t exec = nullptr;
+		hipError_t e2 = hipSuccess;
+		if (rc == TG_OK && e == hipSuccess) e2 = hipGraphInstantiate(&exec, graph, nullptr, nullptr, 0);
+		if (graph) (void)hipGraphDestroy(graph);
+		if (rc != TG_OK) return rc;
+		if (e != hipSuccess || e2 != hipSuccess) return tg_fail(TG_ERR_HIP, std::string("capture of a decode step: ") + hipGetErrorString(e != hipSuccess ? e : e2));
+		it = s->graphs.emplace(key, exec).first;
+	}
+	TG_HIP(hipGraphLaunch(it->second, g_stream));
+	tg_net_replayed(s->seq);
+	s->pos += nsteps;
+	s->bp_local += nsteps;
+	s->bp_global += nsteps;
+	s->steps += nsteps;
+	return TG_OK;
+}
 
 int tg_plan_decode_launch_mode(const tg_config *cfg) {
 	if (!cfg || cfg->n_layers < 1) return -1;
@@ -1718,7 +1762,18 @@ int tg_decode_enqueue(tg_session *s, int n_steps) {
 		s->graph_epoch = g_knob_epoch;
 	}
 	for (int i = 0; i < n_steps; i++) {
-		if (!graph_mode || (graph_mode == 2 && g_fused)) {
+		if (s->m->net && graph_mode && !s->graphs_failed) {
+			if (s->pos >= s->capacity || s->steps >= s->tok_log_cap) return tg_fail(TG_ERR_STATE, "context is full (n_pos)");
+			const int bound = net_context_bound(s);
+			const int ns = n_steps - i >= TG_GRAPH_STEPS && s->pos + TG_GRAPH_STEPS <= bound && s->steps + TG_GRAPH_STEPS <= s->tok_log_cap ? TG_GRAPH_STEPS : 1;
+			if (enqueue_net_graph_steps(s, bound, ns) == TG_OK) {
+				i += ns - 1;
+				continue;
+			}
+			(void)hipGetLastError();  // a capture the runtime refuses leaves nothing enqueued: plain launches from here on
+			s->graphs_failed = true;
+		}
+		if (s->m->net || !graph_mode || (graph_mode == 2 && g_fused)) {
 			if (int rc = enqueue_decode_step(s, nullptr, false, nullptr, g_chain_picks)) {
 				flush_pick(s);
 				return rc;

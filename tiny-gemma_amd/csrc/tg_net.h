@@ -70,5 +70,7 @@ void tg_net_seq_release_workspace(TgNetSeq *q);
 int tg_net_rows(TgNetSeq *q, const int32_t *ids, int n, int pos, const int32_t *want, int n_want, float *logits, const TgHead &h, bool taps);
 // one token, h.ctr[4], at position pos (pos_bound: positions the launch must serve; host_pos false: the kernels read h.ctr[0])
 int tg_net_step(TgNetSeq *q, const TgHead &h, int pos, bool host_pos, int pos_bound);
+// a captured step was replayed: the residual stream kept is that of a step again
+void tg_net_replayed(TgNetSeq *q);
 // residual stream after block b of the last forward (as tg_session_tap); rows must match what was kept
 int tg_net_tap(TgNetSeq *q, int b, float *out, int rows);

@@ -1120,6 +1120,8 @@ int tg_net_rows(TgNetSeq *q, const int32_t *ids, int n, int pos, const int32_t *
 	return TG_OK;
 }
 
+void tg_net_replayed(TgNetSeq *q) { q->tap_rows = 0; }
+
 int tg_net_tap(TgNetSeq *q, int b, float *out, int rows) {
 	const TgNetCfg &c = q->net->cfg;
 	const size_t Dp = (size_t)c.wp(), D = (size_t)c.width;
