@@ -54,16 +54,18 @@ def ids_of(cfg, n, seed=0):
 
 
 # ---- one mechanism at a time: models of a single layer, the others' outputs made zero -------------------------------------
-GLA_SIZES = {"odd": (3, 20, 12, 4.0), "one": (1, 1, 1, 1.0), "slabs": (2, 100, 130, 16.0), "wide": (2, 257, 33, 2.0), "square": (4, 64, 64, 8.0)}
+GLA_SIZES = {"odd": (3, 20, 12, 4.0), "one": (1, 1, 1, 1.0), "slabs": (2, 100, 130, 16.0), "wide": (2, 257, 33, 2.0), "square": (4, 64, 64, 8.0), "tall": (1, 40, 300, 4.0),
+             "v_mid": (2, 48, 200, 8.0)}
 LATENT_SIZES = {"odd": (5, 24, 36, 40, 0.3), "one": (1, 1, 1, 1, 2.0), "many_heads": (33, 32, 16, 70, 0.2), "large": (2, 200, 256, 96, 0.1),
-                "v_small": (4, 128, 32, 600, 0.08), "square": (8, 64, 64, 128, 0.125)}
-MOE_SIZES = {"odd": (6, 2, 40, 1.7), "one": (1, 1, 1, 2.0), "all": (7, 7, 33, 0.3), "many": (130, 6, 20, 2.5), "top1": (16, 1, 96, 1.0)}
+                "v_small": (4, 128, 32, 600, 0.08), "square": (8, 64, 64, 128, 0.125), "v_wide": (3, 40, 100, 50, 0.2),
+                "both_128": (2, 100, 128, 64, 0.15), "q_wide": (2, 160, 96, 64, 0.1), "negative": (2, 32, 32, 48, -0.3)}
+MOE_SIZES = {"odd": (6, 2, 40, 1.7), "one": (1, 1, 1, 2.0), "all": (7, 7, 33, 0.3), "many": (130, 6, 20, 2.5), "top1": (16, 1, 96, 1.0), "crowd": (300, 5, 16, 1.0)}
 
 
 def mixer_case(folder, kind, name, width=84):
     if kind == "gla":
         cfg = nm.config(width, 97, [nm.layer(nm.gla(*GLA_SIZES[name]))])
-        return cfg, *folder(("gla", name), cfg, seed=11, gain=1.5)
+        return cfg, *folder(("gla", name), cfg, seed=11, gain=1.5, rank=23 if name == "slabs" else 7)
     cfg = nm.config(width, 97, [nm.layer(nm.latent(*LATENT_SIZES[name]))])
     return cfg, *folder(("latent", name), cfg, seed=12, gain=2.0)
 
@@ -134,6 +136,61 @@ def test_many_rows_per_expert(tg, folder):
     cfg = nm.config(72, 97, [nm.layer(nm.gla(1, 8, 8), nm.moe(5, 2, 40, 1.5))])
     path, om = folder("moe_rows", cfg, seed=14, edit=edit)
     check_block(tg, cfg, path, om, "float32", 700, block=2)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("n", [700, 2450])
+def test_large_products(tg, folder, dtype, n):
+    """Prompts long enough for the 64- and 128-row tiles of the plain products (3072 columns), with an odd number of stages."""
+    cfg = nm.config(190, 97, [nm.layer(nm.gla(8, 64, 128, 8.0))])
+    path, om = folder("large", cfg, seed=16)
+    ids = ids_of(cfg, n)
+    taps = []
+    om.step(om.state(), ids, taps)
+    s = tg.Transformer.from_dir(path, dtype).open_session(n)
+    want = np.arange(0, n, 7)
+    got = s.forward(ids, want)[1]
+    rows_close(got, om.norm("final.norm", taps[0][want]) @ om.t["head"].T, TOL[dtype], f"{n} tokens")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_many_heads_and_a_long_prompt(tg, folder, dtype):
+    """64 heads and 1030 tokens: the 128-query tiles of the attention kernel; places at their edges against the oracle."""
+    cfg = nm.config(64, 97, [nm.layer(nm.latent(64, 32, 32, 64, 0.4))])
+    path, om = folder("many_heads", cfg, seed=17, gain=1.5)
+    n = 1030
+    ids = ids_of(cfg, n)
+    c = om.norm("l0.norm1", om.t["embed"][ids]) @ om.t["l0.mix.dkv"].T
+    cache = list(layers.rms_norm(c, om.t["l0.mix.dkv.norm"], cfg["norm"]["eps"]))
+    places = [0, 15, 16, 63, 64, 127, 128, 129, 511, 512, 1023, 1024, 1029]
+    want = np.concatenate([om.step([cache[:p]], ids[p:p + 1]) for p in places])
+    s = tg.Transformer.from_dir(path, dtype).open_session(n)
+    rows_close(s.forward(ids, places)[1], want, TOL[dtype], "whole")
+    s.reset()
+    s.forward(ids[:100], [])
+    rows_close(s.forward(ids[100:], [p - 100 for p in places if p >= 100])[1], want[[p >= 100 for p in places]], TOL[dtype], "behind 100 tokens")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_wide_decode_products(tg, folder, dtype):
+    """A vocabulary of thousands of tiles (a wave per tile in the head) and a layer whose products take two tiles per
+    workgroup, with an odd one left over."""
+    cfg = nm.config(32, 33001, [nm.layer(nm.gla(2, 8, 8)), nm.layer(nm.gla(16, 96, 128))])
+    path, om = folder("wide_decode", cfg, seed=18)
+    ids = ids_of(cfg, 24)
+    want = om.step(om.state(), ids)
+    s = tg.Transformer.from_dir(path, dtype).open_session(64)
+    got = np.concatenate([s.forward([t])[1] for t in ids])
+    rows_close(got, want, TOL[dtype], "token by token")
+    s.reset()
+    arg, lg = s.forward(ids, np.arange(24))
+    rows_close(lg, want, TOL[dtype], "prompt")
+    assert arg == int(np.argmax(lg[-1])) or dtype == "bfloat16"
+    if dtype == "float32":
+        s.reset()
+        picks, _, _ = s.greedy(ids, 20)
+        lg = follow(om, ids, picks)
+        assert (lg.max(-1) - lg[np.arange(21), picks]).max() <= 1e-4 * lg.std()
 
 
 def test_norm_and_head_alone(tg, folder):

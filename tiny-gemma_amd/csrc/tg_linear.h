@@ -78,7 +78,7 @@ struct TgPack {
 	int transpose;
 };
 void tg_launch_pack(const TgMat &dst, int dt, const TgPack &p, hipStream_t s);
-// dst[rows][ld] floats (or the transposed [ld columns]...): dst[i * ld + j] = src[row(i)][col(j)], 0 in the padding
+// the same mapping into plain rows of floats: dst[i * ld + j] = source row and column of (i, j), 0 in the padding
 void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s);
 
 // ---- one-row products of a decode step ---------------------------------------------------------------------------------

@@ -110,7 +110,11 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 		for (int u = 0; u < U; u++) {
 			const int kk = kf + u * step, kc = min(kk, p.kfrags - 1);
 #pragma unroll
-			for (int t = 0; t < NTL; t++) wr[t][u] = W[((size_t)(t < tiles_here ? t : 0) * p.kfrags + kc) * 64];
+			for (int t = 0; t < NTL; t++) {
+				const Frag *at = W + ((size_t)(t < tiles_here ? t : 0) * p.kfrags + kc) * 64;
+				// a head is read once per token: past the caches, which keep the layers' matrices
+				wr[t][u] = KW == 1 ? __builtin_nontemporal_load(at) : *at;
+			}
 		}
 	};
 

@@ -28,10 +28,10 @@ void tg_launch_moe_route(const TgMoeRoute &r, hipStream_t s);
 
 // n rows of the fp32 residual x [.][ldx]: optionally x = table row of ids[t], optionally x += mult * (weighted sum of the
 // token's expert rows), then out = tanh(alpha x) w + b in the model's format (out may be null).  gather: row t of out
-// comes from row gather[t] of x (x is then left alone).  Columns width ... ldx are padding.
+// comes from row gather[t] of x (x is then left alone).  (Padding: zero in x, the norm and the table.)
 struct TgRowsDyt {
 	float *x;
-	int ldx, width, n;
+	int ldx, n;
 	const int *gather;
 	const void *embed;
 	const int *ids;

@@ -936,7 +936,6 @@ static int net_pass(TgNetSeq *q, const int32_t *ids, int rows, int pos, const in
 	memset(&d, 0, sizeof(d));
 	d.x = r.x;
 	d.ldx = Dp;
-	d.width = c.width;
 	d.n = rows;
 	d.embed = n->embed;
 	d.ids = r.ids;
