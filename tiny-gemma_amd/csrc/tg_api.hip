@@ -670,7 +670,7 @@ int tg_model_open(const char *dir, int dtype, tg_model **out) {
 	memset(&m->cfg, 0, sizeof(m->cfg));
 	const TgNetCfg &c = tg_net_cfg(net);
 	m->cfg.hidden_size = c.width;
-	m->cfg.n_layers = (int)c.layers.size();
+	m->cfg.n_layers = (int)c.runs.size();
 	m->cfg.n_vocab = c.vocab;
 	m->net = net;
 	m->loaded = true;

@@ -1,4 +1,4 @@
-// Gated linear attention: the step of one token, and the chunked form of many (tg_gla.h).
+// Gated linear attention and the gated delta rule: the step of one token, and the chunked form of many (tg_gla.h).
 //
 // Chunked form.  With b_t the sum of log alpha over the chunk's tokens up to and including t, a chunk of 64 tokens that
 // starts from state S contributes
@@ -89,7 +89,8 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld
 	const int hd = g.heads * g.dimp, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, t0 = blockIdx.x * C;
 	const int c = blockIdx.y * 64 + lane, cc = min(c, hd - 1);
 	const bool real = c < hd && cc % g.dimp < g.dim;
-	const float bias = g.a2b[cc];
+	// softplus(z) = -log(sigmoid(-z))
+	const float bias = g.a2b[cc], flip = g.a_log ? -1.0f : 1.0f, rate = g.a_log ? expf(g.a_log[cc / g.dimp]) : g.inv_tau;
 	float z[16];
 #pragma unroll
 	for (int i = 0; i < 16; i++) z[i] = bias;
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld
 	float run = 0.0f;
 #pragma unroll
 	for (int i = 0; i < 16; i++) {
-		if (real && t0 + 16 * w + i < n) run += tg_log2_sigmoid(z[i]) * g.inv_tau;  // past the end: the sum stays
+		if (real && t0 + 16 * w + i < n) run += tg_log2_sigmoid(flip * z[i]) * rate;  // past the end: the sum stays
 		z[i] = run;
 	}
 	s_sum[w][lane] = run;
@@ -132,20 +133,32 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld
 // ---- A: a workgroup per chunk and head, a wave per block of 16 rows ---------------------------------------------------------
 constexpr int SL = 32, SLP = 36;  // key channels per slab, row pitch
 
-template <class TR>
-__global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qkv, int ld, int k_off, TgGla g, int n, const float *b, float *A) {
+// DELTA: also k . k with the decay between them, T = beta (k . k) below the diagonal, and the chunk's solved keys and values:
+//     u = M (beta v) - M (beta k e^b) S   with M = (1 + T)^-1, S the state in front of the chunk.
+// T's diagonal blocks of 16 are inverted by substitution, a lane per column; the solve runs down the blocks on the matrix
+// instructions, a wave per 16 columns: an accumulator (four consecutive rows of a column per lane) is the next product's
+// second operand as it is, with the first operand's columns taken in the same order.
+struct DeltaIntra {
+	const float *beta;  // [n][ld_beta], before the sigmoid
+	int ld_beta;
+	float *u, *wk, *kt;
+};
+
+template <class TR, bool DELTA>
+__global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qkv, int ld, int k_off, TgGla g, int n, const float *b, float *A,
+                                                        DeltaIntra x) {
 	__shared__ __align__(16) float s_q[C][SLP], s_k[C][SLP], s_b[C][SLP];
-	const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int ch = blockIdx.x, h = blockIdx.y, kh = DELTA ? h / g.group : h, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
 	const int lr = lane & 15, lg = lane >> 4, hd = g.heads * g.dimp, t0 = ch * C;
-	f32x4_t off[3], dia = {0, 0, 0, 0};
+	f32x4_t off[3], dia = {0, 0, 0, 0}, koff[3], kdia = {0, 0, 0, 0};
 #pragma unroll
-	for (int j = 0; j < 3; j++) off[j] = f32x4_t{0, 0, 0, 0};
+	for (int j = 0; j < 3; j++) off[j] = koff[j] = f32x4_t{0, 0, 0, 0};
 	for (int d0 = 0; d0 < g.dimp; d0 += SL) {
 		__syncthreads();
 		for (int e = tid; e < C * SL / 4; e += 256) {
 			const int r = e / (SL / 4), c4 = (e % (SL / 4)) * 4, t = t0 + r;
-			const size_t col = (size_t)h * g.dimp + d0 + c4;
-			f32x4_t q = tg_load4(qkv + (size_t)min(t, n - 1) * ld + col), k = tg_load4(qkv + (size_t)min(t, n - 1) * ld + k_off + col);
+			const size_t col = (size_t)h * g.dimp + d0 + c4, kcol = (size_t)kh * g.dimp + d0 + c4;
+			f32x4_t q = tg_load4(qkv + (size_t)min(t, n - 1) * ld + kcol), k = tg_load4(qkv + (size_t)min(t, n - 1) * ld + k_off + kcol);
 #pragma unroll
 			for (int i = 0; i < 4; i++) {
 				q[i] = t < n ? q[i] * g.qscale : 0.0f;
@@ -161,24 +174,31 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 			for (int st = 0; st < SL / 4; st++) {
 				const int d = 4 * st + lg;
 				const float ref = s_b[16 * w - 1][d];
-				const float qv = s_q[qi][d] * pow2(s_b[qi][d] - ref);
+				const float fade = pow2(s_b[qi][d] - ref), qv = s_q[qi][d] * fade, kq = DELTA ? s_k[qi][d] * fade : 0.0f;
 #pragma unroll
 				for (int j = 0; j < 3; j++)
 					if (j < w) {
 						const float kv = s_k[16 * j + lr][d] * pow2(ref - s_b[16 * j + lr][d]);
 						off[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv, kv, off[j], 0, 0, 0);
+						if constexpr (DELTA) koff[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kq, kv, koff[j], 0, 0, 0);
 					}
 			}
 		}
 		for (int d = 0; d < SL; d += 4) {
 			const f32x4_t q = tg_load4(&s_q[qi][d]), bi = tg_load4(&s_b[qi][d]);
+			f32x4_t ki = {0, 0, 0, 0};
+			if constexpr (DELTA) ki = tg_load4(&s_k[qi][d]);
 #pragma unroll
 			for (int j = 0; j < 4; j++) {
 				const int kj = 16 * w + 4 * lg + j;
 				const f32x4_t k = tg_load4(&s_k[kj][d]), bj = tg_load4(&s_b[kj][d]);
 				if (kj <= qi) {
 #pragma unroll
-					for (int e = 0; e < 4; e++) dia[j] = fmaf(q[e] * k[e], pow2(bi[e] - bj[e]), dia[j]);
+					for (int e = 0; e < 4; e++) {
+						const float fade = pow2(bi[e] - bj[e]);
+						dia[j] = fmaf(q[e] * k[e], fade, dia[j]);
+						if constexpr (DELTA) kdia[j] = fmaf(ki[e] * k[e], fade, kdia[j]);
+					}
 				}
 			}
 		}
@@ -191,6 +211,98 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 		} else {
 #pragma unroll
 			for (int e = 0; e < 4; e++) out[(size_t)(16 * w + 4 * lg + e) * C + 16 * j + lr] = j < w ? off[j < 3 ? j : 0][e] : 0.0f;
+		}
+	}
+	if constexpr (DELTA) {
+		__shared__ __align__(16) float s_t[C][C + 4], s_m[4][16][20];
+		__shared__ float s_beta[C];
+		if (tid < C) s_beta[tid] = t0 + tid < n ? tg_sigmoid(x.beta[(size_t)(t0 + tid) * x.ld_beta + h]) : 0.0f;
+		__syncthreads();
+		const int qi = 16 * w + lr;
+#pragma unroll
+		for (int j = 0; j < 4; j++) s_t[qi][16 * w + 4 * lg + j] = 4 * lg + j < lr ? s_beta[qi] * kdia[j] : 0.0f;
+#pragma unroll
+		for (int j = 0; j < 3; j++)
+			if (j < w) {
+#pragma unroll
+				for (int e = 0; e < 4; e++) s_t[16 * w + 4 * lg + e][16 * j + lr] = s_beta[16 * w + 4 * lg + e] * koff[j][e];
+			}
+		__syncthreads();
+		{
+			float m[16];
+#pragma unroll
+			for (int r = 0; r < 16; r++) {
+				float v = r == lr ? 1.0f : 0.0f;
+				f32x4_t tr[4];
+#pragma unroll
+				for (int j = 0; j < 4; j++) tr[j] = tg_load4(&s_t[16 * w + r][16 * w + 4 * j]);
+#pragma unroll
+				for (int j = 0; j < r; j++) v = fmaf(-tr[j >> 2][j & 3], m[j], v);
+				m[r] = v;
+			}
+			if (lg == 0)
+#pragma unroll
+				for (int r = 0; r < 16; r++) s_m[w][r][lr] = m[r];
+		}
+		__syncthreads();
+		f32x4_t tb[6], mb[4];  // blocks (1,0) (2,0) (2,1) (3,0) (3,1) (3,2), negated; inverses
+#pragma unroll
+		for (int i = 0; i < 4; i++) {
+			mb[i] = tg_load4(&s_m[i][lr][4 * lg]);
+#pragma unroll
+			for (int j = 0; j < i; j++) {
+				tb[i * (i - 1) / 2 + j] = tg_load4(&s_t[16 * i + lr][16 * j + 4 * lg]);
+#pragma unroll
+				for (int e = 0; e < 4; e++) tb[i * (i - 1) / 2 + j][e] *= -1.0f;
+			}
+		}
+		const int nk = g.dimp / 16, ntile = nk + g.vdimp / 16, hv = g.heads * g.vdimp;
+		for (int tile = w; tile < ntile; tile += 4) {
+			const bool key = tile < nk;
+			const int col = (key ? tile : tile - nk) * 16 + lr;
+			f32x4_t X[4], W[4];
+			if (key) {
+				const float be = b[(size_t)(t0 + C - 1) * hd + (size_t)h * g.dimp + col];
+				float *kt = x.kt + (((size_t)ch * g.heads + h) * g.dimp + col) * C + 4 * lg;
+#pragma unroll
+				for (int i = 0; i < 4; i++) {
+					f32x4_t kd;
+#pragma unroll
+					for (int e = 0; e < 4; e++) {
+						const int r = 16 * i + 4 * lg + e, t = t0 + r;
+						const float k = t < n ? (float)qkv[(size_t)min(t, n - 1) * ld + k_off + (size_t)kh * g.dimp + col] : 0.0f;
+						const float bt = b[(size_t)t * hd + (size_t)h * g.dimp + col];
+						X[i][e] = s_beta[r] * k * pow2(bt);
+						kd[e] = k * pow2(be - bt);
+					}
+					tg_store4(kt + 16 * i, kd);
+				}
+			} else {
+#pragma unroll
+				for (int i = 0; i < 4; i++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) {
+						const int r = 16 * i + 4 * lg + e, t = t0 + r;
+						X[i][e] = t < n ? s_beta[r] * x.u[(size_t)t * hv + (size_t)h * g.vdimp + col] : 0.0f;
+					}
+			}
+#pragma unroll
+			for (int i = 0; i < 4; i++) {
+				f32x4_t acc = X[i];
+#pragma unroll
+				for (int j = 0; j < i; j++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(tb[i * (i - 1) / 2 + j][e], W[j][e], acc, 0, 0, 0);
+				W[i] = f32x4_t{0, 0, 0, 0};
+#pragma unroll
+				for (int e = 0; e < 4; e++) W[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(mb[i][e], acc[e], W[i], 0, 0, 0);
+			}
+			float *dst = key ? x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col : x.u + (size_t)t0 * hv + (size_t)h * g.vdimp + col;
+			const int pitch = key ? hd : hv;
+#pragma unroll
+			for (int i = 0; i < 4; i++)
+#pragma unroll
+				for (int e = 0; e < 4; e++) dst[(size_t)(16 * i + 4 * lg + e) * pitch] = W[i][e];
 		}
 	}
 }
@@ -283,9 +395,16 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(float *U, const float *b,
 // ---- o = (q e^b)^T S + A v, the head's root mean square norm and silu(gate): 64 tokens x the whole head per workgroup -------------
 // 8 waves: 16 tokens x half of the value columns each.  Slabs of 32: first the key channels (rows q e^b, columns of S), then
 // the chunk's own tokens (rows A, columns v); a slab's loads are in flight during the one before it.
-template <class TR, int VB>
-__global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv, int ld, int v_off, int g_off, TgGla g, int n, const float *b,
-                                                      const float *A, const float *U, typename TR::T *out, int ld_out) {
+// (delta rule: the rows of v are u, the gate's function is the sigmoid)
+struct OutIn {
+	const void *q, *v, *gate;
+	int ldq, ldv, ldg;
+};
+template <class TI, class TR, int VB, bool DELTA>
+__global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, const float *b, const float *A, const float *U, typename TR::T *out,
+                                                      int ld_out) {
+	const typename TI::T *Q = (const typename TI::T *)in.q + (size_t)(DELTA ? blockIdx.y / g.group : blockIdx.y) * g.dimp,
+	                     *V = (const typename TI::T *)in.v + (size_t)blockIdx.y * g.vdimp;
 	constexpr int XP = 36, YP = VB + 16, NI = VB / 32, NY = 32 * VB / 4 / 512;
 	__shared__ __align__(16) float s_x[C][XP], s_y[32][YP];
 	__shared__ float s_sq[2][C];
@@ -298,7 +417,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv,
 	auto fetch = [&](int sl) {
 		if (sl < slabs) {
 			const size_t qc = (size_t)h * g.dimp + sl * 32 + xc;
-			x = tg_load4(qkv + (size_t)min(t0 + xr, n - 1) * ld + qc);
+			x = tg_load4(Q + (size_t)min(t0 + xr, n - 1) * in.ldq + sl * 32 + xc);
 			bx = tg_load4(b + (size_t)(t0 + xr) * hd + qc);
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
@@ -311,7 +430,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv,
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
 				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-				y[i] = tg_load4(qkv + (size_t)min(t0 + j0 + r, n - 1) * ld + v_off + (size_t)h * g.vdimp + (c4 < g.vdimp ? c4 : 0));
+				y[i] = tg_load4(V + (size_t)min(t0 + j0 + r, n - 1) * in.ldv + (c4 < g.vdimp ? c4 : 0));
 			}
 		}
 	};
@@ -357,7 +476,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv,
 	if (t >= n) return;
 	const float inv = 1.0f / sqrtf((s_sq[0][wt + lr] + s_sq[1][wt + lr]) / (float)g.vdim + g.eps);
 	typename TR::T *dst = out + (size_t)t * ld_out + (size_t)h * g.vdimp;
-	const typename TR::T *gate = qkv + (size_t)t * ld + g_off + (size_t)h * g.vdimp;
+	const typename TR::T *gate = (const typename TR::T *)in.gate + (size_t)t * in.ldg + (size_t)h * g.vdimp;
 #pragma unroll
 	for (int j = 0; j < NI; j++) {
 		const int v = wv + 16 * j + 4 * lg;
@@ -365,7 +484,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv,
 			const f32x4_t gv = tg_load4(gate + v), nw = tg_load4(g.norm + v);
 			f32x4_t r;
 #pragma unroll
-			for (int e = 0; e < 4; e++) r[e] = acc[j][e] * inv * nw[e] * tg_silu(gv[e]);
+			for (int e = 0; e < 4; e++) r[e] = acc[j][e] * inv * nw[e] * (DELTA ? tg_sigmoid(gv[e]) : tg_silu(gv[e]));
 			tg_store4(dst + v, r);
 		}
 	}
@@ -373,11 +492,17 @@ __global__ __launch_bounds__(512) void gla_out_kernel(const typename TR::T *qkv,
 		for (int v = g.heads * g.vdimp + (w >> 2) * 16 + 4 * lg; v < ld_out; v += 32) tg_store4(out + (size_t)t * ld_out + v, f32x4_t{0, 0, 0, 0});
 }
 
-template <class TR, int VB>
-void launch_out(const TgGla &g, const typename TR::T *x, int ld, int v_off, int g_off, int n, const TgGlaScratch &t, typename TR::T *out, int ld_out,
-                hipStream_t s) {
-	hipLaunchKernelGGL((gla_out_kernel<TR, VB>), dim3((unsigned)((n + C - 1) / C), (unsigned)g.heads), dim3(512), 0, s, x, ld, v_off, g_off, g, n, t.b,
-	                   t.a, t.u, out, ld_out);
+template <class TI, class TR, int VB, bool DELTA>
+void launch_out_vb(const TgGla &g, const OutIn &in, int n, const float *b, const float *A, const float *U, void *out, int ld_out, hipStream_t s) {
+	hipLaunchKernelGGL((gla_out_kernel<TI, TR, VB, DELTA>), dim3((unsigned)((n + C - 1) / C), (unsigned)g.heads), dim3(512), 0, s, in, g, n, b, A, U,
+	                   (typename TR::T *)out, ld_out);
+}
+template <class TI, class TR, bool DELTA>
+void launch_out(const TgGla &g, const OutIn &in, int n, const float *b, const float *A, const float *U, void *out, int ld_out, hipStream_t s) {
+	if (g.vdimp <= 64) launch_out_vb<TI, TR, 64, DELTA>(g, in, n, b, A, U, out, ld_out, s);
+	else if (g.vdimp <= 128) launch_out_vb<TI, TR, 128, DELTA>(g, in, n, b, A, U, out, ld_out, s);
+	else if (g.vdimp <= 256) launch_out_vb<TI, TR, 256, DELTA>(g, in, n, b, A, U, out, ld_out, s);
+	else launch_out_vb<TI, TR, TG_GLA_VDIM_MAX, DELTA>(g, in, n, b, A, U, out, ld_out, s);
 }
 
 template <class TR>
@@ -385,10 +510,9 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
                  const TgGlaScratch &t, void *out, int ld_out, hipStream_t s) {
 	typedef typename TR::T T;
 	const T *x = (const T *)qkv;
-	T *o = (T *)out;
 	const unsigned chunks = (unsigned)((n + C - 1) / C), H = (unsigned)g.heads, hd = (unsigned)(g.heads * g.dimp), nd = (unsigned)((g.dimp + 127) / 128);
 	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (hd + 63) / 64), dim3(256), 0, s, low, ld_low, g, n, t.b);
-	hipLaunchKernelGGL((gla_intra_kernel<TR>), dim3(chunks, H), dim3(256), 0, s, x, ld, k_off, g, n, t.b, t.a);
+	hipLaunchKernelGGL((gla_intra_kernel<TR, false>), dim3(chunks, H), dim3(256), 0, s, x, ld, k_off, g, n, t.b, t.a, DeltaIntra{});
 	if (g.vdimp <= 64)
 		hipLaunchKernelGGL((gla_state_kernel<TR, 64>), dim3(chunks, H, nd), dim3(512), 0, s, x, ld, k_off, v_off, g, n, t.b, t.u);
 	else
@@ -396,10 +520,338 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
 		                   n, t.b, t.u);
 	const size_t per = (size_t)hd * g.vdimp;
 	hipLaunchKernelGGL(gla_scan_kernel, dim3((unsigned)((per + 255) / 256)), dim3(256), 0, s, t.u, t.b, g, (int)chunks);
-	if (g.vdimp <= 64) launch_out<TR, 64>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
-	else if (g.vdimp <= 128) launch_out<TR, 128>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
-	else if (g.vdimp <= 256) launch_out<TR, 256>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
-	else launch_out<TR, TG_GLA_VDIM_MAX>(g, x, ld, v_off, g_off, n, t, o, ld_out, s);
+	launch_out<TR, TR, false>(g, OutIn{x, x + v_off, x + g_off, ld, ld, ld}, n, t.b, t.a, t.u, out, ld_out, s);
+}
+
+// ==== the gated delta rule ====================================================================================================
+// Chunked form: with the notation above and T_ij = beta_i sum_d k_id k_jd e^{b_id - b_jd} (j < i),
+//     (1 + T) u = beta (v - (k e^b)^T S),   o_i = (q_i e^{b_i})^T S + sum_{j <= i} A_ij u_j,
+//     S' = diag(e^{b_end}) S + sum_j (k_j e^{b_end - b_j}) u_j^T.
+// Launches: convolution and unit norms; b; A, T and the solved keys and values, all chunks at once; the pass over the chunks
+// (u and the state in front of each), 16 value columns per workgroup; the outputs, all chunks at once.
+
+// ---- convolution, silu, unit norm: 4 tokens per workgroup, a wave each; y: q heads, k heads, blocks of 256 value channels --------
+// Inputs before the portion come from the ring.
+__device__ __forceinline__ f32x4_t ring4(const TgDelta &d, int pos, int c) {
+	return pos < 0 ? f32x4_t{0, 0, 0, 0} : tg_load4(d.ring + (size_t)(pos % d.taps) * d.channels + c);
+}
+template <class TR>
+__global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, float *qk, float *u) {
+	const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, kvh = d.g.heads / d.g.group, qc = d.q_channels();
+	if (t >= n) return;
+	const bool head = (int)blockIdx.y < 2 * kvh;
+	const int base = head ? (int)blockIdx.y * d.g.dimp : 2 * qc + ((int)blockIdx.y - 2 * kvh) * 256;
+	const int len = head ? d.g.dimp : min(256, d.channels - base);
+	constexpr int P = TG_DELTA_DIM_MAX / 256;
+	f32x4_t r[P];
+	float ss = 0.0f;
+#pragma unroll
+	for (int p = 0; p < P; p++) {
+		const int c = 4 * lane + 256 * p;
+		r[p] = f32x4_t{0, 0, 0, 0};
+		if (c < len) {
+			for (int i = 0; i < d.taps; i++) {
+				const int from = t - d.taps + 1 + i;
+				const f32x4_t v = from >= 0 ? tg_load4(x + (size_t)from * ld + base + c) : ring4(d, past + from, base + c);
+				const f32x4_t w = tg_load4(d.conv + (size_t)i * d.channels + base + c);
+#pragma unroll
+				for (int e = 0; e < 4; e++) r[p][e] = fmaf(w[e], v[e], r[p][e]);
+			}
+#pragma unroll
+			for (int e = 0; e < 4; e++) {
+				r[p][e] = tg_silu(r[p][e]);
+				ss = fmaf(r[p][e], r[p][e], ss);
+			}
+		}
+	}
+	float f = 1.0f;
+	if (head) f = 1.0f / sqrtf(tg_wave_sum(ss) + 1e-6f);
+	float *dst = head ? qk + (size_t)t * 2 * qc + base : u + (size_t)t * (d.channels - 2 * qc) + base - 2 * qc;
+#pragma unroll
+	for (int p = 0; p < P; p++) {
+		const int c = 4 * lane + 256 * p;
+		if (c < len) {
+#pragma unroll
+			for (int e = 0; e < 4; e++) r[p][e] *= f;
+			tg_store4(dst + c, r[p]);
+		}
+	}
+}
+
+// ---- the pass over the chunks: 16 value columns of a head per workgroup --------------------------------------------------------
+// Wave w keeps rows 16 (w + 4 i) ... of S in accumulators, which are the second operand of the products with the solved keys as
+// they are; the waves' parts of those products meet in LDS, and u, again in accumulator layout, is the second operand of S's
+// update.  The last inputs of the convolution go to the ring on the way.
+template <class TR, int ND>
+__global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, const float *b, float *u,
+                                                         const float *wk, const float *kt, float *st, int chunks) {
+	__shared__ __align__(16) f32x4_t s_p[4][4][64], s_u[4][64];
+	const TgGla &g = d.g;
+	const int h = blockIdx.x, v0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
+	const int hd = g.heads * g.dimp, hv = g.heads * g.vdimp, ntile = g.dimp / 16;
+	{
+		const int keep = min(d.taps, n), total = keep * d.channels, step = (int)(gridDim.x * gridDim.y) * 256;
+		for (int e = ((int)blockIdx.y * (int)gridDim.x + h) * 256 + tid; e < total; e += step) {
+			const int i = e / d.channels, c = e - i * d.channels, t = n - keep + i;
+			d.ring[(size_t)((past + t) % d.taps) * d.channels + c] = (float)x[(size_t)t * ld + c];
+		}
+	}
+	f32x4_t S[ND];
+	f32x4_t fw[ND][4], fk[ND][4], fb[ND], fv;
+	bool own[ND];
+	int row[ND];  // first row of the tile (the last tile again where there is none; its part counts as zero)
+#pragma unroll
+	for (int i = 0; i < ND; i++) {
+		own[i] = w + 4 * i < ntile;
+		row[i] = 16 * min(w + 4 * i, ntile - 1);
+#pragma unroll
+		for (int e = 0; e < 4; e++) S[i][e] = own[i] ? g.state[((size_t)h * g.dimp + row[i] + 4 * lg + e) * g.vdimp + v0 + lr] : 0.0f;
+	}
+	auto fetch = [&](int ch) {
+		const size_t t0 = (size_t)ch * C;
+#pragma unroll
+		for (int i = 0; i < ND; i++) {
+#pragma unroll
+			for (int tt = 0; tt < 4; tt++) {
+				fw[i][tt] = tg_load4(wk + (t0 + 16 * tt + lr) * hd + (size_t)h * g.dimp + row[i] + 4 * lg);
+				fk[i][tt] = tg_load4(kt + (((size_t)ch * g.heads + h) * g.dimp + row[i] + lr) * C + 16 * tt + 4 * lg);
+			}
+			fb[i] = tg_load4(b + (t0 + C - 1) * hd + (size_t)h * g.dimp + row[i] + 4 * lg);
+		}
+#pragma unroll
+		for (int e = 0; e < 4; e++) fv[e] = u[(t0 + 16 * w + 4 * lg + e) * hv + (size_t)h * g.vdimp + v0 + lr];
+	};
+	fetch(0);
+	for (int ch = 0; ch < chunks; ch++) {
+		f32x4_t part[4];
+#pragma unroll
+		for (int tt = 0; tt < 4; tt++) part[tt] = f32x4_t{0, 0, 0, 0};
+#pragma unroll
+		for (int i = 0; i < ND; i++)
+#pragma unroll
+			for (int e = 0; e < 4; e++)
+#pragma unroll
+				for (int tt = 0; tt < 4; tt++) part[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(fw[i][tt][e], S[i][e], part[tt], 0, 0, 0);
+#pragma unroll
+		for (int tt = 0; tt < 4; tt++) s_p[w][tt][lane] = part[tt];
+		float *front = st + (((size_t)ch * g.heads + h) * g.dimp) * g.vdimp + v0 + lr;
+#pragma unroll
+		for (int i = 0; i < ND; i++)
+			if (own[i])
+#pragma unroll
+				for (int e = 0; e < 4; e++) front[(size_t)(row[i] + 4 * lg + e) * g.vdimp] = S[i][e];
+		f32x4_t kk[ND][4], fade[ND], uv = fv;
+#pragma unroll
+		for (int i = 0; i < ND; i++) {
+#pragma unroll
+			for (int tt = 0; tt < 4; tt++) kk[i][tt] = fk[i][tt];
+#pragma unroll
+			for (int e = 0; e < 4; e++) fade[i][e] = pow2(fb[i][e]);
+		}
+		if (ch + 1 < chunks) fetch(ch + 1);
+		tg_lds_barrier();
+#pragma unroll
+		for (int q = 0; q < 4; q++)
+#pragma unroll
+			for (int e = 0; e < 4; e++) uv[e] -= s_p[q][w][lane][e];
+		s_u[w][lane] = uv;
+#pragma unroll
+		for (int e = 0; e < 4; e++) u[((size_t)ch * C + 16 * w + 4 * lg + e) * hv + (size_t)h * g.vdimp + v0 + lr] = uv[e];
+		tg_lds_barrier();
+		f32x4_t ut[4];
+#pragma unroll
+		for (int tt = 0; tt < 4; tt++) ut[tt] = s_u[tt][lane];
+#pragma unroll
+		for (int i = 0; i < ND; i++) {
+#pragma unroll
+			for (int e = 0; e < 4; e++) S[i][e] *= fade[i][e];
+		}
+#pragma unroll
+		for (int tt = 0; tt < 4; tt++)
+#pragma unroll
+			for (int e = 0; e < 4; e++)
+#pragma unroll
+				for (int i = 0; i < ND; i++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i][tt][e], ut[tt][e], S[i], 0, 0, 0);
+#pragma unroll
+		for (int i = 0; i < ND; i++)
+			if (!own[i]) S[i] = f32x4_t{0, 0, 0, 0};
+	}
+#pragma unroll
+	for (int i = 0; i < ND; i++)
+		if (own[i])
+#pragma unroll
+			for (int e = 0; e < 4; e++) g.state[((size_t)h * g.dimp + row[i] + 4 * lg + e) * g.vdimp + v0 + lr] = S[i][e];
+}
+
+// ---- one token: 32 value columns of a head per workgroup, lane = 4 columns, 32 groups of key channels (R rows of S per lane) ------
+template <int R>
+__global__ __launch_bounds__(256) void delta_step_kernel(const float *y, TgDelta d, int g_off, int b_off, int a_off, const int *ctr, int host_pos,
+                                                         float *o, float *gate) {
+	constexpr int DM = 32 * R;
+	__shared__ __align__(16) float s_q[DM], s_k[DM], s_a[DM], s_z[DM > 256 ? DM : 256], s_v[32], s_g[8][32];
+	__shared__ f32x4_t s_rp[4][8], s_rq[4][8];
+	__shared__ float s_sum[3][4];
+	const TgGla &g = d.g;
+	const int h = blockIdx.x, kh = h / g.group, c0 = blockIdx.y * 32, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int col = c0 + (tid & 7) * 4, dg = tid >> 3, hd = g.heads * g.dimp, hv = g.heads * g.vdimp, qc = d.q_channels();
+	const int pos = host_pos >= 0 ? host_pos : ctr[0];
+	float *S = g.state + ((size_t)h * g.dimp) * g.vdimp + col;
+	f32x4_t st[R];
+#pragma unroll
+	for (int r = 0; r < R; r++) st[r] = tg_load4(S + (size_t)min(dg + 32 * r, g.dimp - 1) * g.vdimp);
+	const float step = y[b_off + h];
+	// silu of the convolution of channel c, and the newest input to the ring where this workgroup is the one that does it
+	const int slot = pos % d.taps;
+	auto conv = [&](int c, bool keep) {
+		const float x = y[c];
+		float r = x * d.conv[(size_t)(d.taps - 1) * d.channels + c];
+		int from = slot + 1 == d.taps ? 0 : slot + 1;  // the row of position pos - taps + 1 (zero before the start)
+		for (int i = 0; i < d.taps - 1; i++) {
+			r = fmaf(d.conv[(size_t)i * d.channels + c], d.ring[(size_t)from * d.channels + c], r);
+			from = from + 1 == d.taps ? 0 : from + 1;
+		}
+		if (keep) d.ring[(size_t)slot * d.channels + c] = x;
+		return tg_silu(r);
+	};
+	const bool keep_qk = h % g.group == 0 && blockIdx.y == 0;
+	for (int e = tid; e < 2 * g.dimp; e += 256) {
+		const bool k = e >= g.dimp;
+		const int c = k ? e - g.dimp : e;
+		(k ? s_k : s_q)[c] = conv((k ? qc : 0) + kh * g.dimp + c, keep_qk);
+	}
+	if (tid >= 224) s_v[tid - 224] = conv(2 * qc + h * g.vdimp + c0 + tid - 224, true);
+	// the decay's low-rank product, its rank split over the lanes that the channels leave
+	const int ns = g.dimp >= 256 ? 1 : 256 / g.dimp, per = (g.rank + ns - 1) / ns;
+	for (int e = tid; e < ns * g.dimp; e += 256) {
+		const int sp = e / g.dimp, c = h * g.dimp + e - sp * g.dimp, hi = min(g.rank, (sp + 1) * per);
+		float z = 0.0f;
+		for (int j0 = sp * per; j0 < hi; j0 += 16) {
+			float wa[16], ya[16];
+#pragma unroll
+			for (int j = 0; j < 16; j++) {
+				wa[j] = g.a2[(size_t)min(j0 + j, g.rank - 1) * hd + c];
+				ya[j] = y[a_off + min(j0 + j, g.rank - 1)];
+			}
+#pragma unroll
+			for (int j = 0; j < 16; j++) z = j0 + j < hi ? fmaf(wa[j], ya[j], z) : z;
+		}
+		s_z[e] = z;
+	}
+	{
+		const int c = h * g.vdimp + c0 + (tid & 31), gp = (d.gate_rank + 7) / 8, lo = (tid >> 5) * gp, hi = min(d.gate_rank, lo + gp);
+		float z = 0.0f;
+		for (int j0 = lo; j0 < hi; j0 += 8) {
+			float wa[8], ya[8];
+#pragma unroll
+			for (int j = 0; j < 8; j++) {
+				wa[j] = d.g2[(size_t)min(j0 + j, d.gate_rank - 1) * hv + c];
+				ya[j] = y[g_off + min(j0 + j, d.gate_rank - 1)];
+			}
+#pragma unroll
+			for (int j = 0; j < 8; j++) z = j0 + j < hi ? fmaf(wa[j], ya[j], z) : z;
+		}
+		s_g[tid >> 5][tid & 31] = z;
+	}
+	__syncthreads();
+	float sq = 0.0f, sk = 0.0f, skq = 0.0f;
+	const float rate = expf(g.a_log[h]);
+	for (int c = tid; c < g.dimp; c += 256) {
+		const float q = s_q[c], k = s_k[c];
+		sq = fmaf(q, q, sq);
+		sk = fmaf(k, k, sk);
+		skq = fmaf(q, k, skq);
+		float z = g.a2b[h * g.dimp + c];
+		for (int sp = 0; sp < ns; sp++) z += s_z[sp * g.dimp + c];
+		s_a[c] = pow2(tg_log2_sigmoid(-z) * rate);
+	}
+	sq = tg_wave_sum(sq);
+	sk = tg_wave_sum(sk);
+	skq = tg_wave_sum(skq);
+	if (lane == 0) {
+		s_sum[0][w] = sq;
+		s_sum[1][w] = sk;
+		s_sum[2][w] = skq;
+	}
+	if (tid < 32) {
+		float z = 0.0f;
+#pragma unroll
+		for (int i = 0; i < 8; i++) z += s_g[i][tid];
+		gate[h * g.vdimp + c0 + tid] = z;
+	}
+	__syncthreads();
+	auto sum4 = [&](int i) { return (s_sum[i][0] + s_sum[i][1]) + (s_sum[i][2] + s_sum[i][3]); };
+	const float fq = g.qscale / sqrtf(sum4(0) + 1e-6f), fk = 1.0f / sqrtf(sum4(1) + 1e-6f), kq = sum4(2) * fk * fq;
+	f32x4_t ap = {0, 0, 0, 0}, aq = {0, 0, 0, 0};
+	float kr[R];
+#pragma unroll
+	for (int r = 0; r < R; r++) {
+		const int c = dg + 32 * r;
+		const bool in = c < g.dimp;
+		const int cc = in ? c : 0;
+		const float a = s_a[cc], q = in ? s_q[cc] * fq : 0.0f;
+		kr[r] = in ? s_k[cc] * fk : 0.0f;
+#pragma unroll
+		for (int e = 0; e < 4; e++) {
+			st[r][e] *= a;
+			ap[e] = fmaf(st[r][e], kr[r], ap[e]);
+			aq[e] = fmaf(st[r][e], q, aq[e]);
+		}
+	}
+#pragma unroll
+	for (int e = 0; e < 4; e++) {
+		ap[e] += tg_red_partner<32>(ap[e]);
+		ap[e] += tg_red_partner<16>(ap[e]);
+		ap[e] += tg_red_partner<8>(ap[e]);
+		aq[e] += tg_red_partner<32>(aq[e]);
+		aq[e] += tg_red_partner<16>(aq[e]);
+		aq[e] += tg_red_partner<8>(aq[e]);
+	}
+	if (lane < 8) {
+		s_rp[w][lane] = ap;
+		s_rq[w][lane] = aq;
+	}
+	__syncthreads();
+	const float beta = tg_sigmoid(step);
+	f32x4_t u, r0;
+#pragma unroll
+	for (int e = 0; e < 4; e++) {
+		const int i = tid & 7;
+		u[e] = beta * (s_v[i * 4 + e] - ((s_rp[0][i][e] + s_rp[1][i][e]) + (s_rp[2][i][e] + s_rp[3][i][e])));
+		r0[e] = fmaf(kq, u[e], (s_rq[0][i][e] + s_rq[1][i][e]) + (s_rq[2][i][e] + s_rq[3][i][e]));
+	}
+#pragma unroll
+	for (int r = 0; r < R; r++) {
+		const int c = dg + 32 * r;
+		if (c < g.dimp) {
+#pragma unroll
+			for (int e = 0; e < 4; e++) st[r][e] = fmaf(kr[r], u[e], st[r][e]);
+			tg_store4(S + (size_t)c * g.vdimp, st[r]);
+		}
+	}
+	if (tid < 8) tg_store4(o + (size_t)h * g.vdimp + col, r0);
+}
+
+template <class TR>
+void launch_delta_rows(const TgDelta &d, const void *xv, int ld, const float *low, int ld_low, int b_off, int a_off, const void *gate, int ldg, int n,
+                       int past, const TgDeltaScratch &t, void *out, int ld_out, hipStream_t s) {
+	const typename TR::T *x = (const typename TR::T *)xv;
+	const TgGla &g = d.g;
+	const int qc = d.q_channels(), hv = g.heads * g.vdimp, hd = g.heads * g.dimp, kvh = g.heads / g.group;
+	const unsigned chunks = (unsigned)((n + C - 1) / C);
+	hipLaunchKernelGGL((delta_prep_kernel<TR>), dim3((unsigned)((n + 3) / 4), (unsigned)(2 * kvh + (hv + 255) / 256)), dim3(256), 0, s, d, x, ld, n, past,
+	                   t.qk, t.u);
+	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (unsigned)((hd + 63) / 64)), dim3(256), 0, s, low + a_off, ld_low, g, n, t.b);
+	hipLaunchKernelGGL((gla_intra_kernel<TgF32, true>), dim3(chunks, (unsigned)g.heads), dim3(256), 0, s, t.qk, 2 * qc, qc, g, n, t.b, t.a,
+	                   DeltaIntra{low + b_off, ld_low, t.u, t.wk, t.kt});
+	const dim3 grid((unsigned)g.heads, (unsigned)(g.vdimp / 16));
+	auto scan = [&](auto *kernel) {
+		hipLaunchKernelGGL(kernel, grid, dim3(256), 0, s, d, x, ld, n, past, (const float *)t.b, t.u, (const float *)t.wk, (const float *)t.kt, t.st,
+		                   (int)chunks);
+	};
+	if (g.dimp <= 64) scan(delta_scan_kernel<TR, 1>);
+	else if (g.dimp <= 128) scan(delta_scan_kernel<TR, 2>);
+	else scan(delta_scan_kernel<TR, 4>);
+	launch_out<TgF32, TR, true>(g, OutIn{t.qk, t.u, gate, 2 * qc, hv, ldg}, n, t.b, t.a, t.st, out, ld_out, s);
 }
 
 }  // namespace
@@ -428,4 +880,39 @@ void tg_launch_gla_rows(const TgGla &g, int dt, const void *qkv, int ld, int k_o
                         const TgGlaScratch &t, void *out, int ld_out, hipStream_t s) {
 	if (dt == TG_DT_BF16) launch_rows<TgB16>(g, qkv, ld, k_off, v_off, g_off, low, ld_low, n, t, out, ld_out, s);
 	else launch_rows<TgF32>(g, qkv, ld, k_off, v_off, g_off, low, ld_low, n, t, out, ld_out, s);
+}
+
+void tg_launch_delta_step(const TgDelta &d, const float *y, int g_off, int b_off, int a_off, const int *ctr, int host_pos, float *o, float *gate,
+                          hipStream_t s) {
+	const dim3 grid((unsigned)d.g.heads, (unsigned)(d.g.vdimp / 32));
+	auto go = [&](auto *kernel) { hipLaunchKernelGGL(kernel, grid, dim3(256), 0, s, y, d, g_off, b_off, a_off, ctr, host_pos, o, gate); };
+	if (d.g.dimp <= 64) go(delta_step_kernel<2>);
+	else if (d.g.dimp <= 128) go(delta_step_kernel<4>);
+	else go(delta_step_kernel<8>);
+}
+
+size_t tg_delta_scratch(const TgDelta &d, int n, TgDeltaScratch *t, unsigned char *base) {
+	const TgGla &g = d.g;
+	const size_t chunks = (size_t)((n + C - 1) / C), hd = (size_t)g.heads * g.dimp, hv = (size_t)g.heads * g.vdimp;
+	size_t off = 0;
+	auto take = [&](float **p, size_t floats) {
+		if (base) *p = (float *)(base + off);
+		off += (floats * sizeof(float) + 255) / 256 * 256;
+	};
+	TgDeltaScratch tmp;
+	if (!t) t = &tmp;
+	take(&t->b, chunks * C * hd);
+	take(&t->a, chunks * g.heads * C * C);
+	take(&t->qk, (size_t)n * 2 * d.q_channels());
+	take(&t->u, chunks * C * hv);
+	take(&t->wk, chunks * C * hd);
+	take(&t->kt, chunks * C * hd);
+	take(&t->st, chunks * hd * g.vdimp);
+	return off;
+}
+
+void tg_launch_delta_rows(const TgDelta &d, int dt, const void *x, int ld, const float *low, int ld_low, int b_off, int a_off, const void *gate, int ldg,
+                          int n, int past, const TgDeltaScratch &t, void *out, int ld_out, hipStream_t s) {
+	if (dt == TG_DT_BF16) launch_delta_rows<TgB16>(d, x, ld, low, ld_low, b_off, a_off, gate, ldg, n, past, t, out, ld_out, s);
+	else launch_delta_rows<TgF32>(d, x, ld, low, ld_low, b_off, a_off, gate, ldg, n, past, t, out, ld_out, s);
 }

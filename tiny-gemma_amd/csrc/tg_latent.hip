@@ -14,9 +14,22 @@ constexpr int ST = 32;         // keys per tile
 constexpr int ST_LOADS = 8;    // 16-byte pieces per lane and round of the tile copy
 
 template <class TR>
-size_t latent_step_lds(int rankp) {  // q' fragments | tile
-	const size_t row = (size_t)rankp * sizeof(typename TR::T);
+size_t latent_step_lds(int rowp) {  // q' fragments | tile
+	const size_t row = (size_t)rowp * sizeof(typename TR::T);
 	return 16 * row + ST * (row + 16);
+}
+
+// Element i of a rotated vector x.
+template <class V>
+__device__ __forceinline__ float rotated(const V *x, int i, const float2 *turn, int dims, int half_layout) {
+	if (i >= dims) return (float)x[i];
+	const int hd = dims / 2;
+	const int pair = half_layout ? (i < hd ? i : i - hd) : i >> 1;
+	const bool second = half_layout ? i >= hd : (i & 1) != 0;
+	const int other = half_layout ? (second ? i - hd : i + hd) : i ^ 1;
+	const float2 t = turn[pair];
+	const float v = (float)x[i], o = (float)x[other];
+	return second ? fmaf(v, t.x, o * t.y) : fmaf(v, t.x, -(o * t.y));
 }
 
 template <class TR>
@@ -24,17 +37,20 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
 	extern __shared__ __align__(16) unsigned char smem[];
-	const int row = a.rankp * (int)sizeof(T), pitch = row + 16, ppr = row / 16;  // bytes; 16-byte pieces per row
-	Frag *s_q = reinterpret_cast<Frag *>(smem);  // [rankp / KF][64]
+	const int rowp = a.rankp + a.rotp, row = rowp * (int)sizeof(T), pitch = row + 16, ppr = row / 16;  // bytes; 16-byte pieces per row
+	Frag *s_q = reinterpret_cast<Frag *>(smem);  // [rowp / KF][64]
 	unsigned char *s_c = smem + 16 * row;
 	__shared__ float s_half[2][ST][16];
 	__shared__ __align__(16) float s_p[16][ST + 4];
 	__shared__ float s_corr[16], s_sq[4];
 	const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
-	const int part = blockIdx.x, h0 = blockIdx.y * 16, heads16 = (int)gridDim.y * 16;
-	const int pos = a.host_pos >= 0 ? a.host_pos : a.ctr[0], ctx = pos + 1;
-	const int kb = part * a.chunk, ke = min(ctx, kb + a.chunk);
-	T *cache = (T *)a.cache;
+	const int blocks = (a.heads + 15) / 16, grp = (int)blockIdx.y / blocks, hb = (int)blockIdx.y - grp * blocks;
+	const int part = blockIdx.x, h0 = hb * 16, heads16 = (int)gridDim.y * 16, g0 = grp * a.heads;  // (h0: inside the group)
+	const int pos = a.host_pos >= 0 ? a.host_pos : a.ctr[0], ctx = pos + 1, lo = max(0, ctx - a.window);
+	const int kb = lo + part * a.chunk, ke = min(ctx, kb + a.chunk);
+	const size_t key_bytes = (size_t)a.groups * row;
+	unsigned char *cache = (unsigned char *)a.cache + (size_t)grp * row;
+	const float2 *turn = a.rot.table + (size_t)pos * (a.rot.dims / 2);
 	typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
 	u32x4 piece[ST_LOADS];
 	// pieces [base, base + 256 * ST_LOADS) of a tile; the new token's row is not in memory yet: it is written to LDS below
@@ -42,7 +58,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 #pragma unroll
 		for (int i = 0; i < ST_LOADS; i++) {
 			const int e = min(base + tid + 256 * i, ST * ppr - 1), r = e / ppr, key = max(min(min(k0 + r, ke - 1), pos - 1), 0);
-			piece[i] = *reinterpret_cast<const u32x4 *>((const unsigned char *)cache + (size_t)key * row + (e - r * ppr) * 16);
+			piece[i] = *reinterpret_cast<const u32x4 *>(cache + (size_t)key * key_bytes + (e - r * ppr) * 16);
 		}
 	};
 	auto place = [&](int base) {
@@ -53,23 +69,37 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		}
 	};
 	const bool mine = pos >= kb && pos < kb + a.chunk;
+	const float *kv = a.kv + (size_t)grp * a.kv_stride;
 	float raw[2], nrm[2];
 #pragma unroll
 	for (int i = 0; i < 2; i++) {
 		const int j = min(tid + 256 * i, a.rank - 1);
-		raw[i] = a.dkv[j];
-		nrm[i] = a.norm[j];
+		raw[i] = kv[j];
+		nrm[i] = a.norm ? a.norm[j] : 1.0f;
 	}
 	request(kb, 0);
 
 	// q' in operand order: lane = head, 16 bytes of the latent
-	const int q4 = a.rankp / 4;
+	const int q4 = rowp / 4, r4 = a.rankp / 4;
 	for (int base = 0; base < 16 * q4; base += 256 * 8) {
 		f32x4_t v[8];
 #pragma unroll
 		for (int i = 0; i < 8; i++) {
-			const int e = min(base + tid + 256 * i, 16 * q4 - 1), h = e / q4;
-			v[i] = tg_load4(a.q + (size_t)min(h0 + h, a.heads - 1) * a.rankp + (e - h * q4) * 4);
+			const int e = min(base + tid + 256 * i, 16 * q4 - 1), h = e / q4, j4 = e - h * q4;
+			const size_t hq = (size_t)(g0 + min(h0 + h, a.heads - 1));
+			v[i] = j4 < r4 ? tg_load4(a.q + hq * a.q_stride + j4 * 4) : f32x4_t{0, 0, 0, 0};
+			if (j4 < r4) {
+#pragma unroll
+				for (int c = 0; c < 4; c++)
+					if (j4 * 4 + c < a.q_zero) v[i][c] = 0.0f;
+			} else {
+				const float *x = a.qr + hq * a.qr_stride;
+#pragma unroll
+				for (int c = 0; c < 4; c++) {
+					const int j = (j4 - r4) * 4 + c;
+					if (j < a.rot_size) v[i][c] = rotated(x, j, turn, a.rot.dims, a.rot.half_layout);
+				}
+			}
 		}
 #pragma unroll
 		for (int i = 0; i < 8; i++) {
@@ -80,11 +110,11 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		}
 	}
 	// the new token's latent, normalised, by the workgroups whose part it ends
-	float inv = 0.0f;
-	if (mine) {
+	float inv = 1.0f;
+	if (mine && a.norm) {
 		float ss = 0.0f;
 		for (int j = tid, i = 0; j < a.rank; j += 256, i++) {
-			const float x = i < 2 ? raw[i & 1] : a.dkv[j];
+			const float x = i < 2 ? raw[i & 1] : kv[j];
 			ss = fmaf(x, x, ss);
 		}
 		ss = tg_wave_sum(ss);
@@ -101,7 +131,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	float m[2], l[2];
 #pragma unroll
 	for (int i = 0; i < 2; i++) { m[i] = -INFINITY; l[i] = 0.0f; }
-	const int kfr = a.rankp / TR::KF, kh = (kfr + 1) / 2, kf_lo = (w >> 1) * kh, kf_hi = min(kfr, kf_lo + kh);
+	const int kfr = rowp / TR::KF, kh = (kfr + 1) / 2, kf_lo = (w >> 1) * kh, kf_hi = min(kfr, kf_lo + kh);
 	for (int k0 = kb; k0 < ke; k0 += ST) {
 		for (int base = 0; base < ST * ppr; base += 256 * ST_LOADS) {
 			if (base) request(k0, base);
@@ -109,12 +139,19 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		}
 		__syncthreads();
 		if (mine && pos < k0 + ST) {
+			T *dst = reinterpret_cast<T *>(cache + (size_t)pos * key_bytes), *tile = reinterpret_cast<T *>(s_c + (size_t)(pos - k0) * pitch);
 			for (int j = tid, i = 0; j < a.rankp; j += 256, i++) {
 				const int jc = j < a.rank ? j : 0;
-				const float x = i < 2 ? raw[i & 1] : a.dkv[jc], g = i < 2 ? nrm[i & 1] : a.norm[jc];
+				const float x = i < 2 ? raw[i & 1] : kv[jc], g = i < 2 ? nrm[i & 1] : (a.norm ? a.norm[jc] : 1.0f);
 				const T c = (T)(j < a.rank ? x * inv * g : 0.0f);
-				*reinterpret_cast<T *>(s_c + (size_t)(pos - k0) * pitch + (size_t)j * sizeof(T)) = c;
-				cache[(size_t)pos * a.rankp + j] = c;
+				tile[j] = c;
+				dst[j] = c;
+			}
+			const float *kr = a.kr + (size_t)grp * a.kr_stride;
+			for (int j = tid; j < a.rotp; j += 256) {
+				const T c = (T)(j < a.rot_size ? rotated(kr, j, turn, a.rot.dims, a.rot.half_layout) : 0.0f);
+				tile[a.rankp + j] = c;
+				dst[a.rankp + j] = c;
 			}
 			__syncthreads();
 		}
@@ -180,7 +217,8 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		}
 		__syncthreads();
 	}
-	float *o = a.part_acc + ((size_t)part * heads16 + h0) * a.rankp;
+	const int hp = (int)blockIdx.y * 16;  // this block's padded heads
+	float *o = a.part_acc + ((size_t)part * heads16 + hp) * a.rankp;
 #pragma unroll
 	for (int c = 0; c < NC; c++) {
 		const int ct = ct0 + 4 * c;
@@ -192,18 +230,20 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	if (blockIdx.z == 0 && (lane & 31) == 0) {
 #pragma unroll
 		for (int i = 0; i < 2; i++) {
-			float *ml = a.part_ml + ((size_t)part * heads16 + h0 + 4 * w + 2 * i + (lane >> 5)) * 2;
+			float *ml = a.part_ml + ((size_t)part * heads16 + hp + 4 * w + 2 * i + (lane >> 5)) * 2;
 			ml[0] = m[i];
 			ml[1] = l[i];
 		}
 	}
 }
 
+// groups > 0: the normalised sum of real head (group, head) instead, [groups * heads][out_stride]
 __global__ __launch_bounds__(256) void latent_fold_kernel(const float *acc, const float *ml, int nb, int heads16, int rankp, float *out_acc,
-                                                          float *out_ml) {
+                                                          float *out_ml, int groups, int heads, int out_stride) {
 	__shared__ float s_f[TG_LATENT_MAX_BLOCKS];
 	__shared__ float s_r[4];
-	const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+	const int hp16 = (heads + 15) / 16 * 16, real = (int)blockIdx.x;
+	const int h = groups ? real / heads * hp16 + real % heads : real, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
 	float m = -INFINITY;
 	for (int b = tid; b < nb; b += 256) m = fmaxf(m, ml[((size_t)b * heads16 + h) * 2]);
 	m = tg_wave_max(m);
@@ -220,40 +260,94 @@ __global__ __launch_bounds__(256) void latent_fold_kernel(const float *acc, cons
 	l = tg_wave_sum(l);
 	if (lane == 0) s_r[w] = l;
 	__syncthreads();
-	if (tid == 0 && blockIdx.y == 0) {
+	l = (s_r[0] + s_r[1]) + (s_r[2] + s_r[3]);
+	if (!groups && tid == 0 && blockIdx.y == 0) {
 		out_ml[2 * h] = m;
-		out_ml[2 * h + 1] = (s_r[0] + s_r[1]) + (s_r[2] + s_r[3]);
+		out_ml[2 * h + 1] = l;
 	}
-	const int j = blockIdx.y * 64 + lane;  // a wave per quarter of the parts
+	const int j = blockIdx.y * 64 + lane, jc = min(j, rankp - 1);  // a wave per quarter of the parts
 	float a = 0.0f;
 	for (int b = w; b < nb; b += 64) {
 		float v[16];
 #pragma unroll
-		for (int i = 0; i < 16; i++) v[i] = acc[((size_t)min(b + 4 * i, nb - 1) * heads16 + h) * rankp + j];
+		for (int i = 0; i < 16; i++) v[i] = acc[((size_t)min(b + 4 * i, nb - 1) * heads16 + h) * rankp + jc];
 #pragma unroll
 		for (int i = 0; i < 16; i++) a = fmaf(b + 4 * i < nb ? s_f[min(b + 4 * i, nb - 1)] : 0.0f, v[i], a);
 	}
 	__shared__ float s_a[4][64];
 	s_a[w][lane] = a;
 	__syncthreads();
-	if (w == 0) out_acc[(size_t)h * rankp + j] = (s_a[0][lane] + s_a[1][lane]) + (s_a[2][lane] + s_a[3][lane]);
+	if (w != 0 || j >= rankp) return;
+	const float sum = (s_a[0][lane] + s_a[1][lane]) + (s_a[2][lane] + s_a[3][lane]);
+	if (groups) out_acc[(size_t)real * out_stride + j] = sum / l;
+	else out_acc[(size_t)h * rankp + j] = sum;
 }
 
 // ---- many tokens -------------------------------------------------------------------------------------------------------------
+// a wave per token and group
+template <class TR, class SRC>
+__global__ __launch_bounds__(256) void latent_rows_kernel(TgLatentCacheRows a) {
+	typedef typename TR::T T;
+	const int e = blockIdx.x * 4 + (threadIdx.x >> 6), t = e / a.groups, grp = e - t * a.groups, lane = threadIdx.x & 63;
+	if (t >= a.n) return;
+	const SRC *x = (const SRC *)a.kv + (size_t)t * a.ld + (size_t)grp * a.kv_stride, *r = (const SRC *)a.kr + (size_t)t * a.ld + (size_t)grp * a.kr_stride;
+	float inv = 1.0f;
+	if (a.norm) {
+		float ss = 0.0f;
+		for (int j = lane; j < a.rank; j += 64) ss = fmaf((float)x[j], (float)x[j], ss);
+		ss = tg_wave_sum(ss);
+		inv = 1.0f / sqrtf(ss / (float)a.rank + a.eps);
+	}
+	const int pos = a.past + t;
+	T *row = (T *)a.cache + ((size_t)pos * a.groups + grp) * (a.rankp + a.rotp);
+	for (int j = lane; j < a.rankp; j += 64) {
+		const int jc = j < a.rank ? j : 0;
+		const float c = (float)x[jc] * inv * (a.norm ? a.norm[jc] : 1.0f);
+		row[j] = (T)(j < a.rank ? c : 0.0f);
+	}
+	const float2 *turn = a.rot.table + (size_t)pos * (a.rot.dims / 2);
+	for (int j = lane; j < a.rotp; j += 64) row[a.rankp + j] = (T)(j < a.rot_size ? rotated(r, j, turn, a.rot.dims, a.rot.half_layout) : 0.0f);
+}
+
+// a lane per pair
+template <class T>
+__global__ __launch_bounds__(256) void rot_rows_kernel(T *rows, int ld, int n, int past, int first, int count, int stride, TgRot rot) {
+	const int hd = rot.dims / 2, per = count * hd, t = blockIdx.y;
+	const int e = blockIdx.x * 256 + threadIdx.x;
+	if (e >= per) return;
+	const int v = e / hd, i = e - v * hd;
+	T *x = rows + (size_t)t * ld + first + (size_t)v * stride;
+	T *p = x + (rot.half_layout ? i : 2 * i), *q = x + (rot.half_layout ? i + hd : 2 * i + 1);
+	const float2 c = rot.table[(size_t)(past + t) * hd + i];
+	const float u = (float)*p, w = (float)*q;
+	*p = (T)fmaf(u, c.x, -(w * c.y));
+	*q = (T)fmaf(w, c.x, u * c.y);
+}
+
+// 64 keys x 32 dimensions of a group per workgroup: rotated keys straight through, values transposed through LDS into the
+// key order of the attention operand; keys past the end are zero values
 template <class TR>
-__global__ __launch_bounds__(256) void latent_rows_kernel(const float *dkv, int ld, int n, int rank, int rankp, const float *norm, float eps,
-                                                          typename TR::T *rows) {
-	const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-	if (t >= n) return;
-	const float *x = dkv + (size_t)t * ld;
-	float ss = 0.0f;
-	for (int j = lane; j < rank; j += 64) ss = fmaf(x[j], x[j], ss);
-	ss = tg_wave_sum(ss);
-	const float inv = 1.0f / sqrtf(ss / (float)rank + eps);
-	for (int j = lane; j < rankp; j += 64) {
-		const int jc = j < rank ? j : 0;
-		const float c = x[jc] * inv * norm[jc];
-		rows[(size_t)t * rankp + j] = (typename TR::T)(j < rank ? c : 0.0f);
+__global__ __launch_bounds__(256) void key_values_kernel(TgKeyValues a) {
+	typedef typename TR::T T;
+	__shared__ T s_v[32][64 + 4];
+	const int grp = blockIdx.y, d0 = blockIdx.z * 32, k0 = blockIdx.x * 64, tid = threadIdx.x;
+	const int rowp = a.dimp + a.rotp;
+	for (int e = tid; e < 64 * 32; e += 256) {
+		const int kk = e >> 5, d = e & 31, key = k0 + kk;
+		T v = (T)0.0f;
+		if (key < a.n) {
+			const T *row = (const T *)a.cache + ((size_t)(a.lo + key) * a.groups + grp) * rowp;
+			v = row[d0 + d];
+			((T *)a.k)[(size_t)key * a.groups * a.dimp + (size_t)grp * a.dimp + d0 + d] = d0 + d < a.rot_size ? row[a.dimp + d0 + d] : v;
+		}
+		int at = kk;
+		if constexpr (TR::DT == TG_DT_BF16) at = (kk & 32) + 8 * ((kk & 15) >> 2) + 4 * ((kk >> 4) & 1) + (kk & 3);
+		s_v[d][at] = v;
+	}
+	__syncthreads();
+	for (int e = tid; e < 64 * 32; e += 256) {
+		const int d = e >> 6, at = e & 63;
+		((T *)a.vt)[(size_t)(grp * a.dimp + d0 + d) * a.ldv + k0 + at] = s_v[d][at];
 	}
 }
 
@@ -275,9 +369,10 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	// Query tiles from both ends: the first half of the launch takes the long rows, longest first, the second half the
 	// short ones, shortest first, so that the workgroups that meet on a compute unit have about the same work together.
 	const int nqt = (int)gridDim.y, y = (int)blockIdx.y, half = (nqt + 1) / 2;
-	const int h = blockIdx.x, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
-	const int kd = a.dimp / TR::KF, nv = a.vdimp / 16;
-	const T *Q = (const T *)a.q, *K = (const T *)a.k + (size_t)h * a.dimp, *V = (const T *)a.vt + (size_t)h * a.vdimp * a.ldv;
+	const int h = blockIdx.x, kh = h / a.group, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
+	const int kn = a.dimp / TR::KF, kd = (a.dimp + a.rotp) / TR::KF, nv = a.vdimp / 16;
+	const T *Q = (const T *)a.q, *K = (const T *)a.k + (size_t)kh * a.dimp, *V = (const T *)a.vt + (size_t)kh * a.vdimp * a.ldv;
+	const T *R = (const T *)a.kr;
 	const float sl2 = fabsf(a.scale) * 1.44269504088896340736f;  // (the sign goes to the queries: maxima are taken before scaling)
 	const bool neg = a.scale < 0.0f;
 
@@ -286,7 +381,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 #pragma unroll
 	for (int s = 0; s < QT; s++) {
 		qi[s] = qb + w * 16 * QT + s * 16 + lr;
-		const T *row = Q + (size_t)min(qi[s], a.n - 1) * a.ldq + (size_t)h * a.dimp + lg * TR::KV;
+		const T *row = Q + (size_t)min(qi[s], a.n - 1) * a.ldq + (size_t)h * (a.dimp + a.rotp) + lg * TR::KV;
 #pragma unroll
 		for (int d = 0; d < ND; d++) {
 			qf[s][d] = *reinterpret_cast<const Frag *>(row + (d < kd ? d : 0) * TR::KF);
@@ -298,13 +393,13 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	float m[QT], l[QT];
 #pragma unroll
 	for (int s = 0; s < QT; s++) {
-		m[s] = -INFINITY;
+		m[s] = -1e30f;  // below every score; finite, so that a tile without a visible key leaves everything as it is
 		l[s] = 0.0f;
 #pragma unroll
 		for (int v = 0; v < NV; v++) o[s][v] = f32x4_t{0, 0, 0, 0};
 	}
 	const int last = a.past + min(qb + 64 * QT, a.n) - 1;  // the last key any of these queries sees
-	const int nt = last / KT + 1, ctx = a.past + a.n;
+	const int nt = last / KT + 1, ctx = a.past + a.n, tb = max(a.past + qb - a.window + 1, 0) / KT;
 	Frag st[PW];
 	auto fetch = [&](int k0) {
 #pragma unroll
@@ -313,7 +408,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 			const T *p;
 			if (f < KFRAGS) {
 				const int kt = f / ND, d = f % ND;
-				p = K + (size_t)min(k0 + kt * 16 + lr, ctx - 1) * a.ldk + (d < kd ? d : 0) * TR::KF + lg * TR::KV;
+				const size_t key = (size_t)min(k0 + kt * 16 + lr, ctx - 1);
+				p = (d < kn || d >= kd ? K + key * a.ldk + (d < kn ? d : 0) * TR::KF : R + key * a.ldkr + (d - kn) * TR::KF) + lg * TR::KV;
 			} else {
 				const int v = (f - KFRAGS) / NB, b = (f - KFRAGS) % NB;
 				p = V + (size_t)((v < nv ? v : 0) * 16 + lr) * a.ldv + k0 + b * TR::KF + lg * TR::KV;
@@ -325,10 +421,10 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 #pragma unroll
 		for (int i = 0; i < PW; i++) lds[(i * 4 + w) * 64 + lane] = st[i];
 	};
-	fetch(0);
+	fetch(tb * KT);
 	put();
 	tg_lds_barrier();
-	for (int t = 0; t < nt; t++) {
+	for (int t = tb; t < nt; t++) {
 		const int k0 = t * KT;
 		fetch((t + 1 < nt ? t + 1 : t) * KT);
 		f32x4_t sc[QT][NK];
@@ -343,16 +439,18 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 				for (int s = 0; s < QT; s++) sc[s][kt] = TR::mma(kf, qf[s][d], sc[s][kt]);
 			}
 		}
-		// keys past a query only in the tiles that reach the wave's first query
-		const bool masked = k0 + KT - 1 > a.past + qb + w * 16 * QT;
+		// keys past a query only in the tiles that reach the wave's first query, keys before its window in those that do not
+		// reach the last query's
+		const int first_q = a.past + qb + w * 16 * QT;
+		const bool masked = k0 + KT - 1 > first_q || k0 < first_q + 16 * QT - a.window;
 #pragma unroll
 		for (int s = 0; s < QT; s++) {
 			if (masked) {
-				const int lim = a.past + qi[s] - k0 - 4 * lg;
+				const int lim = a.past + qi[s] - k0 - 4 * lg, low = lim - a.window;
 #pragma unroll
 				for (int kt = 0; kt < NK; kt++)
 #pragma unroll
-					for (int e = 0; e < 4; e++) sc[s][kt][e] = kt * 16 + e <= lim ? sc[s][kt][e] : -INFINITY;
+					for (int e = 0; e < 4; e++) sc[s][kt][e] = kt * 16 + e <= lim && kt * 16 + e > low ? sc[s][kt][e] : -INFINITY;
 			}
 			float mt = -INFINITY;
 #pragma unroll
@@ -361,7 +459,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 				for (int e = 0; e < 4; e++) mt = fmaxf(mt, sc[s][kt][e]);
 			mt = fmaxf(mt, tg_red_partner<32>(mt));
 			mt = fmaxf(mt, tg_red_partner<16>(mt));
-			const float mn = fmaxf(m[s], mt * sl2);  // key 0 is in the first tile: finite
+			const float mn = fmaxf(m[s], mt * sl2);
 			if (__ballot(mn > m[s])) {
 				const float f = __builtin_amdgcn_exp2f(m[s] - mn);
 				l[s] *= f;
@@ -419,7 +517,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 		ls += tg_red_partner<32>(ls);
 		ls += tg_red_partner<16>(ls);
 		if (qi[s] >= a.n) continue;
-		const float f = tg_sigmoid(a.gate[(size_t)qi[s] * a.ld_gate + h]) / ls;
+		const float f = (a.gate ? tg_sigmoid(a.gate[(size_t)qi[s] * a.ld_gate + h]) : 1.0f) / ls;
 		T *dst = (T *)a.out + (size_t)qi[s] * a.ldo + (size_t)h * a.vdimp + 4 * lg;
 #pragma unroll
 		for (int v = 0; v < NV; v++)
@@ -449,7 +547,7 @@ void launch_bucket(const TgLatentRows &a, hipStream_t s) {
 template <class TR>
 void launch_attention(const TgLatentRows &a, hipStream_t s) {
 	constexpr int W = TR::DT == TG_DT_BF16 ? 64 : 32;  // keys per tile of the wide buckets
-	const int d = a.dimp, v = a.vdimp;
+	const int d = a.dimp + a.rotp, v = a.vdimp;
 	if (d <= 64 && v <= 64) launch_bucket<TR, 64, 64, 64>(a, s);
 	else if (d <= 64 && v <= 128) launch_bucket<TR, 64, 128, 64>(a, s);
 	else if (d <= 128 && v <= 64) launch_bucket<TR, 128, 64, 64>(a, s);
@@ -463,8 +561,8 @@ void launch_attention(const TgLatentRows &a, hipStream_t s) {
 namespace {
 template <class TR>
 void launch_step(const TgLatentStep &a, hipStream_t s) {
-	const dim3 grid((unsigned)a.nb, (unsigned)((a.heads + 15) / 16), (unsigned)((a.rankp + 511) / 512));
-	const size_t lds = latent_step_lds<TR>(a.rankp);
+	const dim3 grid((unsigned)a.nb, (unsigned)(a.groups * ((a.heads + 15) / 16)), (unsigned)((a.rankp + 511) / 512));
+	const size_t lds = latent_step_lds<TR>(a.rowp());
 	if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void *)latent_step_kernel<TR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
 	hipLaunchKernelGGL((latent_step_kernel<TR>), grid, dim3(256), lds, s, a);
 }
@@ -475,20 +573,42 @@ void tg_launch_latent_step(const TgLatentStep &a, int dt, hipStream_t s) {
 	else launch_step<TgF32>(a, s);
 }
 
-size_t tg_latent_step_lds(int rankp, int dt) { return dt == TG_DT_BF16 ? latent_step_lds<TgB16>(rankp) : latent_step_lds<TgF32>(rankp); }
+size_t tg_latent_step_lds(int rowp, int dt) { return dt == TG_DT_BF16 ? latent_step_lds<TgB16>(rowp) : latent_step_lds<TgF32>(rowp); }
 
-void tg_launch_latent_fold(const float *acc, const float *ml, int nb, int heads16, int rankp, float *out_acc, float *out_ml, hipStream_t s) {
-	hipLaunchKernelGGL(latent_fold_kernel, dim3((unsigned)heads16, (unsigned)(rankp / 64)), dim3(256), 0, s, acc, ml, nb, heads16, rankp, out_acc,
-	                   out_ml);
+void tg_launch_latent_fold(const float *acc, const float *ml, int nb, int heads_padded, int rankp, float *out_acc, float *out_ml, hipStream_t s) {
+	hipLaunchKernelGGL(latent_fold_kernel, dim3((unsigned)heads_padded, (unsigned)((rankp + 63) / 64)), dim3(256), 0, s, acc, ml, nb, heads_padded, rankp,
+	                   out_acc, out_ml, 0, 1, 0);
 }
 
-void tg_launch_latent_rows(const float *dkv, int ld, int n, int rank, int rankp, const float *norm, float eps, int dt, void *cache_rows,
-                           hipStream_t s) {
-	const dim3 grid((unsigned)((n + 3) / 4));
-	if (dt == TG_DT_BF16)
-		hipLaunchKernelGGL((latent_rows_kernel<TgB16>), grid, dim3(256), 0, s, dkv, ld, n, rank, rankp, norm, eps, (__bf16 *)cache_rows);
-	else
-		hipLaunchKernelGGL((latent_rows_kernel<TgF32>), grid, dim3(256), 0, s, dkv, ld, n, rank, rankp, norm, eps, (float *)cache_rows);
+void tg_launch_latent_finish(const float *acc, const float *ml, int nb, int groups, int heads, int rankp, float *out, int out_stride, hipStream_t s) {
+	hipLaunchKernelGGL(latent_fold_kernel, dim3((unsigned)(groups * heads), (unsigned)((rankp + 63) / 64)), dim3(256), 0, s, acc, ml, nb,
+	                   groups * tg_up(heads, 16), rankp, out, (float *)nullptr, groups, heads, out_stride);
+}
+
+namespace {
+template <class TR>
+void launch_cache_rows(const TgLatentCacheRows &a, hipStream_t s) {
+	const dim3 grid((unsigned)((a.n * a.groups + 3) / 4));
+	if (a.f32) hipLaunchKernelGGL((latent_rows_kernel<TR, float>), grid, dim3(256), 0, s, a);
+	else hipLaunchKernelGGL((latent_rows_kernel<TR, typename TR::T>), grid, dim3(256), 0, s, a);
+}
+}  // namespace
+
+void tg_launch_latent_rows(const TgLatentCacheRows &a, int dt, hipStream_t s) {
+	if (dt == TG_DT_BF16) launch_cache_rows<TgB16>(a, s);
+	else launch_cache_rows<TgF32>(a, s);
+}
+
+void tg_launch_rot_rows(void *rows, int ld, int n, int past, int first, int count, int stride, const TgRot &rot, int dt, hipStream_t s) {
+	const dim3 grid((unsigned)((count * (rot.dims / 2) + 255) / 256), (unsigned)n);
+	if (dt == TG_DT_BF16) hipLaunchKernelGGL((rot_rows_kernel<__bf16>), grid, dim3(256), 0, s, (__bf16 *)rows, ld, n, past, first, count, stride, rot);
+	else hipLaunchKernelGGL((rot_rows_kernel<float>), grid, dim3(256), 0, s, (float *)rows, ld, n, past, first, count, stride, rot);
+}
+
+void tg_launch_key_values(const TgKeyValues &a, int dt, hipStream_t s) {
+	const dim3 grid((unsigned)((a.n + 63) / 64), (unsigned)a.groups, (unsigned)(a.dimp / 32));
+	if (dt == TG_DT_BF16) hipLaunchKernelGGL((key_values_kernel<TgB16>), grid, dim3(256), 0, s, a);
+	else hipLaunchKernelGGL((key_values_kernel<TgF32>), grid, dim3(256), 0, s, a);
 }
 
 void tg_launch_latent_attention(const TgLatentRows &a, int dt, hipStream_t s) {

@@ -42,6 +42,7 @@ struct TgF32 {
 	}
 };
 __device__ __forceinline__ float tg_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float tg_gelu(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752440f)); }
 __device__ __forceinline__ float tg_silu(float z) { return z / (1.0f + expf(-z)); }
 // log2(sigmoid(z)) = min(z, 0) log2 e - log2(1 + e^-|z|); for a small second term its series, which keeps it exact to the last bits
 __device__ __forceinline__ float tg_log2_sigmoid(float z) {
@@ -76,6 +77,7 @@ struct TgPack {
 	int g, gp, kg, kgp;
 	int frag_step, frag_off;
 	int transpose;
+	float add;               // added to every element that exists
 };
 void tg_launch_pack(const TgMat &dst, int dt, const TgPack &p, hipStream_t s);
 // the same mapping into plain rows of floats: dst[i * ld + j] = source row and column of (i, j), 0 in the padding
@@ -89,12 +91,14 @@ void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s);
 enum {
 	TG_VP_PLAIN = 0,   // x[z]
 	TG_VP_DYT,         // residual sum, then the element-wise tanh norm
-	TG_VP_HEADNORM,    // heads normalised by their root mean square, times silu(gate)
+	TG_VP_RMS,         // residual sum (its addend normed first where there is a weight for it), then the root mean square norm
+	TG_VP_HEADNORM,    // heads normalised by their root mean square, times silu(gate) or sigmoid(gate)
 	TG_VP_MERGE,       // merged attention partials of head z
 	TG_VP_EXPERT       // x, for the z-th of the experts that the router's logits select
 };
 enum {
 	TG_VE_STORE = 0,
+	TG_VE_GELU,        // the exact gelu
 	TG_VE_SWIGLU,      // silu(gate) * up of a tile pair
 	TG_VE_LOGITS,      // store + maximum of the workgroup's outputs
 	TG_VE_GATE,        // times sigmoid(gate[z])
@@ -112,13 +116,17 @@ struct TgVec {
 	const float *pend;         // DYT: x + mult * (sum of nparts vectors, pend_stride apart) is the new residual
 	int nparts, pend_stride;
 	float mult;
-	const float *nw, *nb;      // DYT: weight and bias; HEADNORM: nw = the head norm's weight
+	const float *nw, *nb;      // DYT: weight and bias; RMS, HEADNORM: nw = the norm's weight
+	const float *post;         // RMS: weight of the norm of the sum of parts before it is added (mult is then unused)
+	int width;                 // RMS: elements that the means are over (K without its padding)
 	float alpha;
-	float *x_out, *h_out;      // DYT: the new residual and the normalised vector (may be null)
-	const void *embed;         // DYT: x is row ctr[4] of this table instead (null: x)
+	float *x_out, *h_out;      // DYT, RMS: the new residual and the normalised vector (may be null)
+	const void *embed;         // DYT, RMS: x is row ctr[4] of this table instead (null: x)
 	int embed_ld, vocab;
+	float embed_scale;         // RMS: factor of that row
 	const int *ctr;
 	const float *gate;         // HEADNORM: gate vector laid out like x; GATE: one value per z
+	int gate_sigmoid;          // HEADNORM: sigmoid(gate) instead of silu(gate)
 	int vdim, vdimp;           // HEADNORM: head size and its padded size
 	float eps;
 	const float *part_acc, *part_ml;  // MERGE: [nmerge][heads padded to 16][x_zstride], [nmerge][heads padded to 16][2]
@@ -129,6 +137,7 @@ struct TgVec {
 	int *sel;                  // EXPERT: written by one workgroup; WEIGHTED: read
 	float *wgt;
 	// output
+	const float *bias;         // STORE: added to the outputs (null: none)
 	float *y;
 	int y_zstride, part_stride;
 	int nout;                  // LOGITS: outputs that exist (the rest is padding)
@@ -146,6 +155,7 @@ enum {
 	TG_GE_F32,         // C2 (fp32)
 	TG_GE_RESID,       // C2 += mult * result
 	TG_GE_SWIGLU,      // fragments alternate gate, up: C = silu(gate) * up
+	TG_GE_GELU,        // C = the exact gelu of the result
 	TG_GE_TRANS        // C^T: C[n][ldc], columns in the key order of the attention operand (tg_latent.h)
 };
 struct TgGemm {
@@ -158,6 +168,7 @@ struct TgGemm {
 	float *C2;
 	int ldc2, n_split;
 	float mult;
+	const float *bias;     // STORE: added to the columns below n_split (null: none)
 	int rows_out;          // TRANS: output columns written (>= M: the last row repeats)
 	// grouped: tile t of the list covers rows [tiles[t].y, tiles[t].z) with the matrix of group tiles[t].x
 	const int4 *tiles;     // null: one matrix

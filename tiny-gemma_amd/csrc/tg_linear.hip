@@ -11,7 +11,7 @@ __device__ __forceinline__ float pack_read(const TgPack &p, int i, int j) {
 	const int r = gi * p.g + ri, c = gj * p.kg + rj;
 	if (ri >= p.g || rj >= p.kg || r >= p.rsrc || c >= p.ksrc) return 0.0f;
 	const size_t at = p.transpose ? (size_t)c * p.src_ld + r : (size_t)r * p.src_ld + c;
-	return p.src_f32 ? ((const float *)p.src)[at] : (float)((const __bf16 *)p.src)[at];
+	return (p.src_f32 ? ((const float *)p.src)[at] : (float)((const __bf16 *)p.src)[at]) + p.add;
 }
 
 template <class TR>
@@ -192,6 +192,126 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 				}
 			}
 		}
+	} else if constexpr (PRO == TG_VP_RMS) {
+		// The whole vector in every workgroup (ksplit is 1): four elements per lane and pass; the first RP passes stay in
+		// registers, the rest goes through LDS.  The padding is zero in x, the parts, the weights and the table.
+		constexpr int RP = 2, PQ = 8;
+		int row = 0;
+		if (p.embed) {
+			row = p.ctr[4];
+			row = row < 0 ? 0 : (row >= p.vocab ? p.vocab - 1 : row);
+		}
+		float *sv = reinterpret_cast<float *>(smem + sizeof(T) * (size_t)(per + KW * U) * TR::KF);  // [kn], wider vectors only
+		const int npass = (kn + 4 * NT - 1) / (4 * NT);
+		f32x4_t x[RP], add[RP], nw[RP], pw[RP];
+		auto at = [&](int i) { return min(4 * (tid + i * NT), kn - 4); };
+		auto source = [&](int c) {
+			f32x4_t v;
+			if (p.embed) {
+				v = tg_load4((const __bf16 *)p.embed + (size_t)row * p.embed_ld + c);
+#pragma unroll
+				for (int e = 0; e < 4; e++) v[e] *= p.embed_scale;
+			} else {
+				v = tg_load4(p.x + c);
+			}
+			return v;
+		};
+		auto parts = [&](int c) {
+			f32x4_t r = {0, 0, 0, 0};
+			for (int q0 = 0; q0 < p.nparts; q0 += PQ) {
+				f32x4_t v[PQ];
+#pragma unroll
+				for (int q = 0; q < PQ; q++) v[q] = tg_load4(p.pend + (size_t)min(q0 + q, p.nparts - 1) * p.pend_stride + c);
+#pragma unroll
+				for (int q = 0; q < PQ; q++)
+					if (q0 + q < p.nparts)
+#pragma unroll
+						for (int e = 0; e < 4; e++) r[e] += v[q][e];
+			}
+			return r;
+		};
+		auto total = [&](float v, int slot) {
+			v = tg_wave_sum(v);
+			if (lane == 0) s_misc[slot + w] = v;
+			__syncthreads();
+			return (s_misc[slot] + s_misc[slot + 1]) + (s_misc[slot + 2] + s_misc[slot + 3]);
+		};
+#pragma unroll
+		for (int i = 0; i < RP; i++) {
+			const int c = at(i);
+			x[i] = source(c);
+			nw[i] = tg_load4(p.nw + c);
+			if (p.nparts) pw[i] = p.post ? tg_load4(p.post + c) : f32x4_t{p.mult, p.mult, p.mult, p.mult};
+		}
+		if (p.nparts) {
+#pragma unroll
+			for (int i = 0; i < RP; i++) add[i] = parts(at(i));
+		}
+		load(kf0);
+		auto wide = [&](int i, auto &&f) {  // f(column, its four values in LDS)
+			for (; i < npass; i++) {
+				const int j = 4 * (tid + i * NT);
+				if (j < kn) f(j);
+			}
+		};
+		if (p.nparts) {
+			float inv = 1.0f;
+			if (p.post) {
+				float ss = 0.0f;
+#pragma unroll
+				for (int i = 0; i < RP; i++)
+					if (4 * (tid + i * NT) < kn)
+#pragma unroll
+						for (int e = 0; e < 4; e++) ss = fmaf(add[i][e], add[i][e], ss);
+				wide(RP, [&](int j) {
+					const f32x4_t v = parts(j);
+#pragma unroll
+					for (int e = 0; e < 4; e++) ss = fmaf(v[e], v[e], ss);
+					tg_store4(sv + j, v);
+				});
+				inv = 1.0f / sqrtf(total(ss, 0) / (float)p.width + p.eps);
+			} else {
+				wide(RP, [&](int j) { tg_store4(sv + j, parts(j)); });
+			}
+#pragma unroll
+			for (int i = 0; i < RP; i++)
+#pragma unroll
+				for (int e = 0; e < 4; e++) x[i][e] += add[i][e] * inv * pw[i][e];
+			wide(RP, [&](int j) {
+				f32x4_t v = source(j);
+				const f32x4_t a = tg_load4(sv + j), b = p.post ? tg_load4(p.post + j) : f32x4_t{p.mult, p.mult, p.mult, p.mult};
+#pragma unroll
+				for (int e = 0; e < 4; e++) v[e] += a[e] * inv * b[e];
+				tg_store4(sv + j, v);
+			});
+		} else {
+			wide(RP, [&](int j) { tg_store4(sv + j, source(j)); });
+		}
+		float ss = 0.0f;
+#pragma unroll
+		for (int i = 0; i < RP; i++)
+			if (4 * (tid + i * NT) < kn)
+#pragma unroll
+				for (int e = 0; e < 4; e++) ss = fmaf(x[i][e], x[i][e], ss);
+		wide(RP, [&](int j) {
+			const f32x4_t v = tg_load4(sv + j);
+#pragma unroll
+			for (int e = 0; e < 4; e++) ss = fmaf(v[e], v[e], ss);
+		});
+		const float inv = 1.0f / sqrtf(total(ss, 4) / (float)p.width + p.eps);
+		const bool first = blockIdx.x == 0 && z == 0;
+		auto finish = [&](int j, f32x4_t v, f32x4_t n) {
+			f32x4_t h;
+#pragma unroll
+			for (int e = 0; e < 4; e++) h[e] = v[e] * inv * n[e];
+			tg_store4(xs + j, h);
+			if (first && p.x_out) tg_store4(p.x_out + j, v);
+			if (first && p.h_out) tg_store4(p.h_out + j, h);
+		};
+#pragma unroll
+		for (int i = 0; i < RP; i++)
+			if (4 * (tid + i * NT) < kn) finish(4 * (tid + i * NT), x[i], nw[i]);
+		wide(RP, [&](int j) { finish(j, tg_load4(sv + j), tg_load4(p.nw + j)); });
 	} else if constexpr (PRO == TG_VP_HEADNORM) {
 		// head by head, a wave each, four elements per lane and pass: sum of squares, then the head's elements that lie in
 		// this part of K
@@ -215,7 +335,7 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 				const int j = a * p.vdimp + v - k0;
 				f32x4_t r;
 #pragma unroll
-				for (int e = 0; e < 4; e++) r[e] = ov[e] * inv * wv[e] * tg_silu(gv[e]);
+				for (int e = 0; e < 4; e++) r[e] = ov[e] * inv * wv[e] * (p.gate_sigmoid ? tg_sigmoid(gv[e]) : tg_silu(gv[e]));
 				if (j >= 0 && j < kn) tg_store4(xs + j, r);
 			}
 		}
@@ -284,6 +404,15 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 				y[group * 16 + tid] = tg_silu(v[0]) * v[NTL - 1];
 			} else {
 				float r = v[0];
+				if constexpr (EPI == TG_VE_STORE) {
+					if (p.bias) {
+						r += p.bias[group * NTL * 16 + tid];
+						if constexpr (NTL == 2) {
+							if (group * 2 + 1 < p.ntiles) v[1] += p.bias[group * 32 + 16 + tid];
+						}
+					}
+				}
+				if constexpr (EPI == TG_VE_GELU) r = tg_gelu(r);
 				if constexpr (EPI == TG_VE_GATE) r *= tg_sigmoid(p.gate[z]);
 				if constexpr (EPI == TG_VE_WEIGHTED) r *= p.wgt[z];
 				y[group * NTL * 16 + tid] = r;
@@ -305,8 +434,11 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 		}
 	} else {
 		if (lane < 16) {
-			const float r = acc[0][0];
 			const int o = group * 16 + lane;
+			float r = acc[0][0];
+			if constexpr (EPI == TG_VE_STORE) {
+				if (p.bias && live) r += p.bias[o];
+			}
 			if (live) p.y[(size_t)z * p.y_zstride + o] = r;
 			if constexpr (EPI == TG_VE_LOGITS) s_red[w][lane] = live && o < p.nout ? r : -INFINITY;
 		}
@@ -333,14 +465,17 @@ bool vec_wide(const TgVec &v, int epi) { return (epi == TG_VE_STORE || epi == TG
 // the parts of the residual) is done half as often.
 bool vec_pairs(const TgVec &v, int epi) { return epi == TG_VE_STORE && v.nparts > 0 && v.nz == 1 && v.ksplit == 1 && v.ntiles >= 448; }
 
+// the norm's vector beyond what the registers of a workgroup hold
+size_t rms_lds(int pro, int k) { return pro == TG_VP_RMS && k > 8 * NT ? sizeof(float) * (size_t)k : 0; }
+
 template <class TR, int PRO, int EPI>
 void launch_vec_t(const TgVec &v, hipStream_t s) {
 	constexpr int NTL = EPI == TG_VE_SWIGLU ? 2 : 1;
 	const int per = (v.kfrags + v.ksplit - 1) / v.ksplit;
-	if constexpr (PRO == TG_VP_DYT && EPI == TG_VE_STORE) {
+	if constexpr ((PRO == TG_VP_DYT || PRO == TG_VP_RMS) && EPI == TG_VE_STORE) {
 		if (!vec_wide(v, EPI) && vec_pairs(v, EPI)) {
 			const int n = (per + 3) / 4;
-			auto lds = [&](int pad) { return sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF; };
+			auto lds = [&](int pad) { return sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF + rms_lds(PRO, per * TR::KF); };
 			const dim3 grid((unsigned)tg_vec_blocks(v, EPI), (unsigned)v.ksplit, (unsigned)v.nz);
 			if (n <= 6) hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, 2, 4, 6>), grid, dim3(NT), lds(24), s, v);
 			else hipLaunchKernelGGL((vec_kernel<TR, PRO, EPI, 2, 4, 8>), grid, dim3(NT), lds(32), s, v);
@@ -350,6 +485,7 @@ void launch_vec_t(const TgVec &v, hipStream_t s) {
 	const unsigned bx = (unsigned)tg_vec_blocks(v, EPI);
 	auto lds = [&](int pad) {
 		size_t b = sizeof(typename TR::T) * (size_t)(per + pad) * TR::KF;
+		b += rms_lds(PRO, per * TR::KF);
 		if (PRO == TG_VP_EXPERT) b += sizeof(float) * (size_t)(((v.experts + 3) & ~3) + 2 * v.top);
 		return b;
 	};
@@ -374,6 +510,10 @@ void launch_vec_dt(const TgVec &v, int pro, int epi, hipStream_t s) {
 	if (pro == TG_VP_PLAIN && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_PLAIN, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_DYT && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_DYT, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_DYT && epi == TG_VE_LOGITS) launch_vec_t<TR, TG_VP_DYT, TG_VE_LOGITS>(v, s);
+	else if (pro == TG_VP_RMS && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_RMS, TG_VE_STORE>(v, s);
+	else if (pro == TG_VP_RMS && epi == TG_VE_GELU) launch_vec_t<TR, TG_VP_RMS, TG_VE_GELU>(v, s);
+	else if (pro == TG_VP_RMS && epi == TG_VE_LOGITS) launch_vec_t<TR, TG_VP_RMS, TG_VE_LOGITS>(v, s);
+	else if (pro == TG_VP_MERGE && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_MERGE, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_HEADNORM) launch_vec_t<TR, TG_VP_HEADNORM, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_MERGE) launch_vec_t<TR, TG_VP_MERGE, TG_VE_GATE>(v, s);
 	else if (pro == TG_VP_EXPERT) launch_vec_t<TR, TG_VP_EXPERT, TG_VE_SWIGLU>(v, s);
@@ -558,8 +698,18 @@ __global__ __launch_bounds__(256, 2) void linear_kernel(TgGemm g) {
 					const int n = tn * BN + (wn * NI + j) * 16 + 4 * lg;
 					if (n >= g.N) continue;
 					if constexpr (EPI == TG_GE_STORE) {
+						if (g.bias && n < g.n_split) {
+							const f32x4_t b = tg_load4(g.bias + n);
+#pragma unroll
+							for (int e = 0; e < 4; e++) acc[i][j][e] += b[e];
+						}
 						if (n < g.n_split) tg_store4((T *)g.C + (size_t)m * g.ldc + n, acc[i][j]);
 						else tg_store4(g.C2 + (size_t)m * g.ldc2 + n - g.n_split, acc[i][j]);
+					} else if constexpr (EPI == TG_GE_GELU) {
+						f32x4_t r;
+#pragma unroll
+						for (int e = 0; e < 4; e++) r[e] = tg_gelu(acc[i][j][e]);
+						tg_store4((T *)g.C + (size_t)m * g.ldc + n, r);
 					} else if constexpr (EPI == TG_GE_F32) {
 						tg_store4(g.C2 + (size_t)m * g.ldc2 + n, acc[i][j]);
 					} else {
@@ -653,6 +803,7 @@ void launch_linear_dt(const TgGemm &g, int epi, hipStream_t s) {
 		case TG_GE_STORE: launch_linear_t<TR, TG_GE_STORE>(g, s); break;
 		case TG_GE_F32: launch_linear_t<TR, TG_GE_F32>(g, s); break;
 		case TG_GE_RESID: launch_linear_t<TR, TG_GE_RESID>(g, s); break;
+		case TG_GE_GELU: launch_linear_t<TR, TG_GE_GELU>(g, s); break;
 		case TG_GE_SWIGLU: launch_linear_t<TR, TG_GE_SWIGLU>(g, s); break;
 		default: launch_linear_t<TR, TG_GE_TRANS>(g, s); break;
 	}

@@ -7,32 +7,47 @@
 
 #include "tg_linear.h"
 
-enum { TG_MIX_LATENT = 0, TG_MIX_GLA };
+enum { TG_MIX_LATENT = 0, TG_MIX_GLA, TG_MIX_DELTA, TG_MIX_ATTN };
+enum { TG_FF_NONE = 0, TG_FF_MOE, TG_FF_DENSE };
+// TG_NORM_TANH: an element-wise tanh before each sublayer, whose output is added times residual_mult.
+// TG_NORM_RMS: root mean square norms before and after each sublayer, weights stored around zero.
+enum { TG_NORM_TANH = 0, TG_NORM_RMS };
 
 struct TgMixerCfg {
 	int kind = 0, heads = 0, dim = 0, vdim = 0;
-	int rank = 0;         // latent: kv_rank; gla: rank of the decay projection (from its tensor)
-	float scale = 0.0f;   // latent: factor of q . k
+	int rank = 0;         // latent: kv_rank; gla, delta: rank of the decay projection (from its tensor)
+	float scale = 0.0f;   // latent, attention: factor of q . k
 	float tau = 1.0f;     // gla
+	int kv_heads = 0;     // delta: q/k heads; attention: key heads
+	int q_rank = 0;       // latent: size of the query's latent (0: the query is a projection, and heads have gates)
+	int rot_dim = 0;      // latent: size of the rotated part (0: no positions)
+	int rot_dims = 0;     // rotated dimensions
+	double rot_base = 0;
+	int window = 1 << 30; // latent, attention: newest token and window - 1 before it
+	int taps = 0;         // delta: convolution
+	int gate_rank = 0;    // delta: rank of the output gate (from its tensor)
 	int dimp() const { return tg_up(dim, 32); }
 	int vdimp() const { return tg_up(vdim, 32); }
+	int rotp() const { return tg_up(kind == TG_MIX_ATTN ? rot_dims : rot_dim, 32); }   // rotated part of a cache row
 };
 struct TgMoeCfg {
-	int experts = 0, top = 0, ff = 0;
+	int experts = 0, top = 0, ff = 0;  // (a dense feed-forward: ff only)
 	float scale = 1.0f;
 	int ffp() const { return tg_up(ff, 64); }
 };
 struct TgNetLayerCfg {
 	TgMixerCfg mix;
-	bool mlp = false;
+	int mlp = TG_FF_NONE;
 	TgMoeCfg moe;
 	int weights_of = -1;
 };
 struct TgNetCfg {
 	std::string arch;
 	int width = 0, vocab = 0;
-	float eps = 0.0f, residual_mult = 1.0f;
+	int norm = TG_NORM_TANH;
+	float eps = 0.0f, residual_mult = 1.0f, embed_scale = 1.0f;
 	std::vector<TgNetLayerCfg> layers;
+	std::vector<int> runs;  // the layer of every layer run, in order; each run has its own cache or state
 	int wp() const { return tg_up(width, 64); }
 };
 
