@@ -183,8 +183,36 @@ def design_config(size):
     return cfg(2048, 131072, _design_layers(24, 4, 4, gla(16, 128, 128), lat(16, 128, 128, 512), moe(64, 6, 1024))), None
 
 
+def tutelix_config(size):
+    """Tutelix at the widths and numbers of layers above, with as many parameters of a layer in use (dense instead of experts); the
+    distinct layers are looped."""
+    def lat(heads, dim, rot, vdim, q, kv, window):
+        return {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "q_rank": q, "kv_rank": kv,
+                                                      "mask": {"size": window}, "rot": {"base": 10000.0, "dims": rot}, "scale": (dim + rot) ** -0.5}}
+
+    def att(heads, kv, dim, rot, window):
+        return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "mask": {"size": window},
+                                               "rot": {"base": 1000000.0, "dims": rot}, "scale": dim ** -0.5}}
+
+    def delta(heads, kv, dim, vdim):
+        return {"type": "channel_delta", "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": 4}}
+
+    def cfg(width, vocab, ff, mixers, loop):
+        return {"architecture": "Tutelix", "width": width, "vocab": vocab, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+                "layers": [dict(m, mlp={"kind": "dense", "ff": ff}) for m in mixers], "loop": {"start": loop[0], "stop": loop[1], "times": loop[2]}}
+
+    if size == "640":
+        return cfg(640, 262144, 2304, [delta(4, 4, 64, 128), lat(4, 64, 32, 64, 256, 128, 1024), att(8, 2, 64, 32, 512)] * 6, (0, 1, 1))
+    if size == "1152":
+        a, b, d = delta(4, 4, 128, 256), lat(8, 128, 64, 128, 512, 256, 1024), att(8, 2, 128, 64, 512)
+        return cfg(1152, 262144, 10368, [a, a, d, b, a, a, d, b, a, b], (0, 8, 3))
+    a, b, d = delta(16, 8, 128, 128), lat(16, 128, 64, 128, 768, 512, 2048), att(16, 4, 128, 64, 1024)
+    return cfg(2048, 131072, 9216, [a, a, d, b], (0, 4, 6))
+
+
 def design_bench(args):
-    """Prefill and decode throughput of the design, and of the Gemma shape of equal width in the same process."""
+    """Prefill and decode throughput of the design, and beside it, in the same process, of the closest other model of equal width: the
+    Gemma shape for Madevik, Madevik for Tutelix."""
     import importlib
     import shutil
     import tempfile
@@ -219,8 +247,8 @@ def design_bench(args):
     result = {}
     sizes = [args.size] if args.size else ["640", "1152", "2048"]
     prompts = [int(x) for x in args.prompts.split(",")]
-    for size in sizes:
-        cfg, gemma = design_config(size)
+
+    def design_rates(cfg):
         d = tempfile.mkdtemp(prefix="tg_bench_")
         try:
             tgw.random_model_dir(d, cfg, args.seed)
@@ -230,8 +258,16 @@ def design_bench(args):
         finally:
             shutil.rmtree(d)
         sess = model.open_session(max(prompts) + args.design_steps + 32)
-        r = {"layers": len(cfg["layers"]), "dtype": args.dtype, "load_s": t_load, args.design: rates(sess, cfg["vocab"], prompts, args.design_steps)}
-        del sess, model
+        return model.cfg.n_layers, t_load, rates(sess, cfg["vocab"], prompts, args.design_steps)
+
+    for size in sizes:
+        cfg, gemma = design_config(size)
+        if args.design == "tutelix":
+            other, cfg, gemma = cfg, tutelix_config(size), None
+        layers, t_load, got = design_rates(cfg)
+        r = {"layers": layers, "dtype": args.dtype, "load_s": t_load, args.design: got}
+        if args.design == "tutelix" and not args.headline_only:
+            r["madevik"] = design_rates(other)[2]
         if gemma and not args.headline_only:
             gcfg = tg.named_config(gemma)
             gm = tg.Transformer(gcfg)
@@ -247,8 +283,8 @@ def design_bench(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["madevik"], default=None,
-                    help="instead of the default workload: prefill and decode rates of this design at --size, beside the Gemma shape of equal width")
+    ap.add_argument("--design", choices=["madevik", "tutelix"], default=None,
+                    help="instead of the default workload: prefill and decode rates of this design at --size, beside the closest other model of equal width")
     ap.add_argument("--size", choices=["640", "1152", "2048"], default=None, help="with --design: width (default: all)")
     ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="with --design")
     ap.add_argument("--prompts", default="178,1024,4096", help="with --design: prompt lengths")

@@ -33,7 +33,7 @@ def folder(tmp_path_factory):
             t = nm.weights(cfg, seed, **kw)
             if edit:
                 edit(t)
-            cache[key] = (nm.write(tmp_path_factory.mktemp("net") / "m", cfg, t), layers.LayerModel(cfg, t))
+            cache[key] = (nm.write(tmp_path_factory.mktemp("net") / "m", cfg, t), layers.model_of(cfg, t))
         return cache[key]
 
     return make

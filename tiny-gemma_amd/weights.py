@@ -99,7 +99,7 @@ def random_weight_image(cfg, seed, std=0.02, norm_std=0.1):
 # ---- model folders (layer-list models) ---------------------------------------------------------------------------
 def madevik_tensors(cfg, decay_rank):
     """[(name, shape, kind)] of a Madevik model in file order; kind: "w" matrix, "one" norm weight, "zero" bias,
-    "alpha" scalar of the element-wise tanh norm, "decay" bias of the decay projection."""
+    "alpha" scalar of the element-wise tanh norm, "decay" and "softplus" bias of a decay projection."""
     D, V = cfg["width"], cfg["vocab"]
     out = [("embed", (V, D), "w")]
 
@@ -131,7 +131,36 @@ def madevik_tensors(cfg, decay_rank):
     return out
 
 
-def random_model_dir(path, cfg, seed, decay_rank=16, block=1 << 22):
+def tutelix_tensors(cfg, decay_rank, gate_rank):
+    """The same of a Tutelix model (norm weights stored around zero, A_log and convolutions are "zero" and "w")."""
+    D, V = cfg["width"], cfg["vocab"]
+    out = [("embed", (V, D), "w")]
+    for i, l in enumerate(cfg["layers"]):
+        m, p = l["mixer"], f"l{i}.mix."
+        H, d, v = m["heads"], m["dim"], m["vdim"]
+        mlp = l.get("mlp")
+        out += [(f"l{i}.{n}", (D,), "zero") for n in ("norm1", "norm1b") + (("norm2", "norm2b") if mlp else ())]
+        if l["type"] == "latent_attention":
+            q, r, e = m["q_rank"], m["kv_rank"], m["rot_dim"]
+            out += [(p + "dq", (q, D), "w"), (p + "dq.norm", (q,), "one"), (p + "uq", (H * (d + e), q), "w"), (p + "dkv", (r + e, D), "w"),
+                    (p + "dkv.norm", (r,), "one"), (p + "uk", (H * d, r), "w"), (p + "uv", (H * v, r), "w")]
+        elif l["type"] == "attention":
+            G = m["kv_heads"]
+            out += [(p + "q", (H * d, D), "w"), (p + "q.b", (H * d,), "zero"), (p + "k", (G * d, D), "w"), (p + "k.b", (G * d,), "zero")]
+        else:
+            G = m["kv_heads"]
+            for n, rows in (("q", G * d), ("k", G * d), ("v", H * v)):
+                out += [(p + n, (rows, D), "w"), (f"{p}{n}.conv", (rows, m["conv"]), "w")]
+            out += [(p + "b", (H, D), "w"), (p + "A_log", (H,), "zero"), (p + "norm", (v,), "one"), (p + "a1", (decay_rank, D), "w"),
+                    (p + "a2", (H * d, decay_rank), "w"), (p + "dt_bias", (H * d,), "softplus"), (p + "g1", (gate_rank, D), "w"),
+                    (p + "g2", (H * v, gate_rank), "w")]
+        out.append((p + "o", (D, H * v), "w"))
+        if mlp:
+            out += [(f"l{i}.mlp.up", (mlp["ff"], D), "w"), (f"l{i}.mlp.down", (D, mlp["ff"]), "w")]
+    return out + [("final.norm", (D,), "zero"), ("head", (V, D), "w")]
+
+
+def random_model_dir(path, cfg, seed, decay_rank=16, block=1 << 22, gate_rank=None):
     """Writes config.json and model.safetensors of a random-init model (matrices N(0, 1 / inputs)) into `path`.  Matrices are
     cut at random places out of one block of normal numbers per scale: large models are written at the speed of the disk."""
     os.makedirs(path, exist_ok=True)
@@ -146,7 +175,7 @@ def random_model_dir(path, cfg, seed, decay_rank=16, block=1 << 22):
 
     blocks = {}
     head, off = {}, 0
-    tensors = madevik_tensors(cfg, decay_rank)
+    tensors = tutelix_tensors(cfg, decay_rank, gate_rank or decay_rank) if cfg["architecture"] == "Tutelix" else madevik_tensors(cfg, decay_rank)
     for name, shape, _ in tensors:
         n = 2 * int(np.prod(shape, dtype=np.int64))
         head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [off, off + n]}
@@ -168,7 +197,7 @@ def random_model_dir(path, cfg, seed, decay_rank=16, block=1 << 22):
                     f.write(b[at:at + k].tobytes())
                     n -= k
             else:
-                a = {"one": 1.0, "zero": 0.0, "alpha": 0.7, "decay": 3.0}[kind] * np.ones(n, np.float32)
+                a = {"one": 1.0, "zero": 0.0, "alpha": 0.7, "decay": 3.0, "softplus": -3.0}[kind] * np.ones(n, np.float32)
                 if kind in ("one", "zero"):
                     a += rng.standard_normal(n, dtype=np.float32) * np.float32(0.1)
                 f.write(bf16(a).tobytes())
