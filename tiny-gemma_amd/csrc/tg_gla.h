@@ -56,6 +56,7 @@ void tg_launch_delta_step(const TgDelta &d, const float *y, int g_off, int b_off
 struct TgDeltaScratch {
 	float *b;       // [chunks * 64][heads * dimp] running sums of log2 alpha inside a chunk
 	float *a;       // [chunks][heads][64][64] q . k with the decay between them
+	float *t;       // [chunks][heads][64][64] what the solve multiplies with (tg_gla.hip)
 	float *qk;      // [n][q | k] behind convolution and unit norm
 	float *u;       // [chunks * 64][heads * vdimp] v, then its solved form, then u
 	float *wk;      // [chunks * 64][heads * dimp] solved keys

@@ -133,15 +133,12 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float *low, int ld
 // ---- A: a workgroup per chunk and head, a wave per block of 16 rows ---------------------------------------------------------
 constexpr int SL = 32, SLP = 36;  // key channels per slab, row pitch
 
-// DELTA: also k . k with the decay between them, T = beta (k . k) below the diagonal, and the chunk's solved keys and values:
-//     u = M (beta v) - M (beta k e^b) S   with M = (1 + T)^-1, S the state in front of the chunk.
-// T's diagonal blocks of 16 are inverted by substitution, a lane per column; the solve runs down the blocks on the matrix
-// instructions, a wave per 16 columns: an accumulator (four consecutive rows of a column per lane) is the next product's
-// second operand as it is, with the first operand's columns taken in the same order.
+// DELTA: also k . k with the decay between them, T = beta (k . k) below the diagonal, of which it leaves -T outside the 16 x 16
+// diagonal blocks and in those the inverse of 1 + T's block (by substitution, a lane per column).
 struct DeltaIntra {
 	const float *beta;  // [n][ld_beta], before the sigmoid
 	int ld_beta;
-	float *u, *wk, *kt;
+	float *t;           // [chunks][heads][64][64]
 };
 
 template <class TR, bool DELTA>
@@ -214,96 +211,130 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 		}
 	}
 	if constexpr (DELTA) {
-		__shared__ __align__(16) float s_t[C][C + 4], s_m[4][16][20];
-		__shared__ float s_beta[C];
-		if (tid < C) s_beta[tid] = t0 + tid < n ? tg_sigmoid(x.beta[(size_t)(t0 + tid) * x.ld_beta + h]) : 0.0f;
-		__syncthreads();
-		const int qi = 16 * w + lr;
+		__shared__ __align__(16) float s_t[4][16][20];
+		float *T = x.t + ((size_t)ch * g.heads + h) * C * C;
+		float beta_q = 0.0f, beta_r[4];
+		auto step = [&](int r) { return t0 + r < n ? tg_sigmoid(x.beta[(size_t)(t0 + r) * x.ld_beta + h]) : 0.0f; };
+		beta_q = step(16 * w + lr);
 #pragma unroll
-		for (int j = 0; j < 4; j++) s_t[qi][16 * w + 4 * lg + j] = 4 * lg + j < lr ? s_beta[qi] * kdia[j] : 0.0f;
+		for (int e = 0; e < 4; e++) beta_r[e] = step(16 * w + 4 * lg + e);
+#pragma unroll
+		for (int j = 0; j < 4; j++) s_t[w][lr][4 * lg + j] = 4 * lg + j < lr ? beta_q * kdia[j] : 0.0f;
 #pragma unroll
 		for (int j = 0; j < 3; j++)
 			if (j < w) {
 #pragma unroll
-				for (int e = 0; e < 4; e++) s_t[16 * w + 4 * lg + e][16 * j + lr] = s_beta[16 * w + 4 * lg + e] * koff[j][e];
+				for (int e = 0; e < 4; e++) T[(size_t)(16 * w + 4 * lg + e) * C + 16 * j + lr] = -beta_r[e] * koff[j][e];
 			}
 		__syncthreads();
-		{
-			float m[16];
+		float m[16];
 #pragma unroll
-			for (int r = 0; r < 16; r++) {
-				float v = r == lr ? 1.0f : 0.0f;
-				f32x4_t tr[4];
+		for (int r = 0; r < 16; r++) {
+			float v = r == lr ? 1.0f : 0.0f;
+			f32x4_t tr[4];
 #pragma unroll
-				for (int j = 0; j < 4; j++) tr[j] = tg_load4(&s_t[16 * w + r][16 * w + 4 * j]);
+			for (int j = 0; j < 4; j++) tr[j] = tg_load4(&s_t[w][r][4 * j]);
 #pragma unroll
-				for (int j = 0; j < r; j++) v = fmaf(-tr[j >> 2][j & 3], m[j], v);
-				m[r] = v;
-			}
-			if (lg == 0)
-#pragma unroll
-				for (int r = 0; r < 16; r++) s_m[w][r][lr] = m[r];
+			for (int j = 0; j < r; j++) v = fmaf(-tr[j >> 2][j & 3], m[j], v);
+			m[r] = v;
 		}
-		__syncthreads();
-		f32x4_t tb[6], mb[4];  // blocks (1,0) (2,0) (2,1) (3,0) (3,1) (3,2), negated; inverses
+		if (lg == 0)
 #pragma unroll
-		for (int i = 0; i < 4; i++) {
-			mb[i] = tg_load4(&s_m[i][lr][4 * lg]);
+			for (int r = 0; r < 16; r++) T[(size_t)(16 * w + r) * C + 16 * w + lr] = m[r];
+	}
+}
+
+// ---- the chunk's solved keys and values (delta rule): u = M (beta v) - M (beta k e^b) S with M = (1 + T)^-1, S the state in front of it -
+// The solve runs down the 16 x 16 blocks on the matrix instructions, a wave per two tiles of 16 columns: an accumulator (four
+// consecutive rows of a column per lane) is the next product's second operand as it is, with the first operand's columns taken
+// in the same order.  Also the keys decayed to the chunk's end, transposed.
+struct DeltaSolve {
+	const float *qk, *b, *t, *beta;
+	int ldqk, k_off, ld_beta;
+	float *u, *wk, *kt;
+};
+__global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g, int n) {
+	__shared__ __align__(16) float s_beta[C];
+	const int ch = blockIdx.x, h = blockIdx.y, kh = h / g.group, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
+	const int hd = g.heads * g.dimp, hv = g.heads * g.vdimp, t0 = ch * C;
+	const int nk = g.dimp / 16, ntile = nk + g.vdimp / 16, tile0 = ((int)blockIdx.z * 4 + w) * 2;
+	const float *T = x.t + ((size_t)ch * g.heads + h) * C * C;
+	const float raw = x.beta[(size_t)min(t0 + (tid & 63), n - 1) * x.ld_beta + h];
+	f32x4_t tb[6], mb[4];  // blocks (1,0) (2,0) (2,1) (3,0) (3,1) (3,2); the inverses
 #pragma unroll
-			for (int j = 0; j < i; j++) {
-				tb[i * (i - 1) / 2 + j] = tg_load4(&s_t[16 * i + lr][16 * j + 4 * lg]);
+	for (int i = 0; i < 4; i++) {
+		mb[i] = tg_load4(T + (size_t)(16 * i + lr) * C + 16 * i + 4 * lg);
 #pragma unroll
-				for (int e = 0; e < 4; e++) tb[i * (i - 1) / 2 + j][e] *= -1.0f;
-			}
-		}
-		const int nk = g.dimp / 16, ntile = nk + g.vdimp / 16, hv = g.heads * g.vdimp;
-		for (int tile = w; tile < ntile; tile += 4) {
-			const bool key = tile < nk;
-			const int col = (key ? tile : tile - nk) * 16 + lr;
-			f32x4_t X[4], W[4];
-			if (key) {
-				const float be = b[(size_t)(t0 + C - 1) * hd + (size_t)h * g.dimp + col];
-				float *kt = x.kt + (((size_t)ch * g.heads + h) * g.dimp + col) * C + 4 * lg;
+		for (int j = 0; j < i; j++) tb[i * (i - 1) / 2 + j] = tg_load4(T + (size_t)(16 * i + lr) * C + 16 * j + 4 * lg);
+	}
+	// (a wave past the last tile repeats it and stores nothing; tiles come in pairs: nk and the number of value tiles are even)
+	const bool live = tile0 < ntile;
+	const int tile = live ? tile0 : ntile - 2;
+	const bool key = tile < nk;
+	int col[2];
+	f32x4_t X[2][4], W[2][4], bt[2][4];
+	float be[2] = {0.0f, 0.0f};
 #pragma unroll
-				for (int i = 0; i < 4; i++) {
-					f32x4_t kd;
+	for (int p = 0; p < 2; p++) {
+		col[p] = (key ? tile : tile - nk) * 16 + 16 * p + lr;
+		const float *src = key ? x.qk + x.k_off + (size_t)kh * g.dimp + col[p] : x.u + (size_t)h * g.vdimp + col[p];
+		const int ld = key ? x.ldqk : hv;
 #pragma unroll
-					for (int e = 0; e < 4; e++) {
-						const int r = 16 * i + 4 * lg + e, t = t0 + r;
-						const float k = t < n ? (float)qkv[(size_t)min(t, n - 1) * ld + k_off + (size_t)kh * g.dimp + col] : 0.0f;
-						const float bt = b[(size_t)t * hd + (size_t)h * g.dimp + col];
-						X[i][e] = s_beta[r] * k * pow2(bt);
-						kd[e] = k * pow2(be - bt);
-					}
-					tg_store4(kt + 16 * i, kd);
-				}
-			} else {
+		for (int i = 0; i < 4; i++)
 #pragma unroll
-				for (int i = 0; i < 4; i++)
-#pragma unroll
-					for (int e = 0; e < 4; e++) {
-						const int r = 16 * i + 4 * lg + e, t = t0 + r;
-						X[i][e] = t < n ? s_beta[r] * x.u[(size_t)t * hv + (size_t)h * g.vdimp + col] : 0.0f;
-					}
-			}
-#pragma unroll
-			for (int i = 0; i < 4; i++) {
-				f32x4_t acc = X[i];
-#pragma unroll
-				for (int j = 0; j < i; j++)
-#pragma unroll
-					for (int e = 0; e < 4; e++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(tb[i * (i - 1) / 2 + j][e], W[j][e], acc, 0, 0, 0);
-				W[i] = f32x4_t{0, 0, 0, 0};
-#pragma unroll
-				for (int e = 0; e < 4; e++) W[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(mb[i][e], acc[e], W[i], 0, 0, 0);
-			}
-			float *dst = key ? x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col : x.u + (size_t)t0 * hv + (size_t)h * g.vdimp + col;
-			const int pitch = key ? hd : hv;
+			for (int e = 0; e < 4; e++) X[p][i][e] = src[(size_t)min(t0 + 16 * i + 4 * lg + e, n - 1) * ld];
+		if (key) {
+			const float *bp = x.b + (size_t)t0 * hd + (size_t)h * g.dimp + col[p];
+			be[p] = bp[(size_t)(C - 1) * hd];
 #pragma unroll
 			for (int i = 0; i < 4; i++)
 #pragma unroll
-				for (int e = 0; e < 4; e++) dst[(size_t)(16 * i + 4 * lg + e) * pitch] = W[i][e];
+				for (int e = 0; e < 4; e++) bt[p][i][e] = bp[(size_t)(16 * i + 4 * lg + e) * hd];
 		}
+	}
+	if (tid < C) s_beta[tid] = t0 + tid < n ? tg_sigmoid(raw) : 0.0f;
+	__syncthreads();
+#pragma unroll
+	for (int p = 0; p < 2; p++)
+#pragma unroll
+		for (int i = 0; i < 4; i++) {
+			const f32x4_t beta = tg_load4(&s_beta[16 * i + 4 * lg]);
+			if (key) {
+				f32x4_t kd;
+#pragma unroll
+				for (int e = 0; e < 4; e++) {
+					kd[e] = t0 + 16 * i + 4 * lg + e < n ? X[p][i][e] * pow2(be[p] - bt[p][i][e]) : 0.0f;
+					X[p][i][e] *= pow2(bt[p][i][e]);
+				}
+				if (live) tg_store4(x.kt + (((size_t)ch * g.heads + h) * g.dimp + col[p]) * C + 16 * i + 4 * lg, kd);
+			}
+#pragma unroll
+			for (int e = 0; e < 4; e++) X[p][i][e] *= beta[e];
+		}
+#pragma unroll
+	for (int i = 0; i < 4; i++) {
+#pragma unroll
+		for (int j = 0; j < i; j++)
+#pragma unroll
+			for (int e = 0; e < 4; e++)
+#pragma unroll
+				for (int p = 0; p < 2; p++) X[p][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(tb[i * (i - 1) / 2 + j][e], W[p][j][e], X[p][i], 0, 0, 0);
+#pragma unroll
+		for (int p = 0; p < 2; p++) W[p][i] = f32x4_t{0, 0, 0, 0};
+#pragma unroll
+		for (int e = 0; e < 4; e++)
+#pragma unroll
+			for (int p = 0; p < 2; p++) W[p][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(mb[i][e], X[p][i][e], W[p][i], 0, 0, 0);
+	}
+	if (!live) return;
+	const int pitch = key ? hd : hv;
+#pragma unroll
+	for (int p = 0; p < 2; p++) {
+		float *dst = key ? x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col[p] : x.u + (size_t)t0 * hv + (size_t)h * g.vdimp + col[p];
+#pragma unroll
+		for (int i = 0; i < 4; i++)
+#pragma unroll
+			for (int e = 0; e < 4; e++) dst[(size_t)(16 * i + 4 * lg + e) * pitch] = W[p][i][e];
 	}
 }
 
@@ -530,51 +561,45 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
 // Launches: convolution and unit norms; b; A, T and the solved keys and values, all chunks at once; the pass over the chunks
 // (u and the state in front of each), 16 value columns per workgroup; the outputs, all chunks at once.
 
-// ---- convolution, silu, unit norm: 4 tokens per workgroup, a wave each; y: q heads, k heads, blocks of 256 value channels --------
+// ---- convolution, silu, unit norm: 4 tokens per wave; y: q heads, k heads, blocks of 256 value channels ------------------------------
 // Inputs before the portion come from the ring.
-__device__ __forceinline__ f32x4_t ring4(const TgDelta &d, int pos, int c) {
-	return pos < 0 ? f32x4_t{0, 0, 0, 0} : tg_load4(d.ring + (size_t)(pos % d.taps) * d.channels + c);
-}
+constexpr int PT = 4;
 template <class TR>
 __global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, float *qk, float *u) {
-	const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, kvh = d.g.heads / d.g.group, qc = d.q_channels();
-	if (t >= n) return;
+	const int t0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * PT, lane = threadIdx.x & 63, kvh = d.g.heads / d.g.group, qc = d.q_channels();
+	if (t0 >= n) return;
 	const bool head = (int)blockIdx.y < 2 * kvh;
 	const int base = head ? (int)blockIdx.y * d.g.dimp : 2 * qc + ((int)blockIdx.y - 2 * kvh) * 256;
-	const int len = head ? d.g.dimp : min(256, d.channels - base);
-	constexpr int P = TG_DELTA_DIM_MAX / 256;
-	f32x4_t r[P];
-	float ss = 0.0f;
+	const int len = head ? d.g.dimp : min(256, d.channels - base);  // (at most 256)
+	const int c = base + min(4 * lane, len - 4);
+	const bool in = 4 * lane < len;
+	f32x4_t r[PT];
 #pragma unroll
-	for (int p = 0; p < P; p++) {
-		const int c = 4 * lane + 256 * p;
-		r[p] = f32x4_t{0, 0, 0, 0};
-		if (c < len) {
-			for (int i = 0; i < d.taps; i++) {
-				const int from = t - d.taps + 1 + i;
-				const f32x4_t v = from >= 0 ? tg_load4(x + (size_t)from * ld + base + c) : ring4(d, past + from, base + c);
-				const f32x4_t w = tg_load4(d.conv + (size_t)i * d.channels + base + c);
+	for (int p = 0; p < PT; p++) r[p] = f32x4_t{0, 0, 0, 0};
+	for (int i = 0; i < d.taps; i++) {
+		const f32x4_t w = tg_load4(d.conv + (size_t)i * d.channels + c);
 #pragma unroll
-				for (int e = 0; e < 4; e++) r[p][e] = fmaf(w[e], v[e], r[p][e]);
-			}
+		for (int p = 0; p < PT; p++) {
+			const int from = min(t0 + p, n - 1) - d.taps + 1 + i;
+			f32x4_t v = {0, 0, 0, 0};
+			if (from >= 0) v = tg_load4(x + (size_t)from * ld + c);
+			else if (past + from >= 0) v = tg_load4(d.ring + (size_t)((past + from) % d.taps) * d.channels + c);
 #pragma unroll
-			for (int e = 0; e < 4; e++) {
-				r[p][e] = tg_silu(r[p][e]);
-				ss = fmaf(r[p][e], r[p][e], ss);
-			}
+			for (int e = 0; e < 4; e++) r[p][e] = fmaf(w[e], v[e], r[p][e]);
 		}
 	}
-	float f = 1.0f;
-	if (head) f = 1.0f / sqrtf(tg_wave_sum(ss) + 1e-6f);
-	float *dst = head ? qk + (size_t)t * 2 * qc + base : u + (size_t)t * (d.channels - 2 * qc) + base - 2 * qc;
 #pragma unroll
-	for (int p = 0; p < P; p++) {
-		const int c = 4 * lane + 256 * p;
-		if (c < len) {
+	for (int p = 0; p < PT; p++) {
+		float ss = 0.0f, f = 1.0f;
 #pragma unroll
-			for (int e = 0; e < 4; e++) r[p][e] *= f;
-			tg_store4(dst + c, r[p]);
+		for (int e = 0; e < 4; e++) {
+			r[p][e] = tg_silu(r[p][e]);
+			ss = fmaf(r[p][e], r[p][e], ss);
 		}
+		if (head) f = 1.0f / sqrtf(tg_wave_sum(in ? ss : 0.0f) + 1e-6f);
+#pragma unroll
+		for (int e = 0; e < 4; e++) r[p][e] *= f;
+		if (in && t0 + p < n) tg_store4(head ? qk + (size_t)(t0 + p) * 2 * qc + c : u + (size_t)(t0 + p) * (d.channels - 2 * qc) + c - 2 * qc, r[p]);
 	}
 }
 
@@ -582,12 +607,13 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typena
 // Wave w keeps rows 16 (w + 4 i) ... of S in accumulators, which are the second operand of the products with the solved keys as
 // they are; the waves' parts of those products meet in LDS, and u, again in accumulator layout, is the second operand of S's
 // update.  The last inputs of the convolution go to the ring on the way.
-template <class TR, int ND>
-__global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, const float *b, float *u,
+// AHEAD: chunks whose operands are in registers or on their way.
+template <class TR, int ND, int AHEAD>
+__global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, const float *b, float *u,
                                                          const float *wk, const float *kt, float *st, int chunks) {
 	__shared__ __align__(16) f32x4_t s_p[4][4][64], s_u[4][64];
 	const TgGla &g = d.g;
-	const int h = blockIdx.x, v0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
+	const int h = blockIdx.x, v0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
 	const int hd = g.heads * g.dimp, hv = g.heads * g.vdimp, ntile = g.dimp / 16;
 	{
 		const int keep = min(d.taps, n), total = keep * d.channels, step = (int)(gridDim.x * gridDim.y) * 256;
@@ -597,7 +623,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typena
 		}
 	}
 	f32x4_t S[ND];
-	f32x4_t fw[ND][4], fk[ND][4], fb[ND], fv;
+	f32x4_t fw[AHEAD][ND][4], fk[AHEAD][ND][4], fb[AHEAD][ND], fv[AHEAD];
 	bool own[ND];
 	int row[ND];  // first row of the tile (the last tile again where there is none; its part counts as zero)
 #pragma unroll
@@ -607,22 +633,26 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typena
 #pragma unroll
 		for (int e = 0; e < 4; e++) S[i][e] = own[i] ? g.state[((size_t)h * g.dimp + row[i] + 4 * lg + e) * g.vdimp + v0 + lr] : 0.0f;
 	}
-	auto fetch = [&](int ch) {
-		const size_t t0 = (size_t)ch * C;
+	const unsigned lw = (unsigned)(lr * hd + 4 * lg), lk = (unsigned)(lr * C + 4 * lg), lu = (unsigned)((16 * w + 4 * lg) * hv + lr);
+	const unsigned ls = (unsigned)(4 * lg * g.vdimp + lr);
+	auto fetch = [&](int set, int ch) {
+		// (bases that the workgroup shares, 32-bit offsets per lane)
+		const size_t t0 = (size_t)min(ch, chunks - 1) * C;
+		const float *pw = wk + t0 * hd + (size_t)h * g.dimp, *pk = kt + t0 * hd + (size_t)h * g.dimp * C, *pb = b + (t0 + C - 1) * hd + (size_t)h * g.dimp;
+		const float *pu = u + t0 * hv + (size_t)h * g.vdimp + v0;
 #pragma unroll
 		for (int i = 0; i < ND; i++) {
 #pragma unroll
 			for (int tt = 0; tt < 4; tt++) {
-				fw[i][tt] = tg_load4(wk + (t0 + 16 * tt + lr) * hd + (size_t)h * g.dimp + row[i] + 4 * lg);
-				fk[i][tt] = tg_load4(kt + (((size_t)ch * g.heads + h) * g.dimp + row[i] + lr) * C + 16 * tt + 4 * lg);
+				fw[set][i][tt] = tg_load4(pw + (size_t)(16 * tt) * hd + (lw + (unsigned)row[i]));
+				fk[set][i][tt] = tg_load4(pk + 16 * tt + (lk + (unsigned)row[i] * C));
 			}
-			fb[i] = tg_load4(b + (t0 + C - 1) * hd + (size_t)h * g.dimp + row[i] + 4 * lg);
+			fb[set][i] = tg_load4(pb + (unsigned)(row[i] + 4 * lg));
 		}
 #pragma unroll
-		for (int e = 0; e < 4; e++) fv[e] = u[(t0 + 16 * w + 4 * lg + e) * hv + (size_t)h * g.vdimp + v0 + lr];
+		for (int e = 0; e < 4; e++) fv[set][e] = pu[(size_t)e * hv + lu];
 	};
-	fetch(0);
-	for (int ch = 0; ch < chunks; ch++) {
+	auto chunk = [&](int set, int ch) {
 		f32x4_t part[4];
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) part[tt] = f32x4_t{0, 0, 0, 0};
@@ -631,24 +661,20 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typena
 #pragma unroll
 			for (int e = 0; e < 4; e++)
 #pragma unroll
-				for (int tt = 0; tt < 4; tt++) part[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(fw[i][tt][e], S[i][e], part[tt], 0, 0, 0);
+				for (int tt = 0; tt < 4; tt++) part[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(fw[set][i][tt][e], S[i][e], part[tt], 0, 0, 0);
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) s_p[w][tt][lane] = part[tt];
-		float *front = st + (((size_t)ch * g.heads + h) * g.dimp) * g.vdimp + v0 + lr;
+		float *front = st + (((size_t)ch * g.heads + h) * g.dimp) * g.vdimp + v0;
 #pragma unroll
 		for (int i = 0; i < ND; i++)
 			if (own[i])
 #pragma unroll
-				for (int e = 0; e < 4; e++) front[(size_t)(row[i] + 4 * lg + e) * g.vdimp] = S[i][e];
-		f32x4_t kk[ND][4], fade[ND], uv = fv;
+				for (int e = 0; e < 4; e++) front[(size_t)e * g.vdimp + (ls + (unsigned)(row[i] * g.vdimp))] = S[i][e];
+		f32x4_t uv = fv[set];
 #pragma unroll
-		for (int i = 0; i < ND; i++) {
+		for (int i = 0; i < ND; i++)
 #pragma unroll
-			for (int tt = 0; tt < 4; tt++) kk[i][tt] = fk[i][tt];
-#pragma unroll
-			for (int e = 0; e < 4; e++) fade[i][e] = pow2(fb[i][e]);
-		}
-		if (ch + 1 < chunks) fetch(ch + 1);
+			for (int e = 0; e < 4; e++) S[i][e] *= pow2(fb[set][i][e]);
 		tg_lds_barrier();
 #pragma unroll
 		for (int q = 0; q < 4; q++)
@@ -656,25 +682,30 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(TgDelta d, const typena
 			for (int e = 0; e < 4; e++) uv[e] -= s_p[q][w][lane][e];
 		s_u[w][lane] = uv;
 #pragma unroll
-		for (int e = 0; e < 4; e++) u[((size_t)ch * C + 16 * w + 4 * lg + e) * hv + (size_t)h * g.vdimp + v0 + lr] = uv[e];
+		for (int e = 0; e < 4; e++) u[(size_t)ch * C * hv + (size_t)h * g.vdimp + v0 + (size_t)e * hv + lu] = uv[e];
 		tg_lds_barrier();
 		f32x4_t ut[4];
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) ut[tt] = s_u[tt][lane];
 #pragma unroll
-		for (int i = 0; i < ND; i++) {
-#pragma unroll
-			for (int e = 0; e < 4; e++) S[i][e] *= fade[i][e];
-		}
-#pragma unroll
 		for (int tt = 0; tt < 4; tt++)
 #pragma unroll
 			for (int e = 0; e < 4; e++)
 #pragma unroll
-				for (int i = 0; i < ND; i++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i][tt][e], ut[tt][e], S[i], 0, 0, 0);
+				for (int i = 0; i < ND; i++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(fk[set][i][tt][e], ut[tt][e], S[i], 0, 0, 0);
 #pragma unroll
 		for (int i = 0; i < ND; i++)
 			if (!own[i]) S[i] = f32x4_t{0, 0, 0, 0};
+		fetch(set, ch + AHEAD);  // (past the end: the last chunk again, unused; its u may have changed, and is not looked at)
+	};
+#pragma unroll
+	for (int a = 0; a < AHEAD; a++) fetch(a, a);
+	for (int ch = 0; ch < chunks; ch += AHEAD) {
+#pragma unroll
+		for (int a = 0; a < AHEAD; a++) {
+			if (ch + a < chunks) chunk(a, ch + a);
+			__builtin_amdgcn_sched_barrier(0);
+		}
 	}
 #pragma unroll
 	for (int i = 0; i < ND; i++)
@@ -700,61 +731,96 @@ __global__ __launch_bounds__(256) void delta_step_kernel(const float *y, TgDelta
 #pragma unroll
 	for (int r = 0; r < R; r++) st[r] = tg_load4(S + (size_t)min(dg + 32 * r, g.dimp - 1) * g.vdimp);
 	const float step = y[b_off + h];
-	// silu of the convolution of channel c, and the newest input to the ring where this workgroup is the one that does it
-	const int slot = pos % d.taps;
-	auto conv = [&](int c, bool keep) {
-		const float x = y[c];
-		float r = x * d.conv[(size_t)(d.taps - 1) * d.channels + c];
-		int from = slot + 1 == d.taps ? 0 : slot + 1;  // the row of position pos - taps + 1 (zero before the start)
-		for (int i = 0; i < d.taps - 1; i++) {
-			r = fmaf(d.conv[(size_t)i * d.channels + c], d.ring[(size_t)from * d.channels + c], r);
-			from = from + 1 == d.taps ? 0 : from + 1;
-		}
-		if (keep) d.ring[(size_t)slot * d.channels + c] = x;
-		return tg_silu(r);
+	// Everything is requested before anything is used or stored: the convolution's inputs (CT earlier ones per round) of a key or
+	// query channel and of a value channel, the decay's and the gate's low-rank products.
+	constexpr int CT = 4, RA = 16, RG = 8;
+	const int slot = pos % d.taps, ch_v = 2 * qc + h * g.vdimp + c0 + (tid & 31);
+	struct Conv {
+		float x, wx, w[CT], in[CT];
 	};
-	const bool keep_qk = h % g.group == 0 && blockIdx.y == 0;
+	auto conv_request = [&](int c, int i0, Conv &r) {  // earlier inputs i0 ... i0 + CT - 1, oldest first (zero before the start)
+		r.x = y[c];
+		r.wx = d.conv[(size_t)(d.taps - 1) * d.channels + c];
+#pragma unroll
+		for (int i = 0; i < CT; i++) {
+			const int at = min(i0 + i, d.taps - 1), from = slot + 1 + at;  // row of position pos - taps + 1 + at
+			r.w[i] = d.conv[(size_t)at * d.channels + c];
+			r.in[i] = d.ring[(size_t)(from >= d.taps ? from - d.taps : from) * d.channels + c];
+		}
+	};
+	auto conv_sum = [&](int c, Conv &r) {
+		float v = 0.0f;
+		for (int i0 = 0; i0 < d.taps - 1; i0 += CT) {
+			if (i0) conv_request(c, i0, r);
+#pragma unroll
+			for (int i = 0; i < CT; i++) v = i0 + i < d.taps - 1 ? fmaf(r.w[i], r.in[i], v) : v;
+		}
+		return tg_silu(fmaf(r.x, r.wx, v));
+	};
+	auto qk_channel = [&](int e) { return (e >= g.dimp ? qc - g.dimp : 0) + kh * g.dimp + e; };
+	const int ns = g.dimp >= 256 ? 1 : 256 / g.dimp, per = (g.rank + ns - 1) / ns;  // the rank split over the lanes that the channels leave
+	float wa[RA], ya[RA], wg[RG], yg[RG];
+	auto decay_request = [&](int e, int j0) {
+		const int sp = e / g.dimp, c = h * g.dimp + e - sp * g.dimp;
+#pragma unroll
+		for (int j = 0; j < RA; j++) {
+			const int at = min(sp * per + j0 + j, g.rank - 1);
+			wa[j] = g.a2[(size_t)at * hd + c];
+			ya[j] = y[a_off + at];
+		}
+	};
+	const int gp = (d.gate_rank + 7) / 8, glo = (tid >> 5) * gp, cg = h * g.vdimp + c0 + (tid & 31);
+	auto gate_request = [&](int j0) {
+#pragma unroll
+		for (int j = 0; j < RG; j++) {
+			const int at = min(glo + j0 + j, d.gate_rank - 1);
+			wg[j] = d.g2[(size_t)at * hv + cg];
+			yg[j] = y[g_off + at];
+		}
+	};
+	Conv ck, cv;
+	conv_request(qk_channel(min(tid, 2 * g.dimp - 1)), 0, ck);
+	conv_request(ch_v, 0, cv);
+	decay_request(min(tid, ns * g.dimp - 1), 0);
+	gate_request(0);
+	const float rate = expf(g.a_log[h]);
+
+	const bool keep_qk = h % g.group == 0 && blockIdx.y == 0;  // the workgroup that keeps the newest input of these channels
 	for (int e = tid; e < 2 * g.dimp; e += 256) {
-		const bool k = e >= g.dimp;
-		const int c = k ? e - g.dimp : e;
-		(k ? s_k : s_q)[c] = conv((k ? qc : 0) + kh * g.dimp + c, keep_qk);
+		if (e != tid) conv_request(qk_channel(e), 0, ck);
+		const float v = conv_sum(qk_channel(e), ck);
+		(e >= g.dimp ? s_k[e - g.dimp] : s_q[e]) = v;
+		if (keep_qk) d.ring[(size_t)slot * d.channels + qk_channel(e)] = ck.x;
 	}
-	if (tid >= 224) s_v[tid - 224] = conv(2 * qc + h * g.vdimp + c0 + tid - 224, true);
-	// the decay's low-rank product, its rank split over the lanes that the channels leave
-	const int ns = g.dimp >= 256 ? 1 : 256 / g.dimp, per = (g.rank + ns - 1) / ns;
+	{
+		const float v = conv_sum(ch_v, cv);
+		if (tid < 32) {
+			s_v[tid] = v;
+			d.ring[(size_t)slot * d.channels + ch_v] = cv.x;
+		}
+	}
 	for (int e = tid; e < ns * g.dimp; e += 256) {
-		const int sp = e / g.dimp, c = h * g.dimp + e - sp * g.dimp, hi = min(g.rank, (sp + 1) * per);
+		const int lo = e / g.dimp * per, cnt = min(g.rank - lo, per);
 		float z = 0.0f;
-		for (int j0 = sp * per; j0 < hi; j0 += 16) {
-			float wa[16], ya[16];
+		for (int j0 = 0; j0 < cnt; j0 += RA) {
+			if (e != tid || j0) decay_request(e, j0);
 #pragma unroll
-			for (int j = 0; j < 16; j++) {
-				wa[j] = g.a2[(size_t)min(j0 + j, g.rank - 1) * hd + c];
-				ya[j] = y[a_off + min(j0 + j, g.rank - 1)];
-			}
-#pragma unroll
-			for (int j = 0; j < 16; j++) z = j0 + j < hi ? fmaf(wa[j], ya[j], z) : z;
+			for (int j = 0; j < RA; j++) z = j0 + j < cnt ? fmaf(wa[j], ya[j], z) : z;
 		}
 		s_z[e] = z;
 	}
 	{
-		const int c = h * g.vdimp + c0 + (tid & 31), gp = (d.gate_rank + 7) / 8, lo = (tid >> 5) * gp, hi = min(d.gate_rank, lo + gp);
+		const int cnt = min(d.gate_rank - glo, gp);
 		float z = 0.0f;
-		for (int j0 = lo; j0 < hi; j0 += 8) {
-			float wa[8], ya[8];
+		for (int j0 = 0; j0 < cnt; j0 += RG) {
+			if (j0) gate_request(j0);
 #pragma unroll
-			for (int j = 0; j < 8; j++) {
-				wa[j] = d.g2[(size_t)min(j0 + j, d.gate_rank - 1) * hv + c];
-				ya[j] = y[g_off + min(j0 + j, d.gate_rank - 1)];
-			}
-#pragma unroll
-			for (int j = 0; j < 8; j++) z = j0 + j < hi ? fmaf(wa[j], ya[j], z) : z;
+			for (int j = 0; j < RG; j++) z = j0 + j < cnt ? fmaf(wg[j], yg[j], z) : z;
 		}
 		s_g[tid >> 5][tid & 31] = z;
 	}
 	__syncthreads();
 	float sq = 0.0f, sk = 0.0f, skq = 0.0f;
-	const float rate = expf(g.a_log[h]);
 	for (int c = tid; c < g.dimp; c += 256) {
 		const float q = s_q[c], k = s_k[c];
 		sq = fmaf(q, q, sq);
@@ -838,19 +904,21 @@ void launch_delta_rows(const TgDelta &d, const void *xv, int ld, const float *lo
 	const TgGla &g = d.g;
 	const int qc = d.q_channels(), hv = g.heads * g.vdimp, hd = g.heads * g.dimp, kvh = g.heads / g.group;
 	const unsigned chunks = (unsigned)((n + C - 1) / C);
-	hipLaunchKernelGGL((delta_prep_kernel<TR>), dim3((unsigned)((n + 3) / 4), (unsigned)(2 * kvh + (hv + 255) / 256)), dim3(256), 0, s, d, x, ld, n, past,
+	hipLaunchKernelGGL((delta_prep_kernel<TR>), dim3((unsigned)((n + 4 * PT - 1) / (4 * PT)), (unsigned)(2 * kvh + (hv + 255) / 256)), dim3(256), 0, s, d, x, ld, n, past,
 	                   t.qk, t.u);
 	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (unsigned)((hd + 63) / 64)), dim3(256), 0, s, low + a_off, ld_low, g, n, t.b);
 	hipLaunchKernelGGL((gla_intra_kernel<TgF32, true>), dim3(chunks, (unsigned)g.heads), dim3(256), 0, s, t.qk, 2 * qc, qc, g, n, t.b, t.a,
-	                   DeltaIntra{low + b_off, ld_low, t.u, t.wk, t.kt});
+	                   DeltaIntra{low + b_off, ld_low, t.t});
+	const DeltaSolve solve = {t.qk, t.b, t.t, low + b_off, 2 * qc, qc, ld_low, t.u, t.wk, t.kt};
+	hipLaunchKernelGGL(delta_solve_kernel, dim3(chunks, (unsigned)g.heads, (unsigned)((g.dimp + g.vdimp + 127) / 128)), dim3(256), 0, s, solve, g, n);
 	const dim3 grid((unsigned)g.heads, (unsigned)(g.vdimp / 16));
 	auto scan = [&](auto *kernel) {
 		hipLaunchKernelGGL(kernel, grid, dim3(256), 0, s, d, x, ld, n, past, (const float *)t.b, t.u, (const float *)t.wk, (const float *)t.kt, t.st,
 		                   (int)chunks);
 	};
-	if (g.dimp <= 64) scan(delta_scan_kernel<TR, 1>);
-	else if (g.dimp <= 128) scan(delta_scan_kernel<TR, 2>);
-	else scan(delta_scan_kernel<TR, 4>);
+	if (g.dimp <= 64) scan(delta_scan_kernel<TR, 1, 3>);
+	else if (g.dimp <= 128) scan(delta_scan_kernel<TR, 2, 3>);
+	else scan(delta_scan_kernel<TR, 4, 2>);
 	launch_out<TgF32, TR, true>(g, OutIn{t.qk, t.u, gate, 2 * qc, hv, ldg}, n, t.b, t.a, t.st, out, ld_out, s);
 }
 
@@ -903,6 +971,7 @@ size_t tg_delta_scratch(const TgDelta &d, int n, TgDeltaScratch *t, unsigned cha
 	if (!t) t = &tmp;
 	take(&t->b, chunks * C * hd);
 	take(&t->a, chunks * g.heads * C * C);
+	take(&t->t, chunks * g.heads * C * C);
 	take(&t->qk, (size_t)n * 2 * d.q_channels());
 	take(&t->u, chunks * C * hv);
 	take(&t->wk, chunks * C * hd);

@@ -20,7 +20,7 @@
 #define TG_LATENT_MAX_BLOCKS 128   // key parts per launch
 #define TG_LATENT_TILE 32
 #define TG_LATENT_LDS_MAX (150 * 1024)
-#define TG_LATENT_HEAD_MAX 256     // largest padded head size of the tiled kernel
+#define TG_LATENT_HEAD_MAX 256     // largest padded head size of the tiled kernel, and rotated part of a row
 
 // Rotary positions: dims / 2 pairs of a vector, (2i, 2i + 1) or (i, i + dims / 2); elements behind them pass unchanged.
 struct TgRot {

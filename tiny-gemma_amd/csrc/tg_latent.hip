@@ -11,7 +11,8 @@ namespace {
 // a product of the probabilities [16 heads x 32 keys] (in the bf16 format two planes, value and remainder) with the tile,
 // wave w the column tiles w, w + 4, ..., in passes of 512 columns (blockIdx.z).
 constexpr int ST = 32;         // keys per tile
-constexpr int ST_LOADS = 8;    // 16-byte pieces per lane and round of the tile copy
+template <bool ROT>
+constexpr int ST_LOADS = ROT ? 10 : 8;  // 16-byte pieces per lane and round of the tile copy
 
 template <class TR>
 size_t latent_step_lds(int rowp) {  // q' fragments | tile
@@ -19,25 +20,35 @@ size_t latent_step_lds(int rowp) {  // q' fragments | tile
 	return 16 * row + ST * (row + 16);
 }
 
-// Element i of a rotated vector x.
+// Element i of a rotated vector: itself, turned with its partner.
+struct Turn {
+	int other, pair;
+	bool turns, second;
+	__device__ __forceinline__ Turn(int i, int dims, int half_layout) {
+		const int hd = dims / 2;
+		turns = i < dims;
+		second = half_layout ? i >= hd : (i & 1) != 0;
+		pair = !turns ? 0 : (half_layout ? (second ? i - hd : i) : i >> 1);
+		other = !turns ? i : (half_layout ? (second ? i - hd : i + hd) : i ^ 1);
+	}
+	__device__ __forceinline__ float operator()(float v, float o, float2 t) const {
+		return turns ? fmaf(v, t.x, second ? o * t.y : -(o * t.y)) : v;
+	}
+};
 template <class V>
 __device__ __forceinline__ float rotated(const V *x, int i, const float2 *turn, int dims, int half_layout) {
-	if (i >= dims) return (float)x[i];
-	const int hd = dims / 2;
-	const int pair = half_layout ? (i < hd ? i : i - hd) : i >> 1;
-	const bool second = half_layout ? i >= hd : (i & 1) != 0;
-	const int other = half_layout ? (second ? i - hd : i + hd) : i ^ 1;
-	const float2 t = turn[pair];
-	const float v = (float)x[i], o = (float)x[other];
-	return second ? fmaf(v, t.x, o * t.y) : fmaf(v, t.x, -(o * t.y));
+	const Turn r(i, dims, half_layout);
+	return r((float)x[i], (float)x[r.other], turn[r.pair]);
 }
+// e / d for e * d < 2^22, m = 2^22 / d rounded up
+__device__ __forceinline__ int div_by(int e, unsigned m) { return (int)(((unsigned)e * m) >> 22); }
 
-template <class TR>
+template <class TR, bool ROT>
 __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
 	extern __shared__ __align__(16) unsigned char smem[];
-	const int rowp = a.rankp + a.rotp, row = rowp * (int)sizeof(T), pitch = row + 16, ppr = row / 16;  // bytes; 16-byte pieces per row
+	const int rowp = a.rankp + (ROT ? a.rotp : 0), row = rowp * (int)sizeof(T), pitch = row + 16, ppr = row / 16;  // bytes; 16-byte pieces per row
 	Frag *s_q = reinterpret_cast<Frag *>(smem);  // [rowp / KF][64]
 	unsigned char *s_c = smem + 16 * row;
 	__shared__ float s_half[2][ST][16];
@@ -50,21 +61,23 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	const int kb = lo + part * a.chunk, ke = min(ctx, kb + a.chunk);
 	const size_t key_bytes = (size_t)a.groups * row;
 	unsigned char *cache = (unsigned char *)a.cache + (size_t)grp * row;
-	const float2 *turn = a.rot.table + (size_t)pos * (a.rot.dims / 2);
+	const float2 *turn = ROT ? a.rot.table + (size_t)pos * (a.rot.dims / 2) : nullptr;
+	constexpr int SL = ST_LOADS<ROT>;
+	const unsigned mppr = ((1u << 22) + (unsigned)ppr - 1) / (unsigned)ppr;  // (32 ppr^2 < 2^22: rows below 5 KiB)
 	typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
-	u32x4 piece[ST_LOADS];
-	// pieces [base, base + 256 * ST_LOADS) of a tile; the new token's row is not in memory yet: it is written to LDS below
+	u32x4 piece[SL];
+	// pieces [base, base + 256 * SL) of a tile; the new token's row is not in memory yet: it is written to LDS below
 	auto request = [&](int k0, int base) {
 #pragma unroll
-		for (int i = 0; i < ST_LOADS; i++) {
-			const int e = min(base + tid + 256 * i, ST * ppr - 1), r = e / ppr, key = max(min(min(k0 + r, ke - 1), pos - 1), 0);
+		for (int i = 0; i < SL; i++) {
+			const int e = min(base + tid + 256 * i, ST * ppr - 1), r = div_by(e, mppr), key = max(min(min(k0 + r, ke - 1), pos - 1), 0);
 			piece[i] = *reinterpret_cast<const u32x4 *>(cache + (size_t)key * key_bytes + (e - r * ppr) * 16);
 		}
 	};
 	auto place = [&](int base) {
 #pragma unroll
-		for (int i = 0; i < ST_LOADS; i++) {
-			const int e = base + tid + 256 * i, r = e / ppr;
+		for (int i = 0; i < SL; i++) {
+			const int e = base + tid + 256 * i, r = div_by(e, mppr);
 			if (e < ST * ppr) *reinterpret_cast<u32x4 *>(s_c + (size_t)r * pitch + (e - r * ppr) * 16) = piece[i];
 		}
 	};
@@ -77,36 +90,72 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		raw[i] = kv[j];
 		nrm[i] = a.norm ? a.norm[j] : 1.0f;
 	}
+	// rotated parts: of the queries (16 * rotp elements, RB of them per lane and pass) and of the new row
+	constexpr int RB = 4;
+	float rx[RB], ro[RB], kx = 0.0f, ko = 0.0f;
+	float2 rt[RB], kt = {0.0f, 0.0f};
+	unsigned mrot = 0;
+	auto rot_request = [&](int base) {
+#pragma unroll
+		for (int i = 0; i < RB; i++) {
+			const int e = min(base + tid + 256 * i, 16 * a.rotp - 1), h = div_by(e, mrot), j = min(e - h * a.rotp, a.rot_size - 1);
+			const Turn r(j, a.rot.dims, a.rot.half_layout);
+			const float *x = a.qr + (size_t)(g0 + min(h0 + h, a.heads - 1)) * a.qr_stride;
+			rx[i] = x[j];
+			ro[i] = x[r.other];
+			rt[i] = turn[r.pair];
+		}
+	};
+	auto rot_place = [&](int base) {
+#pragma unroll
+		for (int i = 0; i < RB; i++) {
+			const int e = base + tid + 256 * i, h = div_by(min(e, 16 * a.rotp - 1), mrot), j = e - h * a.rotp, c = a.rankp + j;
+			const Turn r(j, a.rot.dims, a.rot.half_layout);
+			const float v = j < a.rot_size && h0 + h < a.heads ? r(rx[i], ro[i], rt[i]) : 0.0f;
+			if (e < 16 * a.rotp)
+				reinterpret_cast<T *>(s_q)[((size_t)(c / TR::KF) * 64 + h + 16 * ((c % TR::KF) / TR::KV)) * TR::KV + c % TR::KV] = (T)v;
+		}
+	};
+	if constexpr (ROT) {
+		mrot = ((1u << 22) + (unsigned)a.rotp - 1) / (unsigned)a.rotp;
+		const int j = min(tid, a.rot_size - 1);
+		const Turn r(j, a.rot.dims, a.rot.half_layout);
+		const float *x = a.kr + (size_t)grp * a.kr_stride;
+		kx = x[j];
+		ko = x[r.other];
+		kt = turn[r.pair];
+		rot_request(0);
+	}
 	request(kb, 0);
 
-	// q' in operand order: lane = head, 16 bytes of the latent
-	const int q4 = rowp / 4, r4 = a.rankp / 4;
-	for (int base = 0; base < 16 * q4; base += 256 * 8) {
+	// q' in operand order: lane = head, 16 bytes of the row
+	const int r4 = a.rankp / 4;
+	const unsigned mr4 = ((1u << 22) + (unsigned)r4 - 1) / (unsigned)r4;
+	for (int base = 0; base < 16 * r4; base += 256 * 8) {
 		f32x4_t v[8];
 #pragma unroll
 		for (int i = 0; i < 8; i++) {
-			const int e = min(base + tid + 256 * i, 16 * q4 - 1), h = e / q4, j4 = e - h * q4;
-			const size_t hq = (size_t)(g0 + min(h0 + h, a.heads - 1));
-			v[i] = j4 < r4 ? tg_load4(a.q + hq * a.q_stride + j4 * 4) : f32x4_t{0, 0, 0, 0};
-			if (j4 < r4) {
-#pragma unroll
-				for (int c = 0; c < 4; c++)
-					if (j4 * 4 + c < a.q_zero) v[i][c] = 0.0f;
-			} else {
-				const float *x = a.qr + hq * a.qr_stride;
-#pragma unroll
-				for (int c = 0; c < 4; c++) {
-					const int j = (j4 - r4) * 4 + c;
-					if (j < a.rot_size) v[i][c] = rotated(x, j, turn, a.rot.dims, a.rot.half_layout);
-				}
-			}
+			const int e = min(base + tid + 256 * i, 16 * r4 - 1), h = div_by(e, mr4);
+			v[i] = tg_load4(a.q + (size_t)(g0 + min(h0 + h, a.heads - 1)) * a.q_stride + (e - h * r4) * 4);
 		}
 #pragma unroll
 		for (int i = 0; i < 8; i++) {
-			const int e = base + tid + 256 * i, h = e / q4, j = (e - h * q4) * 4;
+			const int e = base + tid + 256 * i, h = div_by(min(e, 16 * r4 - 1), mr4), j = (e - h * r4) * 4;
 			if (h0 + h >= a.heads) v[i] = f32x4_t{0, 0, 0, 0};
-			if (e < 16 * q4)
+			if constexpr (ROT) {
+#pragma unroll
+				for (int c = 0; c < 4; c++)
+					if (j + c < a.q_zero) v[i][c] = 0.0f;
+			}
+			if (e < 16 * r4)
 				tg_store4(reinterpret_cast<T *>(s_q) + ((size_t)(j / TR::KF) * 64 + h + 16 * ((j % TR::KF) / TR::KV)) * TR::KV + j % TR::KV, v[i]);
+		}
+	}
+	if constexpr (ROT) {
+		rot_place(0);
+		for (int base = 256 * RB; base < 16 * a.rotp; base += 256 * RB) {
+			rot_request(base);
+			rot_place(base);
 		}
 	}
 	// the new token's latent, normalised, by the workgroups whose part it ends
@@ -133,7 +182,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	for (int i = 0; i < 2; i++) { m[i] = -INFINITY; l[i] = 0.0f; }
 	const int kfr = rowp / TR::KF, kh = (kfr + 1) / 2, kf_lo = (w >> 1) * kh, kf_hi = min(kfr, kf_lo + kh);
 	for (int k0 = kb; k0 < ke; k0 += ST) {
-		for (int base = 0; base < ST * ppr; base += 256 * ST_LOADS) {
+		for (int base = 0; base < ST * ppr; base += 256 * SL) {
 			if (base) request(k0, base);
 			place(base);
 		}
@@ -147,11 +196,13 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 				tile[j] = c;
 				dst[j] = c;
 			}
-			const float *kr = a.kr + (size_t)grp * a.kr_stride;
-			for (int j = tid; j < a.rotp; j += 256) {
-				const T c = (T)(j < a.rot_size ? rotated(kr, j, turn, a.rot.dims, a.rot.half_layout) : 0.0f);
-				tile[a.rankp + j] = c;
-				dst[a.rankp + j] = c;
+			if constexpr (ROT) {
+				if (tid < a.rotp) {  // (rotp is at most 256)
+					const Turn r(tid, a.rot.dims, a.rot.half_layout);
+					const T c = (T)(tid < a.rot_size ? r(kx, ko, kt) : 0.0f);
+					tile[a.rankp + tid] = c;
+					dst[a.rankp + tid] = c;
+				}
 			}
 			__syncthreads();
 		}
@@ -357,7 +408,8 @@ __global__ __launch_bounds__(256) void key_values_kernel(TgKeyValues a) {
 // enter it as two bf16 planes (value and remainder).
 // Sizes are compile-time buckets (DM >= dimp, VM >= vdimp): query elements past the head are zero, value rows past it are
 // computed from repeated rows and not stored, so that no branch stands between the LDS reads and matrix instructions.
-template <class TR, int DM, int VM, int KT, int QT>
+// WIDE: with a window, a rotated part or grouped heads.
+template <class TR, int DM, int VM, int KT, int QT, bool WIDE>
 __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
@@ -369,8 +421,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	// Query tiles from both ends: the first half of the launch takes the long rows, longest first, the second half the
 	// short ones, shortest first, so that the workgroups that meet on a compute unit have about the same work together.
 	const int nqt = (int)gridDim.y, y = (int)blockIdx.y, half = (nqt + 1) / 2;
-	const int h = blockIdx.x, kh = h / a.group, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
-	const int kn = a.dimp / TR::KF, kd = (a.dimp + a.rotp) / TR::KF, nv = a.vdimp / 16;
+	const int h = blockIdx.x, kh = WIDE ? h / a.group : h, qb = (y < half ? nqt - 1 - y : y - half) * 64 * QT;
+	const int kn = a.dimp / TR::KF, kd = (a.dimp + (WIDE ? a.rotp : 0)) / TR::KF, nv = a.vdimp / 16;
 	const T *Q = (const T *)a.q, *K = (const T *)a.k + (size_t)kh * a.dimp, *V = (const T *)a.vt + (size_t)kh * a.vdimp * a.ldv;
 	const T *R = (const T *)a.kr;
 	const float sl2 = fabsf(a.scale) * 1.44269504088896340736f;  // (the sign goes to the queries: maxima are taken before scaling)
@@ -381,7 +433,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 #pragma unroll
 	for (int s = 0; s < QT; s++) {
 		qi[s] = qb + w * 16 * QT + s * 16 + lr;
-		const T *row = Q + (size_t)min(qi[s], a.n - 1) * a.ldq + (size_t)h * (a.dimp + a.rotp) + lg * TR::KV;
+		const T *row = Q + (size_t)min(qi[s], a.n - 1) * a.ldq + (size_t)h * (a.dimp + (WIDE ? a.rotp : 0)) + lg * TR::KV;
 #pragma unroll
 		for (int d = 0; d < ND; d++) {
 			qf[s][d] = *reinterpret_cast<const Frag *>(row + (d < kd ? d : 0) * TR::KF);
@@ -399,7 +451,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 		for (int v = 0; v < NV; v++) o[s][v] = f32x4_t{0, 0, 0, 0};
 	}
 	const int last = a.past + min(qb + 64 * QT, a.n) - 1;  // the last key any of these queries sees
-	const int nt = last / KT + 1, ctx = a.past + a.n, tb = max(a.past + qb - a.window + 1, 0) / KT;
+	const int nt = last / KT + 1, ctx = a.past + a.n, tb = WIDE ? max(a.past + qb - a.window + 1, 0) / KT : 0;
 	Frag st[PW];
 	auto fetch = [&](int k0) {
 #pragma unroll
@@ -409,7 +461,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 			if (f < KFRAGS) {
 				const int kt = f / ND, d = f % ND;
 				const size_t key = (size_t)min(k0 + kt * 16 + lr, ctx - 1);
-				p = (d < kn || d >= kd ? K + key * a.ldk + (d < kn ? d : 0) * TR::KF : R + key * a.ldkr + (d - kn) * TR::KF) + lg * TR::KV;
+				if constexpr (!WIDE) p = K + key * a.ldk + (d < kd ? d : 0) * TR::KF + lg * TR::KV;
+				else p = (d < kn || d >= kd ? K + key * a.ldk + (d < kn ? d : 0) * TR::KF : R + key * a.ldkr + (d - kn) * TR::KF) + lg * TR::KV;
 			} else {
 				const int v = (f - KFRAGS) / NB, b = (f - KFRAGS) % NB;
 				p = V + (size_t)((v < nv ? v : 0) * 16 + lr) * a.ldv + k0 + b * TR::KF + lg * TR::KV;
@@ -442,15 +495,15 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 		// keys past a query only in the tiles that reach the wave's first query, keys before its window in those that do not
 		// reach the last query's
 		const int first_q = a.past + qb + w * 16 * QT;
-		const bool masked = k0 + KT - 1 > first_q || k0 < first_q + 16 * QT - a.window;
+		const bool masked = k0 + KT - 1 > first_q || (WIDE && k0 < first_q + 16 * QT - a.window);
 #pragma unroll
 		for (int s = 0; s < QT; s++) {
 			if (masked) {
-				const int lim = a.past + qi[s] - k0 - 4 * lg, low = lim - a.window;
+				const int lim = a.past + qi[s] - k0 - 4 * lg, low = WIDE ? lim - a.window : -TG_NO_WINDOW;
 #pragma unroll
 				for (int kt = 0; kt < NK; kt++)
 #pragma unroll
-					for (int e = 0; e < 4; e++) sc[s][kt][e] = kt * 16 + e <= lim && kt * 16 + e > low ? sc[s][kt][e] : -INFINITY;
+					for (int e = 0; e < 4; e++) sc[s][kt][e] = kt * 16 + e <= lim && (!WIDE || kt * 16 + e > low) ? sc[s][kt][e] : -INFINITY;
 			}
 			float mt = -INFINITY;
 #pragma unroll
@@ -532,16 +585,21 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(TgLatentRows a) {
 	}
 }
 
-template <class TR, int DM, int VM, int KT>
-void launch_bucket(const TgLatentRows &a, hipStream_t s) {
+template <class TR, int DM, int VM, int KT, bool WIDE>
+void launch_bucket_w(const TgLatentRows &a, hipStream_t s) {
 	// 128-query tiles (half the LDS reads per product) where they fill the device twice
 	if constexpr (TR::DT == TG_DT_BF16 && DM <= 128 && VM <= 128) {
 		if (a.heads * ((a.n + 127) / 128) >= 512) {
-			hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 2>), dim3((unsigned)a.heads, (unsigned)((a.n + 127) / 128)), dim3(256), 0, s, a);
+			hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 2, WIDE>), dim3((unsigned)a.heads, (unsigned)((a.n + 127) / 128)), dim3(256), 0, s, a);
 			return;
 		}
 	}
-	hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 1>), dim3((unsigned)a.heads, (unsigned)((a.n + 63) / 64)), dim3(256), 0, s, a);
+	hipLaunchKernelGGL((latent_attn_kernel<TR, DM, VM, KT, 1, WIDE>), dim3((unsigned)a.heads, (unsigned)((a.n + 63) / 64)), dim3(256), 0, s, a);
+}
+template <class TR, int DM, int VM, int KT>
+void launch_bucket(const TgLatentRows &a, hipStream_t s) {
+	if (a.rotp || a.group > 1 || a.window < TG_NO_WINDOW) launch_bucket_w<TR, DM, VM, KT, true>(a, s);
+	else launch_bucket_w<TR, DM, VM, KT, false>(a, s);
 }
 
 template <class TR>
@@ -563,8 +621,12 @@ template <class TR>
 void launch_step(const TgLatentStep &a, hipStream_t s) {
 	const dim3 grid((unsigned)a.nb, (unsigned)(a.groups * ((a.heads + 15) / 16)), (unsigned)((a.rankp + 511) / 512));
 	const size_t lds = latent_step_lds<TR>(a.rowp());
-	if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void *)latent_step_kernel<TR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-	hipLaunchKernelGGL((latent_step_kernel<TR>), grid, dim3(256), lds, s, a);
+	auto go = [&](auto *kernel) {
+		if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+		hipLaunchKernelGGL(kernel, grid, dim3(256), lds, s, a);
+	};
+	if (a.rotp) go(latent_step_kernel<TR, true>);
+	else go(latent_step_kernel<TR, false>);
 }
 }  // namespace
 

@@ -87,13 +87,15 @@ void tg_launch_unpack_f32(float *dst, int ld, const TgPack &p, hipStream_t s);
 // y = W x for one vector, or for `nz` of them at once (head blocks, experts).  A workgroup owns one tile of 16 outputs (two
 // for the gate|up pair) over its part of K, or, where there are thousands of tiles, four of them.  The vector is prepared by
 // every workgroup in a prologue and held in LDS.
-#define TG_VEC_MERGE_MAX 16  // attention partials a prologue merges
+#define TG_VEC_MERGE_MAX 16        // attention partials a prologue merges
+#define TG_VEC_MERGE_HEADS_MAX 64  // heads that TG_VP_MERGE_HEADS serves
 enum {
 	TG_VP_PLAIN = 0,   // x[z]
 	TG_VP_DYT,         // residual sum, then the element-wise tanh norm
 	TG_VP_RMS,         // residual sum (its addend normed first where there is a weight for it), then the root mean square norm
 	TG_VP_HEADNORM,    // heads normalised by their root mean square, times silu(gate) or sigmoid(gate)
 	TG_VP_MERGE,       // merged attention partials of head z
+	TG_VP_MERGE_HEADS, // the same of all heads, side by side (vdimp elements each): groups of `group` heads, each padded to 16
 	TG_VP_EXPERT       // x, for the z-th of the experts that the router's logits select
 };
 enum {
@@ -130,7 +132,7 @@ struct TgVec {
 	int vdim, vdimp;           // HEADNORM: head size and its padded size
 	float eps;
 	const float *part_acc, *part_ml;  // MERGE: [nmerge][heads padded to 16][x_zstride], [nmerge][heads padded to 16][2]
-	int nmerge, heads16;
+	int nmerge, heads16, group, heads;  // MERGE_HEADS: heads per group, real heads; heads16 counts the padded heads of all groups
 	const float *logits, *correction;  // EXPERT
 	int experts, top;
 	float rscale;

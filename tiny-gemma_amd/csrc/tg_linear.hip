@@ -342,6 +342,47 @@ __global__ __launch_bounds__(NT) void vec_kernel(TgVec p) {
 		if (first) load(kf0);
 		for (int j = tid; j < kn; j += NT)
 			if ((k0 + j) / p.vdimp >= p.heads16) xs[j] = (T)0.0f;
+	} else if constexpr (PRO == TG_VP_MERGE_HEADS) {
+		// a row of 16 lanes per head: the factors of its partials; then element by element
+		__shared__ float s_f[TG_VEC_MERGE_HEADS_MAX][TG_VEC_MERGE_MAX];
+		const int g16 = (p.group + 15) / 16 * 16, bl = min(lane & 15, p.nmerge - 1);
+		auto padded = [&](int h) { const int g = h / p.group; return g * g16 + h - g * p.group; };
+		const int h_lo = min(k0 / p.vdimp, p.heads - 1), h_hi = min((k0 + max(kn, 1) - 1) / p.vdimp, p.heads - 1);
+		auto column = [&](int j) {
+			const int k = k0 + j, h = min(k / p.vdimp, p.heads - 1);
+			return p.part_acc + (size_t)padded(h) * p.x_zstride + min(k - h * p.vdimp, p.vdimp - 1);
+		};
+		const size_t step_b = (size_t)p.heads16 * p.x_zstride;
+		const int ha = min(h_lo + 4 * w + (lane >> 4), h_hi);
+		float2 ml = *reinterpret_cast<const float2 *>(p.part_ml + ((size_t)bl * p.heads16 + padded(ha)) * 2);
+		float a[TG_VEC_MERGE_MAX];
+		const float *pa = column(min(tid, max(kn - 1, 0)));
+#pragma unroll
+		for (int b = 0; b < TG_VEC_MERGE_MAX; b++) a[b] = pa[(size_t)min(b, p.nmerge - 1) * step_b];
+		load(kf0);
+		const bool in = (lane & 15) < p.nmerge;
+		for (int hb = h_lo; hb <= h_hi; hb += 16) {
+			const int h = min(hb + 4 * w + (lane >> 4), h_hi);
+			if (hb != h_lo) ml = *reinterpret_cast<const float2 *>(p.part_ml + ((size_t)bl * p.heads16 + padded(h)) * 2);
+			const float m = tg_row16_max(in ? ml.x : -INFINITY);
+			const float f = in ? expf(ml.x - m) : 0.0f;
+			const float inv = 1.0f / tg_row16_sum(f * ml.y);
+			s_f[h - h_lo][lane & 15] = f * inv;
+		}
+		__syncthreads();
+		for (int j = tid; j < kn; j += NT) {
+			const int h = (k0 + j) / p.vdimp;
+			if (j != tid) {
+				pa = column(j);
+#pragma unroll
+				for (int b = 0; b < TG_VEC_MERGE_MAX; b++) a[b] = pa[(size_t)min(b, p.nmerge - 1) * step_b];
+			}
+			float r = 0.0f;
+			if (h < p.heads)
+#pragma unroll
+				for (int b = 0; b < TG_VEC_MERGE_MAX; b++) r = fmaf(s_f[h - h_lo][b], a[b], r);
+			xs[j] = (T)r;
+		}
 	} else {  // MERGE: at most 16 partials
 		const int bl = min(lane & 15, p.nmerge - 1);
 		const float2 ml = *reinterpret_cast<const float2 *>(p.part_ml + ((size_t)bl * p.heads16 + z) * 2);
@@ -514,6 +555,7 @@ void launch_vec_dt(const TgVec &v, int pro, int epi, hipStream_t s) {
 	else if (pro == TG_VP_RMS && epi == TG_VE_GELU) launch_vec_t<TR, TG_VP_RMS, TG_VE_GELU>(v, s);
 	else if (pro == TG_VP_RMS && epi == TG_VE_LOGITS) launch_vec_t<TR, TG_VP_RMS, TG_VE_LOGITS>(v, s);
 	else if (pro == TG_VP_MERGE && epi == TG_VE_STORE) launch_vec_t<TR, TG_VP_MERGE, TG_VE_STORE>(v, s);
+	else if (pro == TG_VP_MERGE_HEADS) launch_vec_t<TR, TG_VP_MERGE_HEADS, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_HEADNORM) launch_vec_t<TR, TG_VP_HEADNORM, TG_VE_STORE>(v, s);
 	else if (pro == TG_VP_MERGE) launch_vec_t<TR, TG_VP_MERGE, TG_VE_GATE>(v, s);
 	else if (pro == TG_VP_EXPERT) launch_vec_t<TR, TG_VP_EXPERT, TG_VE_SWIGLU>(v, s);

@@ -735,9 +735,12 @@ void latent_parts(int ctx, int *chunk, int *nb) {
 	}
 	*nb = (ctx + *chunk - 1) / *chunk;
 }
-// The same where the parts always meet in a launch of their own: up to 32 parts per group.
-void group_parts(int ctx, int *chunk, int *nb) {
-	*chunk = tg_up(std::max((ctx + 31) / 32, 1), TG_LATENT_TILE);
+// Grouped rows: as many parts as the output product merges in its prologue, of two tiles at most; more keys go to more parts that
+// meet in a launch of their own.
+void group_parts(int ctx, int heads, int *chunk, int *nb) {
+	const bool merge = ctx <= 2 * TG_LATENT_TILE * TG_VEC_MERGE_MAX && heads <= TG_VEC_MERGE_HEADS_MAX;
+	const int parts = merge ? TG_VEC_MERGE_MAX : 64;
+	*chunk = tg_up(std::max((ctx + parts - 1) / parts, 1), TG_LATENT_TILE);
 	*nb = (ctx + *chunk - 1) / *chunk;
 }
 
@@ -795,7 +798,7 @@ void tg_net_step_cost(const TgNet *n, double *bytes, int *launches) {
 		const TgNetLayerCfg &c = n->cfg.layers[(size_t)l];
 		const LayerW &w = n->lw(l);
 		b += (double)w.in.n * w.in.k + (double)w.out.n * w.out.k;
-		k += c.mix.kind == TG_MIX_ATTN ? 4 : 3;
+		k += 3;
 		if (c.mix.kind == TG_MIX_LATENT) {
 			b += (double)w.uk_t.n * w.uk_t.k + (double)w.uv.n * w.uv.k + (double)w.uq.n * w.uq.k;
 			k += c.mix.q_rank ? 3 : 2;
@@ -1075,7 +1078,7 @@ struct Step {
 		tg_launch_vec(b, dt, TG_VP_MERGE, gate ? TG_VE_GATE : TG_VE_STORE, s);
 		tg_launch_vec(o, dt, TG_VP_PLAIN, TG_VE_STORE, s);
 	}
-	void attention(int l, int r, const TgVec &o) {
+	void attention(int l, int r, TgVec o) {
 		const TgMixerCfg &m = c.layers[(size_t)l].mix;
 		const int dp = m.dimp();
 		const float *k = q->yin + m.heads * dp;
@@ -1089,8 +1092,19 @@ struct Step {
 		t.q_stride = t.qr_stride = dp;
 		t.kv = t.kr = k;
 		t.kv_stride = t.kr_stride = dp;
-		group_parts(std::min(pos_bound + 1, m.window), &t.chunk, &t.nb);
+		group_parts(std::min(pos_bound + 1, m.window), m.heads, &t.chunk, &t.nb);
 		tg_launch_latent_step(t, dt, s);
+		if (t.nb <= TG_VEC_MERGE_MAX && m.heads <= TG_VEC_MERGE_HEADS_MAX) {
+			o.part_acc = q->acc;
+			o.part_ml = q->ml;
+			o.nmerge = t.nb;
+			o.heads16 = t.groups * tg_up(t.heads, 16);
+			o.group = t.heads;
+			o.heads = m.heads;
+			o.vdimp = o.x_zstride = dp;
+			tg_launch_vec(o, dt, TG_VP_MERGE_HEADS, TG_VE_STORE, s);
+			return;
+		}
 		tg_launch_latent_finish(q->acc, q->ml, t.nb, t.groups, t.heads, dp, q->mix, dp, s);
 		tg_launch_vec(o, dt, TG_VP_PLAIN, TG_VE_STORE, s);
 	}
