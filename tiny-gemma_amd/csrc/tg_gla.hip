@@ -251,6 +251,7 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 struct DeltaSolve {
 	const float *qk, *b, *t, *beta;
 	int ldqk, k_off, ld_beta;
+	const float *v;
 	float *u, *wk, *kt;
 };
 __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g, int n) {
@@ -277,7 +278,7 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g,
 #pragma unroll
 	for (int p = 0; p < 2; p++) {
 		col[p] = (key ? tile : tile - nk) * 16 + 16 * p + lr;
-		const float *src = key ? x.qk + x.k_off + (size_t)kh * g.dimp + col[p] : x.u + (size_t)h * g.vdimp + col[p];
+		const float *src = key ? x.qk + x.k_off + (size_t)kh * g.dimp + col[p] : x.v + (size_t)h * g.vdimp + col[p];
 		const int ld = key ? x.ldqk : hv;
 #pragma unroll
 		for (int i = 0; i < 4; i++)
@@ -327,14 +328,18 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g,
 			for (int p = 0; p < 2; p++) W[p][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(mb[i][e], X[p][i][e], W[p][i], 0, 0, 0);
 	}
 	if (!live) return;
-	const int pitch = key ? hd : hv;
 #pragma unroll
 	for (int p = 0; p < 2; p++) {
-		float *dst = key ? x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col[p] : x.u + (size_t)t0 * hv + (size_t)h * g.vdimp + col[p];
+		float *wk = x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col[p], *u = x.u + (((size_t)ch * g.heads + h) * g.vdimp + col[p]) * C;
 #pragma unroll
-		for (int i = 0; i < 4; i++)
+		for (int i = 0; i < 4; i++) {
+			if (key) {
 #pragma unroll
-			for (int e = 0; e < 4; e++) dst[(size_t)(16 * i + 4 * lg + e) * pitch] = W[p][i][e];
+				for (int e = 0; e < 4; e++) wk[(size_t)(16 * i + 4 * lg + e) * hd] = W[p][i][e];
+			} else {
+				tg_store4(u + 16 * i + 4 * lg, W[p][i]);
+			}
+		}
 	}
 }
 
@@ -426,7 +431,7 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(float *U, const float *b,
 // ---- o = (q e^b)^T S + A v, the head's root mean square norm and silu(gate): 64 tokens x the whole head per workgroup -------------
 // 8 waves: 16 tokens x half of the value columns each.  Slabs of 32: first the key channels (rows q e^b, columns of S), then
 // the chunk's own tokens (rows A, columns v); a slab's loads are in flight during the one before it.
-// (delta rule: the rows of v are u, the gate's function is the sigmoid)
+// (delta rule: v is u, [chunks][heads][vdimp][64], the states are [chunks][heads][vdimp][dimp], the gate's function is the sigmoid)
 struct OutIn {
 	const void *q, *v, *gate;
 	int ldq, ldv, ldg;
@@ -435,8 +440,9 @@ template <class TI, class TR, int VB, bool DELTA>
 __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, const float *b, const float *A, const float *U, typename TR::T *out,
                                                       int ld_out) {
 	const typename TI::T *Q = (const typename TI::T *)in.q + (size_t)(DELTA ? blockIdx.y / g.group : blockIdx.y) * g.dimp,
-	                     *V = (const typename TI::T *)in.v + (size_t)blockIdx.y * g.vdimp;
-	constexpr int XP = 36, YP = VB + 16, NI = VB / 32, NY = 32 * VB / 4 / 512;
+	                     *V = (const typename TI::T *)in.v + (DELTA ? ((size_t)blockIdx.x * g.heads + blockIdx.y) * g.vdimp * C : (size_t)blockIdx.y * g.vdimp);
+	// (delta rule: v and S come transposed and are turned on their way into LDS; the pitch keeps those writes apart)
+	constexpr int XP = 36, YP = VB + (DELTA ? 18 : 16), NI = VB / 32, NY = 32 * VB / 4 / 512;
 	__shared__ __align__(16) float s_x[C][XP], s_y[32][YP];
 	__shared__ float s_sq[2][C];
 	const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, wt = (w & 3) * 16, wv = (w >> 2) * (VB / 2);
@@ -453,7 +459,8 @@ __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, 
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
 				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-				y[i] = tg_load4(S + (size_t)(sl * 32 + r) * g.vdimp + (c4 < g.vdimp ? c4 : 0));
+				if constexpr (DELTA) y[i] = tg_load4(S + (size_t)min(e >> 3, g.vdimp - 1) * g.dimp + sl * 32 + (e & 7) * 4);
+				else y[i] = tg_load4(S + (size_t)(sl * 32 + r) * g.vdimp + (c4 < g.vdimp ? c4 : 0));
 			}
 		} else {
 			const int j0 = (sl - slabs) * 32;
@@ -461,7 +468,8 @@ __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, 
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
 				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-				y[i] = tg_load4(V + (size_t)min(t0 + j0 + r, n - 1) * in.ldv + (c4 < g.vdimp ? c4 : 0));
+				if constexpr (DELTA) y[i] = tg_load4(V + (size_t)min(e >> 3, g.vdimp - 1) * C + j0 + (e & 7) * 4);
+				else y[i] = tg_load4(V + (size_t)min(t0 + j0 + r, n - 1) * in.ldv + (c4 < g.vdimp ? c4 : 0));
 			}
 		}
 	};
@@ -474,7 +482,13 @@ __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, 
 #pragma unroll
 		for (int i = 0; i < NY; i++) {
 			const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-			tg_store4(&s_y[r][c4], c4 < g.vdimp ? y[i] : f32x4_t{0, 0, 0, 0});  // (rows of v past the end meet zeros of A)
+			// (rows of v past the end meet zeros of A)
+			if constexpr (DELTA) {
+#pragma unroll
+				for (int q = 0; q < 4; q++) s_y[(e & 7) * 4 + q][e >> 3] = (e >> 3) < g.vdimp ? y[i][q] : 0.0f;
+			} else {
+				tg_store4(&s_y[r][c4], c4 < g.vdimp ? y[i] : f32x4_t{0, 0, 0, 0});
+			}
 		}
 	};
 	f32x4_t acc[NI];
@@ -561,11 +575,12 @@ void launch_rows(const TgGla &g, const void *qkv, int ld, int k_off, int v_off, 
 // Launches: convolution and unit norms; b; A, T and the solved keys and values, all chunks at once; the pass over the chunks
 // (u and the state in front of each), 16 value columns per workgroup; the outputs, all chunks at once.
 
-// ---- convolution, silu, unit norm: 4 tokens per wave; y: q heads, k heads, blocks of 256 value channels ------------------------------
+// ---- convolution, silu, unit norm: 8 tokens per wave; y: q heads, k heads, blocks of 256 value channels ------------------------------
 // Inputs before the portion come from the ring.
-constexpr int PT = 4;
-template <class TR>
-__global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, float *qk, float *u) {
+// TAPS: the number of taps where it is one of the usual ones (every input row is then read once), else 0.
+constexpr int PT = 8;
+template <class TR, int TAPS>
+__global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, float *qk, float *v_out) {
 	const int t0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * PT, lane = threadIdx.x & 63, kvh = d.g.heads / d.g.group, qc = d.q_channels();
 	if (t0 >= n) return;
 	const bool head = (int)blockIdx.y < 2 * kvh;
@@ -576,7 +591,23 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typena
 	f32x4_t r[PT];
 #pragma unroll
 	for (int p = 0; p < PT; p++) r[p] = f32x4_t{0, 0, 0, 0};
-	for (int i = 0; i < d.taps; i++) {
+	const bool inside = TAPS > 0 && t0 >= TAPS - 1 && t0 + PT <= n;
+	if constexpr (TAPS > 0) {
+		if (inside) {
+			f32x4_t v[PT + TAPS - 1], w[TAPS];
+#pragma unroll
+			for (int i = 0; i < TAPS; i++) w[i] = tg_load4(d.conv + (size_t)i * d.channels + c);
+#pragma unroll
+			for (int i = 0; i < PT + TAPS - 1; i++) v[i] = tg_load4(x + (size_t)(t0 - TAPS + 1 + i) * ld + c);
+#pragma unroll
+			for (int i = 0; i < TAPS; i++)
+#pragma unroll
+				for (int p = 0; p < PT; p++)
+#pragma unroll
+					for (int e = 0; e < 4; e++) r[p][e] = fmaf(w[i][e], v[p + i][e], r[p][e]);
+		}
+	}
+	for (int i = 0; i < (inside ? 0 : d.taps); i++) {
 		const f32x4_t w = tg_load4(d.conv + (size_t)i * d.channels + c);
 #pragma unroll
 		for (int p = 0; p < PT; p++) {
@@ -599,7 +630,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typena
 		if (head) f = 1.0f / sqrtf(tg_wave_sum(in ? ss : 0.0f) + 1e-6f);
 #pragma unroll
 		for (int e = 0; e < 4; e++) r[p][e] *= f;
-		if (in && t0 + p < n) tg_store4(head ? qk + (size_t)(t0 + p) * 2 * qc + c : u + (size_t)(t0 + p) * (d.channels - 2 * qc) + c - 2 * qc, r[p]);
+		if (in && t0 + p < n) tg_store4(head ? qk + (size_t)(t0 + p) * 2 * qc + c : v_out + (size_t)(t0 + p) * (d.channels - 2 * qc) + c - 2 * qc, r[p]);
 	}
 }
 
@@ -607,14 +638,16 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(TgDelta d, const typena
 // Wave w keeps rows 16 (w + 4 i) ... of S in accumulators, which are the second operand of the products with the solved keys as
 // they are; the waves' parts of those products meet in LDS, and u, again in accumulator layout, is the second operand of S's
 // update.  The last inputs of the convolution go to the ring on the way.
-// AHEAD: chunks whose operands are in registers or on their way.
+// AHEAD: chunks whose operands are in registers or on their way.  The chunks are padded to a multiple of it (scratch too), with
+// steps that leave S as it is: a branch around a chunk would make every wait cover all loads in flight.
+constexpr int SCAN_AHEAD = 3;
 template <class TR, int ND, int AHEAD>
 __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typename TR::T *x, int ld, int n, int past, const float *b, float *u,
                                                          const float *wk, const float *kt, float *st, int chunks) {
 	__shared__ __align__(16) f32x4_t s_p[4][4][64], s_u[4][64];
 	const TgGla &g = d.g;
 	const int h = blockIdx.x, v0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lg = lane >> 4;
-	const int hd = g.heads * g.dimp, hv = g.heads * g.vdimp, ntile = g.dimp / 16;
+	const int hd = g.heads * g.dimp, ntile = g.dimp / 16;
 	{
 		const int keep = min(d.taps, n), total = keep * d.channels, step = (int)(gridDim.x * gridDim.y) * 256;
 		for (int e = ((int)blockIdx.y * (int)gridDim.x + h) * 256 + tid; e < total; e += step) {
@@ -633,13 +666,12 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 #pragma unroll
 		for (int e = 0; e < 4; e++) S[i][e] = own[i] ? g.state[((size_t)h * g.dimp + row[i] + 4 * lg + e) * g.vdimp + v0 + lr] : 0.0f;
 	}
-	const unsigned lw = (unsigned)(lr * hd + 4 * lg), lk = (unsigned)(lr * C + 4 * lg), lu = (unsigned)((16 * w + 4 * lg) * hv + lr);
-	const unsigned ls = (unsigned)(4 * lg * g.vdimp + lr);
+	const unsigned lw = (unsigned)(lr * hd + 4 * lg), lk = (unsigned)(lr * C + 4 * lg), ls = (unsigned)(lr * g.dimp + 4 * lg);
+	auto column = [&](int ch) { return ((size_t)ch * g.heads + h) * g.vdimp + v0; };  // the first of the workgroup's, of u and of the states
 	auto fetch = [&](int set, int ch) {
 		// (bases that the workgroup shares, 32-bit offsets per lane)
 		const size_t t0 = (size_t)min(ch, chunks - 1) * C;
 		const float *pw = wk + t0 * hd + (size_t)h * g.dimp, *pk = kt + t0 * hd + (size_t)h * g.dimp * C, *pb = b + (t0 + C - 1) * hd + (size_t)h * g.dimp;
-		const float *pu = u + t0 * hv + (size_t)h * g.vdimp + v0;
 #pragma unroll
 		for (int i = 0; i < ND; i++) {
 #pragma unroll
@@ -649,10 +681,10 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 			}
 			fb[set][i] = tg_load4(pb + (unsigned)(row[i] + 4 * lg));
 		}
-#pragma unroll
-		for (int e = 0; e < 4; e++) fv[set][e] = pu[(size_t)e * hv + lu];
+		fv[set] = tg_load4(u + column(min(ch, chunks - 1)) * C + (lk + (unsigned)(16 * w)));
 	};
 	auto chunk = [&](int set, int ch) {
+		const bool live = ch < chunks;
 		f32x4_t part[4];
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) part[tt] = f32x4_t{0, 0, 0, 0};
@@ -664,25 +696,24 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 				for (int tt = 0; tt < 4; tt++) part[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(fw[set][i][tt][e], S[i][e], part[tt], 0, 0, 0);
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) s_p[w][tt][lane] = part[tt];
-		float *front = st + (((size_t)ch * g.heads + h) * g.dimp) * g.vdimp + v0;
+		// (a tile that is not there is written behind the last chunk: no branches, as above)
 #pragma unroll
-		for (int i = 0; i < ND; i++)
-			if (own[i])
-#pragma unroll
-				for (int e = 0; e < 4; e++) front[(size_t)e * g.vdimp + (ls + (unsigned)(row[i] * g.vdimp))] = S[i][e];
+		for (int i = 0; i < ND; i++) {
+			tg_store4(st + column(own[i] ? ch : chunks + AHEAD - 1) * g.dimp + (ls + (unsigned)row[i]), S[i]);
+		}
 		f32x4_t uv = fv[set];
 #pragma unroll
 		for (int i = 0; i < ND; i++)
 #pragma unroll
-			for (int e = 0; e < 4; e++) S[i][e] *= pow2(fb[set][i][e]);
+			for (int e = 0; e < 4; e++) S[i][e] *= live ? pow2(fb[set][i][e]) : 1.0f;
 		tg_lds_barrier();
+		f32x4_t pq[4];
 #pragma unroll
-		for (int q = 0; q < 4; q++)
+		for (int q = 0; q < 4; q++) pq[q] = s_p[q][w][lane];
 #pragma unroll
-			for (int e = 0; e < 4; e++) uv[e] -= s_p[q][w][lane][e];
+		for (int e = 0; e < 4; e++) uv[e] = live ? uv[e] - ((pq[0][e] + pq[1][e]) + (pq[2][e] + pq[3][e])) : 0.0f;
 		s_u[w][lane] = uv;
-#pragma unroll
-		for (int e = 0; e < 4; e++) u[(size_t)ch * C * hv + (size_t)h * g.vdimp + v0 + (size_t)e * hv + lu] = uv[e];
+		tg_store4(u + column(ch) * C + (lk + (unsigned)(16 * w)), uv);
 		tg_lds_barrier();
 		f32x4_t ut[4];
 #pragma unroll
@@ -695,15 +726,19 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 				for (int i = 0; i < ND; i++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(fk[set][i][tt][e], ut[tt][e], S[i], 0, 0, 0);
 #pragma unroll
 		for (int i = 0; i < ND; i++)
-			if (!own[i]) S[i] = f32x4_t{0, 0, 0, 0};
+#pragma unroll
+			for (int e = 0; e < 4; e++) S[i][e] = own[i] ? S[i][e] : 0.0f;
 		fetch(set, ch + AHEAD);  // (past the end: the last chunk again, unused; its u may have changed, and is not looked at)
 	};
 #pragma unroll
-	for (int a = 0; a < AHEAD; a++) fetch(a, a);
+	for (int a = 0; a < AHEAD; a++) {
+		fetch(a, a);
+		__builtin_amdgcn_sched_barrier(0);
+	}
 	for (int ch = 0; ch < chunks; ch += AHEAD) {
 #pragma unroll
 		for (int a = 0; a < AHEAD; a++) {
-			if (ch + a < chunks) chunk(a, ch + a);
+			chunk(a, ch + a);
 			__builtin_amdgcn_sched_barrier(0);
 		}
 	}
@@ -904,22 +939,27 @@ void launch_delta_rows(const TgDelta &d, const void *xv, int ld, const float *lo
 	const TgGla &g = d.g;
 	const int qc = d.q_channels(), hv = g.heads * g.vdimp, hd = g.heads * g.dimp, kvh = g.heads / g.group;
 	const unsigned chunks = (unsigned)((n + C - 1) / C);
-	hipLaunchKernelGGL((delta_prep_kernel<TR>), dim3((unsigned)((n + 4 * PT - 1) / (4 * PT)), (unsigned)(2 * kvh + (hv + 255) / 256)), dim3(256), 0, s, d, x, ld, n, past,
-	                   t.qk, t.u);
+	auto prep = [&](auto *kernel) {
+		hipLaunchKernelGGL(kernel, dim3((unsigned)((n + 4 * PT - 1) / (4 * PT)), (unsigned)(2 * kvh + (hv + 255) / 256)), dim3(256), 0, s, d, x, ld, n, past,
+		                   t.qk, t.v);
+	};
+	if (d.taps == 4) prep(delta_prep_kernel<TR, 4>);
+	else if (d.taps == 3) prep(delta_prep_kernel<TR, 3>);
+	else prep(delta_prep_kernel<TR, 0>);
 	hipLaunchKernelGGL(gla_decay_kernel, dim3(chunks, (unsigned)((hd + 63) / 64)), dim3(256), 0, s, low + a_off, ld_low, g, n, t.b);
 	hipLaunchKernelGGL((gla_intra_kernel<TgF32, true>), dim3(chunks, (unsigned)g.heads), dim3(256), 0, s, t.qk, 2 * qc, qc, g, n, t.b, t.a,
 	                   DeltaIntra{low + b_off, ld_low, t.t});
-	const DeltaSolve solve = {t.qk, t.b, t.t, low + b_off, 2 * qc, qc, ld_low, t.u, t.wk, t.kt};
+	const DeltaSolve solve = {t.qk, t.b, t.t, low + b_off, 2 * qc, qc, ld_low, t.v, t.u, t.wk, t.kt};
 	hipLaunchKernelGGL(delta_solve_kernel, dim3(chunks, (unsigned)g.heads, (unsigned)((g.dimp + g.vdimp + 127) / 128)), dim3(256), 0, s, solve, g, n);
 	const dim3 grid((unsigned)g.heads, (unsigned)(g.vdimp / 16));
 	auto scan = [&](auto *kernel) {
 		hipLaunchKernelGGL(kernel, grid, dim3(256), 0, s, d, x, ld, n, past, (const float *)t.b, t.u, (const float *)t.wk, (const float *)t.kt, t.st,
 		                   (int)chunks);
 	};
-	if (g.dimp <= 64) scan(delta_scan_kernel<TR, 1, 3>);
-	else if (g.dimp <= 128) scan(delta_scan_kernel<TR, 2, 3>);
+	if (g.dimp <= 64) scan(delta_scan_kernel<TR, 1, SCAN_AHEAD>);
+	else if (g.dimp <= 128) scan(delta_scan_kernel<TR, 2, SCAN_AHEAD>);
 	else scan(delta_scan_kernel<TR, 4, 2>);
-	launch_out<TgF32, TR, true>(g, OutIn{t.qk, t.u, gate, 2 * qc, hv, ldg}, n, t.b, t.a, t.st, out, ld_out, s);
+	launch_out<TgF32, TR, true>(g, OutIn{t.qk, t.u, gate, 2 * qc, 0, ldg}, n, t.b, t.a, t.st, out, ld_out, s);
 }
 
 }  // namespace
@@ -962,6 +1002,7 @@ void tg_launch_delta_step(const TgDelta &d, const float *y, int g_off, int b_off
 size_t tg_delta_scratch(const TgDelta &d, int n, TgDeltaScratch *t, unsigned char *base) {
 	const TgGla &g = d.g;
 	const size_t chunks = (size_t)((n + C - 1) / C), hd = (size_t)g.heads * g.dimp, hv = (size_t)g.heads * g.vdimp;
+	const size_t padded = chunks + SCAN_AHEAD;  // (what the pass over the chunks writes)
 	size_t off = 0;
 	auto take = [&](float **p, size_t floats) {
 		if (base) *p = (float *)(base + off);
@@ -973,10 +1014,11 @@ size_t tg_delta_scratch(const TgDelta &d, int n, TgDeltaScratch *t, unsigned cha
 	take(&t->a, chunks * g.heads * C * C);
 	take(&t->t, chunks * g.heads * C * C);
 	take(&t->qk, (size_t)n * 2 * d.q_channels());
-	take(&t->u, chunks * C * hv);
+	take(&t->v, (size_t)n * hv);
+	take(&t->u, padded * C * hv);
 	take(&t->wk, chunks * C * hd);
 	take(&t->kt, chunks * C * hd);
-	take(&t->st, chunks * hd * g.vdimp);
+	take(&t->st, padded * hd * g.vdimp);
 	return off;
 }
 
