@@ -59,10 +59,11 @@ struct TgDeltaScratch {
 	float *t;       // [chunks][heads][64][64] what the solve multiplies with (tg_gla.hip)
 	float *qk;      // [n][q | k] behind convolution and unit norm
 	float *v;       // [n][heads * vdimp] behind the convolution
-	float *u;       // [chunks][heads][vdimp][64] v's solved form, then u
-	float *wk;      // [chunks * 64][heads * dimp] solved keys
-	float *kt;      // [chunks][heads][dimp][64] keys decayed to the chunk's end, transposed
-	float *st;      // [chunks][heads][vdimp][dimp] the state in front of every chunk
+	// in operand order (tg_gla.hip):
+	float *u;       // [chunks][heads][vdimp x 64] v's solved form, then u
+	float *wk;      // [chunks][heads][dimp x 64] solved keys
+	float *kt;      // [chunks][heads][dimp x 64] keys decayed to the chunk's end
+	float *st;      // [chunks][heads][vdimp x dimp] the state in front of every chunk
 };
 size_t tg_delta_scratch(const TgDelta &d, int n, TgDeltaScratch *t, unsigned char *base);
 void tg_launch_delta_rows(const TgDelta &d, int dt, const void *x, int ld, const float *low, int ld_low, int b_off, int a_off, const void *gate, int ldg,

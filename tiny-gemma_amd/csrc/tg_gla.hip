@@ -248,6 +248,9 @@ __global__ __launch_bounds__(256) void gla_intra_kernel(const typename TR::T *qk
 // The solve runs down the 16 x 16 blocks on the matrix instructions, a wave per two tiles of 16 columns: an accumulator (four
 // consecutive rows of a column per lane) is the next product's second operand as it is, with the first operand's columns taken
 // in the same order.  Also the keys decayed to the chunk's end, transposed.
+// Results lie in operand order, 16 x 16 tiles of [lane][4]: wk in tiles (key channels, tokens), lane = token % 16 + 16 (channel % 16
+// / 4), the four values being consecutive channels (turned through LDS); kt and u in tiles (key channels or value columns, tokens),
+// lane = channel % 16 + 16 (token % 16 / 4), consecutive tokens.
 struct DeltaSolve {
 	const float *qk, *b, *t, *beta;
 	int ldqk, k_off, ld_beta;
@@ -255,7 +258,7 @@ struct DeltaSolve {
 	float *u, *wk, *kt;
 };
 __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g, int n) {
-	__shared__ __align__(16) float s_beta[C];
+	__shared__ __align__(16) float s_beta[C], s_turn[4][16][20];
 	const int ch = blockIdx.x, h = blockIdx.y, kh = h / g.group, tid = threadIdx.x, lane = tid & 63, w = tid >> 6, lr = lane & 15, lg = lane >> 4;
 	const int hd = g.heads * g.dimp, hv = g.heads * g.vdimp, t0 = ch * C;
 	const int nk = g.dimp / 16, ntile = nk + g.vdimp / 16, tile0 = ((int)blockIdx.z * 4 + w) * 2;
@@ -307,7 +310,7 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g,
 					kd[e] = t0 + 16 * i + 4 * lg + e < n ? X[p][i][e] * pow2(be[p] - bt[p][i][e]) : 0.0f;
 					X[p][i][e] *= pow2(bt[p][i][e]);
 				}
-				if (live) tg_store4(x.kt + (((size_t)ch * g.heads + h) * g.dimp + col[p]) * C + 16 * i + 4 * lg, kd);
+				if (live) tg_store4(x.kt + (size_t)t0 * hd + (size_t)h * g.dimp * C + (((tile + p) * 4 + i) * 64 + lane) * 4, kd);
 			}
 #pragma unroll
 			for (int e = 0; e < 4; e++) X[p][i][e] *= beta[e];
@@ -330,15 +333,17 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaSolve x, TgGla g,
 	if (!live) return;
 #pragma unroll
 	for (int p = 0; p < 2; p++) {
-		float *wk = x.wk + (size_t)t0 * hd + (size_t)h * g.dimp + col[p], *u = x.u + (((size_t)ch * g.heads + h) * g.vdimp + col[p]) * C;
+		float *dst = key ? x.wk + (size_t)t0 * hd + (size_t)h * g.dimp * C + (tile + p) * 1024 : x.u + (size_t)t0 * hv + (size_t)h * g.vdimp * C + (tile - nk + p) * 1024;
 #pragma unroll
 		for (int i = 0; i < 4; i++) {
 			if (key) {
 #pragma unroll
-				for (int e = 0; e < 4; e++) wk[(size_t)(16 * i + 4 * lg + e) * hd] = W[p][i][e];
-			} else {
-				tg_store4(u + 16 * i + 4 * lg, W[p][i]);
+				for (int e = 0; e < 4; e++) s_turn[w][4 * lg + e][lr] = W[p][i][e];
+				__builtin_amdgcn_wave_barrier();
+				W[p][i] = tg_load4(&s_turn[w][lr][4 * lg]);
+				__builtin_amdgcn_wave_barrier();
 			}
+			tg_store4(dst + (i * 64 + lane) * 4, W[p][i]);
 		}
 	}
 }
@@ -431,7 +436,7 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(float *U, const float *b,
 // ---- o = (q e^b)^T S + A v, the head's root mean square norm and silu(gate): 64 tokens x the whole head per workgroup -------------
 // 8 waves: 16 tokens x half of the value columns each.  Slabs of 32: first the key channels (rows q e^b, columns of S), then
 // the chunk's own tokens (rows A, columns v); a slab's loads are in flight during the one before it.
-// (delta rule: v is u, [chunks][heads][vdimp][64], the states are [chunks][heads][vdimp][dimp], the gate's function is the sigmoid)
+// (delta rule: v is u, the states are tiles (value columns, key channels) like u's, the gate's function is the sigmoid)
 struct OutIn {
 	const void *q, *v, *gate;
 	int ldq, ldv, ldg;
@@ -459,7 +464,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, 
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
 				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-				if constexpr (DELTA) y[i] = tg_load4(S + (size_t)min(e >> 3, g.vdimp - 1) * g.dimp + sl * 32 + (e & 7) * 4);
+				if constexpr (DELTA) y[i] = tg_load4(S + ((size_t)(min(e >> 3, g.vdimp - 1) >> 4) * (g.dimp / 16) + sl * 2 + ((e >> 2) & 1)) * 256 + ((e >> 3) & 15) * 4 + (e & 3) * 64);
 				else y[i] = tg_load4(S + (size_t)(sl * 32 + r) * g.vdimp + (c4 < g.vdimp ? c4 : 0));
 			}
 		} else {
@@ -468,7 +473,7 @@ __global__ __launch_bounds__(512) void gla_out_kernel(OutIn in, TgGla g, int n, 
 #pragma unroll
 			for (int i = 0; i < NY; i++) {
 				const int e = tid + 512 * i, r = e / (VB / 4), c4 = (e % (VB / 4)) * 4;
-				if constexpr (DELTA) y[i] = tg_load4(V + (size_t)min(e >> 3, g.vdimp - 1) * C + j0 + (e & 7) * 4);
+				if constexpr (DELTA) y[i] = tg_load4(V + ((size_t)(min(e >> 3, g.vdimp - 1) >> 4) * 4 + j0 / 16 + ((e >> 2) & 1)) * 256 + ((e >> 3) & 15) * 4 + (e & 3) * 64);
 				else y[i] = tg_load4(V + (size_t)min(t0 + j0 + r, n - 1) * in.ldv + (c4 < g.vdimp ? c4 : 0));
 			}
 		}
@@ -666,28 +671,36 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 #pragma unroll
 		for (int e = 0; e < 4; e++) S[i][e] = own[i] ? g.state[((size_t)h * g.dimp + row[i] + 4 * lg + e) * g.vdimp + v0 + lr] : 0.0f;
 	}
-	const unsigned lw = (unsigned)(lr * hd + 4 * lg), lk = (unsigned)(lr * C + 4 * lg), ls = (unsigned)(lr * g.dimp + 4 * lg);
-	auto column = [&](int ch) { return ((size_t)ch * g.heads + h) * g.vdimp + v0; };  // the first of the workgroup's, of u and of the states
-	auto fetch = [&](int set, int ch) {
-		// (bases that the workgroup shares, 32-bit offsets per lane)
-		const size_t t0 = (size_t)min(ch, chunks - 1) * C;
-		const float *pw = wk + t0 * hd + (size_t)h * g.dimp, *pk = kt + t0 * hd + (size_t)h * g.dimp * C, *pb = b + (t0 + C - 1) * hd + (size_t)h * g.dimp;
+	const int vt = (int)blockIdx.y, vtiles = g.vdimp / 16;
+	const unsigned l4 = (unsigned)(lane * 4);
+	// (bases that the workgroup shares, 32-bit offsets per lane)
+	auto keys = [&](int ch) { return ((size_t)min(ch, chunks - 1) * g.heads + h) * g.dimp * C; };
+	auto values = [&](int ch) { return (((size_t)ch * g.heads + h) * vtiles + vt) * 1024; };
+	auto fetch_w = [&](int set, int ch) {
+		const float *pw = wk + keys(ch), *pb = b + ((size_t)min(ch, chunks - 1) * C + C - 1) * hd + (size_t)h * g.dimp;
 #pragma unroll
 		for (int i = 0; i < ND; i++) {
 #pragma unroll
-			for (int tt = 0; tt < 4; tt++) {
-				fw[set][i][tt] = tg_load4(pw + (size_t)(16 * tt) * hd + (lw + (unsigned)row[i]));
-				fk[set][i][tt] = tg_load4(pk + 16 * tt + (lk + (unsigned)row[i] * C));
-			}
+			for (int tt = 0; tt < 4; tt++) fw[set][i][tt] = tg_load4(pw + (unsigned)(row[i] * C + tt * 256) + l4);
 			fb[set][i] = tg_load4(pb + (unsigned)(row[i] + 4 * lg));
 		}
-		fv[set] = tg_load4(u + column(min(ch, chunks - 1)) * C + (lk + (unsigned)(16 * w)));
+		fv[set] = tg_load4(u + values(min(ch, chunks - 1)) + (unsigned)(w * 256) + l4);
 	};
+	auto fetch_k = [&](int set, int ch) {
+		const float *pk = kt + keys(ch);
+#pragma unroll
+		for (int i = 0; i < ND; i++)
+#pragma unroll
+			for (int tt = 0; tt < 4; tt++) fk[set][i][tt] = tg_load4(pk + (unsigned)(row[i] * C + tt * 256) + l4);
+	};
+	// A wave issues in order and a load takes its time to issue: loads are dealt out among the matrix instructions of the two
+	// products, each set's as soon as it has been used (past the end: the last chunk again, unused).
 	auto chunk = [&](int set, int ch) {
 		const bool live = ch < chunks;
 		f32x4_t part[4];
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) part[tt] = f32x4_t{0, 0, 0, 0};
+		fetch_k((set + AHEAD - 1) % AHEAD, ch + AHEAD - 1);
 #pragma unroll
 		for (int i = 0; i < ND; i++)
 #pragma unroll
@@ -695,11 +708,18 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 #pragma unroll
 				for (int tt = 0; tt < 4; tt++) part[tt] = __builtin_amdgcn_mfma_f32_16x16x4f32(fw[set][i][tt][e], S[i][e], part[tt], 0, 0, 0);
 #pragma unroll
+		for (int i = 0; i < 4 * ND; i++) {
+			__builtin_amdgcn_sched_group_barrier(0x008, 4, 0);  // matrix instructions
+			__builtin_amdgcn_sched_group_barrier(0x020, 1, 0);  // global load
+		}
+		__builtin_amdgcn_sched_barrier(0);
+#pragma unroll
 		for (int tt = 0; tt < 4; tt++) s_p[w][tt][lane] = part[tt];
 		// (a tile that is not there is written behind the last chunk: no branches, as above)
 #pragma unroll
 		for (int i = 0; i < ND; i++) {
-			tg_store4(st + column(own[i] ? ch : chunks + AHEAD - 1) * g.dimp + (ls + (unsigned)row[i]), S[i]);
+			float *front = st + values(own[i] ? ch : chunks + AHEAD - 1) / C * g.dimp;
+			tg_store4(front + (unsigned)(row[i] * 16) + l4, S[i]);
 		}
 		f32x4_t uv = fv[set];
 #pragma unroll
@@ -713,11 +733,13 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 #pragma unroll
 		for (int e = 0; e < 4; e++) uv[e] = live ? uv[e] - ((pq[0][e] + pq[1][e]) + (pq[2][e] + pq[3][e])) : 0.0f;
 		s_u[w][lane] = uv;
-		tg_store4(u + column(ch) * C + (lk + (unsigned)(16 * w)), uv);
+		tg_store4(u + values(ch) + (unsigned)(w * 256) + l4, uv);
 		tg_lds_barrier();
 		f32x4_t ut[4];
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++) ut[tt] = s_u[tt][lane];
+		__builtin_amdgcn_sched_barrier(0);
+		fetch_w(set, ch + AHEAD);
 #pragma unroll
 		for (int tt = 0; tt < 4; tt++)
 #pragma unroll
@@ -725,14 +747,20 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(TgDelta d, const typ
 #pragma unroll
 				for (int i = 0; i < ND; i++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(fk[set][i][tt][e], ut[tt][e], S[i], 0, 0, 0);
 #pragma unroll
+		for (int i = 0; i < 5 * ND + 1; i++) {
+			__builtin_amdgcn_sched_group_barrier(0x008, 3, 0);
+			__builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
+		}
+		__builtin_amdgcn_sched_barrier(0);
+#pragma unroll
 		for (int i = 0; i < ND; i++)
 #pragma unroll
 			for (int e = 0; e < 4; e++) S[i][e] = own[i] ? S[i][e] : 0.0f;
-		fetch(set, ch + AHEAD);  // (past the end: the last chunk again, unused; its u may have changed, and is not looked at)
 	};
 #pragma unroll
 	for (int a = 0; a < AHEAD; a++) {
-		fetch(a, a);
+		fetch_w(a, a);
+		if (a + 1 < AHEAD) fetch_k(a, a);
 		__builtin_amdgcn_sched_barrier(0);
 	}
 	for (int ch = 0; ch < chunks; ch += AHEAD) {
