@@ -84,10 +84,128 @@ def test_routing_uses_the_correction_for_the_choice_only():
     assert np.allclose(w, 0.0)
 
 
-@pytest.mark.parametrize("name", ["ragged", "tiny"])
+def test_rotation_depends_on_the_distance_only():
+    rng = np.random.default_rng(0)
+    for interleaved in (True, False):
+        q, k = rng.standard_normal((2, 12))
+        s = [layers.rotate(q, p + 7, 8, 50.0, interleaved) @ layers.rotate(k, p, 8, 50.0, interleaved) for p in (0, 3, 40)]
+        assert np.allclose(s, s[0])
+        r = layers.rotate(q, 5, 8, 50.0, interleaved)
+        assert np.array_equal(r[8:], q[8:]) and np.isclose(np.linalg.norm(r), np.linalg.norm(q)) and not np.allclose(r[:8], q[:8])
+    x = rng.standard_normal(8)
+    pairs = np.arange(8).reshape(4, 2).T.reshape(-1)          # interleaved pairs brought side by side in halves
+    assert np.allclose(layers.rotate(x, 9, 8, 50.0, True)[pairs], layers.rotate(x[pairs], 9, 8, 50.0, False))
+    z = x[0] + 1j * x[1]                                      # the first pair turns by the position itself
+    assert np.allclose(layers.rotate(x, 2, 8, 50.0, True)[:2], [(z * np.exp(2j)).real, (z * np.exp(2j)).imag])
+
+
+def banded_softmax(s, window):
+    n = s.shape[-1]
+    i, j = np.mgrid[:n, :n]
+    s = np.where((i - j >= 0) & (i - j < window), s, -np.inf)
+    p = np.exp(s - s.max(-1, keepdims=True))
+    return p / p.sum(-1, keepdims=True)
+
+
+def test_rotated_latent_attention_equals_full_matrices():
+    cfg = nm.tutelix(24, 11, [nm.layer(nm.rot_latent(3, 5, 4, 7, 9, 6, 4, 0.7, 30.0))])
+    m = layers.model_of(cfg, nm.weights(cfg, 2))
+    h = np.random.default_rng(0).standard_normal((9, 24))
+    got = m.mixer(0, h, [])
+    t = {k.split("mix.")[-1]: v for k, v in m.t.items()}
+    cq = h @ t["dq"].T
+    q = (cq / np.sqrt((cq ** 2).mean(-1, keepdims=True) + 1e-5) * t["dq.norm"] @ t["uq"].T).reshape(9, 3, 9)
+    kv = h @ t["dkv"].T
+    c = kv[:, :6] / np.sqrt((kv[:, :6] ** 2).mean(-1, keepdims=True) + 1e-5) * t["dkv.norm"]
+    k = np.concatenate([(c @ t["uk"].T).reshape(9, 3, 5), np.repeat(kv[:, None, 6:], 3, 1)], -1)
+    turn = np.exp(1j * np.arange(9)[:, None] * 30.0 ** (-np.arange(0, 4, 2) / 4))
+    for x in (q, k):
+        z = (x[..., 5::2] + 1j * x[..., 6::2]) * turn[:, None]
+        x[..., 5::2], x[..., 6::2] = z.real, z.imag
+    p = banded_softmax(np.einsum("ihd,jhd->hij", q, k) * 0.7, 4)
+    o = np.einsum("hij,jhv->ihv", p, (c @ t["uv"].T).reshape(9, 3, 7))
+    assert np.allclose(got, o.reshape(9, 21) @ t["o"].T, atol=1e-12)
+
+
+def test_attention_on_its_keys_equals_full_matrices():
+    cfg = nm.tutelix(24, 11, [nm.layer(nm.key_values(6, 2, 7, 4, 3, 0.7, 30.0))])
+    m = layers.model_of(cfg, nm.weights(cfg, 2))
+    h = np.random.default_rng(0).standard_normal((9, 24))
+    got = m.mixer(0, h, [])
+    t = {k.split("mix.")[-1]: v for k, v in m.t.items()}
+    q, v = (h @ t["q"].T + t["q.b"]).reshape(9, 6, 7), (h @ t["k"].T + t["k.b"]).reshape(9, 2, 7)
+    k = v.copy()
+    turn = np.exp(1j * np.arange(9)[:, None] * 30.0 ** (-np.arange(0, 4, 2) / 4))[:, None]
+    for x in (q, k):
+        z = (x[..., :2] + 1j * x[..., 2:4]) * turn
+        x[..., :2], x[..., 2:4] = z.real, z.imag
+    own = np.array([0, 0, 0, 1, 1, 1])
+    p = banded_softmax(np.einsum("ihd,jhd->hij", q, k[:, own]) * 0.7, 3)
+    assert np.allclose(got, np.einsum("hij,jhv->ihv", p, v[:, own]).reshape(9, 42) @ t["o"].T, atol=1e-12)
+
+
+def test_short_convolution_is_causal():
+    rng = np.random.default_rng(0)
+    x, w, past = rng.standard_normal((10, 3)), rng.standard_normal((3, 4)), []
+    got = np.array([layers.short_conv(v, past, w) for v in x])
+    want = np.stack([np.convolve(x[:, c], w[c, ::-1])[:10] for c in range(3)], -1)
+    assert np.allclose(got, want)
+    assert np.allclose(layers.short_conv(x[0], [], w), x[0] * w[:, -1])
+
+
+def test_gated_delta_rule_equals_its_transition_matrices():
+    """S_t = (1 - beta k k^T) diag(g) S_(t-1) + beta k v^T, and the state of a portion is carried to the next."""
+    cfg = nm.tutelix(24, 11, [nm.layer(nm.delta(4, 2, 5, 3, 1))])
+    m = layers.model_of(cfg, nm.weights(cfg, 1, rank=4, gate_rank=3))
+    h = np.random.default_rng(0).standard_normal((12, 24))
+    st = m.state()[0]
+    got = np.concatenate([m.mixer(0, h[:5], st), m.mixer(0, h[5:], st)])
+    t = {k.split("mix.")[-1]: v for k, v in m.t.items()}
+
+    def silu(z):
+        return z / (1 + np.exp(-z))
+    q, k, v = (silu(h @ t[n].T * t[n + ".conv"][:, 0]) for n in "qkv")
+    q, k, v = q.reshape(12, 2, 5), k.reshape(12, 2, 5), v.reshape(12, 4, 3)
+    q, k = (x / np.sqrt((x ** 2).sum(-1, keepdims=True) + 1e-6) for x in (q, k))
+    beta = 1 / (1 + np.exp(-h @ t["b"].T))
+    z = (h @ t["a1"].T @ t["a2"].T + t["dt_bias"]).reshape(12, 4, 5)
+    g = np.exp(-np.exp(t["A_log"])[:, None] * np.log1p(np.exp(z)))
+    S, want = np.zeros((4, 5, 3)), np.zeros((12, 4, 3))
+    for i in range(12):
+        for a in range(4):
+            kk = k[i, a // 2]
+            S[a] = (np.eye(5) - beta[i, a] * np.outer(kk, kk)) @ np.diag(g[i, a]) @ S[a] + beta[i, a] * np.outer(kk, v[i, a])
+            o = q[i, a // 2] / np.sqrt(5) @ S[a]
+            want[i, a] = o / np.sqrt((o ** 2).mean() + 1e-5) * t["norm"]
+    want = want.reshape(12, 12) / (1 + np.exp(-(h @ t["g1"].T @ t["g2"].T)))
+    assert np.allclose(got, want @ t["o"].T, atol=1e-10)
+
+
+def test_gelu_is_the_exact_one():
+    z = np.array([-30.0, -1.0, 0.0, 0.5, 30.0])
+    assert np.allclose(layers.gelu(z), [0.0, -0.15865525393145707, 0.0, 0.34573123063700656, 30.0], atol=1e-15)
+
+
+def test_looped_layers_equal_layers_written_out():
+    """A run of layers passed three times has the weights once and a state for each pass."""
+    ls = [nm.layer(nm.delta(2, 1, 5, 3, 2), nm.dense(8)), nm.layer(nm.key_values(2, 1, 6, 4, 3, 0.7)), nm.layer(nm.rot_latent(2, 5, 4, 3, 6, 7, 4, 0.5), nm.dense(5))]
+    cfg = nm.tutelix(16, 11, ls, loop=(1, 3, 3))
+    t = nm.weights(cfg, 5)
+    flat = nm.tutelix(16, 11, [ls[0]] + ls[1:] * 3, loop=(0, 1, 1))
+    t2 = {k: v for k, v in t.items() if not k.startswith(("l1.", "l2."))}
+    for k, v in t.items():
+        if k.startswith(("l1.", "l2.")):
+            t2.update({f"l{int(k[1]) + 2 * i}{k[2:]}": v for i in range(3)})
+    a, b = layers.model_of(cfg, t), layers.model_of(flat, t2)
+    assert a.runs() == [0, 1, 2, 1, 2, 1, 2] and len(a.state()) == 7
+    ids = np.random.default_rng(4).integers(0, 11, 12)
+    assert np.allclose(a.step(a.state(), ids), b.step(b.state(), ids), atol=1e-12)
+
+
+@pytest.mark.parametrize("name", ["ragged", "tiny", "mixed", "ones"])
 def test_portions_of_the_oracle_agree(name):
-    cfg = nm.MODELS[name]
-    m = layers.LayerModel(cfg, nm.weights(cfg, 3))
+    cfg = nm.MODELS.get(name) or nm.TUTELIX[name]
+    m = layers.model_of(cfg, nm.weights(cfg, 3))
     ids = np.random.default_rng(4).integers(0, cfg["vocab"], 12)
     whole = m.step(m.state(), ids)
     st = m.state()
@@ -105,3 +223,6 @@ def test_random_model_dir_is_readable(tmp_path):
     m = layers.LayerModel.from_dir(str(tmp_path / "m"))
     assert np.isfinite(m.step(m.state(), [1, 2, 3])).all()
     assert sum(k.startswith("l3.") or k.startswith("l4.") for k in m.t) == 0   # shared layers have no tensors
+    w.random_model_dir(str(tmp_path / "t"), nm.TUTELIX["mixed"], 5, decay_rank=3, block=1 << 12, gate_rank=4)
+    m = layers.LayerModel.from_dir(str(tmp_path / "t"))
+    assert isinstance(m, layers.TutelixModel) and np.isfinite(m.step(m.state(), [1, 2, 3])).all()
