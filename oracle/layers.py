@@ -187,17 +187,18 @@ def rotated_latent_attention(h, cache, w, heads, dim, rot_dim, vdim, scale, wind
 
 # ---- attention whose values are its keys --------------------------------------------------------------------------
 def key_value_attention(h, cache, w, heads, kv_heads, dim, scale, window, dims, base):
-    """h [n, D]; cache: list of keys [kv_heads, dim] before rotation (extended in place).  Query head a uses key head
+    """h [n, D]; cache: list of (keys [kv_heads, dim] as projected, the same rotated), extended in place.  Query head a uses key head
     a // (heads / kv_heads); scores on rotated queries and keys over the last `window` tokens; the values are the keys as
     projected."""
     out = np.zeros((h.shape[0], w["o"].shape[0]), F)
     for t in range(h.shape[0]):
         pos = len(cache)
-        cache.append((w["k"] @ h[t] + w["k_b"]).reshape(kv_heads, dim))
+        key = (w["k"] @ h[t] + w["k_b"]).reshape(kv_heads, dim)
+        cache.append((key, rotate(key, pos, dims, base, False)))
         q = rotate((w["q"] @ h[t] + w["q_b"]).reshape(heads, dim), pos, dims, base, False)
         lo = max(0, pos - window + 1)
-        v = np.stack(cache[lo:])
-        k = np.stack([rotate(cache[j], j, dims, base, False) for j in range(lo, pos + 1)])
+        v = np.stack([c[0] for c in cache[lo:]])
+        k = np.stack([c[1] for c in cache[lo:]])
         heads_out = []
         for a in range(heads):
             g = a // (heads // kv_heads)

@@ -326,6 +326,12 @@ def test_one_write_that_stays_in_the_state(tg, folder, at):
         rows_close(got, want[None], F32_TOL, f"token {at}, portions {cut}")
 
 
+def key_cache(om, h, m):
+    """The oracle's cache of an attention layer from its normed inputs."""
+    k = (h @ om.t["l0.mix.k"].T + om.t["l0.mix.k.b"]).reshape(len(h), m["kv_heads"], -1)
+    return [(x, layers.rotate(x, p, m["rot"]["dims"], m["rot"]["base"], False)) for p, x in enumerate(k)]
+
+
 @pytest.mark.parametrize("kind", WINDOWED)
 @pytest.mark.parametrize("window", [700, 1100, 1500])
 def test_decoding_in_long_windows(tg, folder, kind, window):
@@ -344,7 +350,7 @@ def test_decoding_in_long_windows(tg, folder, kind, window):
             cache = [(c, layers.rotate(k, p, m["rot"]["dims"], m["rot"]["base"], True))
                      for p, (c, k) in enumerate(zip(layers.rms_norm(kv[:, :r], om.t["l0.mix.dkv.norm"], eps), kv[:, r:]))]
         else:
-            cache = list((h @ om.t["l0.mix.k"].T + om.t["l0.mix.k.b"]).reshape(n, m["kv_heads"], -1))
+            cache = key_cache(om, h, m)
         return om.step([cache[:-1]], tokens[-1:])
 
     want = last(ids)
@@ -382,7 +388,7 @@ def test_large_products_and_tiles(tg, folder, dtype):
     ids = ids_of(cfg, n)
     places = [0, 1, 88, 89, 90, 91, 127, 128, 1023, 1024, 2447, 2449]
     h = om.norm("l0.norm1", om.embed(ids))
-    cache = list((h @ om.t["l0.mix.k"].T + om.t["l0.mix.k.b"]).reshape(n, 4, 64))
+    cache = key_cache(om, h, cfg["layers"][0]["mixer"])
     want = np.concatenate([om.step([cache[:p]], ids[p:p + 1]) for p in places])
     s = tg.Transformer.from_dir(path, dtype).open_session(n)
     rows_close(s.forward(ids, places)[1], want, F32_TOL if dtype == "float32" else 5e-2, "prompt")
