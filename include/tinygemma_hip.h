@@ -119,13 +119,16 @@ void tg_model_destroy(tg_model *m);
 
 /* Any model the library knows by its folder: config.json ("architecture" selects the design, the other keys give its layers
  * and sizes) and model.safetensors.  No counterpart in the reference, whose models are built in.
- * Designs: "Madevik" (layers of gated linear attention and of latent attention, element-wise tanh norms, mixtures of experts).
+ * Designs: "Madevik" (layers of gated linear attention and of latent attention, element-wise tanh norms, mixtures of experts),
+ * "Tutelix" (rotated latent attention and grouped-query attention on its own keys, both in a window, and the gated delta rule;
+ * norms around each sublayer, dense feed-forwards, a run of layers passed several times).
  * dtype: TG_DTYPE_BF16 (weights and matrix operands bfloat16; residual stream, norms, scores, routers and recurrent state
  * fp32) or TG_DTYPE_F32 (everything fp32).  The model comes with its weights; an unknown design or mixer is
  * TG_ERR_UNSUPPORTED_SHAPE, a missing tensor or a wrong shape TG_ERR_BAD_ARG. */
 enum { TG_DTYPE_BF16 = 0, TG_DTYPE_F32 = 1 };
 int tg_model_open(const char *dir, int dtype, tg_model **out);
-/* sizes of a model (of one opened from a folder: hidden_size, n_layers, n_vocab; the other fields are 0) */
+/* sizes of a model (of one opened from a folder: hidden_size, n_layers, n_vocab; the other fields are 0; a layer that is passed
+ * several times counts each time) */
 int tg_model_config(const tg_model *m, tg_config *out);
 const char *tg_model_architecture(const tg_model *m); /* "Gemma3", or config.json's name */
 

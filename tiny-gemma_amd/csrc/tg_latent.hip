@@ -43,7 +43,8 @@ __device__ __forceinline__ float rotated(const V *x, int i, const float2 *turn, 
 // e / d for e * d < 2^22, m = 2^22 / d rounded up
 __device__ __forceinline__ int div_by(int e, unsigned m) { return (int)(((unsigned)e * m) >> 22); }
 
-template <class TR, bool ROT>
+// NC: column tiles of the value part per wave (4 NC tiles of 16 per workgroup).
+template <class TR, bool ROT, int NC>
 __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 	typedef typename TR::T T;
 	typedef typename TR::Frag Frag;
@@ -172,8 +173,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(TgLatentStep a) {
 		inv = 1.0f / sqrtf(((s_sq[0] + s_sq[1]) + (s_sq[2] + s_sq[3])) / (float)a.rank + a.eps);
 	}
 
-	constexpr int NC = 8;  // column tiles per wave
-	const int ct0 = blockIdx.z * 32 + w, nct = a.rankp / 16;
+	const int ct0 = blockIdx.z * (4 * NC) + w, nct = a.rankp / 16;
 	f32x4_t acc[NC];
 #pragma unroll
 	for (int c = 0; c < NC; c++) acc[c] = f32x4_t{0, 0, 0, 0};
@@ -625,8 +625,11 @@ void launch_step(const TgLatentStep &a, hipStream_t s) {
 		if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void *)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
 		hipLaunchKernelGGL(kernel, grid, dim3(256), lds, s, a);
 	};
-	if (a.rotp) go(latent_step_kernel<TR, true>);
-	else go(latent_step_kernel<TR, false>);
+	if (a.rotp && a.rankp <= 128) go(latent_step_kernel<TR, true, 2>);
+	else if (a.rotp && a.rankp <= 256) go(latent_step_kernel<TR, true, 4>);
+	else if (a.rotp) go(latent_step_kernel<TR, true, 8>);
+	else if (a.rankp <= 256) go(latent_step_kernel<TR, false, 4>);
+	else go(latent_step_kernel<TR, false, 8>);
 }
 }  // namespace
 
