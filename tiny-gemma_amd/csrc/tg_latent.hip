@@ -9,7 +9,7 @@ namespace {
 // (the first tile's loads are requested before anything else is done), row pitch 16 bytes more than the row.  Scores: wave w
 // takes keys 16 (w % 2) ... and half w / 2 of the latent; the running softmax is a wave's work for 4 heads; the value sum is
 // a product of the probabilities [16 heads x 32 keys] (in the bf16 format two planes, value and remainder) with the tile,
-// wave w the column tiles w, w + 4, ..., in passes of 512 columns (blockIdx.z).
+// wave w the column tiles w, w + 4, ..., NC of them; wider rows take several workgroups (blockIdx.z).
 constexpr int ST = 32;         // keys per tile
 template <bool ROT>
 constexpr int ST_LOADS = ROT ? 10 : 8;  // 16-byte pieces per lane and round of the tile copy
@@ -362,7 +362,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(TgLatentCacheRows a) {
 
 // a lane per pair
 template <class T>
-__global__ __launch_bounds__(256) void rot_rows_kernel(T *rows, int ld, int n, int past, int first, int count, int stride, TgRot rot) {
+__global__ __launch_bounds__(256) void rot_rows_kernel(T *rows, int ld, int past, int first, int count, int stride, TgRot rot) {
 	const int hd = rot.dims / 2, per = count * hd, t = blockIdx.y;
 	const int e = blockIdx.x * 256 + threadIdx.x;
 	if (e >= per) return;
@@ -666,8 +666,8 @@ void tg_launch_latent_rows(const TgLatentCacheRows &a, int dt, hipStream_t s) {
 
 void tg_launch_rot_rows(void *rows, int ld, int n, int past, int first, int count, int stride, const TgRot &rot, int dt, hipStream_t s) {
 	const dim3 grid((unsigned)((count * (rot.dims / 2) + 255) / 256), (unsigned)n);
-	if (dt == TG_DT_BF16) hipLaunchKernelGGL((rot_rows_kernel<__bf16>), grid, dim3(256), 0, s, (__bf16 *)rows, ld, n, past, first, count, stride, rot);
-	else hipLaunchKernelGGL((rot_rows_kernel<float>), grid, dim3(256), 0, s, (float *)rows, ld, n, past, first, count, stride, rot);
+	if (dt == TG_DT_BF16) hipLaunchKernelGGL((rot_rows_kernel<__bf16>), grid, dim3(256), 0, s, (__bf16 *)rows, ld, past, first, count, stride, rot);
+	else hipLaunchKernelGGL((rot_rows_kernel<float>), grid, dim3(256), 0, s, (float *)rows, ld, past, first, count, stride, rot);
 }
 
 void tg_launch_key_values(const TgKeyValues &a, int dt, hipStream_t s) {

@@ -1314,7 +1314,7 @@ struct Pass {
 	const bool rms = c.norm == TG_NORM_RMS;
 	const size_t eb = tg_dt_bytes(dt);
 	hipStream_t s = n->stream;
-	TgRowsDyt d;                // state of the residual stream: what the next row step still adds
+	TgRowsDyt d = {};           // state of the residual stream: what the next row step still adds
 	const float *post = nullptr;  // (root mean square norms) weight of the norm behind the sublayer in r.sub; null: nothing waits
 	bool embed = true;
 	int due[2] = {-1, -1};      // blocks whose residual is complete behind the next row step
